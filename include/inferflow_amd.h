@@ -716,6 +716,48 @@ int ifa_moe_experts_glu_f32(int glu_kind, float limit, const void *h_f32, size_t
                             const void *gate_up_bf16, const void *down_bf16, const int *idx_dev, const void *wgt_f32, int ops32, void *ws, size_t ws_bytes,
                             void *y_f32, size_t ldy, int accumulate, ifa_stream stream);
 
+/* ---- ops of blocks with several residual streams and of the selective state space (Mamba-2) */
+/* Several residual streams per row, x fp32 [rows][streams][cols] (1 to 16 streams): what lies between two sub-layers in one launch, every stage optional:
+ * embed_bf16: X_s <- embed[token] * embed_scale for every s;  y_f32: X_t <- sum_s mix[s][t] X_s + mult * out[t] * y, all new streams from the
+ * old ones (mix_bf16 [streams][streams] indexed [from][to], out_bf16 [streams]; null: identity / ones);  u = sum_s in[s] X_s (in_bf16 null:
+ * ones), left in sum_f32 if given;  norm_w_bf16: h = u / sqrt(mean(u^2) + eps) * w. */
+int ifa_streams_step_f32(void *x_f32, size_t rows, int streams, size_t cols, const void *embed_bf16, const int *tokens_dev, int vocab, float embed_scale, const void *y_f32,
+                         size_t ldy, const void *mix_bf16, const void *out_bf16, float mult, const void *in_bf16, const void *norm_w_bf16, float eps, void *h_f32,
+                         size_t ldh, void *sum_f32, size_t ldsum, ifa_stream stream);
+/* ifa_shortconv_silu_f32 without unit norms, with a bias per channel in front of the SiLU (bias_bf16 [channels], nullable) */
+int ifa_shortconv_bias_silu_f32(const void *x_f32, size_t ldx, int channels, int taps, const void *w_bf16, const void *bias_bf16, const void *seqs_dev, const int *row_seq_dev,
+                                size_t rows, void *const *slot_base_dev, size_t state_off, void *y_f32, size_t ldy, ifa_stream stream);
+/* step sizes and decays of the state space: dt = softplus(a + dt_bias[h]), decay = exp(-exp(A_log[h]) dt); outputs fp32 [rows][heads] */
+int ifa_ssm_gates_f32(const void *a_f32, size_t lda, int heads, size_t rows, const void *a_log_bf16, const void *dt_bias_bf16, void *dt_f32, void *decay_f32,
+                      ifa_stream stream);
+/* selective state space: per head S [state][vdim] fp32 in the slot ([heads][state][vdim]), S <- decay_t S + dt_t B_t x_t^T,
+ * y_t = S^T C_t + D_h x_t; x fp32 [rows][heads * vdim], B / C fp32 [rows][groups * state] (head h reads group h / (heads / groups)),
+ * dt / decay fp32 [rows][heads], D bf16 [heads].  state <= 256.  Token by token. */
+int ifa_state_scan_ssm_f32(const void *x_f32, size_t ldx, const void *b_f32, size_t ldb, const void *c_f32, size_t ldc, int heads, int groups, int state, int vdim,
+                           const void *dt_f32, const void *decay_f32, const void *skip_bf16, const void *seqs_dev, int n_seqs, void *const *slot_base_dev, size_t state_off,
+                           void *out_f32, size_t ldo, ifa_stream stream);
+/* the gate in front of the norm: v = o * silu(gate); y = v / sqrt(mean_part(v^2) + eps) * w[c] in `groups` equal consecutive parts; y may be o */
+int ifa_gate_groupnorm_f32(const void *o_f32, size_t ldo, size_t rows, int channels, int groups, const void *w_bf16, const void *gate_f32, size_t ldg, float eps,
+                           void *y_f32, size_t ldy, ifa_stream stream);
+/* ifa_latent_prepare_f32 with a choice of the rotated pairs: pairing 0 = interleaved (2i, 2i + 1), 1 = halves (i, i + rot_dims / 2) */
+int ifa_latent_prepare_pairs_f32(int pairing, const void *kv_f32, size_t ldkv, int kv_rank, int rot_dim, int rot_dims, const void *c_norm_w_bf16, float eps,
+                                 void *q_f32, size_t ldq, int heads, int dim, const double *freq_f64_dev, float rot_mult, const void *seqs_dev,
+                                 const int *row_seq_dev, size_t rows, void *const *slot_base_dev, size_t cache_off, ifa_stream stream);
+/* ifa_latent_expand_out_f32 / ifa_attention_latent_tile_f32 with a choice of the gate: gate_cols 0 = sigmoid(g[t][h]) per head (g null: none),
+ * 1 = sigmoid(g[t][h * vdim + e]) per output column */
+int ifa_latent_expand_out_gated_f32(int gate_cols, const void *ol_f32, size_t ldol, int ld_head, int heads, int vdim, int kv_rank, const void *w_uv_bf16,
+                                    const void *g_f32, size_t ldg, size_t rows, void *out_f32, size_t ldo, ifa_stream stream);
+int ifa_attention_latent_tile_gated_f32(int gate_cols, const void *q_f32, size_t ldq, int heads, int dim, int rot_dim, int vdim, int kv_rank, float scale,
+                                        const void *kx_f32, size_t ldkx, const void *vx_f32, size_t ldvx, const int *ctx0_dev, const void *g_f32, size_t ldg,
+                                        const void *seqs_dev, const void *seqs_host, int n_seqs, void *const *slot_base_dev, size_t cache_off,
+                                        void *out_f32, size_t ldo, ifa_stream stream);
+/* ifa_moe_route_scores_f32 / ifa_moe_route_rows_scores_f32 with renormalized weights: renorm != 0: weight = score / (sum of the chosen
+ * scores + renorm_eps) * wgt_scale */
+int ifa_moe_route_renorm_f32(int score_kind, int renorm, float renorm_eps, float wgt_scale, const void *logits_f32, size_t ld, size_t rows, int n_all, int top,
+                             const void *correction_bf16, int *idx_dev, void *wgt_f32, ifa_stream stream);
+int ifa_moe_route_rows_renorm_f32(int score_kind, int renorm, float renorm_eps, float wgt_scale, const void *h_f32, size_t ldh, size_t rows, int width,
+                                  const void *router_bf16, int n_all, int top, const void *correction_bf16, int *idx_dev, void *wgt_f32, ifa_stream stream);
+
 /* ======================================================================== */
 /* Layer-list worker: a decoder whose layers are given one by one, each with its own sequence mixer, a 32-bit residual       */
 /* stream and bfloat16 weights (csrc/ifa_engine_layered.hip).  It is an ifa_model: finalize / kv_slots / select_kv /        */
@@ -730,17 +772,23 @@ enum { IFA_MIX_WINDOW_LINEAR = 1,   /* windowed softmax attention (values = keys
                                      * RMS norm of q and k per head, rotation of the first a_rot_dims dimensions (pairs i, i + a_rot_dims / 2),
                                      * values of their own size, optional sink (fixed score or learned per head), optional window, keys / values
                                      * of an earlier layer, optionally scaled frequencies, normed values, rotated values */
-       IFA_MIX_CHAN_DELTA = 5 };    /* generalized delta rule: decay and removal rate per head and key channel (the decay through a small
+       IFA_MIX_CHAN_DELTA = 5,      /* generalized delta rule: decay and removal rate per head and key channel (the decay through a small
                                      * two-matrix bottleneck), unit keys for the removal, per-head RMS norm x weight x sigmoid gate on the output */
+       IFA_MIX_SSM = 6 };           /* selective state space (Mamba-2): z | x | B | C | dt in one projection, short convolution with bias + SiLU over
+                                     * x | B | C, state per head, skip D x, SiLU gate in front of a grouped RMS norm */
 /* wiring of a layer.  PARALLEL: h = norm1(x); x <- x + ls1 * mixer(h) + ls2 * ffn(h).  POSTNORM: the sub-layers read x itself (plus a
  * short causal convolution of x when canon_taps > 0) and the grouped RMS norm sits on their OUTPUT: x <- x + norm1(mixer(x'));
  * x <- x + norm2(ffn(x')); with depth_avg the next layer reads sum_j dwa[j] X_j over the embedding output X_0 and every layer result.
  * SANDWICH: an RMS norm with weight (1 + w) before AND after each sub-layer: x <- x + norm1b(mixer(norm1(x))); x <- x + norm2b(ffn(norm2(x))).
- * PRENORM: x <- x + mixer(norm1(x)); x <- x + ffn(norm2(x)) with Dynamic Tanh norms tanh(alpha x) w + b (tensors IFA_LT_NORM1 / _B / _ALPHA). */
-enum { IFA_BLOCK_PARALLEL = 0, IFA_BLOCK_POSTNORM = 1, IFA_BLOCK_SANDWICH = 2, IFA_BLOCK_PRENORM = 3 };
+ * PRENORM: x <- x + mixer(norm1(x)); x <- x + ffn(norm2(x)) with Dynamic Tanh norms tanh(alpha x) w + b (tensors IFA_LT_NORM1 / _B / _ALPHA).
+ * STREAMS: cfg.streams residual streams X_s per token and RMS norms in front of the sub-layers q = 1, 2 (mixer, feed-forward): u = sum_s in_q[s] X_s,
+ * y = sub_q(norm_q(u)), X_t <- sum_s mix_q[s][t] X_s + cfg.residual_mult * out_q[t] y (tensors IFA_LT_HC1_* / IFA_LT_HC2_*; cfg.streams 0: one plain
+ * residual x <- x + residual_mult * sub(norm(x)), no such tensors). */
+enum { IFA_BLOCK_PARALLEL = 0, IFA_BLOCK_POSTNORM = 1, IFA_BLOCK_SANDWICH = 2, IFA_BLOCK_PRENORM = 3, IFA_BLOCK_STREAMS = 4 };
 enum { IFA_FFN_GATED = 0,           /* gated feed-forward (GELU tanh, biases), width `ffn` */
        IFA_FFN_MOE = 1,             /* mixture of experts: x_experts experts of width x_ff + x_identity identity experts, x_top per token */
-       IFA_FFN_CLAMPED = 2 };       /* width `ffn`, no biases: g = min(gate, f_limit), u = clamp(up, +-f_limit), y = down(g sigmoid(1.702 g) (u + 1)) */
+       IFA_FFN_CLAMPED = 2,         /* width `ffn`, no biases: g = min(gate, f_limit), u = clamp(up, +-f_limit), y = down(g sigmoid(1.702 g) (u + 1)) */
+       IFA_FFN_SILU = 3 };          /* width `ffn`, no biases: y = down(silu(gate) * up) */
 typedef struct {
     int mixer;                       /* IFA_MIX_* */
     int ffn;                         /* width of the gated feed-forward (GELU tanh, biases); 0 = none */
@@ -755,8 +803,9 @@ typedef struct {
     /* wiring (IFA_BLOCK_*), taps of the input convolution of both sub-layers (0: none), depth average on / off */
     int block, canon_taps, depth_avg;
     /* latent attention: heads of [m_dim unrotated | m_rot_dim rotated] query / key dimensions, values of m_vdim, latent of m_kv_rank;
-     * m_q_rank > 0: the queries go through an RMS-normed latent of that size; m_gate: a sigmoid gate per head on the output;
-     * the first m_rot_dims dimensions of the rotated part turn with base m_rot_base; m_yarn_factor > 0: YaRN frequency scaling */
+     * m_q_rank > 0: the queries go through an RMS-normed latent of that size; m_gate: a sigmoid gate on the output, 1 = per head, 2 = per output column;
+     * the first m_rot_dims dimensions of the rotated part turn with base m_rot_base (m_rot_halves 0: pairs (2i, 2i + 1), 1: pairs (i, i + m_rot_dims / 2));
+     * m_yarn_factor > 0: YaRN frequency scaling */
     int m_heads, m_dim, m_rot_dim, m_vdim, m_kv_rank, m_q_rank, m_gate, m_rot_dims;
     float m_scale, m_rot_base, m_yarn_factor, m_yarn_original, m_yarn_fast, m_yarn_slow;
     /* feed-forward kind (IFA_FFN_*) and the mixture's sizes */
@@ -786,6 +835,13 @@ typedef struct {
     /* mixture: x_score 0 softmax over all, 1 sigmoid per expert (x_route 0); x_glu 0 silu(gate) * up, 3 the clamped form with x_limit (x_gated 1) */
     int x_score, x_glu;
     float x_limit;
+    /* mixture: x_renorm 1: weights = chosen scores / (their sum + x_renorm_eps) * x_wgt_scale */
+    int x_renorm;
+    float x_renorm_eps, x_wgt_scale;
+    int m_rot_halves;
+    /* IFA_MIX_SSM: s_heads heads of s_vdim channels with states of s_state rows, B and C in s_groups groups, s_conv taps, output norm in
+     * s_norm_groups equal parts */
+    int s_heads, s_vdim, s_state, s_groups, s_conv, s_norm_groups;
 } ifa_layer_spec;
 typedef struct {
     int width, vocab, max_ctx, n_layers, device;
@@ -806,6 +862,10 @@ typedef struct {
      * states of its own; before every pass but the first the embedding output is added to the residual, and before every pass row t of
      * IFA_T_LOOP_STEP ([loop_times][width]).  loop_times 0: no group. */
     int loop_start, loop_stop, loop_times;
+    /* stem 4 (every layer wired IFA_BLOCK_STREAMS): the token embedding times embed_scale in every stream, the sum of the streams through an
+     * RMS norm before lm_head; a looped group repeats with nothing between its passes (no IFA_T_LOOP_STEP).  streams 0: one plain residual */
+    int streams;
+    float residual_mult;
 } ifa_layered_config;
 /* tensors of a layer-list model (global ones use IFA_T_EMBD / IFA_T_OUT_NORM / IFA_T_LM_HEAD with layer = -1) */
 enum {
@@ -822,6 +882,8 @@ enum {
     IFA_LT_X_ROUTER_B, IFA_LT_X_SH_GATE, IFA_LT_X_SH_UP, IFA_LT_X_SH_DOWN, IFA_LT_X_SH_SG,
     IFA_LT_NORM1_B, IFA_LT_NORM1_ALPHA, IFA_LT_NORM2_B, IFA_LT_NORM2_ALPHA,                       /* PRENORM: bias and scalar of the Dynamic Tanh norms */
     IFA_LT_C_R, IFA_LT_C_K, IFA_LT_C_V, IFA_LT_C_G, IFA_LT_C_A, IFA_LT_C_A_B, IFA_LT_C_W1, IFA_LT_C_W2, IFA_LT_C_W0, IFA_LT_C_NORM, IFA_LT_C_O,      /* IFA_MIX_CHAN_DELTA */
+    IFA_LT_HC1_IN, IFA_LT_HC1_OUT, IFA_LT_HC1_MIX, IFA_LT_HC2_IN, IFA_LT_HC2_OUT, IFA_LT_HC2_MIX,      /* STREAMS: [streams], [streams], [streams][streams] (from, to) */
+    IFA_LT_S_IN, IFA_LT_S_CONV, IFA_LT_S_CONV_B, IFA_LT_S_DTBIAS, IFA_LT_S_ALOG, IFA_LT_S_D, IFA_LT_S_NORM, IFA_LT_S_O,      /* IFA_MIX_SSM */
     IFA_LT_END
 };
 int ifa_model_create_layered(const ifa_layered_config *cfg, const ifa_layer_spec *layers, ifa_model **out);

@@ -202,6 +202,16 @@ SIGNATURES = {
     "ifa_moe_route_scores_f32": (_i, [_i, _vp, _sz, _sz, _i, _i, _vp, _vp, _vp, _vp]),
     "ifa_moe_route_rows_scores_f32": (_i, [_i, _vp, _sz, _sz, _i, _vp, _i, _i, _vp, _vp, _vp, _vp]),
     "ifa_moe_experts_glu_f32": (_i, [_i, _f, _vp, _sz, _sz, _i, _i, _i, _i, _vp, _vp, _vp, _vp, _i, _vp, _sz, _vp, _sz, _i, _vp]),
+    "ifa_streams_step_f32": (_i, [_vp, _sz, _i, _sz, _vp, _vp, _i, _f, _vp, _sz, _vp, _vp, _f, _vp, _vp, _f, _vp, _sz, _vp, _sz, _vp]),
+    "ifa_shortconv_bias_silu_f32": (_i, [_vp, _sz, _i, _i, _vp, _vp, _vp, _vp, _sz, _vp, _sz, _vp, _sz, _vp]),
+    "ifa_ssm_gates_f32": (_i, [_vp, _sz, _i, _sz, _vp, _vp, _vp, _vp, _vp]),
+    "ifa_state_scan_ssm_f32": (_i, [_vp, _sz, _vp, _sz, _vp, _sz, _i, _i, _i, _i, _vp, _vp, _vp, _vp, _i, _vp, _sz, _vp, _sz, _vp]),
+    "ifa_gate_groupnorm_f32": (_i, [_vp, _sz, _sz, _i, _i, _vp, _vp, _sz, _f, _vp, _sz, _vp]),
+    "ifa_latent_prepare_pairs_f32": (_i, [_i, _vp, _sz, _i, _i, _i, _vp, _f, _vp, _sz, _i, _i, _vp, _f, _vp, _vp, _sz, _vp, _sz, _vp]),
+    "ifa_latent_expand_out_gated_f32": (_i, [_i, _vp, _sz, _i, _i, _i, _i, _vp, _vp, _sz, _sz, _vp, _sz, _vp]),
+    "ifa_attention_latent_tile_gated_f32": (_i, [_i, _vp, _sz, _i, _i, _i, _i, _i, _f, _vp, _sz, _vp, _sz, _vp, _vp, _sz, _vp, _vp, _i, _vp, _sz, _vp, _sz, _vp]),
+    "ifa_moe_route_renorm_f32": (_i, [_i, _i, _f, _f, _vp, _sz, _sz, _i, _i, _vp, _vp, _vp, _vp]),
+    "ifa_moe_route_rows_renorm_f32": (_i, [_i, _i, _f, _f, _vp, _sz, _sz, _i, _vp, _i, _i, _vp, _vp, _vp, _vp]),
     "ifa_model_create_layered": (_i, [_vp, _vp, C.POINTER(_vp)]),
     "ifa_model_set_tensor_host": (_i, [_vp, _i, _i, _i, _vp, _sz, _sz]),
     "ifa_model_logits_f32": (_i, [_vp, C.POINTER(_vp), C.POINTER(_sz), C.POINTER(_sz)]),

@@ -8,11 +8,12 @@
 //   prompts         keys and values of the sequence's positions are expanded by two products over the cached latents
 //                   (ifa_linear_bf16w) and k_attn_latent_tile runs 128 queries of one sequence per workgroup on the fp32 matrix
 //                   cores, reading the rotated key part straight from the cache rows.
-// Rotation: interleaved pairs (2i, 2i + 1) of the first rot_dims dimensions of the rotated part turn by pos * freq[i]; the angle is
+// Rotation: pairs of the first rot_dims dimensions of the rotated part -- interleaved (2i, 2i + 1), or halves (i, i + rot_dims / 2) -- turn by pos * freq[i]; the angle is
 // formed in double (at position 1000 one fp32 ulp of an angle is 1e-4).
 #include <algorithm>
 #include "ifa_host.h"
 #include "ifa_f32_common.h"
+#include "inferflow_amd.h"
 
 using namespace ifa32;
 
@@ -22,7 +23,7 @@ namespace {
 __global__ void __launch_bounds__(256) k_latent_prepare(const float *__restrict__ kv, size_t ldkv, int R, int dr, int rdims, const bf16_t *__restrict__ cw, float eps,
                                                         float *__restrict__ q, size_t ldq, int heads, int dim, const double *__restrict__ freq, float mult,
                                                         const SeqDesc *__restrict__ seqs, const int *__restrict__ row_seq, float *const *__restrict__ slot_base,
-                                                        size_t cache_off)
+                                                        size_t cache_off, int halves)
 {
     extern __shared__ float cs[];          // [rdims / 2] cos, [rdims / 2] sin
     __shared__ float red[17];
@@ -41,18 +42,20 @@ __global__ void __launch_bounds__(256) k_latent_prepare(const float *__restrict_
     const float rinv = 1.0f / sqrtf(block_sum(s, red) / (float)R + eps);          // (the barrier inside also publishes cs)
     for (int c = tid; c < R; c += blockDim.x) row[c] = kr[c] * rinv * bf2f(cw[c]);
     for (int i = tid; i < half; i += blockDim.x) {
-        const float u = kr[R + 2 * i], v = kr[R + 2 * i + 1], co = cs[i], si = cs[half + i];
-        row[R + 2 * i] = u * co - v * si;
-        row[R + 2 * i + 1] = v * co + u * si;
+        const int a = halves ? i : 2 * i, b = halves ? i + half : 2 * i + 1;
+        const float u = kr[R + a], v = kr[R + b], co = cs[i], si = cs[half + i];
+        row[R + a] = u * co - v * si;
+        row[R + b] = v * co + u * si;
     }
     for (int c = rdims + tid; c < dr; c += blockDim.x) row[R + c] = kr[R + c];
     float *qr = q + (size_t)t * ldq;
     for (int e = tid; e < heads * half; e += blockDim.x) {
         const int h = e / half, i = e % half;
-        float *p = qr + (size_t)h * (dim + dr) + dim + 2 * i;
-        const float u = p[0], v = p[1], co = cs[i], si = cs[half + i];
+        float *p = qr + (size_t)h * (dim + dr) + dim + (halves ? i : 2 * i);
+        const int step = halves ? half : 1;
+        const float u = p[0], v = p[step], co = cs[i], si = cs[half + i];
         p[0] = u * co - v * si;
-        p[1] = v * co + u * si;
+        p[step] = v * co + u * si;
     }
 }
 
@@ -78,9 +81,10 @@ __global__ void __launch_bounds__(256) k_latent_absorb_q(const float *__restrict
     if (blockIdx.z == 0) for (int e = threadIdx.x; e < dr; e += blockDim.x) out[R + e] = qh[dim + e];
 }
 
-// grid (rows, groups of four output columns), a wave per column c = h * vdim + e: out[t][c] = gate[t][h] * sum_r W_uv[c][r] ol[t][h * ld_head + r]
+// grid (rows, groups of four output columns), a wave per column c = h * vdim + e: out[t][c] = gate * sum_r W_uv[c][r] ol[t][h * ld_head + r];
+// the gate's argument is g[t][h] (one per head) or g[t][c] (gate_cols: one per column)
 __global__ void __launch_bounds__(256) k_latent_expand_out(const float *__restrict__ ol, size_t ldol, int ld_head, int heads, int vdim, int R, const bf16_t *__restrict__ wuv,
-                                                           const float *__restrict__ g, size_t ldg, float *__restrict__ out, size_t ldo, int vec)
+                                                           const float *__restrict__ g, size_t ldg, int gate_cols, float *__restrict__ out, size_t ldo, int vec)
 {
     const int t = blockIdx.x, lane = threadIdx.x & 63, c = blockIdx.y * 4 + (threadIdx.x >> 6);
     if (c >= heads * vdim) return;
@@ -101,7 +105,7 @@ __global__ void __launch_bounds__(256) k_latent_expand_out(const float *__restri
         for (int r = lane; r < R; r += 64) acc = fmaf(bf2f(w[r]), src[r], acc);
     }
     acc = wave_sum(acc);
-    if (lane == 0) out[(size_t)t * ldo + c] = g ? acc * sigmoid_f(g[(size_t)t * ldg + h]) : acc;
+    if (lane == 0) out[(size_t)t * ldo + c] = g ? acc * sigmoid_f(g[(size_t)t * ldg + (gate_cols ? c : h)]) : acc;
 }
 
 // ---- single tokens, absorbed form: the cache rows are keys (kv_rank + rot_dim) and values (the first kv_rank) of ONE head that all
@@ -287,7 +291,7 @@ struct LatTileArgs {
     const float *kx; size_t ldkx;
     const float *vx; size_t ldvx;
     const int *ctx0;
-    const float *g; size_t ldg;
+    const float *g; size_t ldg; int gate_cols;
     const SeqDesc *seqs; int n_seqs;
     float *const *slot_base; size_t cache_off;
     float *out; size_t ldo;
@@ -421,10 +425,15 @@ __global__ void __launch_bounds__(256) k_attn_latent_tile(LatTileArgs P)
         for (int of = 16; of > 0; of >>= 1) ls += __shfl_xor(ls, of, 64);
         if (qq >= nq_w) continue;
         const size_t row = (size_t)(r0 + 32 * wave + qq);
-        const float gate = P.g ? sigmoid_f(P.g[row * P.ldg + h]) : 1.0f;
+        const float gate = P.g && !P.gate_cols ? sigmoid_f(P.g[row * P.ldg + h]) : 1.0f;
         const float sc = gate / ls;
 #pragma unroll
-        for (int nt = 0; nt < NTV; nt++) if (32 * nt + i < dv) P.out[row * P.ldo + (size_t)h * dv + 32 * nt + i] = o[nt][r] * sc;
+        for (int nt = 0; nt < NTV; nt++)
+            if (32 * nt + i < dv) {
+                const size_t c = (size_t)h * dv + 32 * nt + i;
+                const float v = o[nt][r] * sc;
+                P.out[row * P.ldo + c] = P.gate_cols ? v * sigmoid_f(P.g[row * P.ldg + c]) : v;
+            }
     }
 }
 
@@ -459,12 +468,21 @@ int ifa_latent_prepare_f32(const void *kv_f32, size_t ldkv, int kv_rank, int rot
                            void *q_f32, size_t ldq, int heads, int dim, const double *freq_f64_dev, float rot_mult, const void *seqs_dev,
                            const int *row_seq_dev, size_t rows, void *const *slot_base_dev, size_t cache_off, ifa_stream stream)
 {
+    return ifa_latent_prepare_pairs_f32(0, kv_f32, ldkv, kv_rank, rot_dim, rot_dims, c_norm_w_bf16, eps, q_f32, ldq, heads, dim, freq_f64_dev, rot_mult, seqs_dev, row_seq_dev,
+                                        rows, slot_base_dev, cache_off, stream);
+}
+
+int ifa_latent_prepare_pairs_f32(int pairing, const void *kv_f32, size_t ldkv, int kv_rank, int rot_dim, int rot_dims, const void *c_norm_w_bf16, float eps,
+                                 void *q_f32, size_t ldq, int heads, int dim, const double *freq_f64_dev, float rot_mult, const void *seqs_dev,
+                                 const int *row_seq_dev, size_t rows, void *const *slot_base_dev, size_t cache_off, ifa_stream stream)
+{
+    IFA_REQUIRE(pairing == 0 || pairing == 1, "ifa_latent_prepare_pairs_f32: pairing %d", pairing);
     IFA_REQUIRE(kv_f32 && c_norm_w_bf16 && q_f32 && freq_f64_dev && seqs_dev && row_seq_dev && slot_base_dev, "ifa_latent_prepare_f32: null pointer");
     IFA_REQUIRE(kv_rank > 0 && rot_dim >= 0 && rot_dims >= 0 && rot_dims <= rot_dim && rot_dims % 2 == 0 && heads > 0 && dim >= 0 && rows > 0
                 && ldkv >= (size_t)(kv_rank + rot_dim) && ldq >= (size_t)heads * (dim + rot_dim), "ifa_latent_prepare_f32: bad shape");
     hipLaunchKernelGGL(k_latent_prepare, dim3((unsigned)rows), dim3(256), (size_t)std::max(rot_dims, 2) * 4, ifa_s(stream), (const float *)kv_f32, ldkv, kv_rank, rot_dim,
                        rot_dims, (const bf16_t *)c_norm_w_bf16, eps, (float *)q_f32, ldq, heads, dim, freq_f64_dev, rot_mult, (const SeqDesc *)seqs_dev, row_seq_dev,
-                       (float *const *)slot_base_dev, cache_off);
+                       (float *const *)slot_base_dev, cache_off, pairing);
     IFA_LAUNCH_CHECK();
     return IFA_OK;
 }
@@ -485,14 +503,20 @@ int ifa_latent_absorb_q_f32(const void *q_f32, size_t ldq, int heads, int dim, i
 int ifa_latent_expand_out_f32(const void *ol_f32, size_t ldol, int ld_head, int heads, int vdim, int kv_rank, const void *w_uv_bf16,
                               const void *g_f32, size_t ldg, size_t rows, void *out_f32, size_t ldo, ifa_stream stream)
 {
+    return ifa_latent_expand_out_gated_f32(0, ol_f32, ldol, ld_head, heads, vdim, kv_rank, w_uv_bf16, g_f32, ldg, rows, out_f32, ldo, stream);
+}
+
+int ifa_latent_expand_out_gated_f32(int gate_cols, const void *ol_f32, size_t ldol, int ld_head, int heads, int vdim, int kv_rank, const void *w_uv_bf16,
+                                    const void *g_f32, size_t ldg, size_t rows, void *out_f32, size_t ldo, ifa_stream stream)
+{
     IFA_REQUIRE(ol_f32 && w_uv_bf16 && out_f32, "ifa_latent_expand_out_f32: null pointer");
     IFA_REQUIRE(heads > 0 && heads < 65536 && vdim > 0 && kv_rank > 0 && kv_rank <= 8192 && ld_head >= kv_rank && rows > 0 && ldol >= (size_t)(heads - 1) * ld_head + kv_rank
-                && ldo >= (size_t)heads * vdim && (!g_f32 || ldg >= (size_t)heads), "ifa_latent_expand_out_f32: bad shape");
+                && ldo >= (size_t)heads * vdim && (!g_f32 || ldg >= (size_t)heads * (gate_cols ? vdim : 1)) && (!gate_cols || g_f32), "ifa_latent_expand_out_f32: bad shape");
     IFA_REQUIRE((size_t)heads * vdim <= 4 * 65535, "ifa_latent_expand_out_f32: %d x %d output columns", heads, vdim);
     // 16-byte requests: whole 8-element pieces in every matrix row, every head's part of a latent row on a 16-byte boundary
     const int vec = (kv_rank % 8 == 0 && ld_head % 4 == 0 && ldol % 4 == 0 && ((uintptr_t)ol_f32 & 15) == 0 && ((uintptr_t)w_uv_bf16 & 15) == 0) ? 1 : 0;
     hipLaunchKernelGGL(k_latent_expand_out, dim3((unsigned)rows, ifa_cdiv((size_t)heads * vdim, 4)), dim3(256), 0, ifa_s(stream), (const float *)ol_f32, ldol, ld_head,
-                       heads, vdim, kv_rank, (const bf16_t *)w_uv_bf16, (const float *)g_f32, ldg, (float *)out_f32, ldo, vec);
+                       heads, vdim, kv_rank, (const bf16_t *)w_uv_bf16, (const float *)g_f32, ldg, gate_cols ? 1 : 0, (float *)out_f32, ldo, vec);
     IFA_LAUNCH_CHECK();
     return IFA_OK;
 }
@@ -541,15 +565,24 @@ int ifa_attention_latent_tile_f32(const void *q_f32, size_t ldq, int heads, int 
                                   const void *seqs_dev, const void *seqs_host, int n_seqs, void *const *slot_base_dev, size_t cache_off,
                                   void *out_f32, size_t ldo, ifa_stream stream)
 {
+    return ifa_attention_latent_tile_gated_f32(0, q_f32, ldq, heads, dim, rot_dim, vdim, kv_rank, scale, kx_f32, ldkx, vx_f32, ldvx, ctx0_dev, g_f32, ldg, seqs_dev, seqs_host,
+                                               n_seqs, slot_base_dev, cache_off, out_f32, ldo, stream);
+}
+
+int ifa_attention_latent_tile_gated_f32(int gate_cols, const void *q_f32, size_t ldq, int heads, int dim, int rot_dim, int vdim, int kv_rank, float scale,
+                                        const void *kx_f32, size_t ldkx, const void *vx_f32, size_t ldvx, const int *ctx0_dev, const void *g_f32, size_t ldg,
+                                        const void *seqs_dev, const void *seqs_host, int n_seqs, void *const *slot_base_dev, size_t cache_off,
+                                        void *out_f32, size_t ldo, ifa_stream stream)
+{
     IFA_REQUIRE(q_f32 && kx_f32 && vx_f32 && ctx0_dev && seqs_dev && seqs_host && slot_base_dev && out_f32, "ifa_attention_latent_tile_f32: null pointer");
     IFA_REQUIRE(heads > 0 && heads < 65536 && dim > 0 && rot_dim >= 0 && vdim > 0 && kv_rank > 0 && n_seqs > 0 && ldq >= (size_t)heads * (dim + rot_dim)
-                && ldkx >= (size_t)heads * dim && ldvx >= (size_t)heads * vdim && ldo >= (size_t)heads * vdim && (!g_f32 || ldg >= (size_t)heads),
+                && ldkx >= (size_t)heads * dim && ldvx >= (size_t)heads * vdim && ldo >= (size_t)heads * vdim && (!g_f32 || ldg >= (size_t)heads * (gate_cols ? vdim : 1)) && (!gate_cols || g_f32),
                 "ifa_attention_latent_tile_f32: bad shape");
     const int ntk = (dim + rot_dim + 31) / 32, ntv = (vdim + 31) / 32;
     IFA_REQUIRE(ifa_attention_latent_tile_fits(dim, rot_dim, vdim), "ifa_attention_latent_tile_f32: heads of %d + %d key and %d value dimensions exceed the tile kernel", dim, rot_dim, vdim);
     LatTileArgs P;
     P.q = (const float *)q_f32; P.ldq = ldq; P.heads = heads; P.dim = dim; P.dr = rot_dim; P.vdim = vdim; P.R = kv_rank; P.scale = scale;
-    P.kx = (const float *)kx_f32; P.ldkx = ldkx; P.vx = (const float *)vx_f32; P.ldvx = ldvx; P.ctx0 = ctx0_dev; P.g = (const float *)g_f32; P.ldg = ldg;
+    P.kx = (const float *)kx_f32; P.ldkx = ldkx; P.vx = (const float *)vx_f32; P.ldvx = ldvx; P.ctx0 = ctx0_dev; P.g = (const float *)g_f32; P.ldg = ldg; P.gate_cols = gate_cols ? 1 : 0;
     P.seqs = (const SeqDesc *)seqs_dev; P.n_seqs = n_seqs; P.slot_base = (float *const *)slot_base_dev; P.cache_off = cache_off; P.out = (float *)out_f32; P.ldo = ldo;
     // 16-byte requests: every source row and every part of a row starts on a 16-byte boundary
     P.vec = (dim % 4 == 0 && rot_dim % 4 == 0 && vdim % 4 == 0 && kv_rank % 4 == 0 && ldq % 4 == 0 && ldkx % 4 == 0 && ldvx % 4 == 0 && cache_off % 4 == 0

@@ -7,6 +7,7 @@
 //   windowed attention   K rows (normed keys) and V rows [max_ctx][kv_heads * dim] fp32, addressed by position
 //   linear attention     S [heads][dk][dv] fp32
 //   gated delta rule     S [heads][dk][dv] fp32 + the last conv - 1 inputs of the short convolutions
+//   state space          S [heads][state][vdim] fp32 + the last conv - 1 inputs of the short convolution
 // An arena is allocated when its slot is first used; a sequence that starts at position 0 ignores what the slot held.
 //
 // A step = a list of sequences (ifa_seq_desc): forward() is one sequence of n tokens from position prefix_len,
@@ -28,6 +29,11 @@
 // x <- x + ffn(norm2(x))), mix with the rotary attention (here with a learned sink per head, a sliding window, scaled frequencies, normed
 // values that enter the cache turned by their position and an output turned back) or with the generalized delta rule (IFA_MIX_CHAN_DELTA:
 // state S [dim][dim] per head in the slot), and feed forward through a mixture of clamped gated experts chosen by sigmoid scores.
+// Layers wired IFA_BLOCK_STREAMS keep several residual streams per token ([row][stream][width]) that every sub-layer reads through a learned mix
+// and writes back through another (x_t <- sum_s mix[s][t] x_s + mult * out[t] * sub(rms(sum_s in[s] x_s) w)): everything between two products
+// is ONE launch (ifa_streams_step_f32).  They mix with latent attention (rotation in halves, a gate per output column) or with the selective
+// state space (IFA_MIX_SSM: S [heads][state][vdim] + the convolution's last inputs in the slot) and feed forward through a dense SiLU-gated
+// layer or a mixture whose chosen sigmoid scores are renormalized.
 // A looped layer group runs several times with the same weights: every pass has cache rows and states of its own (a layer's part of the
 // arena is repeated per pass), so the stack is walked as a list of RUNS (layer, pass); stem 3 keeps the embedding output for the passes.
 #include <algorithm>
@@ -66,6 +72,7 @@ struct LLayer {
     // a layer of a looped group repeats its part of the arena per pass, pass_stride floats apart
     double *freq_v = nullptr;
     size_t c_cr = 0, c_ck = 0, c_cv = 0, c_cg = 0, c_ca = 0, c_cw = 0, pass_stride = 0;
+    // (the state space's projection is one matrix already: z at column 0, x | B | C behind it, then dt)
     LTensor &T(int id) { return t[id - IFA_LT_NORM1]; }
     const LTensor &T(int id) const { return t[id - IFA_LT_NORM1]; }
 };
@@ -133,15 +140,16 @@ bool expected_shape(const LayeredNet *n, const ifa_layer_spec &s, int li, int id
     vec = false;
     const bool par = s.mixer == IFA_MIX_WINDOW_LINEAR, del = s.mixer == IFA_MIX_GATED_DELTA, lat = s.mixer == IFA_MIX_LATENT, rot = s.mixer == IFA_MIX_ROTARY;
     const bool post = s.block == IFA_BLOCK_POSTNORM, sand = s.block == IFA_BLOCK_SANDWICH, pre = s.block == IFA_BLOCK_PRENORM, moe = has_moe(s);
-    const bool chan = s.mixer == IFA_MIX_CHAN_DELTA;
+    const bool chan = s.mixer == IFA_MIX_CHAN_DELTA, ssm = s.mixer == IFA_MIX_SSM, strm = s.block == IFA_BLOCK_STREAMS, hc = strm && n->cfg.streams > 0;
+    const size_t SI = (size_t)s.s_heads * s.s_vdim, SC = SI + 2 * (size_t)s.s_groups * s.s_state, NS = (size_t)n->cfg.streams;
     const size_t CH = (size_t)s.c_heads * s.c_dim;
-    const bool own_kv = rot && s.a_kv_layer == 0, gated = s.ffn > 0 && s.ffn_kind == IFA_FFN_GATED, any_ffn = s.ffn > 0 || moe;
+    const bool own_kv = rot && s.a_kv_layer == 0, gated = s.ffn > 0 && s.ffn_kind == IFA_FFN_GATED && !strm, any_ffn = s.ffn > 0 || moe;
     const size_t SF = (size_t)s.x_shared_ff;
     const size_t MH = (size_t)s.m_heads, MQ = MH * (size_t)(s.m_dim + s.m_rot_dim), MR = (size_t)s.m_kv_rank, XA = (size_t)(s.x_experts + s.x_identity);
     switch (id) {
     case IFA_LT_NORM1: r = 1; c = W; vec = true; return true;
-    case IFA_LT_LS1: r = 1; c = W; vec = true; return !post && !sand && !pre;
-    case IFA_LT_NORM2: r = 1; c = W; vec = true; return (post && moe) || ((sand || pre) && any_ffn);
+    case IFA_LT_LS1: r = 1; c = W; vec = true; return !post && !sand && !pre && !strm;
+    case IFA_LT_NORM2: r = 1; c = W; vec = true; return (post && moe) || ((sand || pre || strm) && any_ffn);
     case IFA_LT_NORM1_B: r = 1; c = W; vec = true; return pre;
     case IFA_LT_NORM1_ALPHA: r = 1; c = 1; vec = true; return pre;
     case IFA_LT_NORM2_B: r = 1; c = W; vec = true; return pre && any_ffn;
@@ -151,6 +159,16 @@ bool expected_shape(const LayeredNet *n, const ifa_layer_spec &s, int li, int id
     case IFA_LT_C_W1: r = (size_t)s.c_rank; c = W; return chan;
     case IFA_LT_C_W2: r = CH; c = (size_t)s.c_rank; return chan;
     case IFA_LT_C_O: r = W; c = CH; return chan;
+    case IFA_LT_HC1_IN: case IFA_LT_HC1_OUT: r = 1; c = NS; vec = true; return hc;
+    case IFA_LT_HC2_IN: case IFA_LT_HC2_OUT: r = 1; c = NS; vec = true; return hc && any_ffn;
+    case IFA_LT_HC1_MIX: r = NS; c = NS; return hc;
+    case IFA_LT_HC2_MIX: r = NS; c = NS; return hc && any_ffn;
+    case IFA_LT_S_IN: r = SI + SC + (size_t)s.s_heads; c = W; return ssm;
+    case IFA_LT_S_CONV: r = SC; c = (size_t)s.s_conv; return ssm;
+    case IFA_LT_S_CONV_B: r = 1; c = SC; vec = true; return ssm;
+    case IFA_LT_S_DTBIAS: case IFA_LT_S_ALOG: case IFA_LT_S_D: r = 1; c = (size_t)s.s_heads; vec = true; return ssm;
+    case IFA_LT_S_NORM: r = 1; c = SI; vec = true; return ssm;
+    case IFA_LT_S_O: r = W; c = SI; return ssm;
     case IFA_LT_NORM1B: r = 1; c = W; vec = true; return sand;
     case IFA_LT_NORM2B: r = 1; c = W; vec = true; return sand && any_ffn;
     case IFA_LT_A_V: r = (size_t)s.a_kv_heads * s.a_vdim; c = W; return own_kv;
@@ -174,10 +192,10 @@ bool expected_shape(const LayeredNet *n, const ifa_layer_spec &s, int li, int id
     case IFA_LT_M_DKV_NORM: r = 1; c = MR; vec = true; return lat;
     case IFA_LT_M_UK: r = MH * (size_t)s.m_dim; c = MR; return lat;
     case IFA_LT_M_UV: r = MH * (size_t)s.m_vdim; c = MR; return lat;
-    case IFA_LT_M_G: r = MH; c = W; return lat && s.m_gate;
+    case IFA_LT_M_G: r = s.m_gate == 2 ? MH * (size_t)s.m_vdim : MH; c = W; return lat && s.m_gate;
     case IFA_LT_M_O: r = W; c = MH * (size_t)s.m_vdim; return lat;
     case IFA_LT_X_ROUTER: r = XA; c = W; return moe;
-    case IFA_LT_X_CORR: r = 1; c = XA; vec = true; return moe && s.x_route == 0;
+    case IFA_LT_X_CORR: r = 1; c = XA; vec = true; return moe && s.x_route == 0 && !strm;
     case IFA_LT_X_UP: r = (size_t)s.x_experts * s.x_ff * (s.x_gated ? 2 : 1); c = W; return moe && s.x_experts > 0;
     case IFA_LT_X_DOWN: r = (size_t)s.x_experts * W; c = (size_t)s.x_ff; return moe && s.x_experts > 0;
     case IFA_LT_LS2: case IFA_LT_FFN_DOWN_B: r = 1; c = W; vec = true; return gated;
@@ -238,6 +256,9 @@ int ensure_slot(ifa_model *m, int slot)
     return IFA_OK;
 }
 
+// residual streams per row of n->x
+size_t streams_of(const LayeredNet *n) { return n->cfg.stem == 4 ? (size_t)std::max(n->cfg.streams, 1) : 1; }
+
 int ensure_rows(ifa_model *m, size_t T, size_t nseq)
 {
     LayeredNet *n = m->lay;
@@ -261,7 +282,7 @@ int ensure_rows(ifa_model *m, size_t T, size_t nseq)
         float **bufs[] = {&n->x, &n->h, &n->proj, &n->m1, &n->m2, &n->m3, &n->beta, &n->decay};
         for (float **b : bufs) { lay_free(*b); *b = nullptr; }
         const size_t W = (size_t)n->cfg.width;
-        const size_t sz[] = {W, W, n->n_in_max, n->mix_max, n->mix_max, std::max<size_t>(n->ffn_max, 4), std::max<size_t>(n->heads_max, 4), std::max<size_t>(n->heads_max, 4)};
+        const size_t sz[] = {W * streams_of(n), W, n->n_in_max, n->mix_max, n->mix_max, std::max<size_t>(n->ffn_max, 4), std::max<size_t>(n->heads_max, 4), std::max<size_t>(n->heads_max, 4)};
         for (size_t i = 0; i < 8; i++) IFA_HIP_CHECK(hipMalloc((void **)bufs[i], T * sz[i] * 4));
         {   // the single-row latent attention leaves at least one partial result per (row, head) in the workspace
             size_t need = 0;
@@ -277,7 +298,7 @@ int ensure_rows(ifa_model *m, size_t T, size_t nseq)
         n->m4 = n->m5 = n->stack = n->moe_wgt = nullptr; n->moe_idx = nullptr; n->moe_ws = nullptr; n->moe_ws_bytes = 0;
         lay_free(n->x0); lay_free(n->cg_decay); lay_free(n->cg_unit); lay_free(n->cg_rem);
         n->x0 = n->cg_decay = n->cg_unit = n->cg_rem = nullptr;
-        if (n->cfg.loop_times > 1) IFA_HIP_CHECK(hipMalloc((void **)&n->x0, T * W * 4));
+        if (n->cfg.loop_times > 1 && n->cfg.stem == 3) IFA_HIP_CHECK(hipMalloc((void **)&n->x0, T * W * 4));
         if (n->chan_max) {
             float **gb[] = {&n->cg_decay, &n->cg_unit, &n->cg_rem};
             for (float **b : gb) IFA_HIP_CHECK(hipMalloc((void **)b, T * n->chan_max * 4));
@@ -338,6 +359,53 @@ int post_step(ifa_model *m, size_t T, int nseq, bool fused, const float *sub, co
     return IFA_OK;
 }
 
+// latent attention over T rows of hin -> out (the output product): pass_off = offset of this pass's copy of the layer's part of the arena
+int run_latent_mixer(ifa_model *m, LLayer &L, size_t T, const float *hin, size_t pass_off, float *out)
+{
+    LayeredNet *n = m->lay;
+    const ifa_layered_config &c = n->cfg;
+    const ifa_layer_spec &sp = L.spec;
+    const size_t W = (size_t)c.width, NI = L.n_in, o_c = L.o_c + pass_off;
+    ifa_stream s = (ifa_stream)m->stream;
+    void *const *slots = (void *const *)n->slot_base_dev;
+    int rc;
+    const int H = sp.m_heads, dn = sp.m_dim, dr = sp.m_rot_dim, dv = sp.m_vdim, R = sp.m_kv_rank;
+    const size_t QD = (size_t)H * (dn + dr), CR = (size_t)(R + dr), OV = (size_t)H * dv;
+    if ((rc = linear(m, L.w_in, NI, W, hin, W, T, nullptr, nullptr, 1.0f, 0, n->proj, NI))) return rc;
+    float *q = n->proj + L.c_mq; size_t ldq = NI;
+    if (sp.m_q_rank > 0) {      // queries through their own normed latent
+        const size_t QR = (size_t)sp.m_q_rank;
+        if ((rc = ifa_layernorm_f32(0, n->proj + L.c_mq, NI, T, QR, L.T(IFA_LT_M_DQ_NORM).data, c.eps, n->m3, QR, s))) return rc;
+        if ((rc = linear(m, (const bf16_t *)L.T(IFA_LT_M_UQ).data, QD, QR, n->m3, QR, T, nullptr, nullptr, 1.0f, 0, n->m1, QD))) return rc;
+        q = n->m1; ldq = QD;
+    }
+    if ((rc = ifa_latent_prepare_pairs_f32(sp.m_rot_halves, n->proj + L.c_mkv, NI, R, dr, sp.m_rot_dims, L.T(IFA_LT_M_DKV_NORM).data, c.eps, q, ldq, H, dn, L.freq, L.rot_mult,
+                                     n->seqs_dev, n->row_seq_dev, T, slots, o_c, s))) return rc;
+    const float *gate = sp.m_gate ? n->proj + L.c_mg : nullptr;
+    if (n->step_expand) {
+        // keys and values of every position of the step's sequences from their cached latents, then the tiled kernel
+        const size_t ldk = (size_t)H * dn, ldv = OV;
+        for (size_t qi = 0; qi < n->seqs_host.size(); qi++) {
+            const ifa_seq_desc &sd = n->seqs_host[qi];
+            const float *lat = n->slot_ptr[(size_t)sd.slot] + o_c;
+            const size_t ctx = (size_t)sd.pos0 + sd.n, r0 = (size_t)n->ctx0_host[qi];
+            if ((rc = linear(m, (const bf16_t *)L.T(IFA_LT_M_UK).data, ldk, (size_t)R, lat, CR, ctx, nullptr, nullptr, 1.0f, 0, n->kx + r0 * ldk, ldk))) return rc;
+            if ((rc = linear(m, (const bf16_t *)L.T(IFA_LT_M_UV).data, ldv, (size_t)R, lat, CR, ctx, nullptr, nullptr, 1.0f, 0, n->vx + r0 * ldv, ldv))) return rc;
+        }
+        if ((rc = ifa_attention_latent_tile_gated_f32(sp.m_gate == 2, q, ldq, H, dn, dr, dv, R, sp.m_scale, n->kx, ldk, n->vx, ldv, n->ctx0_dev, gate, NI, n->seqs_dev, n->seqs_host.data(),
+                                                (int)n->seqs_host.size(), slots, o_c, n->m5, OV, s))) return rc;
+    } else {
+        // absorbed form: the cache rows are keys (whole) and values (latent part) of ONE head that all query heads share
+        const size_t QA = (size_t)H * CR;
+        if ((rc = ifa_latent_absorb_q_f32(q, ldq, H, dn, dr, R, L.T(IFA_LT_M_UK).data, T, n->m2, QA, s))) return rc;
+        if ((rc = ifa_attention_latent_rows_f32(n->m2, QA, H, R, dr, sp.m_scale, n->seqs_dev, n->row_seq_dev, T, slots, o_c, c.max_ctx, n->attn_ws, n->attn_ws_bytes,
+                                                n->m4, (size_t)H * R, s))) return rc;
+        if ((rc = ifa_latent_expand_out_gated_f32(sp.m_gate == 2, n->m4, (size_t)H * R, R, H, dv, R, L.T(IFA_LT_M_UV).data, gate, NI, T, n->m5, OV, s))) return rc;
+    }
+    if ((rc = linear(m, (const bf16_t *)L.T(IFA_LT_M_O).data, W, OV, n->m5, OV, T, nullptr, nullptr, 1.0f, 0, out, W))) return rc;
+    return IFA_OK;
+}
+
 // one POSTNORM layer over T rows: x <- x + norm1(mixer(x + conv1(x))); x <- x + norm2(experts(x + conv2(x))); depth average.
 // h_ready: the layer before has already left x + conv1(x) in n->h (its closing step ran this layer's input convolution);
 // next: the layer after, whose input convolution this layer's closing step runs when both are wired alike (*next_h_ready says so).
@@ -360,42 +428,7 @@ int run_postnorm_layer(ifa_model *m, LLayer &L, size_t li, size_t T, int nseq, b
         if (!h_ready && (rc = post_step(m, T, nseq, fused, nullptr, nullptr, nullptr, li, L.T(IFA_LT_CANON1).data, sp.canon_taps, L.o_cv1))) return rc;
         hin = n->h;
     }
-    {   // latent attention
-        const int H = sp.m_heads, dn = sp.m_dim, dr = sp.m_rot_dim, dv = sp.m_vdim, R = sp.m_kv_rank;
-        const size_t QD = (size_t)H * (dn + dr), CR = (size_t)(R + dr), OV = (size_t)H * dv;
-        if ((rc = linear(m, L.w_in, NI, W, hin, W, T, nullptr, nullptr, 1.0f, 0, n->proj, NI))) return rc;
-        float *q = n->proj + L.c_mq; size_t ldq = NI;
-        if (sp.m_q_rank > 0) {      // queries through their own normed latent
-            const size_t QR = (size_t)sp.m_q_rank;
-            if ((rc = ifa_layernorm_f32(0, n->proj + L.c_mq, NI, T, QR, L.T(IFA_LT_M_DQ_NORM).data, c.eps, n->m3, QR, s))) return rc;
-            if ((rc = linear(m, (const bf16_t *)L.T(IFA_LT_M_UQ).data, QD, QR, n->m3, QR, T, nullptr, nullptr, 1.0f, 0, n->m1, QD))) return rc;
-            q = n->m1; ldq = QD;
-        }
-        if ((rc = ifa_latent_prepare_f32(n->proj + L.c_mkv, NI, R, dr, sp.m_rot_dims, L.T(IFA_LT_M_DKV_NORM).data, c.eps, q, ldq, H, dn, L.freq, L.rot_mult,
-                                         n->seqs_dev, n->row_seq_dev, T, slots, L.o_c, s))) return rc;
-        const float *gate = sp.m_gate ? n->proj + L.c_mg : nullptr;
-        if (n->step_expand) {
-            // keys and values of every position of the step's sequences from their cached latents, then the tiled kernel
-            const size_t ldk = (size_t)H * dn, ldv = OV;
-            for (size_t qi = 0; qi < n->seqs_host.size(); qi++) {
-                const ifa_seq_desc &sd = n->seqs_host[qi];
-                const float *lat = n->slot_ptr[(size_t)sd.slot] + L.o_c;
-                const size_t ctx = (size_t)sd.pos0 + sd.n, r0 = (size_t)n->ctx0_host[qi];
-                if ((rc = linear(m, (const bf16_t *)L.T(IFA_LT_M_UK).data, ldk, (size_t)R, lat, CR, ctx, nullptr, nullptr, 1.0f, 0, n->kx + r0 * ldk, ldk))) return rc;
-                if ((rc = linear(m, (const bf16_t *)L.T(IFA_LT_M_UV).data, ldv, (size_t)R, lat, CR, ctx, nullptr, nullptr, 1.0f, 0, n->vx + r0 * ldv, ldv))) return rc;
-            }
-            if ((rc = ifa_attention_latent_tile_f32(q, ldq, H, dn, dr, dv, R, sp.m_scale, n->kx, ldk, n->vx, ldv, n->ctx0_dev, gate, NI, n->seqs_dev, n->seqs_host.data(),
-                                                    (int)n->seqs_host.size(), slots, L.o_c, n->m5, OV, s))) return rc;
-        } else {
-            // absorbed form: the cache rows are keys (whole) and values (latent part) of ONE head that all query heads share
-            const size_t QA = (size_t)H * CR;
-            if ((rc = ifa_latent_absorb_q_f32(q, ldq, H, dn, dr, R, L.T(IFA_LT_M_UK).data, T, n->m2, QA, s))) return rc;
-            if ((rc = ifa_attention_latent_rows_f32(n->m2, QA, H, R, dr, sp.m_scale, n->seqs_dev, n->row_seq_dev, T, slots, L.o_c, c.max_ctx, n->attn_ws, n->attn_ws_bytes,
-                                                    n->m4, (size_t)H * R, s))) return rc;
-            if ((rc = ifa_latent_expand_out_f32(n->m4, (size_t)H * R, R, H, dv, R, L.T(IFA_LT_M_UV).data, gate, NI, T, n->m5, OV, s))) return rc;
-        }
-        if ((rc = linear(m, (const bf16_t *)L.T(IFA_LT_M_O).data, W, OV, n->m5, OV, T, nullptr, nullptr, 1.0f, 0, n->m1, W))) return rc;
-    }
+    if ((rc = run_latent_mixer(m, L, T, hin, 0, n->m1))) return rc;
     const LLayer *depth_of = sp.depth_avg ? &L : nullptr;
     const void *ncw = next_conv ? next->T(IFA_LT_CANON1).data : nullptr;
     const int ntaps = next_conv ? next->spec.canon_taps : 0;
@@ -551,6 +584,83 @@ int run_prenorm_layer(ifa_model *m, LLayer &L, size_t T, int nseq, int pass, boo
                                    n->moe_wgt, c.ops32, n->moe_ws, n->moe_ws_bytes, n->x, W, 1, s);
 }
 
+// selective state space over T rows of h -> out (the output product)
+int run_ssm_mixer(ifa_model *m, LLayer &L, size_t T, int nseq, const float *h, size_t pass_off, float *out)
+{
+    LayeredNet *n = m->lay;
+    const ifa_layered_config &c = n->cfg;
+    const ifa_layer_spec &sp = L.spec;
+    const size_t W = (size_t)c.width, NI = L.n_in, SI = (size_t)sp.s_heads * sp.s_vdim, GN = (size_t)sp.s_groups * sp.s_state, SC = SI + 2 * GN;
+    ifa_stream s = (ifa_stream)m->stream;
+    void *const *slots = (void *const *)n->slot_base_dev;
+    const float *z = n->proj, *xbc = n->proj + SI, *dt = n->proj + SI + SC;
+    int rc;
+    if ((rc = linear(m, L.w_in, NI, W, h, W, T, nullptr, nullptr, 1.0f, 0, n->proj, NI))) return rc;
+    if ((rc = ifa_shortconv_bias_silu_f32(xbc, NI, (int)SC, sp.s_conv, L.T(IFA_LT_S_CONV).data, L.T(IFA_LT_S_CONV_B).data, n->seqs_dev, n->row_seq_dev, T, slots,
+                                          L.o_conv + pass_off, n->m1, SC, s))) return rc;
+    if ((rc = ifa_shortconv_tail_f32(xbc, NI, (int)SC, sp.s_conv, n->seqs_dev, nseq, slots, L.o_conv + pass_off, s))) return rc;
+    if ((rc = ifa_ssm_gates_f32(dt, NI, sp.s_heads, T, L.T(IFA_LT_S_ALOG).data, L.T(IFA_LT_S_DTBIAS).data, n->beta, n->decay, s))) return rc;
+    if ((rc = ifa_state_scan_ssm_f32(n->m1, SC, n->m1 + SI, SC, n->m1 + SI + GN, SC, sp.s_heads, sp.s_groups, sp.s_state, sp.s_vdim, n->beta, n->decay, L.T(IFA_LT_S_D).data,
+                                     n->seqs_dev, nseq, slots, L.o_rec + pass_off, n->m2, SI, s))) return rc;
+    if ((rc = ifa_gate_groupnorm_f32(n->m2, SI, T, (int)SI, sp.s_norm_groups, L.T(IFA_LT_S_NORM).data, z, NI, c.eps, n->m2, SI, s))) return rc;
+    return linear(m, (const bf16_t *)L.T(IFA_LT_S_O).data, W, SI, n->m2, SI, T, nullptr, nullptr, 1.0f, 0, out, W);
+}
+
+// What lies between two sub-layers of STREAMS layers: the sub-layer's output y into the streams with layer L's mixing weights (which = 1: mixer, 2:
+// feed-forward; y null: nothing), then what the next sub-layer reads into n->h: the read-out weights `in` (null: the plain sum) and the RMS
+// norm norm_w.  start: the streams begin with the step's token embeddings.  sum: where the sum of the streams goes (null: nowhere).
+int streams_step(ifa_model *m, size_t T, bool start, const float *y, LLayer *L, int which, const void *in, const void *norm_w)
+{
+    LayeredNet *n = m->lay;
+    const ifa_layered_config &c = n->cfg;
+    const size_t W = (size_t)c.width;
+    ifa_stream s = (ifa_stream)m->stream;
+    const int S = (int)streams_of(n);
+    const void *mix = y ? L->T(which == 1 ? IFA_LT_HC1_MIX : IFA_LT_HC2_MIX).data : nullptr, *out = y ? L->T(which == 1 ? IFA_LT_HC1_OUT : IFA_LT_HC2_OUT).data : nullptr;
+    if (n->opt_fuse_post)
+        return ifa_streams_step_f32(n->x, T, S, W, start ? n->embd.data : nullptr, n->tokens_dev, c.vocab, c.embed_scale, y, W, mix, out, c.residual_mult, in, norm_w, c.eps, n->h,
+                                    W, nullptr, 0, s);
+    int rc = ifa_streams_step_f32(n->x, T, S, W, start ? n->embd.data : nullptr, n->tokens_dev, c.vocab, c.embed_scale, y, W, mix, out, c.residual_mult, nullptr, nullptr, c.eps,
+                                  nullptr, 0, nullptr, 0, s);
+    if (!rc) rc = ifa_streams_step_f32(n->x, T, S, W, nullptr, nullptr, 0, 1.0f, nullptr, 0, nullptr, nullptr, 1.0f, in, norm_w, c.eps, n->h, W, nullptr, 0, s);
+    return rc;
+}
+
+// one STREAMS layer over T rows.  On entry n->h holds norm1 of what the mixer reads; on return norm1 of what `next`'s mixer reads (next null:
+// the norm in front of lm_head over the sum of the streams).
+int run_streams_layer(ifa_model *m, LLayer &L, size_t T, int nseq, int pass, LLayer *next)
+{
+    LayeredNet *n = m->lay;
+    const ifa_layered_config &c = n->cfg;
+    const ifa_layer_spec &sp = L.spec;
+    const size_t W = (size_t)c.width, po = (size_t)pass * L.pass_stride;
+    ifa_stream s = (ifa_stream)m->stream;
+    const bool moe = has_moe(sp), any_ffn = sp.ffn > 0 || moe;
+    const void *next_in = next ? next->T(IFA_LT_HC1_IN).data : nullptr, *next_norm = next ? next->T(IFA_LT_NORM1).data : n->out_norm.data;
+    int rc;
+    if ((rc = sp.mixer == IFA_MIX_LATENT ? run_latent_mixer(m, L, T, n->h, po, n->m3) : run_ssm_mixer(m, L, T, nseq, n->h, po, n->m3))) return rc;
+    if ((rc = streams_step(m, T, false, n->m3, &L, 1, any_ffn ? L.T(IFA_LT_HC2_IN).data : next_in, any_ffn ? L.T(IFA_LT_NORM2).data : next_norm))) return rc;
+    if (!any_ffn) return IFA_OK;
+    if (!moe) {
+        const size_t F = (size_t)sp.ffn, N2 = L.n_in2;
+        if ((rc = linear(m, L.w_in2, N2, W, n->h, W, T, nullptr, nullptr, 1.0f, 0, n->proj, N2))) return rc;
+        if ((rc = ifa_glu_f32(0, n->proj, N2, T, F, n->m3, F, s))) return rc;
+        if ((rc = linear(m, (const bf16_t *)L.T(IFA_LT_FFN_DOWN).data, W, F, n->m3, F, T, nullptr, nullptr, 1.0f, 0, n->m1, W))) return rc;
+    } else {
+        const int XA = sp.x_experts;
+        if (T <= 8 && XA <= 512) {      // a few rows: the router's product inside the choice's launch
+            if ((rc = ifa_moe_route_rows_renorm_f32(sp.x_score, sp.x_renorm, sp.x_renorm_eps, sp.x_wgt_scale, n->h, W, T, (int)W, L.T(IFA_LT_X_ROUTER).data, XA, sp.x_top, nullptr,
+                                                    n->moe_idx, n->moe_wgt, s))) return rc;
+        } else {
+            if ((rc = linear(m, (const bf16_t *)L.T(IFA_LT_X_ROUTER).data, (size_t)XA, W, n->h, W, T, nullptr, nullptr, 1.0f, 0, n->m2, (size_t)XA))) return rc;
+            if ((rc = ifa_moe_route_renorm_f32(sp.x_score, sp.x_renorm, sp.x_renorm_eps, sp.x_wgt_scale, n->m2, (size_t)XA, T, XA, sp.x_top, nullptr, n->moe_idx, n->moe_wgt, s))) return rc;
+        }
+        if ((rc = ifa_moe_experts_glu_f32(sp.x_glu, sp.x_limit, n->h, W, T, (int)W, sp.x_ff, sp.x_experts, sp.x_top, L.T(IFA_LT_X_UP).data, L.T(IFA_LT_X_DOWN).data, n->moe_idx,
+                                          n->moe_wgt, c.ops32, n->moe_ws, n->moe_ws_bytes, n->m1, W, 0, s))) return rc;
+    }
+    return streams_step(m, T, false, n->m1, &L, 2, next_in, next_norm);
+}
+
 // the layers of one step over T rows / nseq sequences whose tables are already on the device; leaves the residual in n->x
 int run_layers(ifa_model *m, size_t T, int nseq)
 {
@@ -571,7 +681,19 @@ int run_layers(ifa_model *m, size_t T, int nseq)
         if ((rc = ifa_embed_pair_scaled_f32(n->embd.data, c.vocab, c.width, c.embed_scale != 0.0f ? c.embed_scale : 1.0f, c.bigram_buckets > 0 ? n->bigram.data : nullptr,
                                             c.bigram_buckets, c.bigram_mul_prev, c.bigram_mul_cur, n->tokens_dev, n->seqs_dev, n->row_seq_dev, T, slots, n->o_prev, n->x,
                                             n->x0, s))) return rc;
-    } else if ((rc = ifa_embed_sinpos_f32(n->embd.data, c.vocab, c.width, n->tokens_dev, n->pos_dev, T, c.pos_base, n->x, s))) return rc;
+    } else if (c.stem == 0 && (rc = ifa_embed_sinpos_f32(n->embd.data, c.vocab, c.width, n->tokens_dev, n->pos_dev, T, c.pos_base, n->x, s))) return rc;
+    if (c.stem == 4) {
+        LLayer &L0 = n->layers[(size_t)n->runs[0].first];
+        if ((rc = streams_step(m, T, true, nullptr, nullptr, 0, L0.T(IFA_LT_HC1_IN).data, L0.T(IFA_LT_NORM1).data))) return rc;
+        for (size_t ri = 0; ri < n->runs.size(); ri++) {
+            LLayer *next = ri + 1 < n->runs.size() ? &n->layers[(size_t)n->runs[ri + 1].first] : nullptr;
+            if ((rc = run_streams_layer(m, n->layers[(size_t)n->runs[ri].first], T, nseq, n->runs[ri].second, next))) return rc;
+            if (n->opt_tap_layers && n->taps && T <= n->taps_rows
+                && (rc = ifa_streams_step_f32(n->x, T, (int)streams_of(n), W, nullptr, nullptr, 0, 1.0f, nullptr, 0, nullptr, nullptr, 1.0f, nullptr, nullptr, c.eps, nullptr, 0,
+                                              n->taps + ri * n->taps_rows * W, W, s))) return rc;
+        }
+        return IFA_OK;
+    }
     bool h_ready = false;
     for (size_t ri = 0; ri < n->runs.size(); ri++) {
         const size_t li = (size_t)n->runs[ri].first;
@@ -669,6 +791,9 @@ int out_norm_rows(ifa_model *m, const float *src, size_t rows, float *dst)
     const size_t W = (size_t)n->cfg.width;
     if (n->cfg.stem == 1) return ifa_group_rmsnorm_f32(src, W, rows, W, n->cfg.norm_groups, n->out_norm.data, n->cfg.eps, 0, dst, W, (ifa_stream)m->stream);
     if (n->cfg.stem == 2) return ifa_rmsnorm_offset_f32(src, W, rows, W, n->out_norm.data, 1.0f, n->cfg.eps, 0, dst, W, (ifa_stream)m->stream);
+    if (n->cfg.stem == 4)      // (the sum of a row's streams)
+        return ifa_streams_step_f32((void *)src, rows, (int)streams_of(n), W, nullptr, nullptr, 0, 1.0f, nullptr, 0, nullptr, nullptr, 1.0f, nullptr, n->out_norm.data, n->cfg.eps, dst,
+                                    W, nullptr, 0, (ifa_stream)m->stream);
     if (n->cfg.stem == 3) return ifa_dyt_f32(src, W, rows, W, n->out_norm_alpha.data, n->out_norm.data, n->out_norm_b.data, dst, W, (ifa_stream)m->stream);
     return ifa_layernorm_f32(1, src, W, rows, W, n->out_norm.data, n->cfg.eps, dst, W, (ifa_stream)m->stream);
 }
@@ -685,8 +810,9 @@ int run_head(ifa_model *m, size_t r0, size_t nr)
         n->logits_rows = nr;
         return IFA_OK;
     }
-    if ((rc = out_norm_rows(m, n->x + r0 * W, nr, n->h))) return rc;
-    if ((rc = linear(m, (const bf16_t *)n->lm_head.data, V, W, n->h, W, nr, nullptr, nullptr, logit_scale_of(n), 0, n->logits, V))) return rc;
+    const float *hn = n->cfg.stem == 4 ? n->h + r0 * W : n->h;      // (stem 4: the last layer's closing step has left the normed rows in n->h)
+    if (n->cfg.stem != 4 && (rc = out_norm_rows(m, n->x + r0 * W, nr, n->h))) return rc;
+    if ((rc = linear(m, (const bf16_t *)n->lm_head.data, V, W, hn, W, nr, nullptr, nullptr, logit_scale_of(n), 0, n->logits, V))) return rc;
     if (n->cfg.logit_softcap > 0.0f && (rc = ifa_softcap_f32(n->logits, nr * V, n->cfg.logit_softcap, (ifa_stream)m->stream))) return rc;
     n->logits_rows = nr;
     return IFA_OK;
@@ -747,7 +873,7 @@ int lay_finalize(ifa_model *m)
     IFA_REQUIRE((n->cfg.stem != 2 && n->cfg.stem != 3) || n->cfg.bigram_buckets <= 0 || n->bigram.present(), "layer-list worker: the token-pair embedding is missing");
     IFA_REQUIRE(n->cfg.stem != 3 || (n->out_norm_b.present() && n->out_norm_alpha.present()), "layer-list worker: bias or scalar of the final norm is missing");
     const bool looped = n->cfg.loop_times > 0 && n->cfg.loop_start < n->cfg.loop_stop;
-    IFA_REQUIRE(!looped || n->loop_step.present(), "layer-list worker: the vectors of the looped group's passes are missing");
+    IFA_REQUIRE(!looped || n->cfg.stem == 4 || n->loop_step.present(), "layer-list worker: the vectors of the looped group's passes are missing");
     size_t off = 0;
     if (n->cfg.stem == 2 || n->cfg.stem == 3) { n->o_prev = off; off += 4; }
     n->n_in_max = n->mix_max = n->ffn_max = n->heads_max = 4;
@@ -793,7 +919,7 @@ int lay_finalize(ifa_model *m)
             n->any_latent = true;
             if ((rc = ifa_attention_latent_rows_reserve(sp.m_kv_rank, sp.m_rot_dim))) return rc;      // (the single-token step may be captured)
             if (!ifa_attention_latent_tile_fits(sp.m_dim, sp.m_rot_dim, sp.m_vdim)) n->latent_tile_ok = false;
-            if (has_moe(sp)) {
+            if (has_moe(sp) && sp.block == IFA_BLOCK_POSTNORM) {
                 if (sp.canon_taps > 1) { L.o_cv2 = off; off += align4((size_t)(sp.canon_taps - 1) * W); }
                 n->mix_max = std::max(n->mix_max, (size_t)(sp.x_experts + sp.x_identity));
                 n->top_max = std::max(n->top_max, (size_t)sp.x_top);
@@ -882,6 +1008,14 @@ int lay_finalize(ifa_model *m)
                 n->top_max = std::max(n->top_max, (size_t)sp.x_top);
                 n->any_moe = true;
             }
+        } else if (sp.mixer == IFA_MIX_SSM) {
+            size_t at = 0;
+            if ((rc = cat_rows(w, b, L.T(IFA_LT_S_IN), nullptr, W, at, m->stream))) return rc;
+            const size_t SI = (size_t)sp.s_heads * sp.s_vdim, SC = SI + 2 * (size_t)sp.s_groups * sp.s_state;
+            L.o_rec = off; off += align4((size_t)sp.s_heads * sp.s_state * sp.s_vdim);
+            L.o_conv = off; off += align4((size_t)std::max(sp.s_conv - 1, 0) * SC);
+            n->mix_max = std::max({n->mix_max, SC, SI, W});
+            n->heads_max = std::max(n->heads_max, (size_t)sp.s_heads);
         } else if (sp.mixer == IFA_MIX_WINDOW_LINEAR) {
             if ((rc = cat_rows(w, b, L.T(IFA_LT_A_Q), nullptr, W, L.c_aq, m->stream)) || (rc = cat_rows(w, b, L.T(IFA_LT_A_K), nullptr, W, L.c_ak, m->stream))
                 || (rc = cat_rows(w, b, L.T(IFA_LT_L_Q), nullptr, W, L.c_lq, m->stream)) || (rc = cat_rows(w, b, L.T(IFA_LT_L_K), nullptr, W, L.c_lk, m->stream))
@@ -913,12 +1047,31 @@ int lay_finalize(ifa_model *m)
             n->mix_max = std::max({n->mix_max, (size_t)L.conv_ch, DV});
             n->heads_max = std::max(n->heads_max, (size_t)sp.d_heads);
         }
+        if (sp.block == IFA_BLOCK_STREAMS) {      // buffers of the feed-forward; dense: gate | up as one product of what norm2 leaves
+            n->ffn_max = std::max(n->ffn_max, W);          // (m3 takes the mixer's output)
+            n->mix_max = std::max(n->mix_max, W);
+            if (has_moe(sp)) {
+                n->mix_max = std::max(n->mix_max, (size_t)sp.x_experts);
+                n->top_max = std::max(n->top_max, (size_t)sp.x_top);
+                n->any_moe = true;
+            } else if (sp.ffn > 0) {
+                std::vector<bf16_t> w2, b2;
+                size_t at = 0;
+                if ((rc = cat_rows(w2, b2, L.T(IFA_LT_FFN_GATE), nullptr, W, L.c2_fg, m->stream)) || (rc = cat_rows(w2, b2, L.T(IFA_LT_FFN_UP), nullptr, W, at, m->stream))) return rc;
+                while (b2.size() % 4) { w2.resize(w2.size() + W, 0); b2.push_back(0); }
+                L.n_in2 = b2.size();
+                IFA_HIP_CHECK(hipMalloc((void **)&L.w_in2, w2.size() * 2));
+                IFA_HIP_CHECK(hipMemcpy(L.w_in2, w2.data(), w2.size() * 2, hipMemcpyHostToDevice));
+                n->n_in_max = std::max(n->n_in_max, L.n_in2);
+                n->ffn_max = std::max(n->ffn_max, (size_t)sp.ffn);
+            }
+        }
         // a layer of a looped group: its part of the arena once per pass
         if (looped && (int)li >= n->cfg.loop_start && (int)li < n->cfg.loop_stop && n->cfg.loop_times > 1) {
             L.pass_stride = off - off_layer;
             off += (size_t)(n->cfg.loop_times - 1) * L.pass_stride;
         }
-        if (sp.ffn > 0 && sp.block != IFA_BLOCK_SANDWICH) {
+        if (sp.ffn > 0 && sp.block != IFA_BLOCK_SANDWICH && sp.block != IFA_BLOCK_STREAMS) {
             size_t up_off;
             if ((rc = cat_rows(w, b, L.T(IFA_LT_FFN_GATE), &L.T(IFA_LT_FFN_GATE_B), W, L.c_fg, m->stream))
                 || (rc = cat_rows(w, b, L.T(IFA_LT_FFN_UP), &L.T(IFA_LT_FFN_UP_B), W, up_off, m->stream))) return rc;
@@ -936,7 +1089,7 @@ int lay_finalize(ifa_model *m)
         for (int id : {IFA_LT_A_Q, IFA_LT_A_K, IFA_LT_L_Q, IFA_LT_L_K, IFA_LT_L_V, IFA_LT_L_G, IFA_LT_D_Q, IFA_LT_D_K, IFA_LT_D_V, IFA_LT_D_B, IFA_LT_D_A,
                        IFA_LT_D_G, IFA_LT_FFN_GATE, IFA_LT_FFN_UP, IFA_LT_M_Q, IFA_LT_M_DQ, IFA_LT_M_DKV, IFA_LT_M_G, IFA_LT_A_V, IFA_LT_A_Q_B, IFA_LT_A_K_B,
                        IFA_LT_A_V_B, IFA_LT_X_ROUTER_B, IFA_LT_X_SH_GATE, IFA_LT_X_SH_UP, IFA_LT_X_SH_SG, IFA_LT_C_R, IFA_LT_C_K, IFA_LT_C_V, IFA_LT_C_G, IFA_LT_C_A,
-                       IFA_LT_C_A_B, IFA_LT_C_W1}) {
+                       IFA_LT_C_A_B, IFA_LT_C_W1, IFA_LT_S_IN}) {
             LTensor &t = L.T(id);
             if (t.data) { lay_free(t.data); t.data = nullptr; }
         }
@@ -1127,7 +1280,7 @@ int lay_step(ifa_model *m, int nseq, const int *tokens_host, const int *lens, co
     } else {
         // the sequences' last rows, normed one by one into consecutive rows of h, then one product
         for (int q = 0; q < nseq; q++)
-            if ((rc = out_norm_rows(m, n->x + (size_t)last[(size_t)q] * W, 1, n->h + (size_t)q * W))) return rc;
+            if ((rc = out_norm_rows(m, n->x + (size_t)last[(size_t)q] * W * streams_of(n), 1, n->h + (size_t)q * W))) return rc;
         if ((rc = linear(m, (const bf16_t *)n->lm_head.data, V, W, n->h, W, (size_t)nseq, nullptr, nullptr, logit_scale_of(n), 0, n->logits, V))) return rc;
         if (n->cfg.logit_softcap > 0.0f && (rc = ifa_softcap_f32(n->logits, (size_t)nseq * V, n->cfg.logit_softcap, s))) return rc;
         n->logits_rows = (size_t)nseq;
@@ -1261,11 +1414,24 @@ int ifa_model_create_layered(const ifa_layered_config *cfg, const ifa_layer_spec
         } else if (s.mixer == IFA_MIX_CHAN_DELTA) {
             IFA_REQUIRE(s.c_heads > 0 && s.c_dim > 0 && s.c_dim <= 256 && s.c_rank >= 1 && s.c_rank <= 8192 && s.c_decay_mult > 0.0f && s.c_l2_eps >= 0.0f,
                         "ifa_model_create_layered: layer %d: bad sizes of the generalized delta rule", l);
+        } else if (s.mixer == IFA_MIX_SSM) {
+            IFA_REQUIRE(s.s_heads > 0 && s.s_vdim > 0 && s.s_state > 0 && s.s_state <= 256 && s.s_groups > 0 && s.s_heads % s.s_groups == 0 && s.s_conv >= 1 && s.s_conv <= 64
+                        && s.s_norm_groups > 0 && ((size_t)s.s_heads * s.s_vdim) % (size_t)s.s_norm_groups == 0,
+                        "ifa_model_create_layered: layer %d: bad state-space sizes", l);
         } else return ifa_fail(IFA_ERR_ARG, "ifa_model_create_layered: layer %d: unknown mixer %d", l, s.mixer);
-        const bool wired = s.mixer == IFA_MIX_LATENT ? s.block == IFA_BLOCK_POSTNORM
+        const bool wired = s.mixer == IFA_MIX_LATENT ? (s.block == IFA_BLOCK_POSTNORM || s.block == IFA_BLOCK_STREAMS)
+                           : s.mixer == IFA_MIX_SSM ? s.block == IFA_BLOCK_STREAMS
                            : s.mixer == IFA_MIX_ROTARY ? (s.block == IFA_BLOCK_SANDWICH || s.block == IFA_BLOCK_PRENORM)
                            : s.mixer == IFA_MIX_CHAN_DELTA ? s.block == IFA_BLOCK_PRENORM : s.block == IFA_BLOCK_PARALLEL;
         IFA_REQUIRE(wired, "ifa_model_create_layered: layer %d: mixer %d is not wired for block kind %d", l, s.mixer, s.block);
+        IFA_REQUIRE((s.block == IFA_BLOCK_STREAMS) == (cfg->stem == 4), "ifa_model_create_layered: layer %d: block kind %d with stem %d", l, s.block, cfg->stem);
+        if (s.block == IFA_BLOCK_STREAMS) {
+            if (s.ffn_kind == IFA_FFN_MOE && s.x_experts + s.x_identity > 0)
+                IFA_REQUIRE(s.ffn == 0 && s.x_identity == 0 && s.x_gated == 1 && s.x_route == 0 && s.x_shared_ff == 0 && s.x_experts >= 1 && s.x_experts <= 4096 && s.x_top >= 1
+                            && s.x_top <= s.x_experts && s.x_ff > 0 && (s.x_score == 0 || s.x_score == 1) && (s.x_glu == 0 || (s.x_glu == 3 && s.x_limit > 0.0f)),
+                            "ifa_model_create_layered: layer %d: bad mixture-of-experts sizes", l);
+            else IFA_REQUIRE(s.ffn == 0 || s.ffn_kind == IFA_FFN_SILU, "ifa_model_create_layered: layer %d: this wiring takes the SiLU-gated feed-forward or a mixture", l);
+        } else
         if (s.block == IFA_BLOCK_PRENORM) {
             IFA_REQUIRE(s.ffn == 0 && s.a_kv_layer == 0, "ifa_model_create_layered: layer %d: this wiring takes a mixture of experts or no feed-forward, and keys of its own", l);
             if (s.ffn_kind == IFA_FFN_MOE && s.x_experts + s.x_identity > 0)
@@ -1287,14 +1453,15 @@ int ifa_model_create_layered(const ifa_layered_config *cfg, const ifa_layer_spec
                             && (s.x_experts == 0 || s.x_ff > 0), "ifa_model_create_layered: layer %d: bad mixture-of-experts sizes", l);
         } else IFA_REQUIRE(s.ffn_kind == IFA_FFN_GATED, "ifa_model_create_layered: layer %d: this wiring takes the gated feed-forward with biases", l);
     }
-    IFA_REQUIRE(cfg->stem == 0 || (cfg->stem == 1 && cfg->norm_groups >= 1 && cfg->width % cfg->norm_groups == 0)
+    IFA_REQUIRE(cfg->stem != 4 || (cfg->streams >= 0 && cfg->streams <= 16), "ifa_model_create_layered: %d residual streams (0 to 16)", cfg->streams);
+    IFA_REQUIRE(cfg->stem == 0 || cfg->stem == 4 || (cfg->stem == 1 && cfg->norm_groups >= 1 && cfg->width % cfg->norm_groups == 0)
                 || ((cfg->stem == 2 || cfg->stem == 3) && cfg->bigram_buckets >= 0 && cfg->bigram_buckets < (1 << 30)), "ifa_model_create_layered: bad stem");
     if (cfg->loop_times > 0 && cfg->loop_start < cfg->loop_stop) {
         IFA_REQUIRE(cfg->loop_start >= 0 && cfg->loop_stop <= cfg->n_layers && cfg->loop_times <= 1024, "ifa_model_create_layered: looped group [%d, %d) x %d of %d layers",
                     cfg->loop_start, cfg->loop_stop, cfg->loop_times, cfg->n_layers);
         for (int l = cfg->loop_start; l < cfg->loop_stop; l++)
-            IFA_REQUIRE(layers[l].block == IFA_BLOCK_PRENORM, "ifa_model_create_layered: layer %d of the looped group is not wired with norms in front of its sub-layers", l);
-        IFA_REQUIRE(cfg->loop_times == 1 || cfg->stem == 3, "ifa_model_create_layered: a looped group of several passes needs the stem that keeps the embedding output");
+            IFA_REQUIRE(layers[l].block == IFA_BLOCK_PRENORM || layers[l].block == IFA_BLOCK_STREAMS, "ifa_model_create_layered: layer %d of the looped group is not wired with norms in front of its sub-layers", l);
+        IFA_REQUIRE(cfg->loop_times == 1 || cfg->stem == 3 || cfg->stem == 4, "ifa_model_create_layered: a looped group of several passes needs the stem that keeps the embedding output");
     }
     IFA_HIP_CHECK(hipSetDevice(cfg->device));
     ifa_model *m = new ifa_model();
@@ -1331,7 +1498,7 @@ int ifa_model_set_tensor_host(ifa_model *m, int layer, int tensor_id, int dtype,
         else if (tensor_id == IFA_T_BIGRAM && (n->cfg.stem == 2 || n->cfg.stem == 3) && n->cfg.bigram_buckets > 0) { t = &n->bigram; er = (size_t)n->cfg.bigram_buckets + 1; ec = W; }
         else if (tensor_id == IFA_T_OUT_NORM_B && n->cfg.stem == 3) { t = &n->out_norm_b; er = 1; ec = W; vec = true; }
         else if (tensor_id == IFA_T_OUT_NORM_ALPHA && n->cfg.stem == 3) { t = &n->out_norm_alpha; er = 1; ec = 1; vec = true; }
-        else if (tensor_id == IFA_T_LOOP_STEP && n->cfg.loop_times > 0) { t = &n->loop_step; er = (size_t)n->cfg.loop_times; ec = W; }
+        else if (tensor_id == IFA_T_LOOP_STEP && n->cfg.loop_times > 0 && n->cfg.stem != 4) { t = &n->loop_step; er = (size_t)n->cfg.loop_times; ec = W; }
         else return ifa_fail(IFA_ERR_ARG, "ifa_model_set_tensor_host: global tensor id %d", tensor_id);
     } else {
         IFA_REQUIRE(layer < (int)n->layers.size() && tensor_id >= IFA_LT_NORM1 && tensor_id < IFA_LT_END, "ifa_model_set_tensor_host: layer %d / tensor id %d", layer, tensor_id);

@@ -1,6 +1,7 @@
 // ifa_moe_f32.hip -- mixture of experts on 32-bit activations with bfloat16 expert matrices:
 //   router   scores = softmax(logits) over `experts` feed-forward experts followed by `identity` identity experts; the `top` largest
 //            (score + correction) are chosen, their weights are the plain scores (not renormalized)
+//            (renorm: the chosen scores are divided by their sum and multiplied by a scale)
 //            (second kind, k_moe_route_top: the `top` largest logit + bias, weights = softmax over the chosen values only)
 //   experts  y[t] (+)= sum_k wgt[t][k] * E_{idx[t][k]}(h[t]),  E_e(h) = W_down[e] act(W_up[e] h),  identity: E(h) = h
 //            (gated experts: E_e(h) = W_down[e] (silu(W_gate[e] h) * (W_up[e] h)), gate and up rows of an expert stored back to back)
@@ -25,7 +26,7 @@ __device__ __forceinline__ float gelu_erf_f(float z) { return 0.5f * z * (1.0f +
 // one wave per row: softmax over n_all logits, then `top` passes of argmax over score + correction (lowest index on ties)
 // (score_kind 1: the scores are the sigmoids of the logits instead of their softmax)
 __global__ void __launch_bounds__(64) k_moe_route(const float *__restrict__ logits, size_t ld, int n_all, int top, const bf16_t *__restrict__ corr,
-                                                  int *__restrict__ idx, float *__restrict__ wgt, int score_kind)
+                                                  int *__restrict__ idx, float *__restrict__ wgt, int score_kind, int renorm, float renorm_eps, float wgt_scale)
 {
     extern __shared__ float sc[];          // [n_all] scores, [n_all] choice scores
     float *ch = sc + n_all;
@@ -43,6 +44,7 @@ __global__ void __launch_bounds__(64) k_moe_route(const float *__restrict__ logi
         for (int e = lane; e < n_all; e += 64) { const float s = sc[e] / sum; sc[e] = s; ch[e] = s + (corr ? bf2f(corr[e]) : 0.0f); }
     }
     __syncthreads();
+    float sum = 0.0f;          // (lane 0: of the chosen scores)
     for (int k = 0; k < top; k++) {
         float best = -INFINITY; int bi = 0x7FFFFFFF;
         for (int e = lane; e < n_all; e += 64) { const float v = ch[e]; if (v > best || (v == best && e < bi)) { best = v; bi = e; } }
@@ -50,9 +52,10 @@ __global__ void __launch_bounds__(64) k_moe_route(const float *__restrict__ logi
             const float ov = __shfl_xor(best, o, 64); const int oi = __shfl_xor(bi, o, 64);
             if (ov > best || (ov == best && oi < bi)) { best = ov; bi = oi; }
         }
-        if (lane == 0) { idx[(size_t)t * top + k] = bi; wgt[(size_t)t * top + k] = sc[bi]; ch[bi] = -INFINITY; }
+        if (lane == 0) { idx[(size_t)t * top + k] = bi; wgt[(size_t)t * top + k] = sc[bi]; ch[bi] = -INFINITY; sum += sc[bi]; }
         __syncthreads();
     }
+    if (renorm && lane == 0) { const float den = sum + renorm_eps; for (int k = 0; k < top; k++) wgt[(size_t)t * top + k] = wgt[(size_t)t * top + k] / den * wgt_scale; }
 }
 
 // one wave per row: `top` passes of argmax over logit + bias (lowest index on ties), then the softmax over the chosen values
@@ -88,7 +91,7 @@ __global__ void __launch_bounds__(64) k_moe_route_top(const float *__restrict__ 
 __global__ void __launch_bounds__(1024) k_moe_route_rows(const float *h, size_t ldh, int W, const bf16_t *__restrict__ router, int n_all, int top,
                                                         const bf16_t *__restrict__ corr, int *__restrict__ idx, float *__restrict__ wgt, int vec, int score_kind,
                                                         const float *__restrict__ x, size_t ldx, const bf16_t *__restrict__ alpha, const bf16_t *__restrict__ nw_,
-                                                        const bf16_t *__restrict__ nb_, float *h_out)
+                                                        const bf16_t *__restrict__ nb_, float *h_out, int renorm, float renorm_eps, float wgt_scale)
 {
     extern __shared__ float sc[];          // [n_all] logits, then scores; [n_all] choice scores
     float *ch = sc + n_all;
@@ -131,6 +134,7 @@ __global__ void __launch_bounds__(1024) k_moe_route_rows(const float *h, size_t 
         for (int e = lane; e < n_all; e += 64) { const float sv = sc[e] / sum; sc[e] = sv; ch[e] = sv + (corr ? bf2f(corr[e]) : 0.0f); }
     }
     __syncthreads();
+    float chosen = 0.0f;          // (thread 0: the sum of the chosen scores)
     for (int k = 0; k < top; k++) {
         if (wave == 0) {
             float best = -INFINITY; int bi = 0x7FFFFFFF;
@@ -139,10 +143,11 @@ __global__ void __launch_bounds__(1024) k_moe_route_rows(const float *h, size_t 
                 const float ov = __shfl_xor(best, o, 64); const int oi = __shfl_xor(bi, o, 64);
                 if (ov > best || (ov == best && oi < bi)) { best = ov; bi = oi; }
             }
-            if (lane == 0) { idx[(size_t)t * top + k] = bi; wgt[(size_t)t * top + k] = sc[bi]; ch[bi] = -INFINITY; }
+            if (lane == 0) { idx[(size_t)t * top + k] = bi; wgt[(size_t)t * top + k] = sc[bi]; ch[bi] = -INFINITY; chosen += sc[bi]; }
         }
         __syncthreads();
     }
+    if (renorm && threadIdx.x == 0) { const float den = chosen + renorm_eps; for (int k = 0; k < top; k++) wgt[(size_t)t * top + k] = wgt[(size_t)t * top + k] / den * wgt_scale; }
 }
 
 // grid (ff chunks, pairs): act[p][n] = gelu(W_up[e][n] . h[t]); a wave per n at a time.  Identity pairs do nothing.
@@ -315,11 +320,17 @@ extern "C" {
 int ifa_moe_route_scores_f32(int score_kind, const void *logits_f32, size_t ld, size_t rows, int n_all, int top, const void *correction_bf16, int *idx_dev,
                              void *wgt_f32, ifa_stream stream)
 {
+    return ifa_moe_route_renorm_f32(score_kind, 0, 0.0f, 1.0f, logits_f32, ld, rows, n_all, top, correction_bf16, idx_dev, wgt_f32, stream);
+}
+
+int ifa_moe_route_renorm_f32(int score_kind, int renorm, float renorm_eps, float wgt_scale, const void *logits_f32, size_t ld, size_t rows, int n_all, int top,
+                             const void *correction_bf16, int *idx_dev, void *wgt_f32, ifa_stream stream)
+{
     IFA_REQUIRE(logits_f32 && idx_dev && wgt_f32, "ifa_moe_route_scores_f32: null pointer");
     IFA_REQUIRE(rows > 0 && n_all >= 1 && n_all <= 4096 && top >= 1 && top <= n_all && ld >= (size_t)n_all && (score_kind == 0 || score_kind == 1),
                 "ifa_moe_route_scores_f32: bad shape (%d router outputs, %d chosen, scores of kind %d)", n_all, top, score_kind);
     hipLaunchKernelGGL(k_moe_route, dim3((unsigned)rows), dim3(64), (size_t)n_all * 8, ifa_s(stream), (const float *)logits_f32, ld, n_all, top,
-                       (const bf16_t *)correction_bf16, idx_dev, (float *)wgt_f32, score_kind);
+                       (const bf16_t *)correction_bf16, idx_dev, (float *)wgt_f32, score_kind, renorm ? 1 : 0, renorm_eps, wgt_scale);
     IFA_LAUNCH_CHECK();
     return IFA_OK;
 }
@@ -339,13 +350,19 @@ int ifa_moe_route_rows_f32(const void *h_f32, size_t ldh, size_t rows, int width
 int ifa_moe_route_rows_scores_f32(int score_kind, const void *h_f32, size_t ldh, size_t rows, int width, const void *router_bf16, int n_all, int top,
                                   const void *correction_bf16, int *idx_dev, void *wgt_f32, ifa_stream stream)
 {
+    return ifa_moe_route_rows_renorm_f32(score_kind, 0, 0.0f, 1.0f, h_f32, ldh, rows, width, router_bf16, n_all, top, correction_bf16, idx_dev, wgt_f32, stream);
+}
+
+int ifa_moe_route_rows_renorm_f32(int score_kind, int renorm, float renorm_eps, float wgt_scale, const void *h_f32, size_t ldh, size_t rows, int width,
+                                  const void *router_bf16, int n_all, int top, const void *correction_bf16, int *idx_dev, void *wgt_f32, ifa_stream stream)
+{
     IFA_REQUIRE(h_f32 && router_bf16 && idx_dev && wgt_f32, "ifa_moe_route_rows_f32: null pointer");
     IFA_REQUIRE(rows > 0 && rows <= 64 && width > 0 && n_all >= 1 && n_all <= 4096 && top >= 1 && top <= n_all && ldh >= (size_t)width && (score_kind == 0 || score_kind == 1),
                 "ifa_moe_route_rows_f32: bad shape");
     const int vec = (width % 8 == 0 && ldh % 4 == 0 && ((uintptr_t)h_f32 & 15) == 0 && ((uintptr_t)router_bf16 & 15) == 0) ? 1 : 0;
     hipLaunchKernelGGL(k_moe_route_rows, dim3((unsigned)rows), dim3(n_all > 8 ? 1024 : 256), (size_t)n_all * 8, ifa_s(stream), (const float *)h_f32, ldh, width,
                        (const bf16_t *)router_bf16, n_all, top, (const bf16_t *)correction_bf16, idx_dev, (float *)wgt_f32, vec, score_kind, (const float *)nullptr, (size_t)0,
-                       (const bf16_t *)nullptr, (const bf16_t *)nullptr, (const bf16_t *)nullptr, (float *)nullptr);
+                       (const bf16_t *)nullptr, (const bf16_t *)nullptr, (const bf16_t *)nullptr, (float *)nullptr, renorm ? 1 : 0, renorm_eps, wgt_scale);
     IFA_LAUNCH_CHECK();
     return IFA_OK;
 }
@@ -360,7 +377,7 @@ int ifa_moe_dyt_route_rows_f32(int score_kind, const void *x_f32, size_t ldx, co
     const int vec = (width % 8 == 0 && ldh % 4 == 0 && ((uintptr_t)h_f32 & 15) == 0 && ((uintptr_t)router_bf16 & 15) == 0) ? 1 : 0;
     hipLaunchKernelGGL(k_moe_route_rows, dim3((unsigned)rows), dim3(n_all > 8 ? 1024 : 256), (size_t)n_all * 8, ifa_s(stream), (const float *)h_f32, ldh, width,
                        (const bf16_t *)router_bf16, n_all, top, (const bf16_t *)correction_bf16, idx_dev, (float *)wgt_f32, vec, score_kind, (const float *)x_f32, ldx,
-                       (const bf16_t *)alpha_bf16, (const bf16_t *)norm_w_bf16, (const bf16_t *)norm_b_bf16, (float *)h_f32);
+                       (const bf16_t *)alpha_bf16, (const bf16_t *)norm_w_bf16, (const bf16_t *)norm_b_bf16, (float *)h_f32, 0, 0.0f, 1.0f);
     IFA_LAUNCH_CHECK();
     return IFA_OK;
 }

@@ -1,13 +1,15 @@
 // ifa_seqmix.hip -- sequence mixers with a recurrent state instead of a key / value cache, on 32-bit activations:
-//   * short causal convolution per channel + SiLU (+ unit-norm of head groups), its tail carried per sequence
+//   * short causal convolution per channel (+ bias) + SiLU (+ unit-norm of head groups), its tail carried per sequence
 //   * per-head matrix state S [dk][dv] advanced token by token:
 //       kind 0  linear attention with a constant decay per head:  S <- d S + k v^T;                      o = S^T q
 //     (in_act = 1: q, k, v pass SiLU as they are read)
 //       kind 1  gated delta rule:                                 S <- g S;  u = beta (v - S^T k);  S <- S + k u^T;  o = S^T q
+//       kind 2  selective state space (Mamba-2):                  S <- g S + k (beta v)^T;  o = S^T q + D v   (beta: the step size)
 //   * the gates of the delta rule (beta = sigmoid, g = exp(-exp(A_log) softplus(a + dt_bias)))
 //   * the generalized delta rule with a decay w and a removal rate per key channel: S <- diag(w) S - b (u^T S) + k v^T, o = S^T q
 //     (u the unit key, b = removal rate * u), and its gates
-//   * RMS norm over channel groups with a weight and an output gate (sigmoid or SiLU)
+//   * the step sizes and decays of the state space (beta = softplus(a + dt_bias), g = exp(-exp(A_log) beta))
+//   * RMS norm over channel groups with a weight and an output gate (sigmoid or SiLU) behind it, or a SiLU gate in front of it
 // Everything that enters a recurrence is fp32; states live in fp32 in the slot arena of the worker (a table of one
 // base pointer per slot + an offset per layer).  A sequence that starts at position 0 starts from a zero state,
 // whatever the slot held before.
@@ -19,14 +21,15 @@ using namespace ifa32;
 
 namespace {
 
-// grid: (rows, channel slices).  y[t][c] = silu(sum_j w[c][j] in(i - (taps - 1) + j)[c]); in(idx) for idx < 0 comes from the
+// grid: (rows, channel slices).  y[t][c] = silu(sum_j w[c][j] in(i - (taps - 1) + j)[c] + b[c]) (b may be absent); in(idx) for idx < 0 comes from the
 // sequence's carried tail (rows [taps - 1][C], oldest first) or is zero at the start of a sequence.  Then channels
 // [0, norm_cols) are turned into unit vectors in groups of gdim (x / sqrt(sum x^2 + l2_eps)) and channels [0, scale_cols)
 // are multiplied by qscale.
 __global__ void __launch_bounds__(256) k_shortconv_silu(const float *__restrict__ x, size_t ldx, int C, int taps, const bf16_t *__restrict__ w,
                                                         const SeqDesc *__restrict__ seqs, const int *__restrict__ row_seq,
                                                         float *const *__restrict__ slot_base, size_t state_off, int norm_cols, int gdim,
-                                                        float l2_eps, int scale_cols, float qscale, float *__restrict__ y, size_t ldy, int slice)
+                                                        float l2_eps, int scale_cols, float qscale, float *__restrict__ y, size_t ldy, int slice,
+                                                        const bf16_t *__restrict__ bias)
 {
     extern __shared__ float ys[];
     const int t = blockIdx.x;
@@ -43,6 +46,7 @@ __global__ void __launch_bounds__(256) k_shortconv_silu(const float *__restrict_
             else v = tail ? tail[(size_t)(taps - 1 + idx) * C + c] : 0.0f;
             acc = fmaf(bf2f(w[(size_t)c * taps + j]), v, acc);
         }
+        if (bias) acc += bf2f(bias[c]);
         ys[c - c_lo] = silu_exact(acc);
     }
     __syncthreads();
@@ -182,10 +186,23 @@ __global__ void __launch_bounds__(256) k_delta_gates(const float *__restrict__ b
     g[idx] = expf(-expf(bf2f(A_log[h])) * softplus_f(a[(size_t)t * lda + h] + bf2f(dt_bias[h])));
 }
 
+// dt[t][h] = softplus(a[t][h] + dt_bias[h]);  g[t][h] = exp(-exp(A_log[h]) * dt[t][h])
+__global__ void __launch_bounds__(256) k_ssm_gates(const float *__restrict__ a, size_t lda, int H, int T, const bf16_t *__restrict__ A_log,
+                                                   const bf16_t *__restrict__ dt_bias, float *__restrict__ dt, float *__restrict__ g)
+{
+    const int idx = blockIdx.x * blockDim.x + threadIdx.x;
+    if (idx >= T * H) return;
+    const int t = idx / H, h = idx % H;
+    const float d = softplus_f(a[(size_t)t * lda + h] + bf2f(dt_bias[h]));
+    dt[idx] = d;
+    g[idx] = expf(-expf(bf2f(A_log[h])) * d);
+}
+
 struct ScanArgs {
     const float *q, *k, *v; size_t ldq, ldk, ldv;
     int heads, qk_heads, dk, dv, in_act;
     const float *decay_head, *decay_row, *beta_row;
+    const bf16_t *skip;          // kind 2: D per head
     const SeqDesc *seqs; float *const *slot_base; size_t state_off;
     float *out; size_t ldo;
 };
@@ -210,7 +227,7 @@ __global__ void __launch_bounds__(64) k_state_scan(ScanArgs P)
     const int dk = P.dk;
     if (sd.pos0 > 0) for (int i = 0; i < dk; i++) S[i * 64 + lane] = state[(size_t)i * P.dv + jc];
     else for (int i = 0; i < dk; i++) S[i * 64 + lane] = 0.0f;
-    const float dconst = KIND == 0 ? P.decay_head[h] : 0.0f;
+    const float dconst = KIND == 0 ? P.decay_head[h] : (KIND == 2 ? bf2f(P.skip[h]) : 0.0f);
     float qr[SCAN_DKL], kr[SCAN_DKL], vr, gr = 0.0f, br = 0.0f;
     auto request = [&](int t) {
         const size_t row = (size_t)(sd.row0 + t);
@@ -224,7 +241,7 @@ __global__ void __launch_bounds__(64) k_state_scan(ScanArgs P)
         }
         vr = P.v[row * P.ldv + (size_t)h * P.dv + jc];
         if (P.in_act) vr = silu_exact(vr);
-        if (KIND == 1) { gr = P.decay_row[row * P.heads + h]; br = P.beta_row[row * P.heads + h]; }
+        if (KIND >= 1) { gr = P.decay_row[row * P.heads + h]; br = P.beta_row[row * P.heads + h]; }
     };
     if (sd.n > 0) request(0);
     for (int t = 0; t < sd.n; t++) {
@@ -241,6 +258,14 @@ __global__ void __launch_bounds__(64) k_state_scan(ScanArgs P)
                 S[i * 64 + lane] = s;
                 o = fmaf(s, qs[i], o);
             }
+        } else if (KIND == 2) {
+            const float bv = bt * vt;
+            for (int i = 0; i < dk; i++) {
+                const float s = fmaf(gt, S[i * 64 + lane], ks[i] * bv);
+                S[i * 64 + lane] = s;
+                o = fmaf(s, qs[i], o);
+            }
+            o = fmaf(dconst, vt, o);
         } else {
             float r = 0.0f;
             for (int i = 0; i < dk; i++) {
@@ -260,7 +285,7 @@ __global__ void __launch_bounds__(64) k_state_scan(ScanArgs P)
     if (live) for (int i = 0; i < dk; i++) state[(size_t)i * P.dv + j] = S[i * 64 + lane];
 }
 
-// The same recurrences for key sizes 16 / 32 / 64 / 128 with the state in REGISTERS and FOUR (key sizes from 64 on: EIGHT) lanes per column:
+// The same recurrences for key sizes 16 / 32 / 48 / 64 / 96 / 128 (kind 2 also 256: sixteen lanes) with the state in REGISTERS and FOUR (key sizes from 64 on: EIGHT) lanes per column:
 // lane 4 c + r of a wave owns rows [r DK / 4, (r + 1) DK / 4) of column c (16 columns per wave), so a token is DK / 4 elements of dependent arithmetic per lane
 // instead of DK -- the recurrence is a chain of dependent instructions of a wave that is alone on its SIMD, and its length per token
 // is what the prompt rate of these layers comes down to.  The sums over a column's rows (the read-out, and S^T k of the delta rule)
@@ -290,7 +315,7 @@ __global__ void __launch_bounds__(64) k_state_scan_reg(ScanArgs P)
 #pragma unroll
         for (int e = 0; e < DKQ; e++) S[e] = 0.0f;
     }
-    const float dconst = KIND == 0 ? P.decay_head[h] : 0.0f;
+    const float dconst = KIND == 0 ? P.decay_head[h] : (KIND == 2 ? bf2f(P.skip[h]) : 0.0f);
     constexpr int PER = SCAN_TB * DK / 64;          // q (and k) values of a group per lane
     float qr[PER], kr[PER], vnext[SCAN_TB], vcur[SCAN_TB], gr = 0.0f, br = 0.0f;
     auto request = [&](int t0) {                    // the group that starts at token t0 -> registers
@@ -307,7 +332,7 @@ __global__ void __launch_bounds__(64) k_state_scan_reg(ScanArgs P)
             vnext[tt] = P.v[row * P.ldv + (size_t)h * P.dv + jc];
             if (P.in_act) vnext[tt] = silu_exact(vnext[tt]);
         }
-        if (KIND == 1 && lane < SCAN_TB) {
+        if (KIND >= 1 && lane < SCAN_TB) {
             const size_t row = (size_t)(sd.row0 + min(t0 + lane, sd.n - 1));
             gr = P.decay_row[row * P.heads + h]; br = P.beta_row[row * P.heads + h];
         }
@@ -315,7 +340,7 @@ __global__ void __launch_bounds__(64) k_state_scan_reg(ScanArgs P)
     auto publish = [&](int buf) {                   // registers -> LDS buffer
 #pragma unroll
         for (int u = 0; u < PER; u++) { const int e = lane + 64 * u; qs[buf][e / DK][e % DK] = qr[u]; ks[buf][e / DK][e % DK] = kr[u]; }
-        if (KIND == 1 && lane < SCAN_TB) { gs[buf][lane] = gr; bs[buf][lane] = br; }
+        if (KIND >= 1 && lane < SCAN_TB) { gs[buf][lane] = gr; bs[buf][lane] = br; }
 #pragma unroll
         for (int tt = 0; tt < SCAN_TB; tt++) vcur[tt] = vnext[tt];
     };
@@ -343,6 +368,13 @@ __global__ void __launch_bounds__(64) k_state_scan_reg(ScanArgs P)
                         S[e] = fmaf(dconst, S[e], kk[e] * vt); o0 = fmaf(S[e], qq[e], o0);
                         S[e + 1] = fmaf(dconst, S[e + 1], kk[e + 1] * vt); o1 = fmaf(S[e + 1], qq[e + 1], o1);
                     }
+                } else if (KIND == 2) {
+                    const float gt = gs[buf][tt], bv = bs[buf][tt] * vt;
+#pragma unroll
+                    for (int e = 0; e < DKQ; e += 2) {
+                        S[e] = fmaf(gt, S[e], kk[e] * bv); o0 = fmaf(S[e], qq[e], o0);
+                        S[e + 1] = fmaf(gt, S[e + 1], kk[e + 1] * bv); o1 = fmaf(S[e + 1], qq[e + 1], o1);
+                    }
                 } else {
                     const float gt = gs[buf][tt], bt = bs[buf][tt];
                     float r0 = 0.0f, r1 = 0.0f;
@@ -358,7 +390,8 @@ __global__ void __launch_bounds__(64) k_state_scan_reg(ScanArgs P)
                         S[e + 1] = fmaf(kk[e + 1], u, S[e + 1]); o1 = fmaf(S[e + 1], qq[e + 1], o1);
                     }
                 }
-                const float o = LPC == 8 ? oct_sum(o0 + o1) : quad_sum(o0 + o1);
+                float o = LPC == 16 ? hex_sum(o0 + o1) : (LPC == 8 ? oct_sum(o0 + o1) : quad_sum(o0 + o1));
+                if (KIND == 2) o = fmaf(dconst, vt, o);
                 if (live && rg == 0) P.out[(size_t)(sd.row0 + t0 + tt) * P.ldo + (size_t)h * P.dv + j] = o;
             }
         }
@@ -615,13 +648,41 @@ __global__ void __launch_bounds__(256) k_gated_groupnorm(const float *__restrict
     }
 }
 
+// y[t][c] = v / sqrt(mean_group(v^2) + eps) * w[c], v = o[t][c] * silu(gate[t][c]): the gate in front of the norm; one workgroup per row
+__global__ void __launch_bounds__(512) k_gate_groupnorm(const float *__restrict__ o, size_t ldo, int C, int group, const bf16_t *__restrict__ w, const float *__restrict__ gate,
+                                                        size_t ldg, float eps, float *__restrict__ y, size_t ldy)
+{
+    extern __shared__ float vs[];          // [C]
+    __shared__ float red[17];
+    const int t = blockIdx.x, lane = threadIdx.x & 63, wave = threadIdx.x >> 6, nw = blockDim.x >> 6;
+    const float *orow = o + (size_t)t * ldo, *grow = gate + (size_t)t * ldg;
+    float *yrow = y + (size_t)t * ldy;
+    for (int c = threadIdx.x; c < C; c += blockDim.x) vs[c] = orow[c] * silu_exact(grow[c]);
+    __syncthreads();
+    if (C / group < nw) {          // fewer groups than waves: the whole workgroup works on each group
+        for (int gi = 0; gi < C / group; gi++) {
+            float s = 0.0f;
+            for (int e = threadIdx.x; e < group; e += blockDim.x) { const float v = vs[gi * group + e]; s = fmaf(v, v, s); }
+            const float r = 1.0f / sqrtf(block_sum(s, red) / (float)group + eps);
+            for (int e = threadIdx.x; e < group; e += blockDim.x) { const int c = gi * group + e; yrow[c] = vs[c] * r * bf2f(w[c]); }
+        }
+        return;
+    }
+    for (int gi = wave; gi < C / group; gi += nw) {
+        float s = 0.0f;
+        for (int e = lane; e < group; e += 64) { const float v = vs[gi * group + e]; s = fmaf(v, v, s); }
+        const float r = 1.0f / sqrtf(wave_sum(s) / (float)group + eps);
+        for (int e = lane; e < group; e += 64) { const int c = gi * group + e; yrow[c] = vs[c] * r * bf2f(w[c]); }
+    }
+}
+
 } // namespace
 
 extern "C" {
 
-int ifa_shortconv_silu_f32(const void *x_f32, size_t ldx, int channels, int taps, const void *w_bf16, const void *seqs_dev, const int *row_seq_dev,
-                           size_t rows, void *const *slot_base_dev, size_t state_off, int norm_cols, int group_dim, float l2_eps, int scale_cols,
-                           float scale, void *y_f32, size_t ldy, ifa_stream stream)
+static int shortconv_silu(const void *x_f32, size_t ldx, int channels, int taps, const void *w_bf16, const void *bias_bf16, const void *seqs_dev, const int *row_seq_dev,
+                          size_t rows, void *const *slot_base_dev, size_t state_off, int norm_cols, int group_dim, float l2_eps, int scale_cols,
+                          float scale, void *y_f32, size_t ldy, ifa_stream stream)
 {
     IFA_REQUIRE(x_f32 && w_bf16 && seqs_dev && row_seq_dev && slot_base_dev && y_f32, "ifa_shortconv_silu_f32: null pointer");
     IFA_REQUIRE(channels > 0 && taps >= 1 && taps <= 64 && rows > 0 && ldx >= (size_t)channels && ldy >= (size_t)channels, "ifa_shortconv_silu_f32: bad shape");
@@ -634,9 +695,23 @@ int ifa_shortconv_silu_f32(const void *x_f32, size_t ldx, int channels, int taps
     IFA_REQUIRE((size_t)slice * 4 <= 64 * 1024, "ifa_shortconv_silu_f32: norm groups of %d channels do not fit the LDS", group_dim);
     hipLaunchKernelGGL(k_shortconv_silu, dim3((unsigned)rows, ifa_cdiv((size_t)channels, (size_t)slice)), dim3(256), (size_t)slice * 4, ifa_s(stream),
                        (const float *)x_f32, ldx, channels, taps, (const bf16_t *)w_bf16, (const SeqDesc *)seqs_dev, row_seq_dev, (float *const *)slot_base_dev,
-                       state_off, norm_cols, group_dim, l2_eps, scale_cols, scale, (float *)y_f32, ldy, slice);
+                       state_off, norm_cols, group_dim, l2_eps, scale_cols, scale, (float *)y_f32, ldy, slice, (const bf16_t *)bias_bf16);
     IFA_LAUNCH_CHECK();
     return IFA_OK;
+}
+
+int ifa_shortconv_silu_f32(const void *x_f32, size_t ldx, int channels, int taps, const void *w_bf16, const void *seqs_dev, const int *row_seq_dev,
+                           size_t rows, void *const *slot_base_dev, size_t state_off, int norm_cols, int group_dim, float l2_eps, int scale_cols,
+                           float scale, void *y_f32, size_t ldy, ifa_stream stream)
+{
+    return shortconv_silu(x_f32, ldx, channels, taps, w_bf16, nullptr, seqs_dev, row_seq_dev, rows, slot_base_dev, state_off, norm_cols, group_dim, l2_eps, scale_cols, scale,
+                          y_f32, ldy, stream);
+}
+
+int ifa_shortconv_bias_silu_f32(const void *x_f32, size_t ldx, int channels, int taps, const void *w_bf16, const void *bias_bf16, const void *seqs_dev, const int *row_seq_dev,
+                                size_t rows, void *const *slot_base_dev, size_t state_off, void *y_f32, size_t ldy, ifa_stream stream)
+{
+    return shortconv_silu(x_f32, ldx, channels, taps, w_bf16, bias_bf16, seqs_dev, row_seq_dev, rows, slot_base_dev, state_off, 0, 0, 0.0f, 0, 1.0f, y_f32, ldy, stream);
 }
 
 int ifa_shortconv_residual_f32(const void *x_f32, size_t ldx, int channels, int taps, const void *w_bf16, const void *seqs_dev, const int *row_seq_dev,
@@ -693,19 +768,31 @@ int ifa_delta_gates_f32(const void *b_f32, size_t ldb, const void *a_f32, size_t
     return IFA_OK;
 }
 
-int ifa_state_scan_f32(int kind, int in_act, const void *q_f32, size_t ldq, const void *k_f32, size_t ldk, const void *v_f32, size_t ldv, int heads, int qk_heads,
-                       int dk, int dv, const void *decay_head_f32, const void *decay_row_f32, const void *beta_row_f32, const void *seqs_dev, int n_seqs,
-                       void *const *slot_base_dev, size_t state_off, void *out_f32, size_t ldo, ifa_stream stream)
+int ifa_ssm_gates_f32(const void *a_f32, size_t lda, int heads, size_t rows, const void *a_log_bf16, const void *dt_bias_bf16, void *dt_f32, void *decay_f32,
+                      ifa_stream stream)
+{
+    IFA_REQUIRE(a_f32 && a_log_bf16 && dt_bias_bf16 && dt_f32 && decay_f32, "ifa_ssm_gates_f32: null pointer");
+    IFA_REQUIRE(heads > 0 && rows > 0 && lda >= (size_t)heads && rows * (size_t)heads < (1u << 31), "ifa_ssm_gates_f32: bad shape");
+    hipLaunchKernelGGL(k_ssm_gates, dim3(ifa_cdiv(rows * heads, 256)), dim3(256), 0, ifa_s(stream), (const float *)a_f32, lda, heads, (int)rows, (const bf16_t *)a_log_bf16,
+                       (const bf16_t *)dt_bias_bf16, (float *)dt_f32, (float *)decay_f32);
+    IFA_LAUNCH_CHECK();
+    return IFA_OK;
+}
+
+static int state_scan(int kind, int in_act, const void *q_f32, size_t ldq, const void *k_f32, size_t ldk, const void *v_f32, size_t ldv, int heads, int qk_heads,
+                      int dk, int dv, const void *decay_head_f32, const void *decay_row_f32, const void *beta_row_f32, const void *skip_bf16, const void *seqs_dev, int n_seqs,
+                      void *const *slot_base_dev, size_t state_off, void *out_f32, size_t ldo, ifa_stream stream)
 {
     IFA_REQUIRE(q_f32 && k_f32 && v_f32 && seqs_dev && slot_base_dev && out_f32, "ifa_state_scan_f32: null pointer");
-    IFA_REQUIRE(kind == 0 || kind == 1, "ifa_state_scan_f32: kind %d", kind);
+    IFA_REQUIRE(kind >= 0 && kind <= 2, "ifa_state_scan_f32: kind %d", kind);
     IFA_REQUIRE(heads > 0 && qk_heads > 0 && heads % qk_heads == 0 && dk > 0 && dv > 0 && n_seqs > 0, "ifa_state_scan_f32: bad shape");
     IFA_REQUIRE(dk <= 64 * SCAN_DKL, "ifa_state_scan_f32: key size %d above %d", dk, 64 * SCAN_DKL);
-    IFA_REQUIRE(kind == 0 ? decay_head_f32 != nullptr : (decay_row_f32 && beta_row_f32), "ifa_state_scan_f32: the gates of kind %d are missing", kind);
+    IFA_REQUIRE(kind == 0 ? decay_head_f32 != nullptr : (decay_row_f32 && beta_row_f32 && (kind == 1 || skip_bf16)), "ifa_state_scan_f32: the gates of kind %d are missing", kind);
     ScanArgs P;
     P.q = (const float *)q_f32; P.k = (const float *)k_f32; P.v = (const float *)v_f32; P.ldq = ldq; P.ldk = ldk; P.ldv = ldv;
     P.heads = heads; P.qk_heads = qk_heads; P.dk = dk; P.dv = dv; P.in_act = in_act ? 1 : 0;
     P.decay_head = (const float *)decay_head_f32; P.decay_row = (const float *)decay_row_f32; P.beta_row = (const float *)beta_row_f32;
+    P.skip = (const bf16_t *)skip_bf16;
     P.seqs = (const SeqDesc *)seqs_dev; P.slot_base = (float *const *)slot_base_dev; P.state_off = state_off;
     P.out = (float *)out_f32; P.ldo = ldo;
     const size_t smem = ((size_t)dk * 64 + 2 * (size_t)dk) * 4;
@@ -722,15 +809,52 @@ int ifa_state_scan_f32(int kind, int in_act, const void *q_f32, size_t ldq, cons
         IFA_LAUNCH_CHECK(); \
         return IFA_OK; \
     }
-    IFA_SCAN_REG(16) IFA_SCAN_REG(32) IFA_SCAN_REG(64) IFA_SCAN_REG(128)
+    if (kind < 2) { IFA_SCAN_REG(16) IFA_SCAN_REG(32) IFA_SCAN_REG(64) IFA_SCAN_REG(128) }
 #undef IFA_SCAN_REG
-    if (kind == 0) {
+    const dim3 grid4((unsigned)(n_seqs * heads), ifa_cdiv((size_t)dv, 4));
+#define IFA_SSM_REG(DKV, L, G) if (kind == 2 && dk == DKV) { hipLaunchKernelGGL((k_state_scan_reg<2, DKV, L>), G, dim3(64), 0, ifa_s(stream), P); IFA_LAUNCH_CHECK(); return IFA_OK; }
+    IFA_SSM_REG(16, 4, grid16) IFA_SSM_REG(32, 4, grid16) IFA_SSM_REG(48, 4, grid16) IFA_SSM_REG(64, 8, grid8) IFA_SSM_REG(96, 8, grid8) IFA_SSM_REG(128, 8, grid8)
+    IFA_SSM_REG(256, 16, grid4)
+#undef IFA_SSM_REG
+    if (kind == 2) {
+        IFA_HIP_CHECK(hipFuncSetAttribute((const void *)k_state_scan<2>, hipFuncAttributeMaxDynamicSharedMemorySize, (int)smem));
+        hipLaunchKernelGGL(k_state_scan<2>, grid, dim3(64), smem, ifa_s(stream), P);
+    } else if (kind == 0) {
         IFA_HIP_CHECK(hipFuncSetAttribute((const void *)k_state_scan<0>, hipFuncAttributeMaxDynamicSharedMemorySize, (int)smem));
         hipLaunchKernelGGL(k_state_scan<0>, grid, dim3(64), smem, ifa_s(stream), P);
     } else {
         IFA_HIP_CHECK(hipFuncSetAttribute((const void *)k_state_scan<1>, hipFuncAttributeMaxDynamicSharedMemorySize, (int)smem));
         hipLaunchKernelGGL(k_state_scan<1>, grid, dim3(64), smem, ifa_s(stream), P);
     }
+    IFA_LAUNCH_CHECK();
+    return IFA_OK;
+}
+
+int ifa_state_scan_f32(int kind, int in_act, const void *q_f32, size_t ldq, const void *k_f32, size_t ldk, const void *v_f32, size_t ldv, int heads, int qk_heads,
+                       int dk, int dv, const void *decay_head_f32, const void *decay_row_f32, const void *beta_row_f32, const void *seqs_dev, int n_seqs,
+                       void *const *slot_base_dev, size_t state_off, void *out_f32, size_t ldo, ifa_stream stream)
+{
+    IFA_REQUIRE(kind == 0 || kind == 1, "ifa_state_scan_f32: kind %d", kind);
+    return state_scan(kind, in_act, q_f32, ldq, k_f32, ldk, v_f32, ldv, heads, qk_heads, dk, dv, decay_head_f32, decay_row_f32, beta_row_f32, nullptr, seqs_dev, n_seqs,
+                      slot_base_dev, state_off, out_f32, ldo, stream);
+}
+
+int ifa_state_scan_ssm_f32(const void *x_f32, size_t ldx, const void *b_f32, size_t ldb, const void *c_f32, size_t ldc, int heads, int groups, int state, int vdim,
+                           const void *dt_f32, const void *decay_f32, const void *skip_bf16, const void *seqs_dev, int n_seqs, void *const *slot_base_dev, size_t state_off,
+                           void *out_f32, size_t ldo, ifa_stream stream)
+{
+    return state_scan(2, 0, c_f32, ldc, b_f32, ldb, x_f32, ldx, heads, groups, state, vdim, nullptr, decay_f32, dt_f32, skip_bf16, seqs_dev, n_seqs, slot_base_dev, state_off,
+                      out_f32, ldo, stream);
+}
+
+int ifa_gate_groupnorm_f32(const void *o_f32, size_t ldo, size_t rows, int channels, int groups, const void *w_bf16, const void *gate_f32, size_t ldg, float eps,
+                           void *y_f32, size_t ldy, ifa_stream stream)
+{
+    IFA_REQUIRE(o_f32 && w_bf16 && gate_f32 && y_f32, "ifa_gate_groupnorm_f32: null pointer");
+    IFA_REQUIRE(rows > 0 && channels > 0 && groups > 0 && channels % groups == 0 && ldo >= (size_t)channels && ldg >= (size_t)channels && ldy >= (size_t)channels
+                && (size_t)channels * 4 <= 64 * 1024 - 256, "ifa_gate_groupnorm_f32: bad arguments (%d channels in %d groups)", channels, groups);
+    hipLaunchKernelGGL(k_gate_groupnorm, dim3((unsigned)rows), dim3(channels >= 2048 ? 512 : 256), (size_t)channels * 4, ifa_s(stream), (const float *)o_f32, ldo, channels,
+                       channels / groups, (const bf16_t *)w_bf16, (const float *)gate_f32, ldg, eps, (float *)y_f32, ldy);
     IFA_LAUNCH_CHECK();
     return IFA_OK;
 }

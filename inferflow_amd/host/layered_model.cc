@@ -32,6 +32,14 @@
 //                    turned by their position over all of vdim (the head's output turned back), sliding window mask.size, a learned sink per head
 //   "general_delta"  generalized delta rule with a decay and a removal rate per head and key channel, per-head RMS norm, sigmoid gate
 // and a mixture of clamped gated experts (sigmoid scores, choice by score + correction, weights = the scores), or no feed-forward.
+//
+// Kamelorn: width / vocab / norm.eps / embedding.scale / residual_mult / streams / loop {start, stop, times}; `streams` residual streams per token, all
+// equal to the scaled embedding at the start, read and written by every sub-layer through learned mixing weights (hc1 / hc2), RMS norms in
+// front of the sub-layers and, over the sum of the streams, of the head; layers [loop.start, loop.stop) run loop.times times with the same
+// weights, every pass on a cache or state of its own; mixer types
+//   "latent_attention"  queries straight from the input, rotation in halves, one cached row per position, a sigmoid gate per output column
+//   "mamba2"            selective state space behind a short convolution with bias, SiLU gate in front of an RMS norm in norm_groups parts
+// and a feed-forward of kind "dense" (SiLU-gated) or "moe" (sigmoid scores, renormalized over the chosen and multiplied by router.scale), or none.
 #include <cmath>
 #include <cstdio>
 #include <cstring>
@@ -342,6 +350,101 @@ void BogupelNames(const LayeredDesc &d, std::vector<std::pair<std::string, std::
     }
 }
 
+// ---- Kamelorn
+bool ParseKamelorn(const JsonValue &root, LayeredDesc &d)
+{
+    memset(&d.cfg, 0, sizeof(d.cfg));
+    if (!Need(root, "width", d.cfg.width, "config") || !Need(root, "vocab", d.cfg.vocab, "config")) return false;
+    const JsonValue *norm = root.Get("norm");
+    if (!norm || !Need(*norm, "eps", d.cfg.eps, "norm")) { if (!norm) EngineSetError("config.json: norm is missing"); return false; }
+    d.cfg.stem = 4;
+    d.cfg.embed_scale = 1.0f; d.cfg.residual_mult = 1.0f;
+    if (const JsonValue *emb = root.Get("embedding")) emb->GetNumber("scale", d.cfg.embed_scale);
+    root.GetNumber("residual_mult", d.cfg.residual_mult);
+    root.GetNumber("streams", d.cfg.streams);
+    const JsonValue *loop = root.Get("loop");
+    if (loop && loop->type == JsonValue::Object
+        && (!Need(*loop, "start", d.cfg.loop_start, "loop") || !Need(*loop, "stop", d.cfg.loop_stop, "loop") || !Need(*loop, "times", d.cfg.loop_times, "loop"))) return false;
+    const JsonValue *layers = root.Get("layers");
+    if (!layers || layers->type != JsonValue::Array || layers->arr.empty()) { EngineSetError("config.json: layers is missing or empty"); return false; }
+    for (size_t li = 0; li < layers->arr.size(); li++) {
+        const JsonValue &L = layers->arr[li];
+        ifa_layer_spec s; memset(&s, 0, sizeof(s));
+        std::string type;
+        const JsonValue *mx = L.Get("mixer");
+        if (!L.GetString("type", type) || !mx || mx->type != JsonValue::Object) { EngineSetError("config.json: layer %zu has no type / mixer", li); return false; }
+        s.block = IFA_BLOCK_STREAMS;
+        if (type == "latent_attention") {
+            s.mixer = IFA_MIX_LATENT; s.m_gate = 2; s.m_rot_halves = 1;
+            if (!Need(*mx, "heads", s.m_heads, "mixer") || !Need(*mx, "dim", s.m_dim, "mixer") || !Need(*mx, "rot_dim", s.m_rot_dim, "mixer") || !Need(*mx, "vdim", s.m_vdim, "mixer")
+                || !Need(*mx, "kv_rank", s.m_kv_rank, "mixer") || !Need(*mx, "scale", s.m_scale, "mixer")) return false;
+            const JsonValue *rot = mx->Get("rot");
+            if (!rot || !Need(*rot, "base", s.m_rot_base, "mixer.rot") || !Need(*rot, "dims", s.m_rot_dims, "mixer.rot")) {
+                if (!rot) EngineSetError("config.json: layer %zu: mixer.rot is missing", li);
+                return false;
+            }
+        } else if (type == "mamba2") {
+            s.mixer = IFA_MIX_SSM;
+            if (!Need(*mx, "heads", s.s_heads, "mixer") || !Need(*mx, "vdim", s.s_vdim, "mixer") || !Need(*mx, "state", s.s_state, "mixer") || !Need(*mx, "groups", s.s_groups, "mixer")
+                || !Need(*mx, "conv", s.s_conv, "mixer") || !Need(*mx, "norm_groups", s.s_norm_groups, "mixer")) return false;
+        } else { EngineSetError("config.json: layer %zu: unknown type \"%s\"", li, type.c_str()); return false; }
+        const JsonValue *mlp = L.Get("mlp");
+        if (mlp && mlp->type == JsonValue::Object) {
+            std::string kind;
+            mlp->GetString("kind", kind);
+            if (kind == "dense") {
+                s.ffn_kind = IFA_FFN_SILU;
+                if (!Need(*mlp, "ff", s.ffn, "mlp")) return false;
+            } else if (kind == "moe") {
+                const JsonValue *ex = mlp->Get("expert"), *ro = mlp->Get("router");
+                if (!ex || !ro) { EngineSetError("config.json: layer %zu: mlp needs expert and router", li); return false; }
+                s.ffn_kind = IFA_FFN_MOE; s.x_gated = 1; s.x_route = 0; s.x_score = 1; s.x_glu = 0; s.x_renorm = 1; s.x_renorm_eps = 1e-20f; s.x_wgt_scale = 1.0f;
+                if (!Need(*ex, "ff", s.x_ff, "mlp.expert") || !Need(*ro, "experts", s.x_experts, "mlp.router") || !Need(*ro, "top", s.x_top, "mlp.router")) return false;
+                ro->GetNumber("scale", s.x_wgt_scale);
+            } else { EngineSetError("config.json: layer %zu: mlp.kind \"%s\" is not supported (dense, moe)", li, kind.c_str()); return false; }
+        }
+        d.layers.push_back(s);
+        d.decays.push_back(std::vector<float>());
+    }
+    d.cfg.n_layers = (int)d.layers.size();
+    return true;
+}
+
+void KamelornNames(const LayeredDesc &d, std::vector<std::pair<std::string, std::pair<int, int>>> &out)
+{
+    out.push_back({"embed", {-1, IFA_T_EMBD}}); out.push_back({"final.norm", {-1, IFA_T_OUT_NORM}}); out.push_back({"head", {-1, IFA_T_LM_HEAD}});
+    for (size_t li = 0; li < d.layers.size(); li++) {
+        const ifa_layer_spec &s = d.layers[li];
+        const std::string p = "l" + std::to_string(li) + ".";
+        const int l = (int)li;
+        const bool moe = s.ffn_kind == IFA_FFN_MOE && s.x_experts > 0, any_ffn = moe || s.ffn > 0;
+        out.push_back({p + "norm1", {l, IFA_LT_NORM1}});
+        if (d.cfg.streams > 0) { out.push_back({p + "hc1.in", {l, IFA_LT_HC1_IN}}); out.push_back({p + "hc1.out", {l, IFA_LT_HC1_OUT}}); out.push_back({p + "hc1.mix", {l, IFA_LT_HC1_MIX}}); }
+        if (s.mixer == IFA_MIX_LATENT) {
+            out.push_back({p + "mix.q", {l, IFA_LT_M_Q}}); out.push_back({p + "mix.dkv", {l, IFA_LT_M_DKV}}); out.push_back({p + "mix.dkv.norm", {l, IFA_LT_M_DKV_NORM}});
+            out.push_back({p + "mix.uk", {l, IFA_LT_M_UK}}); out.push_back({p + "mix.uv", {l, IFA_LT_M_UV}}); out.push_back({p + "mix.g", {l, IFA_LT_M_G}});
+            out.push_back({p + "mix.o", {l, IFA_LT_M_O}});
+        } else {
+            out.push_back({p + "mix.in", {l, IFA_LT_S_IN}}); out.push_back({p + "mix.conv", {l, IFA_LT_S_CONV}}); out.push_back({p + "mix.conv.b", {l, IFA_LT_S_CONV_B}});
+            out.push_back({p + "mix.dt_bias", {l, IFA_LT_S_DTBIAS}}); out.push_back({p + "mix.A_log", {l, IFA_LT_S_ALOG}}); out.push_back({p + "mix.D", {l, IFA_LT_S_D}});
+            out.push_back({p + "mix.norm", {l, IFA_LT_S_NORM}}); out.push_back({p + "mix.o", {l, IFA_LT_S_O}});
+        }
+        if (!any_ffn) continue;
+        out.push_back({p + "norm2", {l, IFA_LT_NORM2}});
+        if (d.cfg.streams > 0) { out.push_back({p + "hc2.in", {l, IFA_LT_HC2_IN}}); out.push_back({p + "hc2.out", {l, IFA_LT_HC2_OUT}}); out.push_back({p + "hc2.mix", {l, IFA_LT_HC2_MIX}}); }
+        if (!moe) {
+            out.push_back({p + "mlp.gate", {l, IFA_LT_FFN_GATE}}); out.push_back({p + "mlp.up", {l, IFA_LT_FFN_UP}}); out.push_back({p + "mlp.down", {l, IFA_LT_FFN_DOWN}});
+            continue;
+        }
+        out.push_back({p + "mlp.router", {l, IFA_LT_X_ROUTER}});
+        for (int e = 0; e < s.x_experts; e++) {      // per expert: its gate rows, then its up rows
+            out.push_back({p + "mlp.e" + std::to_string(e) + ".gate", {l, IFA_LT_X_UP}});
+            out.push_back({p + "mlp.e" + std::to_string(e) + ".up", {l, IFA_LT_X_UP}});
+        }
+        for (int e = 0; e < s.x_experts; e++) out.push_back({p + "mlp.e" + std::to_string(e) + ".down", {l, IFA_LT_X_DOWN}});
+    }
+}
+
 void SopulornNames(const LayeredDesc &d, std::vector<std::pair<std::string, std::pair<int, int>>> &out)
 {
     out.push_back({"embed", {-1, IFA_T_EMBD}});
@@ -462,7 +565,8 @@ struct ArchEntry {
 const ArchEntry kArchitectures[] = {{"Gelarax", ParseGelarax, GelaraxSizesFromTensors, GelaraxNames},
                                     {"Muzopel", ParseMuzopel, NoSizesFromTensors, MuzopelNames},
                                     {"Sopulorn", ParseSopulorn, NoSizesFromTensors, SopulornNames},
-                                    {"Bogupel", ParseBogupel, BogupelSizesFromTensors, BogupelNames}};
+                                    {"Bogupel", ParseBogupel, BogupelSizesFromTensors, BogupelNames},
+                                    {"Kamelorn", ParseKamelorn, NoSizesFromTensors, KamelornNames}};
 
 const ArchEntry *FindArch(const std::string &name)
 {
