@@ -394,8 +394,18 @@ BOGUPEL_SIZES = {   # --arch bogupel: six layers in eight layer runs (attention,
 }
 
 
+KAMELORN_SIZES = {  # --arch kamelorn: six layers in eight layer runs (latent attention, state space, a group of state space + latent attention that runs twice, state space twice), dense and mixture feed-forwards
+    "w1024": dict(width=1024, heads=8, dim=96, rot_dim=32, vdim=128, kv_rank=256, ssm_heads=32, ssm_vdim=64, state=128, groups=4, norm_groups=4, dense_ff=2816, experts=16, top=4,
+                  ff=704, streams=4),
+    "w2048": dict(width=2048, heads=16, dim=128, rot_dim=64, vdim=128, kv_rank=512, ssm_heads=64, ssm_vdim=64, state=128, groups=8, norm_groups=8, dense_ff=5632, experts=32, top=6,
+                  ff=1408, streams=4),
+}
+
+
 def run_arch_bench(args):
-    """--arch gelarax | muzopel | sopulorn | bogupel: see run_gelarax_bench / run_muzopel_bench"""
+    """--arch gelarax | muzopel | sopulorn | bogupel | kamelorn: see run_gelarax_bench / run_muzopel_bench"""
+    if args.arch.lower() == "kamelorn":
+        return run_muzopel_bench(args, "kamelorn")
     if args.arch.lower() == "muzopel":
         return run_muzopel_bench(args)
     if args.arch.lower() == "bogupel":
@@ -406,7 +416,7 @@ def run_arch_bench(args):
 
 
 def run_muzopel_bench(args, design="muzopel"):
-    """--arch muzopel | sopulorn: prefill and decode throughput of models of that design with random bfloat16 weights (layer-list worker: latent attention
+    """--arch muzopel | sopulorn | bogupel | kamelorn: prefill and decode throughput of models of that design with random bfloat16 weights (layer-list worker: latent attention
     or rotary attention with shared key / value rows, mixture of experts, fp32 residual) beside the closest standard model of this framework at equal
     width / heads / KV heads / layers / experts / expert width (Mixtral wiring: attention with an F16 KV cache, gated experts, F16 weights).  One JSON
     line; `value` = decode tokens/s of the largest size."""
@@ -430,20 +440,17 @@ def run_muzopel_bench(args, design="muzopel"):
 
     sop = design == "sopulorn"
     label = design.capitalize()
-    size_table = {"sopulorn": SOPULORN_SIZES, "muzopel": MUZOPEL_SIZES, "bogupel": BOGUPEL_SIZES}[design]
-    make_cfg = {"sopulorn": synth.sopulorn_config, "muzopel": synth.muzopel_config, "bogupel": synth.bogupel_config}[design]
-    write_dir = {"sopulorn": synth.write_sopulorn_dir, "muzopel": synth.write_muzopel_dir, "bogupel": synth.write_bogupel_dir}[design]
-    shapes_of = {"sopulorn": synth.sopulorn_tensor_shapes, "muzopel": synth.muzopel_tensor_shapes, "bogupel": synth.bogupel_tensor_shapes}[design]
-    for name in sizes:
-        sz = size_table[name]
-        cfg = make_cfg(vocab=32000, **sz)
+    size_table = {"sopulorn": SOPULORN_SIZES, "muzopel": MUZOPEL_SIZES, "bogupel": BOGUPEL_SIZES, "kamelorn": KAMELORN_SIZES}[design]
+    make_cfg = {"sopulorn": synth.sopulorn_config, "muzopel": synth.muzopel_config, "bogupel": synth.bogupel_config, "kamelorn": synth.kamelorn_config}[design]
+    write_dir = {"sopulorn": synth.write_sopulorn_dir, "muzopel": synth.write_muzopel_dir, "bogupel": synth.write_bogupel_dir, "kamelorn": synth.write_kamelorn_dir}[design]
+    shapes_of = {"sopulorn": synth.sopulorn_tensor_shapes, "muzopel": synth.muzopel_tensor_shapes, "bogupel": synth.bogupel_tensor_shapes, "kamelorn": synth.kamelorn_tensor_shapes}[design]
+    def layered_rates(cfg, write_dir, shapes):
         d = tempfile.mkdtemp(prefix="ifa_%s_" % design, dir="/dev/shm" if os.path.isdir("/dev/shm") else None)
         try:
             write_dir(d, cfg, seed=1)
             eng = InferenceEngine.from_model_dir(d, "bfloat16", ctx, 2, False)
         finally:
             shutil.rmtree(d, ignore_errors=True)
-        shapes = shapes_of(cfg)
         g = {"prefill_tok_s": {}, "params": int(sum(int(np.prod(s)) for s in shapes.values()))}
         for n in lens:
             prompt = [int(t) for t in rng.integers(3, 32000, n)]
@@ -459,6 +466,17 @@ def run_muzopel_bench(args, design="muzopel"):
         wall = timed(lambda: eng.generate(q, steps))
         g["decode_tok_s"] = steps / wall; g["decode_ms_per_step"] = wall * 1e3 / steps; g["decode_context"] = "%d..%d" % (lens[-1] + warmup, lens[-1] + warmup + steps)
         eng.close()
+        return g
+
+    for name in sizes:
+        sz = size_table[name]
+        cfg = make_cfg(vocab=32000, **sz)
+        g = layered_rates(cfg, write_dir, shapes_of(cfg))
+        extra = {}
+        if design == "kamelorn":      # the closest layer-list model: latent attention of the same sizes and the same mixture of experts in each of eight layers
+            mz = synth.muzopel_config(width=sz["width"], vocab=32000, heads=sz["heads"], dim=sz["dim"], rot_dim=sz["rot_dim"], vdim=sz["vdim"], kv_rank=sz["kv_rank"],
+                                      q_rank=3 * sz["kv_rank"] // 2, experts=sz["experts"], identity=0, top=sz["top"], ff=sz["ff"])
+            extra["closest_layered_model"] = {"design": "Muzopel", **layered_rates(mz, synth.write_muzopel_dir, synth.muzopel_tensor_shapes(mz))}
         # the closest standard model: same width, heads, layer count, experts, choices per token and expert width, F16 weights
         synth.SHAPES["cmp_" + name] = dict(dim=sz["width"], layers=8, heads=sz["heads"], kv_heads=sz.get("kv_heads", sz["heads"]), head_dim=128, ffn=sz["ff"], vocab=32000,
                                            experts=sz["experts"], moe_top_k=sz["top"])
@@ -474,7 +492,7 @@ def run_muzopel_bench(args, design="muzopel"):
         wall = timed(lambda: wk.decode(nxt, lens[-1] + warmup, steps))
         c["decode_tok_s"] = steps / wall; c["decode_ms_per_step"] = wall * 1e3 / steps
         del wk
-        rows.append({"size": name, "layers": 8, **sz, design: g, "closest_standard_model": c})
+        rows.append({"size": name, "layers": 8, **sz, design: g, **extra, "closest_standard_model": c})
     last = rows[-1][design]
     print(json.dumps({"metric": "decode tokens/sec, %s-shaped model (%s), batch=1 greedy" % (label, sizes[-1]), "value": last["decode_tok_s"], "unit": "tokens/s", "n_gpus": 1,
                       "steps": steps, "warmup": warmup, "ms_per_step": last["decode_ms_per_step"], "higher_is_better": True, "scaling": "strong", "vs_baseline": None,
@@ -571,13 +589,13 @@ def main():
                     "a functional check of the N > 1 step logic on a one-GPU box, not a scaling number")
     ap.add_argument("--no-cpu-baseline", action="store_true")
     ap.add_argument("--cpu-tokens", type=int, default=0, help="CPU baseline sample size (0 = auto)")
-    ap.add_argument("--arch", default="", help="'gelarax', 'muzopel', 'sopulorn' or 'bogupel': instead of the headline workload, prefill / decode rates of models of that design beside the "
+    ap.add_argument("--arch", default="", help="'gelarax', 'muzopel', 'sopulorn', 'bogupel' or 'kamelorn': instead of the headline workload, prefill / decode rates of models of that design beside the "
                     "closest standard model at equal size (one GPU; --prefill-lens, --steps, --warmup apply)")
     ap.add_argument("--arch-sizes", default="w1024,w2048")
     args = ap.parse_args()
     if args.arch:
-        if args.arch.lower() not in ("gelarax", "muzopel", "sopulorn", "bogupel"):
-            raise SystemExit("unknown --arch %s (gelarax, muzopel, sopulorn, bogupel)" % args.arch)
+        if args.arch.lower() not in ("gelarax", "muzopel", "sopulorn", "bogupel", "kamelorn"):
+            raise SystemExit("unknown --arch %s (gelarax, muzopel, sopulorn, bogupel, kamelorn)" % args.arch)
         if args.gpus > 1 or int(os.environ.get("WORLD_SIZE", "1")) > 1:
             raise SystemExit("--arch runs on one GPU")
         return run_arch_bench(args)

@@ -296,6 +296,55 @@ def bogupel_tensor_shapes(cfg):
     return s
 
 
+def kamelorn_config(width=2048, vocab=32000, heads=16, dim=128, rot_dim=64, vdim=128, kv_rank=512, ssm_heads=64, ssm_vdim=64, state=128, groups=8, conv=4, norm_groups=8,
+                    dense_ff=5632, experts=32, top=6, ff=1408, streams=4):
+    """six layers, eight layer runs: latent attention (dense), state space, a looped group of (state space, latent attention) that runs twice, state space (dense),
+    state space; a mixture of experts wherever not dense"""
+    lat = {"heads": heads, "dim": dim, "rot_dim": rot_dim, "vdim": vdim, "kv_rank": kv_rank, "scale": float((dim + rot_dim) ** -0.5), "rot": {"base": 10000.0, "dims": rot_dim}}
+    ssm = {"heads": ssm_heads, "vdim": ssm_vdim, "state": state, "groups": groups, "conv": conv, "norm_groups": norm_groups}
+    dense = {"kind": "dense", "ff": dense_ff}
+    moe = {"kind": "moe", "expert": {"ff": ff}, "router": {"experts": experts, "top": top, "scale": 2.0}}
+
+    def layer(kind, mlp):
+        return {"type": kind, "mixer": lat if kind == "latent_attention" else ssm, "mlp": mlp}
+    L, M = "latent_attention", "mamba2"
+    return {"architecture": "Kamelorn", "width": width, "vocab": vocab, "norm": {"eps": 1e-6}, "embedding": {"scale": 4.0}, "residual_mult": 0.5, "streams": streams,
+            "loop": {"start": 2, "stop": 4, "times": 2}, "layers": [layer(L, dense), layer(M, moe), layer(M, moe), layer(L, moe), layer(M, dense), layer(M, moe)]}
+
+
+def kamelorn_tensor_shapes(cfg):
+    W_, V, S = cfg["width"], cfg["vocab"], cfg["streams"]
+    s = {"embed": (V, W_), "final.norm": (W_,), "head": (V, W_)}
+    for li, L in enumerate(cfg["layers"]):
+        p, m = "l%d." % li, L["mixer"]
+        s.update({p + "norm1": (W_,), p + "hc1.in": (S,), p + "hc1.out": (S,), p + "hc1.mix": (S, S)})
+        if L["type"] == "latent_attention":
+            H, dn, dr, dv, R = m["heads"], m["dim"], m["rot_dim"], m["vdim"], m["kv_rank"]
+            s.update({p + "mix.q": (H * (dn + dr), W_), p + "mix.dkv": (R + dr, W_), p + "mix.dkv.norm": (R,), p + "mix.uk": (H * dn, R), p + "mix.uv": (H * dv, R),
+                      p + "mix.g": (H * dv, W_), p + "mix.o": (W_, H * dv)})
+        else:
+            H, inner = m["heads"], m["heads"] * m["vdim"]
+            C = inner + 2 * m["groups"] * m["state"]
+            s.update({p + "mix.in": (inner + C + H, W_), p + "mix.conv": (C, m["conv"]), p + "mix.conv.b": (C,), p + "mix.dt_bias": (H,), p + "mix.A_log": (H,), p + "mix.D": (H,),
+                      p + "mix.norm": (inner,), p + "mix.o": (W_, inner)})
+        mlp = L.get("mlp")
+        if not mlp:
+            continue
+        s.update({p + "norm2": (W_,), p + "hc2.in": (S,), p + "hc2.out": (S,), p + "hc2.mix": (S, S)})
+        if mlp["kind"] == "dense":
+            s.update({p + "mlp.gate": (mlp["ff"], W_), p + "mlp.up": (mlp["ff"], W_), p + "mlp.down": (W_, mlp["ff"])})
+            continue
+        E, F = mlp["router"]["experts"], mlp["expert"]["ff"]
+        s[p + "mlp.router"] = (E, W_)
+        for e in range(E):
+            s.update({p + "mlp.e%d.gate" % e: (F, W_), p + "mlp.e%d.up" % e: (F, W_), p + "mlp.e%d.down" % e: (W_, F)})
+    return s
+
+
+def write_kamelorn_dir(path, cfg, seed=0):
+    return write_gelarax_dir(path, cfg, seed, kamelorn_tensor_shapes(cfg))
+
+
 def write_bogupel_dir(path, cfg, seed=0):
     clean = dict(cfg)
     clean["layers"] = [{k: v for k, v in L.items() if not k.startswith("_")} for L in cfg["layers"]]
@@ -345,6 +394,10 @@ def write_gelarax_dir(path, cfg, seed=0, shapes=None):
                 a = 0.01 * rng.standard_normal(shape, dtype=np.float32)
             elif leaf in ("canon1", "canon2"):
                 a = 0.2 * rng.standard_normal(shape, dtype=np.float32)
+            elif leaf == "mix":          # (between residual streams: close to the identity; read-out and write-back weights near 1 / streams and 1)
+                a = np.eye(shape[0], dtype=np.float32) + 0.1 * rng.standard_normal(shape, dtype=np.float32)
+            elif ".hc1." in name or ".hc2." in name:
+                a = (1.0 / shape[0] if leaf == "in" else 1.0) + 0.1 * rng.standard_normal(shape, dtype=np.float32)
             elif leaf == "A_log":
                 a = rng.uniform(-3.0, 0.0, shape).astype(np.float32)
             elif len(shape) == 1 or leaf in ("rel", "conv"):
