@@ -724,12 +724,26 @@ int ifa_moe_experts_glu_f32(int glu_kind, float limit, const void *h_f32, size_t
 int ifa_streams_step_f32(void *x_f32, size_t rows, int streams, size_t cols, const void *embed_bf16, const int *tokens_dev, int vocab, float embed_scale, const void *y_f32,
                          size_t ldy, const void *mix_bf16, const void *out_bf16, float mult, const void *in_bf16, const void *norm_w_bf16, float eps, void *h_f32,
                          size_t ldh, void *sum_f32, size_t ldsum, ifa_stream stream);
-/* ifa_shortconv_silu_f32 without unit norms, with a bias per channel in front of the SiLU (bias_bf16 [channels], nullable) */
-int ifa_shortconv_bias_silu_f32(const void *x_f32, size_t ldx, int channels, int taps, const void *w_bf16, const void *bias_bf16, const void *seqs_dev, const int *row_seq_dev,
-                                size_t rows, void *const *slot_base_dev, size_t state_off, void *y_f32, size_t ldy, ifa_stream stream);
-/* step sizes and decays of the state space: dt = softplus(a + dt_bias[h]), decay = exp(-exp(A_log[h]) dt); outputs fp32 [rows][heads] */
-int ifa_ssm_gates_f32(const void *a_f32, size_t lda, int heads, size_t rows, const void *a_log_bf16, const void *dt_bias_bf16, void *dt_f32, void *decay_f32,
-                      ifa_stream stream);
+/* short causal convolution per channel with a bias + SiLU whose history is a RING in the slot: the input of position p lives in row p % taps of [taps][channels]
+ * (ifa_ssm_gates_ring_f32 / ifa_ssm_step_f32 write a step's last inputs there; positions before the start read as zero).  bias_bf16 nullable. */
+int ifa_conv_ring_silu_f32(const void *x_f32, size_t ldx, int channels, int taps, const void *w_bf16, const void *bias_bf16, const void *seqs_dev, const int *row_seq_dev,
+                           size_t rows, void *const *slot_base_dev, size_t ring_off, void *y_f32, size_t ldy, ifa_stream stream);
+/* step sizes and decays of the state space: dt = softplus(a + dt_bias[h]), decay = exp(-exp(A_log[h]) dt), outputs fp32 [rows][heads]; and, in the same
+ * launch, the last taps - 1 inputs x of every sequence of the step into its ring (AFTER ifa_conv_ring_silu_f32 has read it) */
+int ifa_ssm_gates_ring_f32(const void *a_f32, size_t lda, int heads, size_t rows, const void *a_log_bf16, const void *dt_bias_bf16, void *dt_f32, void *decay_f32,
+                           const void *x_f32, size_t ldx, int channels, int taps, const void *seqs_dev, int n_seqs, void *const *slot_base_dev, size_t ring_off,
+                           ifa_stream stream);
+/* ONE token per sequence (rows = sequences): convolution + SiLU of xbc = [x: heads * vdim | B: groups * state | C: groups * state] over the ring and the ring's
+ * new row, step size and decay from dt (before softplus), state update, y = S^T C + D x, in one launch.  state <= 256. */
+int ifa_ssm_step_f32(const void *xbc_f32, size_t ldx, const void *dt_f32, size_t ldd, int heads, int groups, int state, int vdim, int taps, const void *conv_w_bf16,
+                     const void *conv_b_bf16, const void *a_log_bf16, const void *dt_bias_bf16, const void *skip_bf16, const void *seqs_dev, const int *row_seq_dev, size_t rows,
+                     void *const *slot_base_dev, size_t ring_off, size_t state_off, void *out_f32, size_t ldo, ifa_stream stream);
+/* the same recurrence for prompts in chunks of 64 tokens of one sequence on the fp32 matrix cores (inputs behind the convolution, dt behind softplus, the
+ * decays' logarithms summed in double inside); ws: ifa_ssm_chunked_workspace_bytes(chunks of the step, ...), chunks = sum over the sequences of ceil(n / 64) */
+size_t ifa_ssm_chunked_workspace_bytes(size_t chunks, int heads, int groups, int state, int vdim);
+int ifa_ssm_chunked_f32(const void *x_f32, size_t ldx, const void *b_f32, size_t ldb, const void *c_f32, size_t ldc, int heads, int groups, int state, int vdim,
+                        const void *dt_f32, const void *a_log_bf16, const void *skip_bf16, const void *seqs_dev, const void *seqs_host, int n_seqs, void *const *slot_base_dev,
+                        size_t state_off, void *ws, size_t ws_bytes, void *out_f32, size_t ldo, ifa_stream stream);
 /* selective state space: per head S [state][vdim] fp32 in the slot ([heads][state][vdim]), S <- decay_t S + dt_t B_t x_t^T,
  * y_t = S^T C_t + D_h x_t; x fp32 [rows][heads * vdim], B / C fp32 [rows][groups * state] (head h reads group h / (heads / groups)),
  * dt / decay fp32 [rows][heads], D bf16 [heads].  state <= 256.  Token by token. */
@@ -757,6 +771,12 @@ int ifa_moe_route_renorm_f32(int score_kind, int renorm, float renorm_eps, float
                              const void *correction_bf16, int *idx_dev, void *wgt_f32, ifa_stream stream);
 int ifa_moe_route_rows_renorm_f32(int score_kind, int renorm, float renorm_eps, float wgt_scale, const void *h_f32, size_t ldh, size_t rows, int width,
                                   const void *router_bf16, int n_all, int top, const void *correction_bf16, int *idx_dev, void *wgt_f32, ifa_stream stream);
+/* steps of at most 64 rows: ifa_streams_step_f32 (with y and the norm) and the routing of its h (ifa_moe_route_rows_renorm_f32) in one launch.  Needs
+ * ifa_moe_streams_route_rows_fits(...) and 16-byte aligned rows. */
+int ifa_moe_streams_route_rows_fits(int streams, int width, int n_all, int top);
+int ifa_moe_streams_route_rows_f32(int score_kind, int renorm, float renorm_eps, float wgt_scale, void *x_f32, size_t rows, int streams, int width, const void *y_f32, size_t ldy,
+                                   const void *mix_bf16, const void *out_bf16, float mult, const void *in_bf16, const void *norm_w_bf16, float eps, void *h_f32, size_t ldh,
+                                   const void *router_bf16, int n_all, int top, const void *correction_bf16, int *idx_dev, void *wgt_f32, ifa_stream stream);
 
 /* ======================================================================== */
 /* Layer-list worker: a decoder whose layers are given one by one, each with its own sequence mixer, a 32-bit residual       */

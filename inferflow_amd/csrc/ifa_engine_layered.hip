@@ -7,7 +7,7 @@
 //   windowed attention   K rows (normed keys) and V rows [max_ctx][kv_heads * dim] fp32, addressed by position
 //   linear attention     S [heads][dk][dv] fp32
 //   gated delta rule     S [heads][dk][dv] fp32 + the last conv - 1 inputs of the short convolutions
-//   state space          S [heads][state][vdim] fp32 + the last conv - 1 inputs of the short convolution
+//   state space          S [heads][state][vdim] fp32 + a ring of the last inputs of the short convolution
 // An arena is allocated when its slot is first used; a sequence that starts at position 0 ignores what the slot held.
 //
 // A step = a list of sequences (ifa_seq_desc): forward() is one sequence of n tokens from position prefix_len,
@@ -32,7 +32,7 @@
 // Layers wired IFA_BLOCK_STREAMS keep several residual streams per token ([row][stream][width]) that every sub-layer reads through a learned mix
 // and writes back through another (x_t <- sum_s mix[s][t] x_s + mult * out[t] * sub(rms(sum_s in[s] x_s) w)): everything between two products
 // is ONE launch (ifa_streams_step_f32).  They mix with latent attention (rotation in halves, a gate per output column) or with the selective
-// state space (IFA_MIX_SSM: S [heads][state][vdim] + the convolution's last inputs in the slot) and feed forward through a dense SiLU-gated
+// state space (IFA_MIX_SSM: S [heads][state][vdim] + a ring of the convolution's inputs in the slot) and feed forward through a dense SiLU-gated
 // layer or a mixture whose chosen sigmoid scores are renormalized.
 // A looped layer group runs several times with the same weights: every pass has cache rows and states of its own (a layer's part of the
 // arena is repeated per pass), so the stack is walked as a list of RUNS (layer, pass); stem 3 keeps the embedding output for the passes.
@@ -117,6 +117,8 @@ struct LayeredNet {
     int *moe_idx = nullptr, *ctx0_dev = nullptr; void *moe_ws = nullptr; size_t moe_ws_bytes = 0, expand_rows = 0, kx_max = 0, vx_max = 0, top_max = 0;
     bool any_depth_avg = false, any_latent = false, any_moe = false, latent_tile_ok = true, step_expand = false;
     std::vector<int> ctx0_host; size_t step_ctx_rows = 0;
+    // state-space layers: steps whose longest sequence brings at least opt_ssm_chunk_min tokens run in chunks (ssm_chunks > 0), their workspace
+    bool any_ssm = false; int opt_ssm_chunk_min = 48; size_t ssm_chunks = 0, ssm_ws_bytes = 0; void *ssm_ws = nullptr;
     hipGraphExec_t step_exec = nullptr; hipGraph_t step_graph = nullptr; int step_slot = -1;
 };
 
@@ -596,12 +598,23 @@ int run_ssm_mixer(ifa_model *m, LLayer &L, size_t T, int nseq, const float *h, s
     const float *z = n->proj, *xbc = n->proj + SI, *dt = n->proj + SI + SC;
     int rc;
     if ((rc = linear(m, L.w_in, NI, W, h, W, T, nullptr, nullptr, 1.0f, 0, n->proj, NI))) return rc;
-    if ((rc = ifa_shortconv_bias_silu_f32(xbc, NI, (int)SC, sp.s_conv, L.T(IFA_LT_S_CONV).data, L.T(IFA_LT_S_CONV_B).data, n->seqs_dev, n->row_seq_dev, T, slots,
-                                          L.o_conv + pass_off, n->m1, SC, s))) return rc;
-    if ((rc = ifa_shortconv_tail_f32(xbc, NI, (int)SC, sp.s_conv, n->seqs_dev, nseq, slots, L.o_conv + pass_off, s))) return rc;
-    if ((rc = ifa_ssm_gates_f32(dt, NI, sp.s_heads, T, L.T(IFA_LT_S_ALOG).data, L.T(IFA_LT_S_DTBIAS).data, n->beta, n->decay, s))) return rc;
-    if ((rc = ifa_state_scan_ssm_f32(n->m1, SC, n->m1 + SI, SC, n->m1 + SI + GN, SC, sp.s_heads, sp.s_groups, sp.s_state, sp.s_vdim, n->beta, n->decay, L.T(IFA_LT_S_D).data,
-                                     n->seqs_dev, nseq, slots, L.o_rec + pass_off, n->m2, SI, s))) return rc;
+    if ((size_t)nseq == T) {      // one token per sequence: everything between the two products but the norm in one launch
+        if ((rc = ifa_ssm_step_f32(xbc, NI, dt, NI, sp.s_heads, sp.s_groups, sp.s_state, sp.s_vdim, sp.s_conv, L.T(IFA_LT_S_CONV).data, L.T(IFA_LT_S_CONV_B).data,
+                                   L.T(IFA_LT_S_ALOG).data, L.T(IFA_LT_S_DTBIAS).data, L.T(IFA_LT_S_D).data, n->seqs_dev, n->row_seq_dev, T, slots, L.o_conv + pass_off,
+                                   L.o_rec + pass_off, n->m2, SI, s))) return rc;
+    } else {
+        if ((rc = ifa_conv_ring_silu_f32(xbc, NI, (int)SC, sp.s_conv, L.T(IFA_LT_S_CONV).data, L.T(IFA_LT_S_CONV_B).data, n->seqs_dev, n->row_seq_dev, T, slots,
+                                         L.o_conv + pass_off, n->m1, SC, s))) return rc;
+        if ((rc = ifa_ssm_gates_ring_f32(dt, NI, sp.s_heads, T, L.T(IFA_LT_S_ALOG).data, L.T(IFA_LT_S_DTBIAS).data, n->beta, n->decay, xbc, NI, (int)SC, sp.s_conv, n->seqs_dev,
+                                         nseq, slots, L.o_conv + pass_off, s))) return rc;
+        if (n->ssm_chunks)
+            rc = ifa_ssm_chunked_f32(n->m1, SC, n->m1 + SI, SC, n->m1 + SI + GN, SC, sp.s_heads, sp.s_groups, sp.s_state, sp.s_vdim, n->beta, L.T(IFA_LT_S_ALOG).data,
+                                     L.T(IFA_LT_S_D).data, n->seqs_dev, n->seqs_host.data(), nseq, slots, L.o_rec + pass_off, n->ssm_ws, n->ssm_ws_bytes, n->m2, SI, s);
+        else
+            rc = ifa_state_scan_ssm_f32(n->m1, SC, n->m1 + SI, SC, n->m1 + SI + GN, SC, sp.s_heads, sp.s_groups, sp.s_state, sp.s_vdim, n->beta, n->decay, L.T(IFA_LT_S_D).data,
+                                        n->seqs_dev, nseq, slots, L.o_rec + pass_off, n->m2, SI, s);
+        if (rc) return rc;
+    }
     if ((rc = ifa_gate_groupnorm_f32(n->m2, SI, T, (int)SI, sp.s_norm_groups, L.T(IFA_LT_S_NORM).data, z, NI, c.eps, n->m2, SI, s))) return rc;
     return linear(m, (const bf16_t *)L.T(IFA_LT_S_O).data, W, SI, n->m2, SI, T, nullptr, nullptr, 1.0f, 0, out, W);
 }
@@ -639,6 +652,15 @@ int run_streams_layer(ifa_model *m, LLayer &L, size_t T, int nseq, int pass, LLa
     const void *next_in = next ? next->T(IFA_LT_HC1_IN).data : nullptr, *next_norm = next ? next->T(IFA_LT_NORM1).data : n->out_norm.data;
     int rc;
     if ((rc = sp.mixer == IFA_MIX_LATENT ? run_latent_mixer(m, L, T, n->h, po, n->m3) : run_ssm_mixer(m, L, T, nseq, n->h, po, n->m3))) return rc;
+    if (moe && n->opt_fuse_post && T <= 8 && ifa_moe_streams_route_rows_fits((int)streams_of(n), c.width, sp.x_experts, sp.x_top)) {
+        // a few rows: the streams' update, the norm, the router's product and its choice in one launch
+        if ((rc = ifa_moe_streams_route_rows_f32(sp.x_score, sp.x_renorm, sp.x_renorm_eps, sp.x_wgt_scale, n->x, T, (int)streams_of(n), c.width, n->m3, W, L.T(IFA_LT_HC1_MIX).data,
+                                                 L.T(IFA_LT_HC1_OUT).data, c.residual_mult, L.T(IFA_LT_HC2_IN).data, L.T(IFA_LT_NORM2).data, c.eps, n->h, W,
+                                                 L.T(IFA_LT_X_ROUTER).data, sp.x_experts, sp.x_top, nullptr, n->moe_idx, n->moe_wgt, s))) return rc;
+        if ((rc = ifa_moe_experts_glu_f32(sp.x_glu, sp.x_limit, n->h, W, T, (int)W, sp.x_ff, sp.x_experts, sp.x_top, L.T(IFA_LT_X_UP).data, L.T(IFA_LT_X_DOWN).data, n->moe_idx,
+                                          n->moe_wgt, c.ops32, n->moe_ws, n->moe_ws_bytes, n->m1, W, 0, s))) return rc;
+        return streams_step(m, T, false, n->m1, &L, 2, next_in, next_norm);
+    }
     if ((rc = streams_step(m, T, false, n->m3, &L, 1, any_ffn ? L.T(IFA_LT_HC2_IN).data : next_in, any_ffn ? L.T(IFA_LT_NORM2).data : next_norm))) return rc;
     if (!any_ffn) return IFA_OK;
     if (!moe) {
@@ -837,7 +859,7 @@ int lay_destroy(ifa_model *m)
     lay_free(n->embd.data); lay_free(n->out_norm.data); lay_free(n->lm_head.data); lay_free(n->embd_norm.data); lay_free(n->bigram.data);
     lay_free(n->out_norm_b.data); lay_free(n->out_norm_alpha.data); lay_free(n->loop_step.data);
     lay_free(n->x0); lay_free(n->cg_decay); lay_free(n->cg_unit); lay_free(n->cg_rem);
-    lay_free(n->m4); lay_free(n->m5); lay_free(n->stack); lay_free(n->moe_wgt); lay_free(n->moe_idx); lay_free(n->moe_ws); lay_free(n->kx); lay_free(n->vx);
+    lay_free(n->m4); lay_free(n->m5); lay_free(n->stack); lay_free(n->moe_wgt); lay_free(n->moe_idx); lay_free(n->moe_ws); lay_free(n->kx); lay_free(n->vx); lay_free(n->ssm_ws);
     for (float *p : n->slot_ptr) lay_free(p);
     lay_free(n->slot_base_dev);
     if (n->tab_pin) (void)hipHostFree(n->tab_pin);
@@ -1013,7 +1035,8 @@ int lay_finalize(ifa_model *m)
             if ((rc = cat_rows(w, b, L.T(IFA_LT_S_IN), nullptr, W, at, m->stream))) return rc;
             const size_t SI = (size_t)sp.s_heads * sp.s_vdim, SC = SI + 2 * (size_t)sp.s_groups * sp.s_state;
             L.o_rec = off; off += align4((size_t)sp.s_heads * sp.s_state * sp.s_vdim);
-            L.o_conv = off; off += align4((size_t)std::max(sp.s_conv - 1, 0) * SC);
+            L.o_conv = off; off += align4((size_t)sp.s_conv * SC);          // (a ring: row = position modulo taps)
+            n->any_ssm = true;
             n->mix_max = std::max({n->mix_max, SC, SI, W});
             n->heads_max = std::max(n->heads_max, (size_t)sp.s_heads);
         } else if (sp.mixer == IFA_MIX_WINDOW_LINEAR) {
@@ -1154,10 +1177,11 @@ int lay_set_option(ifa_model *m, const char *name, int value)
     if (!strcmp(name, "tap_layers")) { n->opt_tap_layers = value; drop_step_graph(n); return IFA_OK; }
     if (!strcmp(name, "fuse_rows")) { n->opt_fuse_rows = value; drop_step_graph(n); return IFA_OK; }
     if (!strcmp(name, "fuse_post")) { n->opt_fuse_post = value; drop_step_graph(n); return IFA_OK; }
+    if (!strcmp(name, "ssm_chunk_min")) { n->opt_ssm_chunk_min = value; return IFA_OK; }
     if (!strcmp(name, "attn_tile_min")) { n->opt_attn_tile_min = value; return IFA_OK; }
     if (!strcmp(name, "graph")) { n->opt_graph = value; drop_step_graph(n); return IFA_OK; }
     if (!strcmp(name, "ops32")) { IFA_HIP_CHECK(hipStreamSynchronize(m->stream)); n->cfg.ops32 = value ? 1 : 0; drop_step_graph(n); return IFA_OK; }
-    return ifa_fail(IFA_ERR_ARG, "ifa_model_set_option: unknown option '%s' (layer-list model: tap_layers, graph, ops32, attn_tile_min, fuse_rows, fuse_post)", name);
+    return ifa_fail(IFA_ERR_ARG, "ifa_model_set_option: unknown option '%s' (layer-list model: tap_layers, graph, ops32, attn_tile_min, fuse_rows, fuse_post, ssm_chunk_min)", name);
 }
 
 int lay_set_excluded(ifa_model *m, const int *ids_host, int cnt)
@@ -1270,6 +1294,22 @@ int lay_step(ifa_model *m, int nseq, const int *tokens_host, const int *lens, co
         IFA_HIP_CHECK(hipMalloc((void **)&n->kx, n->step_ctx_rows * n->kx_max * 4));
         IFA_HIP_CHECK(hipMalloc((void **)&n->vx, n->step_ctx_rows * n->vx_max * 4));
         n->expand_rows = n->step_ctx_rows;
+    }
+    n->ssm_chunks = 0;
+    if (n->any_ssm) {
+        int longest = 0; size_t chunks = 0, need = 0;
+        for (int q = 0; q < nseq; q++) { longest = std::max(longest, lens[q]); chunks += ((size_t)lens[q] + 63) / 64; }
+        if (longest >= std::max(n->opt_ssm_chunk_min, 2)) {
+            n->ssm_chunks = chunks;
+            for (const LLayer &L : n->layers)
+                if (L.spec.mixer == IFA_MIX_SSM) need = std::max(need, ifa_ssm_chunked_workspace_bytes(chunks, L.spec.s_heads, L.spec.s_groups, L.spec.s_state, L.spec.s_vdim));
+            if (need > n->ssm_ws_bytes) {
+                IFA_HIP_CHECK(hipStreamSynchronize(m->stream));
+                lay_free(n->ssm_ws); n->ssm_ws = nullptr; n->ssm_ws_bytes = 0;
+                IFA_HIP_CHECK(hipMalloc(&n->ssm_ws, need));
+                n->ssm_ws_bytes = need;
+            }
+        }
     }
     if ((rc = run_layers(m, T, nseq))) return rc;
     ifa_stream s = (ifa_stream)m->stream;

@@ -13,6 +13,7 @@
 #include <algorithm>
 #include "ifa_host.h"
 #include "ifa_f32_common.h"
+#include "ifa_streams.h"
 #include "inferflow_amd.h"
 
 using namespace ifa32;
@@ -148,6 +149,94 @@ __global__ void __launch_bounds__(1024) k_moe_route_rows(const float *h, size_t 
         __syncthreads();
     }
     if (renorm && threadIdx.x == 0) { const float den = chosen + renorm_eps; for (int k = 0; k < top; k++) wgt[(size_t)t * top + k] = wgt[(size_t)t * top + k] / den * wgt_scale; }
+}
+
+// Steps of a few rows of blocks with several residual streams, one launch: what lies between the mixer and the experts (streams_row), the
+// router's product and its choice.  One workgroup of sixteen waves per row; the router's rows are requested before anything else (they do
+// not depend on the row) as far as they fit RW_PRE pieces per thread; the choice runs in the first wave's registers (n_all <= 64 RW_E).
+constexpr int RW_PRE = 8, RW_E = 8;
+struct RouteArgs {
+    const bf16_t *router; int n_all, top, score_kind, renorm; float renorm_eps, wgt_scale;
+    const bf16_t *corr; int *idx; float *wgt; int pre;      // pre: every wave's share of the router in registers ahead
+};
+
+template <int SMAX>
+__global__ void __launch_bounds__(1024) k_streams_route_rows(StreamArgs P, RouteArgs R)
+{
+    __shared__ float lds[SMAX * SMAX + 2 * SMAX + 17];
+    extern __shared__ float hs[];          // [cols] the normed row, [n_all] logits
+    float *sc = hs + P.cols;
+    const int t = blockIdx.x, lane = threadIdx.x & 63, wave = threadIdx.x >> 6, W = P.cols, nk = (W + 511) / 512;
+    u32x4m pw[RW_PRE];
+    if (R.pre) {
+#pragma unroll
+        for (int a = 0; a < RW_PRE; a++) {
+            const int e = wave + 16 * (a / nk), k = lane * 8 + 512 * (a % nk);
+            if (e < R.n_all && k < W) pw[a] = *reinterpret_cast<const u32x4m *>(R.router + (size_t)e * W + k);
+        }
+    }
+    streams_row<SMAX, true>(P, t, lds, hs);
+    __syncthreads();
+    auto dot8 = [&](const u32x4m &w, int k, float acc) {
+        const float4 a0 = *reinterpret_cast<const float4 *>(hs + k), a1 = *reinterpret_cast<const float4 *>(hs + k + 4);
+        acc = fmaf(a0.x, __uint_as_float(w[0] << 16), acc); acc = fmaf(a0.y, __uint_as_float(w[0] & 0xFFFF0000u), acc);
+        acc = fmaf(a0.z, __uint_as_float(w[1] << 16), acc); acc = fmaf(a0.w, __uint_as_float(w[1] & 0xFFFF0000u), acc);
+        acc = fmaf(a1.x, __uint_as_float(w[2] << 16), acc); acc = fmaf(a1.y, __uint_as_float(w[2] & 0xFFFF0000u), acc);
+        acc = fmaf(a1.z, __uint_as_float(w[3] << 16), acc); return fmaf(a1.w, __uint_as_float(w[3] & 0xFFFF0000u), acc);
+    };
+    if (R.pre) {
+        float acc = 0.0f;
+#pragma unroll
+        for (int a = 0; a < RW_PRE; a++) {
+            const int e = wave + 16 * (a / nk), k = lane * 8 + 512 * (a % nk);
+            if (e < R.n_all) {
+                if (k < W) acc = dot8(pw[a], k, acc);
+                if (a % nk == nk - 1) { acc = wave_sum(acc); if (lane == 0) sc[e] = acc; acc = 0.0f; }
+            }
+        }
+    } else {
+        for (int e = wave; e < R.n_all; e += 16) {
+            float acc = 0.0f;
+#pragma unroll 4
+            for (int k = lane * 8; k < W; k += 512) acc = dot8(*reinterpret_cast<const u32x4m *>(R.router + (size_t)e * W + k), k, acc);
+            acc = wave_sum(acc);
+            if (lane == 0) sc[e] = acc;
+        }
+    }
+    __syncthreads();
+    if (wave) return;
+    float s[RW_E], ch[RW_E], mx = -INFINITY;
+#pragma unroll
+    for (int r = 0; r < RW_E; r++) { const int e = lane + 64 * r; s[r] = e < R.n_all ? sc[e] : -INFINITY; mx = fmaxf(mx, s[r]); }
+    if (R.score_kind == 1) {
+#pragma unroll
+        for (int r = 0; r < RW_E; r++) s[r] = sigmoid_f(s[r]);
+    } else {
+        mx = wave_max(mx);
+        float sum = 0.0f;
+#pragma unroll
+        for (int r = 0; r < RW_E; r++) { s[r] = expf(s[r] - mx); sum += s[r]; }
+        sum = wave_sum(sum);
+#pragma unroll
+        for (int r = 0; r < RW_E; r++) s[r] /= sum;
+    }
+#pragma unroll
+    for (int r = 0; r < RW_E; r++) { const int e = lane + 64 * r; ch[r] = e < R.n_all ? s[r] + (R.corr ? bf2f(R.corr[e]) : 0.0f) : -INFINITY; }
+    float chosen = 0.0f;
+    for (int k = 0; k < R.top; k++) {
+        float best = -INFINITY, bs = 0.0f; int bi = 0x7FFFFFFF;
+#pragma unroll
+        for (int r = 0; r < RW_E; r++) { const int e = lane + 64 * r; if (e < R.n_all && (ch[r] > best || (ch[r] == best && e < bi))) { best = ch[r]; bs = s[r]; bi = e; } }
+        for (int o = 32; o > 0; o >>= 1) {
+            const float ov = __shfl_xor(best, o, 64), os = __shfl_xor(bs, o, 64); const int oi = __shfl_xor(bi, o, 64);
+            if (ov > best || (ov == best && oi < bi)) { best = ov; bs = os; bi = oi; }
+        }
+        chosen += bs;
+#pragma unroll
+        for (int r = 0; r < RW_E; r++) if (lane + 64 * r == bi) ch[r] = -INFINITY;
+        if (lane == 0) { R.idx[(size_t)t * R.top + k] = bi; R.wgt[(size_t)t * R.top + k] = bs; }
+    }
+    if (R.renorm && lane == 0) { const float den = chosen + R.renorm_eps; for (int k = 0; k < R.top; k++) R.wgt[(size_t)t * R.top + k] = R.wgt[(size_t)t * R.top + k] / den * R.wgt_scale; }
 }
 
 // grid (ff chunks, pairs): act[p][n] = gelu(W_up[e][n] . h[t]); a wave per n at a time.  Identity pairs do nothing.
@@ -363,6 +452,34 @@ int ifa_moe_route_rows_renorm_f32(int score_kind, int renorm, float renorm_eps, 
     hipLaunchKernelGGL(k_moe_route_rows, dim3((unsigned)rows), dim3(n_all > 8 ? 1024 : 256), (size_t)n_all * 8, ifa_s(stream), (const float *)h_f32, ldh, width,
                        (const bf16_t *)router_bf16, n_all, top, (const bf16_t *)correction_bf16, idx_dev, (float *)wgt_f32, vec, score_kind, (const float *)nullptr, (size_t)0,
                        (const bf16_t *)nullptr, (const bf16_t *)nullptr, (const bf16_t *)nullptr, (float *)nullptr, renorm ? 1 : 0, renorm_eps, wgt_scale);
+    IFA_LAUNCH_CHECK();
+    return IFA_OK;
+}
+
+int ifa_moe_streams_route_rows_fits(int streams, int width, int n_all, int top)
+{
+    return streams >= 1 && streams <= 16 && width > 0 && width % 8 == 0 && n_all >= 1 && n_all <= 64 * RW_E && top >= 1 && top <= n_all && ((size_t)width + n_all) * 4 <= 60 * 1024;
+}
+
+int ifa_moe_streams_route_rows_f32(int score_kind, int renorm, float renorm_eps, float wgt_scale, void *x_f32, size_t rows, int streams, int width, const void *y_f32, size_t ldy,
+                                   const void *mix_bf16, const void *out_bf16, float mult, const void *in_bf16, const void *norm_w_bf16, float eps, void *h_f32, size_t ldh,
+                                   const void *router_bf16, int n_all, int top, const void *correction_bf16, int *idx_dev, void *wgt_f32, ifa_stream stream)
+{
+    IFA_REQUIRE(x_f32 && y_f32 && norm_w_bf16 && h_f32 && router_bf16 && idx_dev && wgt_f32, "ifa_moe_streams_route_rows_f32: null pointer");
+    IFA_REQUIRE(rows > 0 && rows <= 64 && ifa_moe_streams_route_rows_fits(streams, width, n_all, top) && ldy >= (size_t)width && ldh >= (size_t)width && ldy % 4 == 0 && ldh % 4 == 0
+                && (((uintptr_t)x_f32 | (uintptr_t)y_f32 | (uintptr_t)h_f32 | (uintptr_t)router_bf16) & 15) == 0 && (score_kind == 0 || score_kind == 1),
+                "ifa_moe_streams_route_rows_f32: bad shape or alignment");
+    StreamArgs P;
+    P.x = (float *)x_f32; P.S = streams; P.cols = width; P.embed = nullptr; P.tokens = nullptr; P.vocab = 0; P.scale = 1.0f; P.y = (const float *)y_f32; P.ldy = ldy;
+    P.mix = (const bf16_t *)mix_bf16; P.out = (const bf16_t *)out_bf16; P.mult = mult; P.in = (const bf16_t *)in_bf16; P.w = (const bf16_t *)norm_w_bf16; P.eps = eps;
+    P.h = (float *)h_f32; P.ldh = ldh; P.sum_out = nullptr; P.ldsum = 0;
+    RouteArgs R;
+    R.router = (const bf16_t *)router_bf16; R.n_all = n_all; R.top = top; R.score_kind = score_kind; R.renorm = renorm ? 1 : 0; R.renorm_eps = renorm_eps; R.wgt_scale = wgt_scale;
+    R.corr = (const bf16_t *)correction_bf16; R.idx = idx_dev; R.wgt = (float *)wgt_f32; R.pre = ((n_all + 15) / 16) * ((width + 511) / 512) <= RW_PRE ? 1 : 0;
+    const size_t smem = ((size_t)width + n_all) * 4;
+#define IFA_SR(SM) hipLaunchKernelGGL(k_streams_route_rows<SM>, dim3((unsigned)rows), dim3(1024), smem, ifa_s(stream), P, R)
+    if (streams == 1) IFA_SR(1); else if (streams == 2) IFA_SR(2); else if (streams <= 4) IFA_SR(4); else if (streams <= 8) IFA_SR(8); else IFA_SR(16);
+#undef IFA_SR
     IFA_LAUNCH_CHECK();
     return IFA_OK;
 }

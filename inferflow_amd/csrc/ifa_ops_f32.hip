@@ -3,6 +3,7 @@
 #include <algorithm>
 #include "ifa_host.h"
 #include "ifa_f32_common.h"
+#include "ifa_streams.h"
 
 using namespace ifa32;
 
@@ -188,121 +189,12 @@ __global__ void __launch_bounds__(256) k_norm_add_norm(float *__restrict__ x, si
     for (int c = threadIdx.x; c < cols; c += blockDim.x) hr[c] = xr[c] * rinv2 * (w_off + bf2f(w_before[c]));
 }
 
-// Several residual streams per row (x [rows][S][cols]), one workgroup per row; what lies between two sub-layers:
-//   0. (embed not null) X_s <- embed[token] * scale for every s          (the start of the stack)
-//   1. (y not null)     X_t <- sum_s mix[s][t] X_s + mult * out[t] * y    (all new streams from the old ones; mix / out null: identity / ones)
-//   2. u = sum_s in[s] X_s (in null: ones);  sum_out <- u (if asked for)
-//   3. (w not null)     h = u / sqrt(mean(u^2) + eps) * w
-// A thread keeps its columns of all streams in registers, and its pieces of u (16-byte pieces when VEC) from stage 2 to stage 3.
-struct StreamArgs {
-    float *x; int S, cols;
-    const bf16_t *embed; const int *tokens; int vocab; float scale;
-    const float *y; size_t ldy; const bf16_t *mix, *out; float mult;
-    const bf16_t *in, *w; float eps;
-    float *h; size_t ldh; float *sum_out; size_t ldsum;
-};
-
-template <bool VEC> struct StreamPiece;
-template <> struct StreamPiece<true> { static constexpr int N = 4; };
-template <> struct StreamPiece<false> { static constexpr int N = 1; };
-
-constexpr int ST_KEEP = 4;          // pieces of u per thread that stay in registers (more columns: they are read back from h)
-
+// one workgroup per row (ifa_streams.h)
 template <int SMAX, bool VEC>
 __global__ void __launch_bounds__(1024) k_streams_step(StreamArgs P)
 {
-    constexpr int N = StreamPiece<VEC>::N;
-    __shared__ float red[17], mx[SMAX * SMAX], ob[SMAX], ib[SMAX];
-    const int S = P.S, cols = P.cols, tid = threadIdx.x, nt = blockDim.x;
-    for (int e = tid; e < S * S; e += nt) mx[e] = P.mix ? bf2f(P.mix[e]) : (e / S == e % S ? 1.0f : 0.0f);
-    for (int e = tid; e < S; e += nt) { ob[e] = (P.out ? bf2f(P.out[e]) : 1.0f) * P.mult; ib[e] = P.in ? bf2f(P.in[e]) : 1.0f; }
-    __syncthreads();
-    float *xr = P.x + (size_t)blockIdx.x * S * cols;
-    const float *yr = P.y ? P.y + (size_t)blockIdx.x * P.ldy : nullptr;
-    float *hr = P.h ? P.h + (size_t)blockIdx.x * P.ldh : nullptr, *sr = P.sum_out ? P.sum_out + (size_t)blockIdx.x * P.ldsum : nullptr;
-    const bf16_t *er = P.embed ? P.embed + (size_t)min(max(P.tokens[blockIdx.x], 0), P.vocab - 1) * cols : nullptr;
-    const int pieces = cols / N;
-    float keep[ST_KEEP][N];
-    float q = 0.0f;
-    auto piece = [&](int c, float (&u)[N]) {
-        float xs[SMAX][N];
-        if (er) {
-#pragma unroll
-            for (int k = 0; k < N; k++) { const float v = bf2f(er[c + k]) * P.scale; 
-#pragma unroll
-                for (int s = 0; s < SMAX; s++) xs[s][k] = v; }
-        } else {
-#pragma unroll
-            for (int s = 0; s < SMAX; s++)
-                if (s < S) {
-                    if constexpr (VEC) { const float4 v = *reinterpret_cast<const float4 *>(xr + (size_t)s * cols + c); xs[s][0] = v.x; xs[s][1] = v.y; xs[s][2] = v.z; xs[s][3] = v.w; }
-                    else xs[s][0] = xr[(size_t)s * cols + c];
-                }
-        }
-#pragma unroll
-        for (int k = 0; k < N; k++) u[k] = 0.0f;
-        float yv[N];
-        if (yr) {
-            if constexpr (VEC) { const float4 v = *reinterpret_cast<const float4 *>(yr + c); yv[0] = v.x; yv[1] = v.y; yv[2] = v.z; yv[3] = v.w; }
-            else yv[0] = yr[c];
-        }
-#pragma unroll
-        for (int t = 0; t < SMAX; t++)
-            if (t < S) {
-                float n[N];
-                if (yr) {
-#pragma unroll
-                    for (int k = 0; k < N; k++) n[k] = ob[t] * yv[k];
-#pragma unroll
-                    for (int s = 0; s < SMAX; s++)
-                        if (s < S) {
-#pragma unroll
-                            for (int k = 0; k < N; k++) n[k] = fmaf(mx[s * S + t], xs[s][k], n[k]);
-                        }
-                } else {
-#pragma unroll
-                    for (int k = 0; k < N; k++) n[k] = xs[t][k];
-                }
-                if (yr || er) {
-                    if constexpr (VEC) *reinterpret_cast<float4 *>(xr + (size_t)t * cols + c) = make_float4(n[0], n[1], n[2], n[3]);
-                    else xr[(size_t)t * cols + c] = n[0];
-                }
-#pragma unroll
-                for (int k = 0; k < N; k++) u[k] = fmaf(ib[t], n[k], u[k]);
-            }
-        if (sr) {
-#pragma unroll
-            for (int k = 0; k < N; k++) sr[c + k] = u[k];
-        }
-#pragma unroll
-        for (int k = 0; k < N; k++) q = fmaf(u[k], u[k], q);
-    };
-#pragma unroll
-    for (int i = 0; i < ST_KEEP; i++) { const int p = tid + i * nt; if (p < pieces) piece(p * N, keep[i]); }
-    for (int p = tid + ST_KEEP * nt; p < pieces; p += nt) {
-        float u[N];
-        piece(p * N, u);
-        if (P.w) {
-#pragma unroll
-            for (int k = 0; k < N; k++) hr[p * N + k] = u[k];
-        }
-    }
-    if (!P.w) return;
-    const float rinv = 1.0f / sqrtf(block_sum(q, red) / (float)cols + P.eps);
-#pragma unroll
-    for (int i = 0; i < ST_KEEP; i++) {
-        const int p = tid + i * nt;
-        if (p < pieces) {
-            if constexpr (VEC) {
-                const int c = p * 4;
-                *reinterpret_cast<float4 *>(hr + c) = make_float4(keep[i][0] * rinv * bf2f(P.w[c]), keep[i][1] * rinv * bf2f(P.w[c + 1]), keep[i][2] * rinv * bf2f(P.w[c + 2]),
-                                                                  keep[i][3] * rinv * bf2f(P.w[c + 3]));
-            } else hr[p] = keep[i][0] * rinv * bf2f(P.w[p]);
-        }
-    }
-    for (int p = tid + ST_KEEP * nt; p < pieces; p += nt)
-#pragma unroll
-        for (int k = 0; k < N; k++) hr[p * N + k] = hr[p * N + k] * rinv * bf2f(P.w[p * N + k]);
+    __shared__ float lds[SMAX * SMAX + 2 * SMAX + 17];
+    streams_row<SMAX, VEC>(P, blockIdx.x, lds, nullptr);
 }
 
 // stack[count - 1] <- x; x <- sum_j w[j] stack[j]  (element-wise over n = rows * cols values)
@@ -563,7 +455,7 @@ int ifa_streams_step_f32(void *x_f32, size_t rows, int streams, size_t cols, con
     const bool vec = cols % 4 == 0 && ((uintptr_t)x_f32 & 15) == 0 && (!y_f32 || (ldy % 4 == 0 && ((uintptr_t)y_f32 & 15) == 0))
                      && (!norm_w_bf16 || (ldh % 4 == 0 && ((uintptr_t)h_f32 & 15) == 0));
     const size_t pieces = vec ? cols / 4 : cols;
-    const unsigned nt = pieces <= 64 ? 64 : (pieces <= 128 ? 128 : (pieces <= 512 ? 256 : (pieces <= 2048 ? 512 : 1024)));
+    const unsigned nt = (unsigned)std::min<size_t>(1024, std::max<size_t>(64, (pieces + 63) / 64 * 64));
 #define IFA_ST(SM) { if (vec) hipLaunchKernelGGL((k_streams_step<SM, true>), dim3((unsigned)rows), dim3(nt), 0, ifa_s(stream), P); \
                      else hipLaunchKernelGGL((k_streams_step<SM, false>), dim3((unsigned)rows), dim3(nt), 0, ifa_s(stream), P); }
     if (streams == 1) IFA_ST(1) else if (streams == 2) IFA_ST(2) else if (streams <= 4) IFA_ST(4) else if (streams <= 8) IFA_ST(8) else IFA_ST(16)

@@ -1,5 +1,5 @@
 // ifa_seqmix.hip -- sequence mixers with a recurrent state instead of a key / value cache, on 32-bit activations:
-//   * short causal convolution per channel (+ bias) + SiLU (+ unit-norm of head groups), its tail carried per sequence
+//   * short causal convolution per channel + SiLU (+ unit-norm of head groups), its tail carried per sequence
 //   * per-head matrix state S [dk][dv] advanced token by token:
 //       kind 0  linear attention with a constant decay per head:  S <- d S + k v^T;                      o = S^T q
 //     (in_act = 1: q, k, v pass SiLU as they are read)
@@ -8,8 +8,7 @@
 //   * the gates of the delta rule (beta = sigmoid, g = exp(-exp(A_log) softplus(a + dt_bias)))
 //   * the generalized delta rule with a decay w and a removal rate per key channel: S <- diag(w) S - b (u^T S) + k v^T, o = S^T q
 //     (u the unit key, b = removal rate * u), and its gates
-//   * the step sizes and decays of the state space (beta = softplus(a + dt_bias), g = exp(-exp(A_log) beta))
-//   * RMS norm over channel groups with a weight and an output gate (sigmoid or SiLU) behind it, or a SiLU gate in front of it
+//   * RMS norm over channel groups with a weight and an output gate (sigmoid or SiLU)
 // Everything that enters a recurrence is fp32; states live in fp32 in the slot arena of the worker (a table of one
 // base pointer per slot + an offset per layer).  A sequence that starts at position 0 starts from a zero state,
 // whatever the slot held before.
@@ -21,15 +20,14 @@ using namespace ifa32;
 
 namespace {
 
-// grid: (rows, channel slices).  y[t][c] = silu(sum_j w[c][j] in(i - (taps - 1) + j)[c] + b[c]) (b may be absent); in(idx) for idx < 0 comes from the
+// grid: (rows, channel slices).  y[t][c] = silu(sum_j w[c][j] in(i - (taps - 1) + j)[c]); in(idx) for idx < 0 comes from the
 // sequence's carried tail (rows [taps - 1][C], oldest first) or is zero at the start of a sequence.  Then channels
 // [0, norm_cols) are turned into unit vectors in groups of gdim (x / sqrt(sum x^2 + l2_eps)) and channels [0, scale_cols)
 // are multiplied by qscale.
 __global__ void __launch_bounds__(256) k_shortconv_silu(const float *__restrict__ x, size_t ldx, int C, int taps, const bf16_t *__restrict__ w,
                                                         const SeqDesc *__restrict__ seqs, const int *__restrict__ row_seq,
                                                         float *const *__restrict__ slot_base, size_t state_off, int norm_cols, int gdim,
-                                                        float l2_eps, int scale_cols, float qscale, float *__restrict__ y, size_t ldy, int slice,
-                                                        const bf16_t *__restrict__ bias)
+                                                        float l2_eps, int scale_cols, float qscale, float *__restrict__ y, size_t ldy, int slice)
 {
     extern __shared__ float ys[];
     const int t = blockIdx.x;
@@ -46,7 +44,6 @@ __global__ void __launch_bounds__(256) k_shortconv_silu(const float *__restrict_
             else v = tail ? tail[(size_t)(taps - 1 + idx) * C + c] : 0.0f;
             acc = fmaf(bf2f(w[(size_t)c * taps + j]), v, acc);
         }
-        if (bias) acc += bf2f(bias[c]);
         ys[c - c_lo] = silu_exact(acc);
     }
     __syncthreads();
@@ -184,18 +181,6 @@ __global__ void __launch_bounds__(256) k_delta_gates(const float *__restrict__ b
     const int t = idx / H, h = idx % H;
     beta[idx] = sigmoid_f(b[(size_t)t * ldb + h]);
     g[idx] = expf(-expf(bf2f(A_log[h])) * softplus_f(a[(size_t)t * lda + h] + bf2f(dt_bias[h])));
-}
-
-// dt[t][h] = softplus(a[t][h] + dt_bias[h]);  g[t][h] = exp(-exp(A_log[h]) * dt[t][h])
-__global__ void __launch_bounds__(256) k_ssm_gates(const float *__restrict__ a, size_t lda, int H, int T, const bf16_t *__restrict__ A_log,
-                                                   const bf16_t *__restrict__ dt_bias, float *__restrict__ dt, float *__restrict__ g)
-{
-    const int idx = blockIdx.x * blockDim.x + threadIdx.x;
-    if (idx >= T * H) return;
-    const int t = idx / H, h = idx % H;
-    const float d = softplus_f(a[(size_t)t * lda + h] + bf2f(dt_bias[h]));
-    dt[idx] = d;
-    g[idx] = expf(-expf(bf2f(A_log[h])) * d);
 }
 
 struct ScanArgs {
@@ -648,41 +633,13 @@ __global__ void __launch_bounds__(256) k_gated_groupnorm(const float *__restrict
     }
 }
 
-// y[t][c] = v / sqrt(mean_group(v^2) + eps) * w[c], v = o[t][c] * silu(gate[t][c]): the gate in front of the norm; one workgroup per row
-__global__ void __launch_bounds__(512) k_gate_groupnorm(const float *__restrict__ o, size_t ldo, int C, int group, const bf16_t *__restrict__ w, const float *__restrict__ gate,
-                                                        size_t ldg, float eps, float *__restrict__ y, size_t ldy)
-{
-    extern __shared__ float vs[];          // [C]
-    __shared__ float red[17];
-    const int t = blockIdx.x, lane = threadIdx.x & 63, wave = threadIdx.x >> 6, nw = blockDim.x >> 6;
-    const float *orow = o + (size_t)t * ldo, *grow = gate + (size_t)t * ldg;
-    float *yrow = y + (size_t)t * ldy;
-    for (int c = threadIdx.x; c < C; c += blockDim.x) vs[c] = orow[c] * silu_exact(grow[c]);
-    __syncthreads();
-    if (C / group < nw) {          // fewer groups than waves: the whole workgroup works on each group
-        for (int gi = 0; gi < C / group; gi++) {
-            float s = 0.0f;
-            for (int e = threadIdx.x; e < group; e += blockDim.x) { const float v = vs[gi * group + e]; s = fmaf(v, v, s); }
-            const float r = 1.0f / sqrtf(block_sum(s, red) / (float)group + eps);
-            for (int e = threadIdx.x; e < group; e += blockDim.x) { const int c = gi * group + e; yrow[c] = vs[c] * r * bf2f(w[c]); }
-        }
-        return;
-    }
-    for (int gi = wave; gi < C / group; gi += nw) {
-        float s = 0.0f;
-        for (int e = lane; e < group; e += 64) { const float v = vs[gi * group + e]; s = fmaf(v, v, s); }
-        const float r = 1.0f / sqrtf(wave_sum(s) / (float)group + eps);
-        for (int e = lane; e < group; e += 64) { const int c = gi * group + e; yrow[c] = vs[c] * r * bf2f(w[c]); }
-    }
-}
-
 } // namespace
 
 extern "C" {
 
-static int shortconv_silu(const void *x_f32, size_t ldx, int channels, int taps, const void *w_bf16, const void *bias_bf16, const void *seqs_dev, const int *row_seq_dev,
-                          size_t rows, void *const *slot_base_dev, size_t state_off, int norm_cols, int group_dim, float l2_eps, int scale_cols,
-                          float scale, void *y_f32, size_t ldy, ifa_stream stream)
+int ifa_shortconv_silu_f32(const void *x_f32, size_t ldx, int channels, int taps, const void *w_bf16, const void *seqs_dev, const int *row_seq_dev,
+                           size_t rows, void *const *slot_base_dev, size_t state_off, int norm_cols, int group_dim, float l2_eps, int scale_cols,
+                           float scale, void *y_f32, size_t ldy, ifa_stream stream)
 {
     IFA_REQUIRE(x_f32 && w_bf16 && seqs_dev && row_seq_dev && slot_base_dev && y_f32, "ifa_shortconv_silu_f32: null pointer");
     IFA_REQUIRE(channels > 0 && taps >= 1 && taps <= 64 && rows > 0 && ldx >= (size_t)channels && ldy >= (size_t)channels, "ifa_shortconv_silu_f32: bad shape");
@@ -695,23 +652,9 @@ static int shortconv_silu(const void *x_f32, size_t ldx, int channels, int taps,
     IFA_REQUIRE((size_t)slice * 4 <= 64 * 1024, "ifa_shortconv_silu_f32: norm groups of %d channels do not fit the LDS", group_dim);
     hipLaunchKernelGGL(k_shortconv_silu, dim3((unsigned)rows, ifa_cdiv((size_t)channels, (size_t)slice)), dim3(256), (size_t)slice * 4, ifa_s(stream),
                        (const float *)x_f32, ldx, channels, taps, (const bf16_t *)w_bf16, (const SeqDesc *)seqs_dev, row_seq_dev, (float *const *)slot_base_dev,
-                       state_off, norm_cols, group_dim, l2_eps, scale_cols, scale, (float *)y_f32, ldy, slice, (const bf16_t *)bias_bf16);
+                       state_off, norm_cols, group_dim, l2_eps, scale_cols, scale, (float *)y_f32, ldy, slice);
     IFA_LAUNCH_CHECK();
     return IFA_OK;
-}
-
-int ifa_shortconv_silu_f32(const void *x_f32, size_t ldx, int channels, int taps, const void *w_bf16, const void *seqs_dev, const int *row_seq_dev,
-                           size_t rows, void *const *slot_base_dev, size_t state_off, int norm_cols, int group_dim, float l2_eps, int scale_cols,
-                           float scale, void *y_f32, size_t ldy, ifa_stream stream)
-{
-    return shortconv_silu(x_f32, ldx, channels, taps, w_bf16, nullptr, seqs_dev, row_seq_dev, rows, slot_base_dev, state_off, norm_cols, group_dim, l2_eps, scale_cols, scale,
-                          y_f32, ldy, stream);
-}
-
-int ifa_shortconv_bias_silu_f32(const void *x_f32, size_t ldx, int channels, int taps, const void *w_bf16, const void *bias_bf16, const void *seqs_dev, const int *row_seq_dev,
-                                size_t rows, void *const *slot_base_dev, size_t state_off, void *y_f32, size_t ldy, ifa_stream stream)
-{
-    return shortconv_silu(x_f32, ldx, channels, taps, w_bf16, bias_bf16, seqs_dev, row_seq_dev, rows, slot_base_dev, state_off, 0, 0, 0.0f, 0, 1.0f, y_f32, ldy, stream);
 }
 
 int ifa_shortconv_residual_f32(const void *x_f32, size_t ldx, int channels, int taps, const void *w_bf16, const void *seqs_dev, const int *row_seq_dev,
@@ -764,17 +707,6 @@ int ifa_delta_gates_f32(const void *b_f32, size_t ldb, const void *a_f32, size_t
     IFA_REQUIRE(heads > 0 && rows > 0 && ldb >= (size_t)heads && lda >= (size_t)heads, "ifa_delta_gates_f32: bad shape");
     hipLaunchKernelGGL(k_delta_gates, dim3(ifa_cdiv(rows * heads, 256)), dim3(256), 0, ifa_s(stream), (const float *)b_f32, ldb, (const float *)a_f32, lda,
                        heads, (int)rows, (const bf16_t *)a_log_bf16, (const bf16_t *)dt_bias_bf16, (float *)beta_f32, (float *)decay_f32);
-    IFA_LAUNCH_CHECK();
-    return IFA_OK;
-}
-
-int ifa_ssm_gates_f32(const void *a_f32, size_t lda, int heads, size_t rows, const void *a_log_bf16, const void *dt_bias_bf16, void *dt_f32, void *decay_f32,
-                      ifa_stream stream)
-{
-    IFA_REQUIRE(a_f32 && a_log_bf16 && dt_bias_bf16 && dt_f32 && decay_f32, "ifa_ssm_gates_f32: null pointer");
-    IFA_REQUIRE(heads > 0 && rows > 0 && lda >= (size_t)heads && rows * (size_t)heads < (1u << 31), "ifa_ssm_gates_f32: bad shape");
-    hipLaunchKernelGGL(k_ssm_gates, dim3(ifa_cdiv(rows * heads, 256)), dim3(256), 0, ifa_s(stream), (const float *)a_f32, lda, heads, (int)rows, (const bf16_t *)a_log_bf16,
-                       (const bf16_t *)dt_bias_bf16, (float *)dt_f32, (float *)decay_f32);
     IFA_LAUNCH_CHECK();
     return IFA_OK;
 }
@@ -845,18 +777,6 @@ int ifa_state_scan_ssm_f32(const void *x_f32, size_t ldx, const void *b_f32, siz
 {
     return state_scan(2, 0, c_f32, ldc, b_f32, ldb, x_f32, ldx, heads, groups, state, vdim, nullptr, decay_f32, dt_f32, skip_bf16, seqs_dev, n_seqs, slot_base_dev, state_off,
                       out_f32, ldo, stream);
-}
-
-int ifa_gate_groupnorm_f32(const void *o_f32, size_t ldo, size_t rows, int channels, int groups, const void *w_bf16, const void *gate_f32, size_t ldg, float eps,
-                           void *y_f32, size_t ldy, ifa_stream stream)
-{
-    IFA_REQUIRE(o_f32 && w_bf16 && gate_f32 && y_f32, "ifa_gate_groupnorm_f32: null pointer");
-    IFA_REQUIRE(rows > 0 && channels > 0 && groups > 0 && channels % groups == 0 && ldo >= (size_t)channels && ldg >= (size_t)channels && ldy >= (size_t)channels
-                && (size_t)channels * 4 <= 64 * 1024 - 256, "ifa_gate_groupnorm_f32: bad arguments (%d channels in %d groups)", channels, groups);
-    hipLaunchKernelGGL(k_gate_groupnorm, dim3((unsigned)rows), dim3(channels >= 2048 ? 512 : 256), (size_t)channels * 4, ifa_s(stream), (const float *)o_f32, ldo, channels,
-                       channels / groups, (const bf16_t *)w_bf16, (const float *)gate_f32, ldg, eps, (float *)y_f32, ldy);
-    IFA_LAUNCH_CHECK();
-    return IFA_OK;
 }
 
 int ifa_chan_delta_gates_f32(const void *lr_f32, size_t ldl, int rank, const void *w2_bf16, const void *w0_bf16, float decay_mult, const void *a_f32, size_t lda,
