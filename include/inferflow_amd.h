@@ -771,12 +771,12 @@ int ifa_moe_route_renorm_f32(int score_kind, int renorm, float renorm_eps, float
                              const void *correction_bf16, int *idx_dev, void *wgt_f32, ifa_stream stream);
 int ifa_moe_route_rows_renorm_f32(int score_kind, int renorm, float renorm_eps, float wgt_scale, const void *h_f32, size_t ldh, size_t rows, int width,
                                   const void *router_bf16, int n_all, int top, const void *correction_bf16, int *idx_dev, void *wgt_f32, ifa_stream stream);
-/* steps of at most 64 rows: ifa_streams_step_f32 (with y and the norm) and the routing of its h (ifa_moe_route_rows_renorm_f32) in one launch.  Needs
- * ifa_moe_streams_route_rows_fits(...) and 16-byte aligned rows. */
-int ifa_moe_streams_route_rows_fits(int streams, int width, int n_all, int top);
-int ifa_moe_streams_route_rows_f32(int score_kind, int renorm, float renorm_eps, float wgt_scale, void *x_f32, size_t rows, int streams, int width, const void *y_f32, size_t ldy,
-                                   const void *mix_bf16, const void *out_bf16, float mult, const void *in_bf16, const void *norm_w_bf16, float eps, void *h_f32, size_t ldh,
-                                   const void *router_bf16, int n_all, int top, const void *correction_bf16, int *idx_dev, void *wgt_f32, ifa_stream stream);
+/* steps of at most 8 rows, at most 256 experts: ifa_moe_experts_glu_f32 with the choice (as ifa_moe_route_renorm_f32, from the router's logits fp32 [rows][experts])
+ * made inside the experts' first launch, which leaves it in idx_dev / wgt_f32 */
+int ifa_moe_experts_routed_rows_f32(int score_kind, int renorm, float renorm_eps, float wgt_scale, const void *logits_f32, size_t ldl, const void *correction_bf16,
+                                    int glu_kind, float limit, const void *h_f32, size_t ldh, size_t rows, int width, int ff, int experts, int top,
+                                    const void *gate_up_bf16, const void *down_bf16, int *idx_dev, void *wgt_f32, void *ws, size_t ws_bytes, void *y_f32, size_t ldy,
+                                    int accumulate, ifa_stream stream);
 
 /* ======================================================================== */
 /* Layer-list worker: a decoder whose layers are given one by one, each with its own sequence mixer, a 32-bit residual       */

@@ -208,8 +208,7 @@ SIGNATURES = {
     "ifa_ssm_step_f32": (_i, [_vp, _sz, _vp, _sz, _i, _i, _i, _i, _i, _vp, _vp, _vp, _vp, _vp, _vp, _vp, _sz, _vp, _sz, _sz, _vp, _sz, _vp]),
     "ifa_ssm_chunked_workspace_bytes": (_sz, [_sz, _i, _i, _i, _i]),
     "ifa_ssm_chunked_f32": (_i, [_vp, _sz, _vp, _sz, _vp, _sz, _i, _i, _i, _i, _vp, _vp, _vp, _vp, _vp, _i, _vp, _sz, _vp, _sz, _vp, _sz, _vp]),
-    "ifa_moe_streams_route_rows_fits": (_i, [_i, _i, _i, _i]),
-    "ifa_moe_streams_route_rows_f32": (_i, [_i, _i, _f, _f, _vp, _sz, _i, _i, _vp, _sz, _vp, _vp, _f, _vp, _vp, _f, _vp, _sz, _vp, _i, _i, _vp, _vp, _vp, _vp]),
+    "ifa_moe_experts_routed_rows_f32": (_i, [_i, _i, _f, _f, _vp, _sz, _vp, _i, _f, _vp, _sz, _sz, _i, _i, _i, _i, _vp, _vp, _vp, _vp, _vp, _sz, _vp, _sz, _i, _vp]),
     "ifa_state_scan_ssm_f32": (_i, [_vp, _sz, _vp, _sz, _vp, _sz, _i, _i, _i, _i, _vp, _vp, _vp, _vp, _i, _vp, _sz, _vp, _sz, _vp]),
     "ifa_gate_groupnorm_f32": (_i, [_vp, _sz, _sz, _i, _i, _vp, _vp, _sz, _f, _vp, _sz, _vp]),
     "ifa_latent_prepare_pairs_f32": (_i, [_i, _vp, _sz, _i, _i, _i, _vp, _f, _vp, _sz, _i, _i, _vp, _f, _vp, _vp, _sz, _vp, _sz, _vp]),

@@ -126,7 +126,7 @@ struct LatRowArgs {
 template <int HB, int CPL>
 __global__ void __launch_bounds__(256) k_attn_latent_rows(LatRowArgs P)
 {
-    extern __shared__ float sm[];
+    extern __shared__ __attribute__((aligned(16))) float sm[];
     const int D = P.R + P.dr, dv = P.R;
     float *qs = sm;                              // [HB][D]
     float *wm = qs + HB * D, *wl = wm + 4 * HB;  // [4][HB] each
@@ -157,12 +157,21 @@ __global__ void __launch_bounds__(256) k_attn_latent_rows(LatRowArgs P)
 #pragma unroll
         for (int hh = 0; hh < HB; hh++) s[hh] = 0.0f;
         if (P.vec) {
-            for (int c = 4 * sub; c < D; c += 16) {
-                const float4 kv = *reinterpret_cast<const float4 *>(kr + c);
+            constexpr int KB = 12;          // pieces of the key row requested side by side (a chunk is bound by the latency of its requests)
+            for (int c0 = 4 * sub; c0 < D; c0 += 16 * KB) {
+                float4 kv[KB];
 #pragma unroll
-                for (int hh = 0; hh < HB; hh++) {
-                    const float *qq = qs + hh * D + c;
-                    s[hh] = fmaf(qq[0], kv.x, s[hh]); s[hh] = fmaf(qq[1], kv.y, s[hh]); s[hh] = fmaf(qq[2], kv.z, s[hh]); s[hh] = fmaf(qq[3], kv.w, s[hh]);
+                for (int u = 0; u < KB; u++) kv[u] = *reinterpret_cast<const float4 *>(kr + min(c0 + 16 * u, D - 4));
+#pragma unroll
+                for (int u = 0; u < KB; u++) {
+                    const int c = c0 + 16 * u;
+                    if (c < D) {
+#pragma unroll
+                        for (int hh = 0; hh < HB; hh++) {
+                            const float4 qq = *reinterpret_cast<const float4 *>(qs + hh * D + c);
+                            s[hh] = fmaf(qq.x, kv[u].x, s[hh]); s[hh] = fmaf(qq.y, kv[u].y, s[hh]); s[hh] = fmaf(qq.z, kv[u].z, s[hh]); s[hh] = fmaf(qq.w, kv[u].w, s[hh]);
+                        }
+                    }
                 }
             }
         } else {
@@ -185,17 +194,23 @@ __global__ void __launch_bounds__(256) k_attn_latent_rows(LatRowArgs P)
             m[hh] = m_new;
         }
         const int cnt = min(16, nk - ch * 16);
-        for (int jj = 0; jj < cnt; jj++) {
-            const float *vr = kc + (size_t)(ch * 16 + jj) * D;
-            float v[CPL];
+        constexpr int JB = CPL <= 8 ? 4 : 2;          // value rows requested side by side (beyond cnt: the last one again, with weight zero)
+        for (int j0 = 0; j0 < cnt; j0 += JB) {
+            float v[JB][CPL];
 #pragma unroll
-            for (int e = 0; e < CPL; e++) { const int d = lane + 64 * e; v[e] = d < dv ? vr[d] : 0.0f; }
+            for (int u = 0; u < JB; u++) {
+                const float *vr = kc + (size_t)min(ch * 16 + j0 + u, nk - 1) * D;
 #pragma unroll
-            for (int hh = 0; hh < HB; hh++) {
-                const float pj = __shfl(p[hh], 4 * jj, 64);
-#pragma unroll
-                for (int e = 0; e < CPL; e++) acc[hh][e] = fmaf(pj, v[e], acc[hh][e]);
+                for (int e = 0; e < CPL; e++) v[u][e] = vr[min(lane + 64 * e, dv - 1)];
             }
+#pragma unroll
+            for (int u = 0; u < JB; u++)
+#pragma unroll
+                for (int hh = 0; hh < HB; hh++) {
+                    const float pj = __shfl(p[hh], 4 * (j0 + u), 64);
+#pragma unroll
+                    for (int e = 0; e < CPL; e++) acc[hh][e] = fmaf(pj, v[u][e], acc[hh][e]);
+                }
         }
     }
 #pragma unroll
@@ -278,9 +293,11 @@ void launch_latent_rows(const LatRowArgs &P, unsigned rows, hipStream_t s)
 }
 
 // ---- prompts: 128 queries of one sequence per workgroup, the keys 0 .. last query walked in blocks of 32 staged once per workgroup in
-// LDS; each wave owns 32 queries: S = Q K^T and O += P V on the fp32 matrix cores (v_mfma_f32_32x32x2_f32: scores and weights stay
-// 32-bit), online softmax per query row, P turned from the accumulator layout into an A operand through LDS.  Key columns beyond
-// dim + rot_dim and value columns beyond vdim are zero padding up to 32 NTK / 32 NTV.
+// LDS; each wave owns 32 queries, one per lane of each half, held in registers as the B operand of S^T = K Q^T; O^T += V^T P^T; both on the fp32
+// matrix cores (v_mfma_f32_32x32x2_f32: scores and weights stay 32-bit).  In the transposed products a lane's accumulators hold 16 keys of ITS
+// query, so the online softmax is lane-local but for one exchange between the halves of the wave and the weights are the second product's B
+// operand as they lie in the accumulators.  The next block's keys and values are requested before the current one is worked on.  Key columns
+// beyond dim + rot_dim and value columns beyond vdim are zero padding up to 32 NTK / 32 NTV.
 typedef float f32x16l __attribute__((ext_vector_type(16)));
 constexpr int LT_Q = 128, LT_K = 32;
 
@@ -298,25 +315,17 @@ struct LatTileArgs {
     int vec;
 };
 
-__device__ __forceinline__ float lt_half_wave_max(float v)      // over the 32 lanes that share lane >> 5
-{
-#pragma unroll
-    for (int o = 16; o > 0; o >>= 1) v = fmaxf(v, __shfl_xor(v, o, 64));
-    return v;
-}
-
 template <int NTK, int NTV>
 __global__ void __launch_bounds__(256) k_attn_latent_tile(LatTileArgs P)
 {
     constexpr int DK = 32 * NTK, DKP = DK + 1, DV = 32 * NTV, DVP = DV + 1;
     extern __shared__ float sm[];
-    float *Qs = sm;                          // [128][DKP]
-    float *Ks = Qs + LT_Q * DKP;             // [32][DKP]
+    float *Ks = sm;                          // [32][DKP]
     float *Vs = Ks + LT_K * DKP;             // [32][DVP]
-    float *Ps = Vs + LT_K * DVP;             // [4][32][33]
     const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, i = lane & 31, g = lane >> 5;
-    const int h = blockIdx.y, dim = P.dim, dk = P.dim + P.dr, dv = P.vdim;
-    int tile = blockIdx.x, sq = 0;
+    const int h = blockIdx.x, dim = P.dim, dk = P.dim + P.dr, dv = P.vdim;
+    // the head is the grid's fast index, the tiles run from the last one down: the tiles with the most key blocks start first
+    int tile = (int)(gridDim.y - 1 - blockIdx.y), sq = 0;
     for (; sq < P.n_seqs; sq++) {
         const int nt = (P.seqs[sq].n + LT_Q - 1) / LT_Q;
         if (tile < nt) break;
@@ -328,122 +337,136 @@ __global__ void __launch_bounds__(256) k_attn_latent_tile(LatTileArgs P)
     const float *cache = P.slot_base[sd.slot] + P.cache_off + P.R;              // rotated key part of position j: cache + j (R + dr)
     const size_t crow = (size_t)(P.R + P.dr);
     const float *kx = P.kx + (size_t)P.ctx0[sq] * P.ldkx + (size_t)h * dim, *vx = P.vx + (size_t)P.ctx0[sq] * P.ldvx + (size_t)h * dv;
-    for (int e = tid; e < LT_Q * (DK / 4); e += 256) {
-        const int row = e / (DK / 4), c4 = (e % (DK / 4)) * 4;
-        float v4[4] = {0.f, 0.f, 0.f, 0.f};
-        if (row < nq) {
-            const float *src = P.q + (size_t)(r0 + row) * P.ldq + (size_t)h * dk + c4;
-            if (P.vec && c4 + 4 <= dk) { const float4 t4 = *reinterpret_cast<const float4 *>(src); v4[0] = t4.x; v4[1] = t4.y; v4[2] = t4.z; v4[3] = t4.w; }
-            else for (int u = 0; u < 4; u++) if (c4 + u < dk) v4[u] = src[u];
-        }
-        float *d = Qs + row * DKP + c4;
-        d[0] = v4[0]; d[1] = v4[1]; d[2] = v4[2]; d[3] = v4[3];
-    }
     const int nq_w = min(32, max(0, nq - 32 * wave));             // queries of this wave
     const int qlo = p0 + 32 * wave, qhi = qlo + nq_w - 1;          // their positions
     const int p_last = p0 + nq - 1, nb = p_last / LT_K + 1;
+    // the waves' queries in turn through the key buffer into registers: lane (i, g) takes the elements 2 s + g of query i
+    float qr[16 * NTK];
+#pragma unroll
+    for (int w = 0; w < 4; w++) {
+        for (int e = tid; e < 32 * DK; e += 256) {
+            const int row = e / DK, c = e % DK;
+            Ks[row * DKP + c] = 32 * w + row < nq && c < dk ? P.q[(size_t)(r0 + 32 * w + row) * P.ldq + (size_t)h * dk + c] : 0.0f;
+        }
+        __syncthreads();
+        if (wave == w) {
+#pragma unroll
+            for (int s = 0; s < 16 * NTK; s++) qr[s] = Ks[i * DKP + 2 * s + g];
+        }
+        __syncthreads();
+    }
     f32x16l o[NTV];
-    float m[16], l[16];
+    float m = -INFINITY, l = 0.0f;          // of the lane's query (lane & 31)
 #pragma unroll
     for (int nt = 0; nt < NTV; nt++)
 #pragma unroll
         for (int r = 0; r < 16; r++) o[nt][r] = 0.0f;
+    float4 kreg[NTK], vreg[NTV];
+    auto fetch = [&](int b) {
+        const int kb0 = b * LT_K, kc_n = min(LT_K, p_last - kb0 + 1);
 #pragma unroll
-    for (int r = 0; r < 16; r++) { m[r] = -INFINITY; l[r] = 0.0f; }
-    float *Pw = Ps + wave * 32 * 33;
+        for (int u = 0; u < NTK; u++) {
+            const int e = tid + 256 * u, row = e / (DK / 4), c4 = (e % (DK / 4)) * 4;
+            kreg[u] = make_float4(0.f, 0.f, 0.f, 0.f);
+            if (row < kc_n && c4 < dk)
+                kreg[u] = *reinterpret_cast<const float4 *>(c4 < dim ? kx + (size_t)(kb0 + row) * P.ldkx + c4 : cache + (size_t)(kb0 + row) * crow + (c4 - dim));
+        }
+#pragma unroll
+        for (int u = 0; u < NTV; u++) {
+            const int e = tid + 256 * u, row = e / (DV / 4), c4 = (e % (DV / 4)) * 4;
+            vreg[u] = make_float4(0.f, 0.f, 0.f, 0.f);
+            if (row < kc_n && c4 < dv) vreg[u] = *reinterpret_cast<const float4 *>(vx + (size_t)(kb0 + row) * P.ldvx + c4);
+        }
+    };
+    if (P.vec) fetch(0);
     for (int b = 0; b < nb; b++) {
         const int kb0 = b * LT_K, kc_n = min(LT_K, p_last - kb0 + 1);
-        __syncthreads();                 // the previous block's K / V reads are done (and Q is staged)
-        for (int e = tid; e < LT_K * (DK / 4); e += 256) {
-            const int row = e / (DK / 4), c4 = (e % (DK / 4)) * 4;
-            float v4[4] = {0.f, 0.f, 0.f, 0.f};
-            if (row < kc_n) {
-                const float *su = kx + (size_t)(kb0 + row) * P.ldkx, *sr = cache + (size_t)(kb0 + row) * crow;
-                if (P.vec && c4 + 4 <= dk) {
-                    const float4 t4 = *reinterpret_cast<const float4 *>(c4 < dim ? su + c4 : sr + (c4 - dim));
-                    v4[0] = t4.x; v4[1] = t4.y; v4[2] = t4.z; v4[3] = t4.w;
-                } else {
-                    for (int u = 0; u < 4; u++) { const int c = c4 + u; if (c < dk) v4[u] = c < dim ? su[c] : sr[c - dim]; }
-                }
+        __syncthreads();                 // the previous block's K / V reads are done
+        if (P.vec) {
+#pragma unroll
+            for (int u = 0; u < NTK; u++) {
+                const int e = tid + 256 * u, row = e / (DK / 4), c4 = (e % (DK / 4)) * 4;
+                float *d = Ks + row * DKP + c4;
+                d[0] = kreg[u].x; d[1] = kreg[u].y; d[2] = kreg[u].z; d[3] = kreg[u].w;
             }
-            float *d = Ks + row * DKP + c4;
-            d[0] = v4[0]; d[1] = v4[1]; d[2] = v4[2]; d[3] = v4[3];
-        }
-        for (int e = tid; e < LT_K * (DV / 4); e += 256) {
-            const int row = e / (DV / 4), c4 = (e % (DV / 4)) * 4;
-            float v4[4] = {0.f, 0.f, 0.f, 0.f};
-            if (row < kc_n) {
-                const float *sv = vx + (size_t)(kb0 + row) * P.ldvx + c4;
-                if (P.vec && c4 + 4 <= dv) { const float4 t4 = *reinterpret_cast<const float4 *>(sv); v4[0] = t4.x; v4[1] = t4.y; v4[2] = t4.z; v4[3] = t4.w; }
-                else for (int u = 0; u < 4; u++) if (c4 + u < dv) v4[u] = sv[u];
+#pragma unroll
+            for (int u = 0; u < NTV; u++) {
+                const int e = tid + 256 * u, row = e / (DV / 4), c4 = (e % (DV / 4)) * 4;
+                float *d = Vs + row * DVP + c4;
+                d[0] = vreg[u].x; d[1] = vreg[u].y; d[2] = vreg[u].z; d[3] = vreg[u].w;
             }
-            float *d = Vs + row * DVP + c4;
-            d[0] = v4[0]; d[1] = v4[1]; d[2] = v4[2]; d[3] = v4[3];
+            if (b + 1 < nb) fetch(b + 1);
+        } else {
+            for (int e = tid; e < LT_K * DK; e += 256) {
+                const int row = e / DK, c = e % DK;
+                Ks[row * DKP + c] = row < kc_n && c < dk ? (c < dim ? kx[(size_t)(kb0 + row) * P.ldkx + c] : cache[(size_t)(kb0 + row) * crow + (c - dim)]) : 0.0f;
+            }
+            for (int e = tid; e < LT_K * DV; e += 256) {
+                const int row = e / DV, c = e % DV;
+                Vs[row * DVP + c] = row < kc_n && c < dv ? vx[(size_t)(kb0 + row) * P.ldvx + c] : 0.0f;
+            }
         }
         __syncthreads();
-        const bool active = nq_w > 0 && kb0 <= qhi;
-        if (active) {
+        if (nq_w > 0 && kb0 <= qhi) {
             f32x16l acc;
 #pragma unroll
             for (int r = 0; r < 16; r++) acc[r] = 0.0f;
-            const float *qa = Qs + (32 * wave + i) * DKP + g, *ka = Ks + i * DKP + g;
-#pragma unroll 8
-            for (int s2 = 0; s2 < DK / 2; s2++) acc = __builtin_amdgcn_mfma_f32_32x32x2f32(qa[2 * s2], ka[2 * s2], acc, 0, 0, 0);
-            const int j = kb0 + i;
-            const bool jin = i < kc_n;
+            const float *ka = Ks + i * DKP + g;
+#pragma unroll
+            for (int s = 0; s < 16 * NTK; s++) acc = __builtin_amdgcn_mfma_f32_32x32x2f32(ka[2 * s], qr[s], acc, 0, 0, 0);
+            const int iq = qlo + i;
+            const bool qin = i < nq_w;
+            float mloc = -INFINITY;
 #pragma unroll
             for (int r = 0; r < 16; r++) {
-                const int qq = (r & 3) + 8 * (r >> 2) + 4 * g, iq = qlo + qq;
-                const bool vis = jin && qq < nq_w && j <= iq;
-                const float sc = vis ? acc[r] * P.scale : -INFINITY;
-                const float m_new = fmaxf(m[r], lt_half_wave_max(sc));
-                const float pr = vis ? expf(sc - m_new) : 0.0f;
-                const float corr = m[r] == -INFINITY ? 1.0f : expf(m[r] - m_new);      // (m_new == -inf only while nothing was visible: sums are 0)
-                l[r] = l[r] * corr + pr;
-                m[r] = m_new;
-#pragma unroll
-                for (int nt = 0; nt < NTV; nt++) o[nt][r] *= corr;
-                Pw[qq * 33 + i] = pr;
+                const int kk = (r & 3) + 8 * (r >> 2) + 4 * g;
+                acc[r] = qin && kk < kc_n && kb0 + kk <= iq ? acc[r] * P.scale : -INFINITY;
+                mloc = fmaxf(mloc, acc[r]);
             }
-        }
-        __syncthreads();                 // P of every wave is in LDS
-        if (active) {
-            const float *pa = Pw + i * 33 + g;
+            mloc = fmaxf(mloc, __shfl_xor(mloc, 32, 64));
+            const float m_new = fmaxf(m, mloc);
+            const float corr = m == -INFINITY ? 1.0f : expf(m - m_new);      // (m_new == -inf only while nothing was visible: sums are 0)
+            float psum = 0.0f;
+#pragma unroll
+            for (int r = 0; r < 16; r++) { acc[r] = acc[r] == -INFINITY ? 0.0f : expf(acc[r] - m_new); psum += acc[r]; }
+            l = l * corr + psum;             // (the keys of this half of the wave; the halves are added at the end)
+            m = m_new;
+            // step s takes keys (s & 3) + 8 (s >> 2) + 4 g
 #pragma unroll
             for (int nt = 0; nt < NTV; nt++) {
-                const float *va = Vs + g * DVP + 32 * nt + i;
-#pragma unroll 8
-                for (int s2 = 0; s2 < LT_K / 2; s2++) o[nt] = __builtin_amdgcn_mfma_f32_32x32x2f32(pa[2 * s2], va[2 * s2 * DVP], o[nt], 0, 0, 0);
+#pragma unroll
+                for (int r = 0; r < 16; r++) o[nt][r] *= corr;
+                const float *va = Vs + 4 * g * DVP + 32 * nt + i;
+#pragma unroll
+                for (int s = 0; s < 16; s++)
+                    o[nt] = __builtin_amdgcn_mfma_f32_32x32x2f32(va[((s & 3) + 8 * (s >> 2)) * DVP], acc[s], o[nt], 0, 0, 0);
             }
         }
     }
+    // the lane holds value columns 32 nt + (r & 3) + 8 (r >> 2) + 4 g of its query
+    const float ls = l + __shfl_xor(l, 32, 64);
+    if (i >= nq_w) return;
+    const size_t row = (size_t)(r0 + 32 * wave + i);
+    const float gate = P.g && !P.gate_cols ? sigmoid_f(P.g[row * P.ldg + h]) : 1.0f;
+    const float sc = gate / ls;
 #pragma unroll
-    for (int r = 0; r < 16; r++) {
-        const int qq = (r & 3) + 8 * (r >> 2) + 4 * g;
-        float ls = l[r];
+    for (int nt = 0; nt < NTV; nt++)
 #pragma unroll
-        for (int of = 16; of > 0; of >>= 1) ls += __shfl_xor(ls, of, 64);
-        if (qq >= nq_w) continue;
-        const size_t row = (size_t)(r0 + 32 * wave + qq);
-        const float gate = P.g && !P.gate_cols ? sigmoid_f(P.g[row * P.ldg + h]) : 1.0f;
-        const float sc = gate / ls;
-#pragma unroll
-        for (int nt = 0; nt < NTV; nt++)
-            if (32 * nt + i < dv) {
-                const size_t c = (size_t)h * dv + 32 * nt + i;
+        for (int r = 0; r < 16; r++) {
+            const int e = 32 * nt + (r & 3) + 8 * (r >> 2) + 4 * g;
+            if (e < dv) {
+                const size_t c = (size_t)h * dv + e;
                 const float v = o[nt][r] * sc;
                 P.out[row * P.ldo + c] = P.gate_cols ? v * sigmoid_f(P.g[row * P.ldg + c]) : v;
             }
-    }
+        }
 }
 
 template <int NTK, int NTV>
 int launch_latent_tile(const LatTileArgs &P, unsigned tiles, hipStream_t s)
 {
-    const size_t smem = ((size_t)(LT_Q + LT_K) * (32 * NTK + 1) + (size_t)LT_K * (32 * NTV + 1) + 4 * 32 * 33) * 4;
-    IFA_REQUIRE(smem <= 160 * 1024, "ifa_attention_latent_tile_f32: head sizes need %zu bytes of LDS", smem);
-    IFA_HIP_CHECK(hipFuncSetAttribute((const void *)k_attn_latent_tile<NTK, NTV>, hipFuncAttributeMaxDynamicSharedMemorySize, (int)smem));
-    hipLaunchKernelGGL((k_attn_latent_tile<NTK, NTV>), dim3(tiles, (unsigned)P.heads), dim3(256), smem, s, P);
+    const size_t smem = (size_t)LT_K * (32 * NTK + 1 + 32 * NTV + 1) * 4;          // (at most 41 KB)
+    hipLaunchKernelGGL((k_attn_latent_tile<NTK, NTV>), dim3((unsigned)P.heads, tiles), dim3(256), smem, s, P);
     IFA_LAUNCH_CHECK();
     return IFA_OK;
 }
@@ -590,6 +613,7 @@ int ifa_attention_latent_tile_gated_f32(int gate_cols, const void *q_f32, size_t
     const ifa_seq_desc *sh = (const ifa_seq_desc *)seqs_host;
     size_t tiles = 0;
     for (int q = 0; q < n_seqs; q++) tiles += ((size_t)sh[q].n + LT_Q - 1) / LT_Q;
+    IFA_REQUIRE(tiles > 0 && tiles < 65536, "ifa_attention_latent_tile_f32: %zu query tiles", tiles);
     hipStream_t s = ifa_s(stream);
     switch (ntk) {
     case 1: return dispatch_latent_tile_v<1>(P, (unsigned)tiles, ntv, s);
@@ -605,9 +629,7 @@ int ifa_attention_latent_tile_gated_f32(int gate_cols, const void *q_f32, size_t
 int ifa_attention_latent_tile_fits(int dim, int rot_dim, int vdim)
 {
     const int ntk = (dim + rot_dim + 31) / 32, ntv = (vdim + 31) / 32;
-    if (ntk < 1 || ntk > 6 || ntv < 1 || ntv > 4) return 0;
-    const size_t smem = ((size_t)(LT_Q + LT_K) * (32 * ntk + 1) + (size_t)LT_K * (32 * ntv + 1) + 4 * 32 * 33) * 4;
-    return smem <= 160 * 1024 ? 1 : 0;
+    return ntk >= 1 && ntk <= 6 && ntv >= 1 && ntv <= 4 ? 1 : 0;
 }
 
 } // extern "C"

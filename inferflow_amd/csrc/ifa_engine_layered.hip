@@ -652,15 +652,6 @@ int run_streams_layer(ifa_model *m, LLayer &L, size_t T, int nseq, int pass, LLa
     const void *next_in = next ? next->T(IFA_LT_HC1_IN).data : nullptr, *next_norm = next ? next->T(IFA_LT_NORM1).data : n->out_norm.data;
     int rc;
     if ((rc = sp.mixer == IFA_MIX_LATENT ? run_latent_mixer(m, L, T, n->h, po, n->m3) : run_ssm_mixer(m, L, T, nseq, n->h, po, n->m3))) return rc;
-    if (moe && n->opt_fuse_post && T <= 8 && ifa_moe_streams_route_rows_fits((int)streams_of(n), c.width, sp.x_experts, sp.x_top)) {
-        // a few rows: the streams' update, the norm, the router's product and its choice in one launch
-        if ((rc = ifa_moe_streams_route_rows_f32(sp.x_score, sp.x_renorm, sp.x_renorm_eps, sp.x_wgt_scale, n->x, T, (int)streams_of(n), c.width, n->m3, W, L.T(IFA_LT_HC1_MIX).data,
-                                                 L.T(IFA_LT_HC1_OUT).data, c.residual_mult, L.T(IFA_LT_HC2_IN).data, L.T(IFA_LT_NORM2).data, c.eps, n->h, W,
-                                                 L.T(IFA_LT_X_ROUTER).data, sp.x_experts, sp.x_top, nullptr, n->moe_idx, n->moe_wgt, s))) return rc;
-        if ((rc = ifa_moe_experts_glu_f32(sp.x_glu, sp.x_limit, n->h, W, T, (int)W, sp.x_ff, sp.x_experts, sp.x_top, L.T(IFA_LT_X_UP).data, L.T(IFA_LT_X_DOWN).data, n->moe_idx,
-                                          n->moe_wgt, c.ops32, n->moe_ws, n->moe_ws_bytes, n->m1, W, 0, s))) return rc;
-        return streams_step(m, T, false, n->m1, &L, 2, next_in, next_norm);
-    }
     if ((rc = streams_step(m, T, false, n->m3, &L, 1, any_ffn ? L.T(IFA_LT_HC2_IN).data : next_in, any_ffn ? L.T(IFA_LT_NORM2).data : next_norm))) return rc;
     if (!any_ffn) return IFA_OK;
     if (!moe) {
@@ -670,6 +661,13 @@ int run_streams_layer(ifa_model *m, LLayer &L, size_t T, int nseq, int pass, LLa
         if ((rc = linear(m, (const bf16_t *)L.T(IFA_LT_FFN_DOWN).data, W, F, n->m3, F, T, nullptr, nullptr, 1.0f, 0, n->m1, W))) return rc;
     } else {
         const int XA = sp.x_experts;
+        if (T <= 8 && XA <= 256 && n->opt_fuse_post) {      // a few rows: the choice inside the experts' first launch
+            if ((rc = linear(m, (const bf16_t *)L.T(IFA_LT_X_ROUTER).data, (size_t)XA, W, n->h, W, T, nullptr, nullptr, 1.0f, 0, n->m2, (size_t)XA))) return rc;
+            if ((rc = ifa_moe_experts_routed_rows_f32(sp.x_score, sp.x_renorm, sp.x_renorm_eps, sp.x_wgt_scale, n->m2, (size_t)XA, nullptr, sp.x_glu, sp.x_limit, n->h, W, T, (int)W,
+                                                      sp.x_ff, XA, sp.x_top, L.T(IFA_LT_X_UP).data, L.T(IFA_LT_X_DOWN).data, n->moe_idx, n->moe_wgt, n->moe_ws, n->moe_ws_bytes,
+                                                      n->m1, W, 0, s))) return rc;
+            return streams_step(m, T, false, n->m1, &L, 2, next_in, next_norm);
+        }
         if (T <= 8 && XA <= 512) {      // a few rows: the router's product inside the choice's launch
             if ((rc = ifa_moe_route_rows_renorm_f32(sp.x_score, sp.x_renorm, sp.x_renorm_eps, sp.x_wgt_scale, n->h, W, T, (int)W, L.T(IFA_LT_X_ROUTER).data, XA, sp.x_top, nullptr,
                                                     n->moe_idx, n->moe_wgt, s))) return rc;

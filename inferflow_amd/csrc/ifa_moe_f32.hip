@@ -13,7 +13,6 @@
 #include <algorithm>
 #include "ifa_host.h"
 #include "ifa_f32_common.h"
-#include "ifa_streams.h"
 #include "inferflow_amd.h"
 
 using namespace ifa32;
@@ -151,100 +150,56 @@ __global__ void __launch_bounds__(1024) k_moe_route_rows(const float *h, size_t 
     if (renorm && threadIdx.x == 0) { const float den = chosen + renorm_eps; for (int k = 0; k < top; k++) wgt[(size_t)t * top + k] = wgt[(size_t)t * top + k] / den * wgt_scale; }
 }
 
-// Steps of a few rows of blocks with several residual streams, one launch: what lies between the mixer and the experts (streams_row), the
-// router's product and its choice.  One workgroup of sixteen waves per row; the router's rows are requested before anything else (they do
-// not depend on the row) as far as they fit RW_PRE pieces per thread; the choice runs in the first wave's registers (n_all <= 64 RW_E).
-constexpr int RW_PRE = 8, RW_E = 8;
-struct RouteArgs {
-    const bf16_t *router; int n_all, top, score_kind, renorm; float renorm_eps, wgt_scale;
-    const bf16_t *corr; int *idx; float *wgt; int pre;      // pre: every wave's share of the router in registers ahead
+// Steps of a few rows whose choice is made by the first experts' launch itself: every workgroup forms the scores of its row from the router's logits
+// and finds the expert of its pair as the one whose RANK (larger choice scores, lower index on ties) is the pair's place; the pair's first
+// workgroup leaves expert and weight for the launches behind.  At most 256 router outputs (one per thread).
+struct RouteSel {
+    const float *logits; size_t ld; int n_all, score_kind, renorm; float renorm_eps, wgt_scale;
+    const bf16_t *corr; int *idx; float *wgt;
 };
 
-template <int SMAX>
-__global__ void __launch_bounds__(1024) k_streams_route_rows(StreamArgs P, RouteArgs R)
+__device__ int route_pair(const RouteSel &R, int t, int k, int top, bool leave)
 {
-    __shared__ float lds[SMAX * SMAX + 2 * SMAX + 17];
-    extern __shared__ float hs[];          // [cols] the normed row, [n_all] logits
-    float *sc = hs + P.cols;
-    const int t = blockIdx.x, lane = threadIdx.x & 63, wave = threadIdx.x >> 6, W = P.cols, nk = (W + 511) / 512;
-    u32x4m pw[RW_PRE];
-    if (R.pre) {
-#pragma unroll
-        for (int a = 0; a < RW_PRE; a++) {
-            const int e = wave + 16 * (a / nk), k = lane * 8 + 512 * (a % nk);
-            if (e < R.n_all && k < W) pw[a] = *reinterpret_cast<const u32x4m *>(R.router + (size_t)e * W + k);
-        }
+    __shared__ float ch[256], red[17];
+    __shared__ int mine;
+    const int e = threadIdx.x;
+    const bool live = e < R.n_all;
+    float s = live ? R.logits[(size_t)t * R.ld + e] : -INFINITY;
+    if (R.score_kind == 1) s = live ? sigmoid_f(s) : 0.0f;
+    else {          // softmax: the maximum over the row, then the sum
+        const float wm = wave_max(s);
+        if ((e & 63) == 0) red[e >> 6] = wm;
+        __syncthreads();
+        float mx = -INFINITY;
+        for (int w = 0; w < (int)(blockDim.x >> 6); w++) mx = fmaxf(mx, red[w]);
+        s = live ? expf(s - mx) : 0.0f;
+        s /= block_sum(s, red);
     }
-    streams_row<SMAX, true>(P, t, lds, hs);
+    const float c = live ? s + (R.corr ? bf2f(R.corr[e]) : 0.0f) : -INFINITY;
+    ch[e] = c;
     __syncthreads();
-    auto dot8 = [&](const u32x4m &w, int k, float acc) {
-        const float4 a0 = *reinterpret_cast<const float4 *>(hs + k), a1 = *reinterpret_cast<const float4 *>(hs + k + 4);
-        acc = fmaf(a0.x, __uint_as_float(w[0] << 16), acc); acc = fmaf(a0.y, __uint_as_float(w[0] & 0xFFFF0000u), acc);
-        acc = fmaf(a0.z, __uint_as_float(w[1] << 16), acc); acc = fmaf(a0.w, __uint_as_float(w[1] & 0xFFFF0000u), acc);
-        acc = fmaf(a1.x, __uint_as_float(w[2] << 16), acc); acc = fmaf(a1.y, __uint_as_float(w[2] & 0xFFFF0000u), acc);
-        acc = fmaf(a1.z, __uint_as_float(w[3] << 16), acc); return fmaf(a1.w, __uint_as_float(w[3] & 0xFFFF0000u), acc);
-    };
-    if (R.pre) {
-        float acc = 0.0f;
-#pragma unroll
-        for (int a = 0; a < RW_PRE; a++) {
-            const int e = wave + 16 * (a / nk), k = lane * 8 + 512 * (a % nk);
-            if (e < R.n_all) {
-                if (k < W) acc = dot8(pw[a], k, acc);
-                if (a % nk == nk - 1) { acc = wave_sum(acc); if (lane == 0) sc[e] = acc; acc = 0.0f; }
-            }
-        }
-    } else {
-        for (int e = wave; e < R.n_all; e += 16) {
-            float acc = 0.0f;
-#pragma unroll 4
-            for (int k = lane * 8; k < W; k += 512) acc = dot8(*reinterpret_cast<const u32x4m *>(R.router + (size_t)e * W + k), k, acc);
-            acc = wave_sum(acc);
-            if (lane == 0) sc[e] = acc;
-        }
+    int rank = 0;
+    if (live) {
+#pragma unroll 8
+        for (int j = 0; j < R.n_all; j++) { const float v = ch[j]; rank += (v > c || (v == c && j < e)) ? 1 : 0; }
+    }
+    if (live && rank == k) mine = e;
+    float sum = 0.0f;
+    if (leave && R.renorm) sum = block_sum(live && rank < top ? s : 0.0f, red);
+    if (leave && live && rank == k) {
+        R.idx[(size_t)t * top + k] = e;
+        R.wgt[(size_t)t * top + k] = R.renorm ? s / (sum + R.renorm_eps) * R.wgt_scale : s;
     }
     __syncthreads();
-    if (wave) return;
-    float s[RW_E], ch[RW_E], mx = -INFINITY;
-#pragma unroll
-    for (int r = 0; r < RW_E; r++) { const int e = lane + 64 * r; s[r] = e < R.n_all ? sc[e] : -INFINITY; mx = fmaxf(mx, s[r]); }
-    if (R.score_kind == 1) {
-#pragma unroll
-        for (int r = 0; r < RW_E; r++) s[r] = sigmoid_f(s[r]);
-    } else {
-        mx = wave_max(mx);
-        float sum = 0.0f;
-#pragma unroll
-        for (int r = 0; r < RW_E; r++) { s[r] = expf(s[r] - mx); sum += s[r]; }
-        sum = wave_sum(sum);
-#pragma unroll
-        for (int r = 0; r < RW_E; r++) s[r] /= sum;
-    }
-#pragma unroll
-    for (int r = 0; r < RW_E; r++) { const int e = lane + 64 * r; ch[r] = e < R.n_all ? s[r] + (R.corr ? bf2f(R.corr[e]) : 0.0f) : -INFINITY; }
-    float chosen = 0.0f;
-    for (int k = 0; k < R.top; k++) {
-        float best = -INFINITY, bs = 0.0f; int bi = 0x7FFFFFFF;
-#pragma unroll
-        for (int r = 0; r < RW_E; r++) { const int e = lane + 64 * r; if (e < R.n_all && (ch[r] > best || (ch[r] == best && e < bi))) { best = ch[r]; bs = s[r]; bi = e; } }
-        for (int o = 32; o > 0; o >>= 1) {
-            const float ov = __shfl_xor(best, o, 64), os = __shfl_xor(bs, o, 64); const int oi = __shfl_xor(bi, o, 64);
-            if (ov > best || (ov == best && oi < bi)) { best = ov; bs = os; bi = oi; }
-        }
-        chosen += bs;
-#pragma unroll
-        for (int r = 0; r < RW_E; r++) if (lane + 64 * r == bi) ch[r] = -INFINITY;
-        if (lane == 0) { R.idx[(size_t)t * R.top + k] = bi; R.wgt[(size_t)t * R.top + k] = bs; }
-    }
-    if (R.renorm && lane == 0) { const float den = chosen + R.renorm_eps; for (int k = 0; k < R.top; k++) R.wgt[(size_t)t * R.top + k] = R.wgt[(size_t)t * R.top + k] / den * R.wgt_scale; }
+    return mine;
 }
 
 // grid (ff chunks, pairs): act[p][n] = gelu(W_up[e][n] . h[t]); a wave per n at a time.  Identity pairs do nothing.
-template <bool GATED>
+template <bool GATED, bool SEL>
 __global__ void __launch_bounds__(256) k_moe_up_rows(const float *__restrict__ h, size_t ldh, int W, int F, int experts, int top, const bf16_t *__restrict__ up,
-                                                     const int *__restrict__ idx, float *__restrict__ act, int vec, int glu_kind, float limit)
+                                                     const int *__restrict__ idx, float *__restrict__ act, int vec, int glu_kind, float limit, RouteSel R)
 {
-    const int p = blockIdx.y, e = idx[p];
+    const int p = blockIdx.y, e = SEL ? route_pair(R, p / top, p % top, top, blockIdx.x == 0) : idx[p];
     if (e >= experts) return;
     const int lane = threadIdx.x & 63, wave = blockIdx.x * (blockDim.x >> 6) + (threadIdx.x >> 6), nwaves = gridDim.x * (blockDim.x >> 6);
     const float *hr = h + (size_t)(p / top) * ldh;
@@ -456,34 +411,6 @@ int ifa_moe_route_rows_renorm_f32(int score_kind, int renorm, float renorm_eps, 
     return IFA_OK;
 }
 
-int ifa_moe_streams_route_rows_fits(int streams, int width, int n_all, int top)
-{
-    return streams >= 1 && streams <= 16 && width > 0 && width % 8 == 0 && n_all >= 1 && n_all <= 64 * RW_E && top >= 1 && top <= n_all && ((size_t)width + n_all) * 4 <= 60 * 1024;
-}
-
-int ifa_moe_streams_route_rows_f32(int score_kind, int renorm, float renorm_eps, float wgt_scale, void *x_f32, size_t rows, int streams, int width, const void *y_f32, size_t ldy,
-                                   const void *mix_bf16, const void *out_bf16, float mult, const void *in_bf16, const void *norm_w_bf16, float eps, void *h_f32, size_t ldh,
-                                   const void *router_bf16, int n_all, int top, const void *correction_bf16, int *idx_dev, void *wgt_f32, ifa_stream stream)
-{
-    IFA_REQUIRE(x_f32 && y_f32 && norm_w_bf16 && h_f32 && router_bf16 && idx_dev && wgt_f32, "ifa_moe_streams_route_rows_f32: null pointer");
-    IFA_REQUIRE(rows > 0 && rows <= 64 && ifa_moe_streams_route_rows_fits(streams, width, n_all, top) && ldy >= (size_t)width && ldh >= (size_t)width && ldy % 4 == 0 && ldh % 4 == 0
-                && (((uintptr_t)x_f32 | (uintptr_t)y_f32 | (uintptr_t)h_f32 | (uintptr_t)router_bf16) & 15) == 0 && (score_kind == 0 || score_kind == 1),
-                "ifa_moe_streams_route_rows_f32: bad shape or alignment");
-    StreamArgs P;
-    P.x = (float *)x_f32; P.S = streams; P.cols = width; P.embed = nullptr; P.tokens = nullptr; P.vocab = 0; P.scale = 1.0f; P.y = (const float *)y_f32; P.ldy = ldy;
-    P.mix = (const bf16_t *)mix_bf16; P.out = (const bf16_t *)out_bf16; P.mult = mult; P.in = (const bf16_t *)in_bf16; P.w = (const bf16_t *)norm_w_bf16; P.eps = eps;
-    P.h = (float *)h_f32; P.ldh = ldh; P.sum_out = nullptr; P.ldsum = 0;
-    RouteArgs R;
-    R.router = (const bf16_t *)router_bf16; R.n_all = n_all; R.top = top; R.score_kind = score_kind; R.renorm = renorm ? 1 : 0; R.renorm_eps = renorm_eps; R.wgt_scale = wgt_scale;
-    R.corr = (const bf16_t *)correction_bf16; R.idx = idx_dev; R.wgt = (float *)wgt_f32; R.pre = ((n_all + 15) / 16) * ((width + 511) / 512) <= RW_PRE ? 1 : 0;
-    const size_t smem = ((size_t)width + n_all) * 4;
-#define IFA_SR(SM) hipLaunchKernelGGL(k_streams_route_rows<SM>, dim3((unsigned)rows), dim3(1024), smem, ifa_s(stream), P, R)
-    if (streams == 1) IFA_SR(1); else if (streams == 2) IFA_SR(2); else if (streams <= 4) IFA_SR(4); else if (streams <= 8) IFA_SR(8); else IFA_SR(16);
-#undef IFA_SR
-    IFA_LAUNCH_CHECK();
-    return IFA_OK;
-}
-
 int ifa_moe_dyt_route_rows_f32(int score_kind, const void *x_f32, size_t ldx, const void *alpha_bf16, const void *norm_w_bf16, const void *norm_b_bf16, void *h_f32,
                                size_t ldh, size_t rows, int width, const void *router_bf16, int n_all, int top, const void *correction_bf16, int *idx_dev,
                                void *wgt_f32, ifa_stream stream)
@@ -518,7 +445,7 @@ size_t ifa_moe_workspace_bytes(size_t rows, int top, int width, int ff, int expe
 
 static int moe_experts(const char *who, int gated, int glu_kind, float limit, const void *h_f32, size_t ldh, size_t rows, int width, int ff, int experts, int identity, int top, int act,
                        const void *up_bf16, const void *down_bf16, const int *idx_dev, const void *wgt_f32, int ops32, void *ws, size_t ws_bytes,
-                       void *y_f32, size_t ldy, int accumulate, ifa_stream stream)
+                       void *y_f32, size_t ldy, int accumulate, ifa_stream stream, const RouteSel *sel = nullptr)
 {
     IFA_REQUIRE(h_f32 && idx_dev && wgt_f32 && ws && y_f32 && (experts == 0 || (up_bf16 && down_bf16)), "%s: null pointer", who);
     IFA_REQUIRE(rows > 0 && rows < 65536 && width > 0 && ff > 0 && experts >= 0 && experts <= 4096 && identity >= 0 && top >= 1 && top <= experts + identity && act == 0
@@ -542,12 +469,15 @@ static int moe_experts(const char *who, int gated, int glu_kind, float limit, co
     if (rows <= 8 || experts == 0) {
         const int vec_u = (width % 8 == 0 && ldh % 4 == 0 && ((uintptr_t)h_f32 & 15) == 0 && ((uintptr_t)up_bf16 & 15) == 0) ? 1 : 0;
         const int vec_d = (ff % 8 == 0 && ((uintptr_t)down_bf16 & 15) == 0) ? 1 : 0;
-        if (experts > 0 && gated)
-            hipLaunchKernelGGL(k_moe_up_rows<true>, dim3(std::min(512u, ifa_cdiv((size_t)ff, 4)), (unsigned)pairs), dim3(256), 0, s, h, ldh, width, ff, experts, top,
-                               (const bf16_t *)up_bf16, idx_dev, actb, vec_u, glu_kind, limit);
+        if (experts > 0 && gated && sel)
+            hipLaunchKernelGGL((k_moe_up_rows<true, true>), dim3(std::min(512u, ifa_cdiv((size_t)ff, 4)), (unsigned)pairs), dim3(256), 0, s, h, ldh, width, ff, experts, top,
+                               (const bf16_t *)up_bf16, idx_dev, actb, vec_u, glu_kind, limit, *sel);
+        else if (experts > 0 && gated)
+            hipLaunchKernelGGL((k_moe_up_rows<true, false>), dim3(std::min(512u, ifa_cdiv((size_t)ff, 4)), (unsigned)pairs), dim3(256), 0, s, h, ldh, width, ff, experts, top,
+                               (const bf16_t *)up_bf16, idx_dev, actb, vec_u, glu_kind, limit, RouteSel());
         else if (experts > 0)
-            hipLaunchKernelGGL(k_moe_up_rows<false>, dim3(std::min(512u, ifa_cdiv((size_t)ff, 4)), (unsigned)pairs), dim3(256), 0, s, h, ldh, width, ff, experts, top,
-                               (const bf16_t *)up_bf16, idx_dev, actb, vec_u, 0, 0.0f);
+            hipLaunchKernelGGL((k_moe_up_rows<false, false>), dim3(std::min(512u, ifa_cdiv((size_t)ff, 4)), (unsigned)pairs), dim3(256), 0, s, h, ldh, width, ff, experts, top,
+                               (const bf16_t *)up_bf16, idx_dev, actb, vec_u, 0, 0.0f, RouteSel());
         hipLaunchKernelGGL(k_moe_down_rows, dim3(std::min(1024u, ifa_cdiv((size_t)width, 4)), (unsigned)rows), dim3(256), 0, s, h, ldh, width, ff, experts, top,
                            (const bf16_t *)down_bf16, idx_dev, (const float *)wgt_f32, actb, accumulate ? 1 : 0, (float *)y_f32, ldy, vec_d);
         IFA_LAUNCH_CHECK();
@@ -595,6 +525,20 @@ int ifa_moe_experts_glu_f32(int glu_kind, float limit, const void *h_f32, size_t
     IFA_REQUIRE(experts > 0 && (glu_kind == 0 || (glu_kind == 3 && limit > 0.0f)), "ifa_moe_experts_glu_f32: no experts, or gate kind %d (0, or 3 with a limit)", glu_kind);
     return moe_experts("ifa_moe_experts_glu_f32", 1, glu_kind, limit, h_f32, ldh, rows, width, ff, experts, 0, top, 0, gate_up_bf16, down_bf16, idx_dev, wgt_f32, ops32, ws,
                        ws_bytes, y_f32, ldy, accumulate, stream);
+}
+
+int ifa_moe_experts_routed_rows_f32(int score_kind, int renorm, float renorm_eps, float wgt_scale, const void *logits_f32, size_t ldl, const void *correction_bf16,
+                                    int glu_kind, float limit, const void *h_f32, size_t ldh, size_t rows, int width, int ff, int experts, int top,
+                                    const void *gate_up_bf16, const void *down_bf16, int *idx_dev, void *wgt_f32, void *ws, size_t ws_bytes, void *y_f32, size_t ldy,
+                                    int accumulate, ifa_stream stream)
+{
+    IFA_REQUIRE(logits_f32 && rows <= 8 && experts > 0 && experts <= 256 && ldl >= (size_t)experts && (score_kind == 0 || score_kind == 1)
+                && (glu_kind == 0 || (glu_kind == 3 && limit > 0.0f)), "ifa_moe_experts_routed_rows_f32: bad arguments (%zu rows: at most 8, %d experts: at most 256)", rows, experts);
+    RouteSel R;
+    R.logits = (const float *)logits_f32; R.ld = ldl; R.n_all = experts; R.score_kind = score_kind; R.renorm = renorm ? 1 : 0; R.renorm_eps = renorm_eps; R.wgt_scale = wgt_scale;
+    R.corr = (const bf16_t *)correction_bf16; R.idx = idx_dev; R.wgt = (float *)wgt_f32;
+    return moe_experts("ifa_moe_experts_routed_rows_f32", 1, glu_kind, limit, h_f32, ldh, rows, width, ff, experts, 0, top, 0, gate_up_bf16, down_bf16, idx_dev, wgt_f32, 1, ws,
+                       ws_bytes, y_f32, ldy, accumulate, stream, &R);
 }
 
 } // extern "C"

@@ -123,11 +123,30 @@ __global__ void __launch_bounds__(512) k_ssm_step(SsmStepArgs A)
     float *ring = base + A.conv_off;
     const float *xr = A.xbc + (size_t)t * A.ldx;
     const bool shared_writer = h == g * hpg && p0 == 0;
+    auto item = [&](int e, float *&dst, bool &wr) -> int {          // channel of the slice's e-th input, where it goes, whether this workgroup writes its ring row
+        if (e < pc) { dst = xs + e; wr = true; return h * P + p0 + e; }
+        if (e < pc + N) { dst = Bs + (e - pc); wr = shared_writer; return inner + g * N + (e - pc); }
+        dst = Cs + (e - pc - N); wr = shared_writer;
+        return inner + GN + g * N + (e - pc - N);
+    };
+    if (taps == 4) {          // the usual number of taps: every request of an input at once
+        for (int e = tid; e < pc + 2 * N; e += 512) {
+            float *dst; bool wr;
+            const int ch = item(e, dst, wr), p = sd.pos0;
+            const float cur = xr[ch], h1 = ring[(size_t)((p + 3) % 4) * C + ch], h2 = ring[(size_t)((p + 2) % 4) * C + ch], h3 = ring[(size_t)((p + 1) % 4) * C + ch];
+            const bf16_t *w = A.w + (size_t)ch * 4;
+            const float w0 = bf2f(w[0]), w1 = bf2f(w[1]), w2 = bf2f(w[2]), w3 = bf2f(w[3]), b = A.bias ? bf2f(A.bias[ch]) : 0.0f;
+            float acc = fmaf(w0, p >= 3 ? h3 : 0.0f, 0.0f);
+            acc = fmaf(w1, p >= 2 ? h2 : 0.0f, acc);
+            acc = fmaf(w2, p >= 1 ? h1 : 0.0f, acc);
+            acc = fmaf(w3, cur, acc);
+            *dst = silu_exact(acc + b);
+            if (wr) ring[(size_t)(p % 4) * C + ch] = cur;
+        }
+    } else
     for (int e = tid; e < pc + 2 * N; e += 512) {
-        int ch; float *dst; bool wr;
-        if (e < pc) { ch = h * P + p0 + e; dst = xs + e; wr = true; }
-        else if (e < pc + N) { ch = inner + g * N + (e - pc); dst = Bs + (e - pc); wr = shared_writer; }
-        else { ch = inner + GN + g * N + (e - pc - N); dst = Cs + (e - pc - N); wr = shared_writer; }
+        float *dst; bool wr;
+        const int ch = item(e, dst, wr);
         const float cur = xr[ch];
         float acc = 0.0f;
         for (int j = 0; j < taps - 1; j++) {
@@ -365,32 +384,28 @@ __global__ void __launch_bounds__(256) k_ssd_out(SsdArgs A)
     }
 }
 
-// y[t][c] = v / sqrt(mean_group(v^2) + eps) * w[c], v = o[t][c] * silu(gate[t][c]): the gate in front of the norm; one workgroup per row
-__global__ void __launch_bounds__(512) k_gate_groupnorm(const float *__restrict__ o, size_t ldo, int C, int group, const bf16_t *__restrict__ w, const float *__restrict__ gate,
+// y[t][c] = v / sqrt(mean_part(v^2) + eps) * w[c], v = o[t][c] * silu(gate[t][c]): the gate in front of the norm.  grid (rows, parts or
+// groups of four parts): a workgroup or a wave per part; a thread keeps its first GN_KEEP values, more are formed again
+constexpr int GN_KEEP = 8;
+template <bool WHOLE>      // WHOLE: one part per workgroup; else one part per wave
+__global__ void __launch_bounds__(256) k_gate_groupnorm(const float *__restrict__ o, size_t ldo, int parts, int group, const bf16_t *__restrict__ w, const float *__restrict__ gate,
                                                         size_t ldg, float eps, float *__restrict__ y, size_t ldy)
 {
-    extern __shared__ float vs[];          // [C]
     __shared__ float red[17];
-    const int t = blockIdx.x, lane = threadIdx.x & 63, wave = threadIdx.x >> 6, nw = blockDim.x >> 6;
-    const float *orow = o + (size_t)t * ldo, *grow = gate + (size_t)t * ldg;
-    float *yrow = y + (size_t)t * ldy;
-    for (int c = threadIdx.x; c < C; c += blockDim.x) vs[c] = orow[c] * silu_exact(grow[c]);
-    __syncthreads();
-    if (C / group < nw) {          // fewer groups than waves: the whole workgroup works on each group
-        for (int gi = 0; gi < C / group; gi++) {
-            float s = 0.0f;
-            for (int e = threadIdx.x; e < group; e += blockDim.x) { const float v = vs[gi * group + e]; s = fmaf(v, v, s); }
-            const float r = 1.0f / sqrtf(block_sum(s, red) / (float)group + eps);
-            for (int e = threadIdx.x; e < group; e += blockDim.x) { const int c = gi * group + e; yrow[c] = vs[c] * r * bf2f(w[c]); }
-        }
-        return;
-    }
-    for (int gi = wave; gi < C / group; gi += nw) {
-        float s = 0.0f;
-        for (int e = lane; e < group; e += 64) { const float v = vs[gi * group + e]; s = fmaf(v, v, s); }
-        const float r = 1.0f / sqrtf(wave_sum(s) / (float)group + eps);
-        for (int e = lane; e < group; e += 64) { const int c = gi * group + e; yrow[c] = vs[c] * r * bf2f(w[c]); }
-    }
+    const int t = blockIdx.x, part = WHOLE ? blockIdx.y : blockIdx.y * (blockDim.x >> 6) + (threadIdx.x >> 6);
+    const int i0 = WHOLE ? threadIdx.x : threadIdx.x & 63, step = WHOLE ? blockDim.x : 64;
+    if (!WHOLE && part >= parts) return;
+    const float *orow = o + (size_t)t * ldo + (size_t)part * group, *grow = gate + (size_t)t * ldg + (size_t)part * group;
+    const bf16_t *wr = w + (size_t)part * group;
+    float *yrow = y + (size_t)t * ldy + (size_t)part * group;
+    float v[GN_KEEP], q = 0.0f;
+#pragma unroll
+    for (int k = 0; k < GN_KEEP; k++) { const int c = i0 + k * step; v[k] = c < group ? orow[c] * silu_exact(grow[c]) : 0.0f; q = fmaf(v[k], v[k], q); }
+    for (int c = i0 + GN_KEEP * step; c < group; c += step) { const float u = orow[c] * silu_exact(grow[c]); q = fmaf(u, u, q); }
+    const float r = 1.0f / sqrtf((WHOLE ? block_sum(q, red) : wave_sum(q)) / (float)group + eps);
+#pragma unroll
+    for (int k = 0; k < GN_KEEP; k++) { const int c = i0 + k * step; if (c < group) yrow[c] = v[k] * r * bf2f(wr[c]); }
+    for (int c = i0 + GN_KEEP * step; c < group; c += step) yrow[c] = orow[c] * silu_exact(grow[c]) * r * bf2f(wr[c]);      // (y may be o: a value is read before it is written)
 }
 
 size_t al16s(size_t v) { return (v + 15) & ~(size_t)15; }
@@ -495,10 +510,15 @@ int ifa_gate_groupnorm_f32(const void *o_f32, size_t ldo, size_t rows, int chann
                            void *y_f32, size_t ldy, ifa_stream stream)
 {
     IFA_REQUIRE(o_f32 && w_bf16 && gate_f32 && y_f32, "ifa_gate_groupnorm_f32: null pointer");
-    IFA_REQUIRE(rows > 0 && channels > 0 && groups > 0 && channels % groups == 0 && ldo >= (size_t)channels && ldg >= (size_t)channels && ldy >= (size_t)channels
-                && (size_t)channels * 4 <= 64 * 1024 - 256, "ifa_gate_groupnorm_f32: bad arguments (%d channels in %d groups)", channels, groups);
-    hipLaunchKernelGGL(k_gate_groupnorm, dim3((unsigned)rows), dim3(channels >= 2048 ? 512 : 256), (size_t)channels * 4, ifa_s(stream), (const float *)o_f32, ldo, channels,
-                       channels / groups, (const bf16_t *)w_bf16, (const float *)gate_f32, ldg, eps, (float *)y_f32, ldy);
+    IFA_REQUIRE(rows > 0 && rows < (1u << 31) && channels > 0 && groups > 0 && groups < 65536 && channels % groups == 0 && ldo >= (size_t)channels && ldg >= (size_t)channels
+                && ldy >= (size_t)channels, "ifa_gate_groupnorm_f32: bad arguments (%d channels in %d groups)", channels, groups);
+    const int group = channels / groups;
+    if (group > 256)
+        hipLaunchKernelGGL(k_gate_groupnorm<true>, dim3((unsigned)rows, (unsigned)groups), dim3(group > 512 ? 256 : 128), 0, ifa_s(stream), (const float *)o_f32, ldo, groups, group,
+                           (const bf16_t *)w_bf16, (const float *)gate_f32, ldg, eps, (float *)y_f32, ldy);
+    else
+        hipLaunchKernelGGL(k_gate_groupnorm<false>, dim3((unsigned)rows, ifa_cdiv((size_t)groups, 4)), dim3(256), 0, ifa_s(stream), (const float *)o_f32, ldo, groups, group,
+                           (const bf16_t *)w_bf16, (const float *)gate_f32, ldg, eps, (float *)y_f32, ldy);
     IFA_LAUNCH_CHECK();
     return IFA_OK;
 }

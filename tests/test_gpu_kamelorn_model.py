@@ -149,7 +149,7 @@ def test_portions_and_token_by_token_equal_the_whole_prompt(tmp_path, sizes):
 
 
 def test_folded_launches_and_separate_ops_agree(tmp_path):
-    """the streams' update with the norm behind it, and with the router behind that, against the same steps as launches of their own"""
+    """the streams' update with the norm behind it, and the router's choice inside the experts' launch, against the same steps as launches of their own"""
     import inferflow_amd as ia
     w = fx.random_weights(MIXED, 25)
     toks = tokens_for(MIXED, 60, 26)
@@ -371,7 +371,7 @@ CASES = {
     # many experts of which eight are chosen, sixteen streams, the largest state
     "many": lambda: fx.config([fx.ssm_layer(heads=4, vdim=16, state=256, groups=4, norm_groups=2, mlp=fx.moe(experts=70, top=8, ff=16, scale=3.0)),
                                fx.latent_layer(heads=5, dim=24, rot_dim=12, vdim=20, kv_rank=40, mlp=fx.moe(experts=17, top=17, ff=8))], width=32, vocab=29, streams=16),
-    # more router outputs than the fused choice keeps in registers; a group at the end with four passes
+    # more router outputs than the experts' launch chooses from; a group at the end with four passes
     "huge_router": lambda: fx.config([fx.ssm_layer(heads=2, vdim=16, state=64, groups=1, mlp=fx.dense(24)), fx.latent_layer(mlp=fx.moe(experts=530, top=3, ff=4)),
                                       fx.ssm_layer(heads=3, vdim=32, state=96, groups=1, norm_groups=3, mlp=None)], width=32, vocab=40, streams=2, loop=(1, 3, 4)),
 }

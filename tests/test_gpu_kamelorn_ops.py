@@ -1,7 +1,8 @@
 """Each mechanism that the Kamelorn layers add to the layer-list worker alone, through its C-ABI op, against the float64 functions of
-tests/kamelorn_oracle.py: the residual streams' step (embedding, update, read-out, norm, sum; with the router behind it), the convolution over a
+tests/kamelorn_oracle.py: the residual streams' step (embedding, update, read-out, norm, sum), the convolution over a
 ring, the state space in its three forms (single tokens, chunks, token by token; continued states, several sequences, reused slots), the gate in
-front of the norm in parts, latent attention rotated in halves with a gate per column in both forms, the renormalized router."""
+front of the norm in parts, latent attention rotated in halves with a gate per column in both forms, the renormalized router, also inside the
+experts' first launch."""
 import ctypes as C
 
 import numpy as np
@@ -60,35 +61,46 @@ def test_streams_step(rows, S, cols):
     assert near(xd.cpu().numpy(), np.stack([e + mult * y[:, :cols]] * S, 1))
 
 
-@pytest.mark.parametrize("rows,S,W,n_all,top,kind", [(1, 2, 64, 6, 2, 1), (3, 4, 2048, 32, 6, 1), (8, 3, 40, 16, 1, 1), (2, 1, 512, 5, 5, 1), (2, 4, 1032, 70, 8, 0), (1, 2, 8, 500, 3, 1),
-                                                     (2, 16, 264, 3, 2, 0)])
-def test_streams_step_with_the_router_behind_it_equals_the_separate_ops(rows, S, W, n_all, top, kind):
-    rng = np.random.default_rng(rows + W + n_all)
-    X, y = rng.standard_normal((rows, S, W)).astype(np.float32), rng.standard_normal((rows, W)).astype(np.float32)
-    mix, out, nin = bf16_round(rng.standard_normal((S, S))), bf16_round(rng.standard_normal(S)), bf16_round(1 + 0.2 * rng.standard_normal(S))
-    nw, router = bf16_round(1 + 0.3 * rng.standard_normal(W)), bf16_round(rng.standard_normal((n_all, W)) * 2 / np.sqrt(W))
-    corr = bf16_round(0.2 * rng.standard_normal(n_all)) if kind == 0 else None
-    if n_all >= 5:
-        router[3] = router[1]
+@pytest.mark.parametrize("rows,W,F,E,top,kind", [(1, 64, 24, 6, 2, 1), (3, 256, 40, 32, 6, 1), (8, 40, 10, 16, 1, 1), (2, 64, 16, 5, 5, 1), (2, 72, 9, 70, 8, 0), (1, 14, 6, 256, 3, 1),
+                                                  (2, 16, 8, 3, 2, 0), (1, 8, 1, 1, 1, 1)])
+def test_experts_with_the_choice_inside_their_first_launch(rows, W, F, E, top, kind):
+    rng = np.random.default_rng(rows + W + E)
+    h = rng.standard_normal((rows, W)).astype(np.float32)
+    router = bf16_round(rng.standard_normal((E, W)) * 2 / np.sqrt(W))
+    corr = bf16_round(0.2 * rng.standard_normal(E)) if kind == 0 else None
+    if E >= 5:
+        router[3] = router[1]          # a tie: the lower index wins
         if corr is not None:
             corr[3] = corr[1]
+    gate, up, down = (bf16_round(rng.standard_normal(s) * 0.3) for s in ((E, F, W), (E, F, W), (E, W, F)))
+    logits = (orc.f64(h) @ orc.f64(router).T).astype(np.float32)
+    if kind == 1:
+        idx_w, wgt_w = orc.route(orc.f64(h), orc.f64(router), top, 1.7)
+    else:
+        z = orc.f64(logits); sc = np.exp(z - z.max(-1, keepdims=True)); sc /= sc.sum(-1, keepdims=True)
+        idx_w = np.argsort(-(sc + orc.f64(corr)), axis=-1, kind="stable")[:, :top]
+        wgt_w = np.take_along_axis(sc, idx_w, -1); wgt_w = wgt_w / wgt_w.sum(-1, keepdims=True) * 1.7
+    want = np.zeros((rows, W))
+    for t in range(rows):
+        for e, wv in zip(idx_w[t], wgt_w[t]):
+            want[t] += wv * orc.gated_ffn(orc.f64(h[t:t + 1]), orc.f64(gate[e]), orc.f64(up[e]), orc.f64(down[e]))[0]
     L = capi()
-    assert L.ifa_moe_streams_route_rows_fits(S, W, n_all, top) == 1
-    res = []
-    for fused in (1, 0):
-        xd, h = dev32(X), torch.zeros((rows, W), dtype=torch.float32, device="cuda")
-        idx, wgt = torch.full((rows, top), -1, dtype=torch.int32, device="cuda"), torch.zeros((rows, top), dtype=torch.float32, device="cuda")
-        dy, dm, do, di, dn, dr, dc = dev32(y), devbf(mix), devbf(out), devbf(nin), devbf(nw), devbf(router), devbf(corr) if corr is not None else None
-        pc = p(dc) if dc is not None else None
-        if fused:
-            ia.check(L.ifa_moe_streams_route_rows_f32(kind, 1, 1e-20, 1.7, p(xd), rows, S, W, p(dy), W, p(dm), p(do), 0.4, p(di), p(dn), 1e-5, p(h), W, p(dr), n_all, top, pc, p(idx),
-                                                      p(wgt), None))
-        else:
-            ia.check(L.ifa_streams_step_f32(p(xd), rows, S, W, None, None, 0, 1.0, p(dy), W, p(dm), p(do), 0.4, p(di), p(dn), 1e-5, p(h), W, None, 0, None))
-            ia.check(L.ifa_moe_route_rows_renorm_f32(kind, 1, 1e-20, 1.7, p(h), W, rows, W, p(dr), n_all, top, pc, p(idx), p(wgt), None))
-        sync(); res.append([t.cpu().numpy() for t in (xd, h, idx, wgt)])
-    assert np.array_equal(res[0][0], res[1][0]) and near(res[0][1], res[1][1]) and np.array_equal(res[0][2], res[1][2]) and near(res[0][3], res[1][3], 5e-6)
-    assert np.abs(res[0][3].sum(-1) - 1.7).max() < 1e-5
+    nb = L.ifa_moe_workspace_bytes(rows, top, W, 3 * F, E)
+    ws = torch.empty((nb,), dtype=torch.uint8, device="cuda")
+    idx, wgt = torch.full((rows, top), -1, dtype=torch.int32, device="cuda"), torch.zeros((rows, top), dtype=torch.float32, device="cuda")
+    y = torch.zeros((rows, W), dtype=torch.float32, device="cuda")
+    gu, dd, dh, dl = devbf(np.concatenate([gate, up], 1).reshape(E * 2 * F, W)), devbf(down.reshape(E * W, F)), dev32(h), dev32(logits)
+    dc = devbf(corr) if corr is not None else None
+    ia.check(L.ifa_moe_experts_routed_rows_f32(kind, 1, 1e-20, 1.7, p(dl), E, p(dc) if dc is not None else None, 0, 0.0, p(dh), W, rows, W, F, E, top, p(gu), p(dd), p(idx), p(wgt), p(ws),
+                                               nb, p(y), W, 0, None)); sync()
+    assert np.array_equal(idx.cpu().numpy(), idx_w) and near(wgt.cpu().numpy(), wgt_w, 5e-6) and near(y.cpu().numpy(), want, 2e-5)
+    # without renormalization: the plain scores
+    ia.check(L.ifa_moe_experts_routed_rows_f32(kind, 0, 0.0, 1.0, p(dl), E, p(dc) if dc is not None else None, 0, 0.0, p(dh), W, rows, W, F, E, top, p(gu), p(dd), p(idx), p(wgt), p(ws),
+                                               nb, p(y), W, 0, None)); sync()
+    plain = wgt.cpu().numpy()
+    assert near(plain / plain.sum(-1, keepdims=True) * 1.7, wgt_w, 5e-6)
+    if kind == 1:
+        assert near(plain, orc.logistic(np.take_along_axis(orc.f64(logits), idx_w, -1)), 5e-6)
 
 
 @pytest.mark.parametrize("T,n_all,top,scale", [(9, 6, 2, 2.5), (70, 16, 1, 0.3), (5, 5, 5, 1.0), (12, 70, 8, 3.0)])
