@@ -194,7 +194,7 @@ template <int SMAX, bool VEC>
 __global__ void __launch_bounds__(1024) k_streams_step(StreamArgs P)
 {
     __shared__ float lds[SMAX * SMAX + 2 * SMAX + 17];
-    streams_row<SMAX, VEC>(P, blockIdx.x, lds, nullptr);
+    streams_row<SMAX, VEC>(P, blockIdx.x, lds);
 }
 
 // stack[count - 1] <- x; x <- sum_j w[j] stack[j]  (element-wise over n = rows * cols values)

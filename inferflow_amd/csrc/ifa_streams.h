@@ -1,9 +1,8 @@
-// ifa_streams.h -- what lies between two sub-layers of a block with several residual streams, for one row by one workgroup
-// (k_streams_step, and the fused router of steps of a few rows).  x [rows][S][cols]:
+// ifa_streams.h -- what lies between two sub-layers of a block with several residual streams, for one row by one workgroup.  x [rows][S][cols]:
 //   0. (embed not null) X_s <- embed[token] * scale for every s          (the start of the stack)
 //   1. (y not null)     X_t <- sum_s mix[s][t] X_s + mult * out[t] * y    (all new streams from the old ones; mix / out null: identity / ones)
 //   2. u = sum_s in[s] X_s (in null: ones);  sum_out <- u (if asked for)
-//   3. (w not null)     h = u / sqrt(mean(u^2) + eps) * w                 (also into LDS when h_lds is given)
+//   3. (w not null)     h = u / sqrt(mean(u^2) + eps) * w
 // A thread keeps its pieces of a row (16 bytes when VEC) in registers from stage 1 to stage 3; all of a row's loads are issued before the first barrier.
 #pragma once
 #include "ifa_f32_common.h"
@@ -31,7 +30,7 @@ template <int N> __device__ __forceinline__ void st_store(float *p, const float 
 
 // lds: SMAX * SMAX + 2 SMAX + 17 floats
 template <int SMAX, bool VEC>
-__device__ void streams_row(const StreamArgs &P, int row, float *lds, float *h_lds)
+__device__ void streams_row(const StreamArgs &P, int row, float *lds)
 {
     constexpr int N = VEC ? 4 : 1, KEEP = SMAX <= 4 ? 2 : 1;
     float *red = lds, *mx = lds + 17, *ob = mx + SMAX * SMAX, *ib = ob + SMAX;
@@ -111,10 +110,6 @@ __device__ void streams_row(const StreamArgs &P, int row, float *lds, float *h_l
 #pragma unroll
         for (int k = 0; k < N; k++) uu[k] = uu[k] * rinv * bf2f(P.w[c + k]);
         st_store<N>(hr + c, uu);
-        if (h_lds) {
-#pragma unroll
-            for (int k = 0; k < N; k++) h_lds[c + k] = uu[k];
-        }
     };
 #pragma unroll
     for (int i = 0; i < KEEP; i++) { const int p = tid + i * nt; if (p < pieces) finish(p * N, u[i]); }
