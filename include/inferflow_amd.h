@@ -765,6 +765,37 @@ int ifa_attention_latent_tile_gated_f32(int gate_cols, const void *q_f32, size_t
                                         const void *kx_f32, size_t ldkx, const void *vx_f32, size_t ldvx, const int *ctx0_dev, const void *g_f32, size_t ldg,
                                         const void *seqs_dev, const void *seqs_host, int n_seqs, void *const *slot_base_dev, size_t cache_off,
                                         void *out_f32, size_t ldo, ifa_stream stream);
+/* the two forms above with a learned sink per head (sink_bf16 [heads], null: none): exp(sink[h]) joins the softmax's denominator, once, unscaled, with no
+ * key and no value */
+int ifa_attention_latent_rows_sinks_f32(const void *qa_f32, size_t ldqa, int heads, int kv_rank, int rot_dim, float scale, const void *sink_bf16, const void *seqs_dev,
+                                        const int *row_seq_dev, size_t rows, void *const *slot_base_dev, size_t cache_off, int max_keys, void *ws_f32,
+                                        size_t ws_bytes, void *out_f32, size_t ldo, ifa_stream stream);
+int ifa_attention_latent_tile_sinks_f32(int gate_cols, const void *q_f32, size_t ldq, int heads, int dim, int rot_dim, int vdim, int kv_rank, float scale,
+                                        const void *sink_bf16, const void *kx_f32, size_t ldkx, const void *vx_f32, size_t ldvx, const int *ctx0_dev, const void *g_f32,
+                                        size_t ldg, const void *seqs_dev, const void *seqs_host, int n_seqs, void *const *slot_base_dev, size_t cache_off, void *out_f32,
+                                        size_t ldo, ifa_stream stream);
+/* the queries' part of ifa_latent_prepare_pairs_f32 alone (a layer that reads another layer's cache rows): the rotated part of every query head in place */
+int ifa_latent_rotate_q_f32(int pairing, int rot_dim, int rot_dims, void *q_f32, size_t ldq, int heads, int dim, const double *freq_f64_dev, float rot_mult,
+                            const void *seqs_dev, const int *row_seq_dev, size_t rows, ifa_stream stream);
+/* ifa_qk_rope_store_f32 with a choice of the rotated pairs (pairing 1 = interleaved (2i, 2i + 1), 0 = halves (i, i + rot_dims / 2)) and a number of value
+ * heads of its own: k has k_heads heads of dim, v has v_heads heads of vdim (differential attention: two key heads per value head) */
+int ifa_qk_rope_store_pairs_f32(int pairing, void *q_f32, size_t ldq, int heads, const void *k_f32, size_t ldk, const void *v_f32, size_t ldv, int k_heads, int v_heads,
+                                int dim, int vdim, const void *q_norm_w_bf16, const void *k_norm_w_bf16, float eps, int rot_dims, const double *freq_f64_dev,
+                                const void *seqs_dev, const int *row_seq_dev, size_t rows, void *const *slot_base_dev, size_t k_off, size_t v_off, ifa_stream stream);
+/* Differential attention over cached rows (ifa_qk_rope_store_pairs_f32): K rows [kv_heads][2 maps][dim], V rows [kv_heads][vdim], queries
+ * [rows][heads][2 maps][dim]; query head h reads key / value head h / (heads / kv_heads).  Position i sees key j iff j <= i, i - j < window (window 0: any
+ * distance) and, chunk > 0, i / chunk == j / chunk.  With a_m = softmax(q_m . k_m * scale) v per map: o = a_1 - lambda a_2,
+ * out = o / sqrt(mean(o^2) + eps) * out_scale * sigmoid(g[t][h]) (g null: no gate).  Steps whose longest sequence brings tile_min_rows rows or more run 64
+ * queries of one sequence per workgroup on the fp32 matrix cores (dim <= 128, vdim <= 128 or 193 .. 256); others a workgroup per (row, up to four heads
+ * of a group, share of the keys) through ws_f32 (rows * heads * shares * 2 * (vdim + 2) floats; max_keys > 0 bounds the shares) and a second launch that merges
+ * the shares, takes the difference, norms and gates.  dim, vdim <= 1024. */
+int ifa_attention_diff_f32(const void *q_f32, size_t ldq, int heads, int kv_heads, int dim, int vdim, float scale, int window, int chunk, float lambda, float out_scale,
+                           float eps, const void *g_f32, size_t ldg, const void *seqs_dev, const int *row_seq_dev, size_t rows, void *const *slot_base_dev, size_t k_off,
+                           size_t v_off, void *out_f32, size_t ldo, const void *seqs_host, int n_seqs, int tile_min_rows, int max_keys, void *ws_f32, size_t ws_bytes,
+                           ifa_stream stream);
+/* ifa_linear_bf16w with an activation of every output after the bias: act 0 none, 1 erf-GELU, 2 relu(z)^2 */
+int ifa_linear_bf16w_act(const void *w_bf16, size_t rows, size_t cols, const void *a_f32, size_t lda, size_t tokens, const void *bias_bf16, int act, int ops32,
+                         void *c_f32, size_t ldc, ifa_stream stream);
 /* ifa_moe_route_scores_f32 / ifa_moe_route_rows_scores_f32 with renormalized weights: renorm != 0: weight = score / (sum of the chosen
  * scores + renorm_eps) * wgt_scale */
 int ifa_moe_route_renorm_f32(int score_kind, int renorm, float renorm_eps, float wgt_scale, const void *logits_f32, size_t ld, size_t rows, int n_all, int top,
@@ -794,12 +825,15 @@ enum { IFA_MIX_WINDOW_LINEAR = 1,   /* windowed softmax attention (values = keys
                                      * of an earlier layer, optionally scaled frequencies, normed values, rotated values */
        IFA_MIX_CHAN_DELTA = 5,      /* generalized delta rule: decay and removal rate per head and key channel (the decay through a small
                                      * two-matrix bottleneck), unit keys for the removal, per-head RMS norm x weight x sigmoid gate on the output */
-       IFA_MIX_SSM = 6 };           /* selective state space (Mamba-2): z | x | B | C | dt in one projection, short convolution with bias + SiLU over
+       IFA_MIX_SSM = 6,             /* selective state space (Mamba-2): z | x | B | C | dt in one projection, short convolution with bias + SiLU over
                                      * x | B | C, state per head, skip D x, SiLU gate in front of a grouped RMS norm */
+       IFA_MIX_DIFF = 7 };          /* differential attention: two softmax maps per head over the same values, the second times a learned factor taken off
+                                     * the first, the difference normed per head; grouped queries, rotation, window and / or chunks, gate per head */
 /* wiring of a layer.  PARALLEL: h = norm1(x); x <- x + ls1 * mixer(h) + ls2 * ffn(h).  POSTNORM: the sub-layers read x itself (plus a
  * short causal convolution of x when canon_taps > 0) and the grouped RMS norm sits on their OUTPUT: x <- x + norm1(mixer(x'));
  * x <- x + norm2(ffn(x')); with depth_avg the next layer reads sum_j dwa[j] X_j over the embedding output X_0 and every layer result.
- * SANDWICH: an RMS norm with weight (1 + w) before AND after each sub-layer: x <- x + norm1b(mixer(norm1(x))); x <- x + norm2b(ffn(norm2(x))).
+ * SANDWICH: an RMS norm before AND after each sub-layer: x <- x + norm1b(mixer(norm1(x))); x <- x + norm2b(ffn(norm2(x))), weights (1 + w), or w as
+ * stored with cfg.norm_plain.
  * PRENORM: x <- x + mixer(norm1(x)); x <- x + ffn(norm2(x)) with Dynamic Tanh norms tanh(alpha x) w + b (tensors IFA_LT_NORM1 / _B / _ALPHA).
  * STREAMS: cfg.streams residual streams X_s per token and RMS norms in front of the sub-layers q = 1, 2 (mixer, feed-forward): u = sum_s in_q[s] X_s,
  * y = sub_q(norm_q(u)), X_t <- sum_s mix_q[s][t] X_s + cfg.residual_mult * out_q[t] y (tensors IFA_LT_HC1_* / IFA_LT_HC2_*; cfg.streams 0: one plain
@@ -808,7 +842,8 @@ enum { IFA_BLOCK_PARALLEL = 0, IFA_BLOCK_POSTNORM = 1, IFA_BLOCK_SANDWICH = 2, I
 enum { IFA_FFN_GATED = 0,           /* gated feed-forward (GELU tanh, biases), width `ffn` */
        IFA_FFN_MOE = 1,             /* mixture of experts: x_experts experts of width x_ff + x_identity identity experts, x_top per token */
        IFA_FFN_CLAMPED = 2,         /* width `ffn`, no biases: g = min(gate, f_limit), u = clamp(up, +-f_limit), y = down(g sigmoid(1.702 g) (u + 1)) */
-       IFA_FFN_SILU = 3 };          /* width `ffn`, no biases: y = down(silu(gate) * up) */
+       IFA_FFN_SILU = 3,            /* width `ffn`, no biases: y = down(silu(gate) * up) */
+       IFA_FFN_RELU2 = 4 };         /* width `ffn`, no biases, no gate: y = down(relu(up)^2) */
 typedef struct {
     int mixer;                       /* IFA_MIX_* */
     int ffn;                         /* width of the gated feed-forward (GELU tanh, biases); 0 = none */
@@ -862,6 +897,16 @@ typedef struct {
     /* IFA_MIX_SSM: s_heads heads of s_vdim channels with states of s_state rows, B and C in s_groups groups, s_conv taps, output norm in
      * s_norm_groups equal parts */
     int s_heads, s_vdim, s_state, s_groups, s_conv, s_norm_groups;
+    /* more of latent attention (SANDWICH wiring): m_sink 1: a learned sink per head (tensor IFA_LT_M_SINK); m_kv_layer: 0 = cache rows of its own, j + 1 =
+     * the cache rows of layer j (an earlier latent layer with rows of its own, the same m_kv_rank / m_rot_dim and the same rotation): the layer
+     * then has no IFA_LT_M_DKV / _NORM */
+    int m_sink, m_kv_layer;
+    /* IFA_MIX_DIFF (with a_heads, a_kv_heads, a_dim = size of a head in ONE map, a_vdim, a_scale, a_window 0 = unlimited, a_rot_dims, a_rot_base):
+     * a_rot_pairs 1: dimensions (2i, 2i + 1) turn together, 0: (i, i + a_rot_dims / 2); a_chunk > 0: a position sees its own chunk of that many positions
+     * only; a_gate 1: sigmoid gate per head (IFA_LT_A_G).  o = a_1 - lambda a_2, lambda = exp(lq1 . lk1) - exp(lq2 . lk2) + a_diff; the head's output is
+     * o / rms(o) * (1 - a_diff) */
+    int a_rot_pairs, a_chunk, a_gate;
+    float a_diff;
 } ifa_layer_spec;
 typedef struct {
     int width, vocab, max_ctx, n_layers, device;
@@ -873,7 +918,7 @@ typedef struct {
     float logit_softcap;             /* > 0: logits <- cap * tanh(logits / cap) */
     /* stem 2: embedding + hashed token-pair embedding (IFA_T_BIGRAM row (prev * bigram_mul_prev + token * bigram_mul_cur) mod
      * bigram_buckets; row bigram_buckets for a sequence's first token; bigram_buckets 0: none), no position vector, RMS norm with
-     * weight (1 + w) before lm_head.  The previous token of a sequence is kept in its slot. */
+     * weight (1 + w) (norm_plain: w) before lm_head; the token embedding times embed_scale (0: 1).  The previous token of a sequence is kept in its slot. */
     int bigram_buckets, bigram_mul_prev, bigram_mul_cur;
     /* stem 3: stem 2 with the token embedding times embed_scale (0: 1), a Dynamic Tanh norm before lm_head (IFA_T_OUT_NORM / _B / _ALPHA)
      * and logits times logit_scale (0: 1) */
@@ -886,6 +931,7 @@ typedef struct {
      * RMS norm before lm_head; a looped group repeats with nothing between its passes (no IFA_T_LOOP_STEP).  streams 0: one plain residual */
     int streams;
     float residual_mult;
+    int norm_plain;                  /* 1: the norms of SANDWICH layers and of stem 2 multiply by the stored weight, 0: by one plus the stored weight */
 } ifa_layered_config;
 /* tensors of a layer-list model (global ones use IFA_T_EMBD / IFA_T_OUT_NORM / IFA_T_LM_HEAD with layer = -1) */
 enum {
@@ -904,6 +950,8 @@ enum {
     IFA_LT_C_R, IFA_LT_C_K, IFA_LT_C_V, IFA_LT_C_G, IFA_LT_C_A, IFA_LT_C_A_B, IFA_LT_C_W1, IFA_LT_C_W2, IFA_LT_C_W0, IFA_LT_C_NORM, IFA_LT_C_O,      /* IFA_MIX_CHAN_DELTA */
     IFA_LT_HC1_IN, IFA_LT_HC1_OUT, IFA_LT_HC1_MIX, IFA_LT_HC2_IN, IFA_LT_HC2_OUT, IFA_LT_HC2_MIX,      /* STREAMS: [streams], [streams], [streams][streams] (from, to) */
     IFA_LT_S_IN, IFA_LT_S_CONV, IFA_LT_S_CONV_B, IFA_LT_S_DTBIAS, IFA_LT_S_ALOG, IFA_LT_S_D, IFA_LT_S_NORM, IFA_LT_S_O,      /* IFA_MIX_SSM */
+    IFA_LT_M_SINK,                                 /* latent attention with m_sink: [heads] */
+    IFA_LT_A_G, IFA_LT_A_LQ1, IFA_LT_A_LK1, IFA_LT_A_LQ2, IFA_LT_A_LK2,      /* IFA_MIX_DIFF (with IFA_LT_A_Q / _K / _V / _O): [heads][width], [a_dim] each */
     IFA_LT_END
 };
 int ifa_model_create_layered(const ifa_layered_config *cfg, const ifa_layer_spec *layers, ifa_model **out);

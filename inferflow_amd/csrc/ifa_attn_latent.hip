@@ -1,6 +1,7 @@
 // ifa_attn_latent.hip -- latent attention: every position leaves ONE cache row [kv_rank latent c | rot_dim rotated key part] in
 // 32-bit floats that all heads share; a head's unrotated key is W_uk[h] c, its value W_uv[h] c, and
-//     score(i, j, h) = (q_u[i][h] . W_uk[h] c_j + q_r[i][h] . k_r[j]) * scale,   causal, ordinary softmax.
+//     score(i, j, h) = (q_u[i][h] . W_uk[h] c_j + q_r[i][h] . k_r[j]) * scale,   causal, ordinary softmax, optionally with a learned sink per head
+// (exp(sink[h]) joins the denominator).  A layer may read the cache rows that an earlier layer has written; it then turns its queries only.
 // Two forms of the same sums:
 //   single tokens   the key map is absorbed into the query, qa[h] = [W_uk[h]^T q_u | q_r], which is then a query of kv_rank + rot_dim
 //                   dimensions against the cache rows themselves (one shared "KV head": ifa_attention_window_f32 with the value row =
@@ -20,6 +21,7 @@ using namespace ifa32;
 namespace {
 
 // one workgroup per row: latent normed into the cache, key part rotated into the cache, the rotated part of every query head in place
+// (kv null: the queries only)
 __global__ void __launch_bounds__(256) k_latent_prepare(const float *__restrict__ kv, size_t ldkv, int R, int dr, int rdims, const bf16_t *__restrict__ cw, float eps,
                                                         float *__restrict__ q, size_t ldq, int heads, int dim, const double *__restrict__ freq, float mult,
                                                         const SeqDesc *__restrict__ seqs, const int *__restrict__ row_seq, float *const *__restrict__ slot_base,
@@ -35,19 +37,21 @@ __global__ void __launch_bounds__(256) k_latent_prepare(const float *__restrict_
         cs[i] = (float)(cos(a) * (double)mult);
         cs[half + i] = (float)(sin(a) * (double)mult);
     }
-    const float *kr = kv + (size_t)t * ldkv;
-    float *row = slot_base[sd.slot] + cache_off + (size_t)pos * (R + dr);
-    float s = 0.0f;
-    for (int c = tid; c < R; c += blockDim.x) s = fmaf(kr[c], kr[c], s);
-    const float rinv = 1.0f / sqrtf(block_sum(s, red) / (float)R + eps);          // (the barrier inside also publishes cs)
-    for (int c = tid; c < R; c += blockDim.x) row[c] = kr[c] * rinv * bf2f(cw[c]);
-    for (int i = tid; i < half; i += blockDim.x) {
-        const int a = halves ? i : 2 * i, b = halves ? i + half : 2 * i + 1;
-        const float u = kr[R + a], v = kr[R + b], co = cs[i], si = cs[half + i];
-        row[R + a] = u * co - v * si;
-        row[R + b] = v * co + u * si;
-    }
-    for (int c = rdims + tid; c < dr; c += blockDim.x) row[R + c] = kr[R + c];
+    if (kv) {
+        const float *kr = kv + (size_t)t * ldkv;
+        float *row = slot_base[sd.slot] + cache_off + (size_t)pos * (R + dr);
+        float s = 0.0f;
+        for (int c = tid; c < R; c += blockDim.x) s = fmaf(kr[c], kr[c], s);
+        const float rinv = 1.0f / sqrtf(block_sum(s, red) / (float)R + eps);          // (the barrier inside also publishes cs)
+        for (int c = tid; c < R; c += blockDim.x) row[c] = kr[c] * rinv * bf2f(cw[c]);
+        for (int i = tid; i < half; i += blockDim.x) {
+            const int a = halves ? i : 2 * i, b = halves ? i + half : 2 * i + 1;
+            const float u = kr[R + a], v = kr[R + b], co = cs[i], si = cs[half + i];
+            row[R + a] = u * co - v * si;
+            row[R + b] = v * co + u * si;
+        }
+        for (int c = rdims + tid; c < dr; c += blockDim.x) row[R + c] = kr[R + c];
+    } else __syncthreads();
     float *qr = q + (size_t)t * ldq;
     for (int e = tid; e < heads * half; e += blockDim.x) {
         const int h = e / half, i = e % half;
@@ -121,6 +125,7 @@ struct LatRowArgs {
     float *ws; int nsplit;                      // [rows][heads][nsplit][R + 2]
     float *out; size_t ldo;                     // [rows][heads * R]
     int vec;
+    const bf16_t *sink;                         // [heads] or null
 };
 
 template <int HB, int CPL>
@@ -242,9 +247,10 @@ __global__ void __launch_bounds__(64) k_attn_latent_rows_combine(LatRowArgs P)
     const int t = blockIdx.x, h = blockIdx.y, dv = P.R, nsplit = P.nsplit, lane = threadIdx.x;
     const float *src = P.ws + ((size_t)t * P.heads + h) * nsplit * (dv + 2);
     const float m_sp = lane < nsplit ? src[(size_t)lane * (dv + 2)] : -INFINITY, l_sp = lane < nsplit ? src[(size_t)lane * (dv + 2) + 1] : 0.0f;
-    const float M = wave_max(m_sp);
+    const float snk = P.sink ? bf2f(P.sink[h]) : -INFINITY;
+    const float M = fmaxf(snk, wave_max(m_sp));
     const float f_sp = m_sp == -INFINITY ? 0.0f : expf(m_sp - M);
-    const float L = wave_sum(l_sp * f_sp);
+    const float L = wave_sum(l_sp * f_sp) + (P.sink ? expf(snk - M) : 0.0f);
     const int d = blockIdx.z * 64 + lane;
     const float *col = src + 2 + min(d, dv - 1);
     float o0 = 0.0f, o1 = 0.0f, o2 = 0.0f, o3 = 0.0f;
@@ -313,6 +319,7 @@ struct LatTileArgs {
     float *const *slot_base; size_t cache_off;
     float *out; size_t ldo;
     int vec;
+    const bf16_t *sink;          // [heads] or null
 };
 
 template <int NTK, int NTV>
@@ -448,7 +455,11 @@ __global__ void __launch_bounds__(256) k_attn_latent_tile(LatTileArgs P)
     if (i >= nq_w) return;
     const size_t row = (size_t)(r0 + 32 * wave + i);
     const float gate = P.g && !P.gate_cols ? sigmoid_f(P.g[row * P.ldg + h]) : 1.0f;
-    const float sc = gate / ls;
+    float sc = gate / ls;
+    if (P.sink) {          // (a large sink: both sums relative to the larger of the two maxima)
+        const float snk = bf2f(P.sink[h]), M = fmaxf(m, snk), f = expf(m - M);
+        sc = gate * f / (ls * f + expf(snk - M));
+    }
 #pragma unroll
     for (int nt = 0; nt < NTV; nt++)
 #pragma unroll
@@ -510,6 +521,21 @@ int ifa_latent_prepare_pairs_f32(int pairing, const void *kv_f32, size_t ldkv, i
     return IFA_OK;
 }
 
+int ifa_latent_rotate_q_f32(int pairing, int rot_dim, int rot_dims, void *q_f32, size_t ldq, int heads, int dim, const double *freq_f64_dev, float rot_mult,
+                            const void *seqs_dev, const int *row_seq_dev, size_t rows, ifa_stream stream)
+{
+    IFA_REQUIRE(pairing == 0 || pairing == 1, "ifa_latent_rotate_q_f32: pairing %d", pairing);
+    IFA_REQUIRE(q_f32 && freq_f64_dev && seqs_dev && row_seq_dev, "ifa_latent_rotate_q_f32: null pointer");
+    IFA_REQUIRE(rot_dim >= 0 && rot_dims >= 0 && rot_dims <= rot_dim && rot_dims % 2 == 0 && heads > 0 && dim >= 0 && rows > 0 && ldq >= (size_t)heads * (dim + rot_dim),
+                "ifa_latent_rotate_q_f32: bad shape");
+    if (rot_dims == 0) return IFA_OK;
+    hipLaunchKernelGGL(k_latent_prepare, dim3((unsigned)rows), dim3(256), (size_t)std::max(rot_dims, 2) * 4, ifa_s(stream), (const float *)nullptr, (size_t)0, 0, rot_dim,
+                       rot_dims, (const bf16_t *)nullptr, 0.0f, (float *)q_f32, ldq, heads, dim, freq_f64_dev, rot_mult, (const SeqDesc *)seqs_dev, row_seq_dev,
+                       (float *const *)nullptr, (size_t)0, pairing);
+    IFA_LAUNCH_CHECK();
+    return IFA_OK;
+}
+
 int ifa_latent_absorb_q_f32(const void *q_f32, size_t ldq, int heads, int dim, int rot_dim, int kv_rank, const void *w_uk_bf16, size_t rows,
                             void *qa_f32, size_t ldqa, ifa_stream stream)
 {
@@ -548,6 +574,14 @@ int ifa_attention_latent_rows_f32(const void *qa_f32, size_t ldqa, int heads, in
                                   const int *row_seq_dev, size_t rows, void *const *slot_base_dev, size_t cache_off, int max_keys, void *ws_f32,
                                   size_t ws_bytes, void *out_f32, size_t ldo, ifa_stream stream)
 {
+    return ifa_attention_latent_rows_sinks_f32(qa_f32, ldqa, heads, kv_rank, rot_dim, scale, nullptr, seqs_dev, row_seq_dev, rows, slot_base_dev, cache_off, max_keys, ws_f32,
+                                               ws_bytes, out_f32, ldo, stream);
+}
+
+int ifa_attention_latent_rows_sinks_f32(const void *qa_f32, size_t ldqa, int heads, int kv_rank, int rot_dim, float scale, const void *sink_bf16, const void *seqs_dev,
+                                        const int *row_seq_dev, size_t rows, void *const *slot_base_dev, size_t cache_off, int max_keys, void *ws_f32,
+                                        size_t ws_bytes, void *out_f32, size_t ldo, ifa_stream stream)
+{
     IFA_REQUIRE(qa_f32 && seqs_dev && row_seq_dev && slot_base_dev && ws_f32 && out_f32, "ifa_attention_latent_rows_f32: null pointer");
     IFA_REQUIRE(heads > 0 && heads < 65536 * LR_HB && kv_rank > 0 && kv_rank <= 1024 && rot_dim >= 0 && rows > 0 && rows < 65536 && max_keys >= 1
                 && ldqa >= (size_t)heads * (kv_rank + rot_dim) && ldo >= (size_t)heads * kv_rank, "ifa_attention_latent_rows_f32: bad shape");
@@ -555,6 +589,7 @@ int ifa_attention_latent_rows_f32(const void *qa_f32, size_t ldqa, int heads, in
     P.q = (const float *)qa_f32; P.ldq = ldqa; P.heads = heads; P.R = kv_rank; P.dr = rot_dim; P.scale = scale; P.seqs = (const SeqDesc *)seqs_dev;
     P.row_seq = row_seq_dev; P.slot_base = (float *const *)slot_base_dev; P.cache_off = cache_off; P.ws = (float *)ws_f32; P.out = (float *)out_f32; P.ldo = ldo;
     P.vec = ((kv_rank + rot_dim) % 4 == 0 && cache_off % 4 == 0) ? 1 : 0;
+    P.sink = (const bf16_t *)sink_bf16;
     // key shares: 64 keys a share over the longest sequence the cache holds (the same for every step, so that a captured step replays),
     // fewer where many rows already fill the chip or the workspace is small
     int nsplit = std::min(LR_MAX_SPLITS, (max_keys + 63) / 64);
@@ -597,6 +632,15 @@ int ifa_attention_latent_tile_gated_f32(int gate_cols, const void *q_f32, size_t
                                         const void *seqs_dev, const void *seqs_host, int n_seqs, void *const *slot_base_dev, size_t cache_off,
                                         void *out_f32, size_t ldo, ifa_stream stream)
 {
+    return ifa_attention_latent_tile_sinks_f32(gate_cols, q_f32, ldq, heads, dim, rot_dim, vdim, kv_rank, scale, nullptr, kx_f32, ldkx, vx_f32, ldvx, ctx0_dev, g_f32, ldg,
+                                               seqs_dev, seqs_host, n_seqs, slot_base_dev, cache_off, out_f32, ldo, stream);
+}
+
+int ifa_attention_latent_tile_sinks_f32(int gate_cols, const void *q_f32, size_t ldq, int heads, int dim, int rot_dim, int vdim, int kv_rank, float scale,
+                                        const void *sink_bf16, const void *kx_f32, size_t ldkx, const void *vx_f32, size_t ldvx, const int *ctx0_dev, const void *g_f32,
+                                        size_t ldg, const void *seqs_dev, const void *seqs_host, int n_seqs, void *const *slot_base_dev, size_t cache_off, void *out_f32,
+                                        size_t ldo, ifa_stream stream)
+{
     IFA_REQUIRE(q_f32 && kx_f32 && vx_f32 && ctx0_dev && seqs_dev && seqs_host && slot_base_dev && out_f32, "ifa_attention_latent_tile_f32: null pointer");
     IFA_REQUIRE(heads > 0 && heads < 65536 && dim > 0 && rot_dim >= 0 && vdim > 0 && kv_rank > 0 && n_seqs > 0 && ldq >= (size_t)heads * (dim + rot_dim)
                 && ldkx >= (size_t)heads * dim && ldvx >= (size_t)heads * vdim && ldo >= (size_t)heads * vdim && (!g_f32 || ldg >= (size_t)heads * (gate_cols ? vdim : 1)) && (!gate_cols || g_f32),
@@ -606,6 +650,7 @@ int ifa_attention_latent_tile_gated_f32(int gate_cols, const void *q_f32, size_t
     LatTileArgs P;
     P.q = (const float *)q_f32; P.ldq = ldq; P.heads = heads; P.dim = dim; P.dr = rot_dim; P.vdim = vdim; P.R = kv_rank; P.scale = scale;
     P.kx = (const float *)kx_f32; P.ldkx = ldkx; P.vx = (const float *)vx_f32; P.ldvx = ldvx; P.ctx0 = ctx0_dev; P.g = (const float *)g_f32; P.ldg = ldg; P.gate_cols = gate_cols ? 1 : 0;
+    P.sink = (const bf16_t *)sink_bf16;
     P.seqs = (const SeqDesc *)seqs_dev; P.n_seqs = n_seqs; P.slot_base = (float *const *)slot_base_dev; P.cache_off = cache_off; P.out = (float *)out_f32; P.ldo = ldo;
     // 16-byte requests: every source row and every part of a row starts on a 16-byte boundary
     P.vec = (dim % 4 == 0 && rot_dim % 4 == 0 && vdim % 4 == 0 && kv_rank % 4 == 0 && ldq % 4 == 0 && ldkx % 4 == 0 && ldvx % 4 == 0 && cache_off % 4 == 0

@@ -12,6 +12,7 @@
 #include <algorithm>
 #include "ifa_host.h"
 #include "ifa_f32_common.h"
+#include "inferflow_amd.h"
 
 using namespace ifa32;
 
@@ -353,7 +354,7 @@ __global__ void __launch_bounds__(256) k_attn_window_tile(WinAttnArgs P, int n_s
 }
 
 // ---- rotated queries and keys.  One workgroup per row, a wave per head at a time: RMS norm over the head's dim values with a weight
-// (norm_w bf16 [dim], null: none), then the first rot_dims dimensions turn in pairs (i, i + rot_dims / 2) by the angle pos * freq[i]
+// (norm_w bf16 [dim], null: none), then the first rot_dims dimensions turn in pairs (i, i + rot_dims / 2) -- pairing 1: (2i, 2i + 1) -- by the angle pos * freq[i]
 // (formed in double: at position 1000 one fp32 ulp of the angle is already 1e-4); the rest pass unchanged.  Query heads are rewritten in
 // place; key heads go into the K rows of the cache, the value heads (as projected) into its V rows.  k null: the row brings no keys
 // and values of its own (the layer reads another layer's cache rows).
@@ -365,7 +366,7 @@ __global__ void __launch_bounds__(256) k_qk_rope_store(float *__restrict__ q, si
                                                        const bf16_t *__restrict__ q_norm_w, const bf16_t *__restrict__ k_norm_w, float eps, int rot_dims,
                                                        const double *__restrict__ freq, const SeqDesc *__restrict__ seqs, const int *__restrict__ row_seq,
                                                        float *const *__restrict__ slot_base, size_t k_off, size_t v_off, int v_norm,
-                                                       const double *__restrict__ v_freq)
+                                                       const double *__restrict__ v_freq, int pairing, int v_heads)
 {
     extern __shared__ float cs[];          // [rot_dims / 2] cos, [rot_dims / 2] sin; VX: [vdim / 2] cos, [vdim / 2] sin behind them
     const int t = blockIdx.x, tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, nw = blockDim.x >> 6;
@@ -410,7 +411,7 @@ __global__ void __launch_bounds__(256) k_qk_rope_store(float *__restrict__ q, si
             val[e] = oth[e] = 0.0f;
             if (c < dim) {
                 val[e] = src[c] * r * (nw_ ? bf2f(nw_[c]) : 1.0f);
-                if (c < rot_dims) { const int pc = c < half ? c + half : c - half; oth[e] = src[pc] * r * (nw_ ? bf2f(nw_[pc]) : 1.0f); }
+                if (c < rot_dims) { const int pc = pairing ? c ^ 1 : (c < half ? c + half : c - half); oth[e] = src[pc] * r * (nw_ ? bf2f(nw_[pc]) : 1.0f); }
             }
         }
 #pragma unroll
@@ -419,8 +420,9 @@ __global__ void __launch_bounds__(256) k_qk_rope_store(float *__restrict__ q, si
             if (c >= dim) continue;
             float out = val[e];
             if (c < rot_dims) {
-                const int fi = c < half ? c : c - half;
-                out = c < half ? val[e] * cs[fi] - oth[e] * cs[half + fi] : val[e] * cs[fi] + oth[e] * cs[half + fi];
+                const bool first = pairing ? (c & 1) == 0 : c < half;          // first or second member of its pair
+                const int fi = pairing ? c >> 1 : (c < half ? c : c - half);
+                out = first ? val[e] * cs[fi] - oth[e] * cs[half + fi] : val[e] * cs[fi] + oth[e] * cs[half + fi];
             }
             dst[c] = out;
         }
@@ -450,9 +452,9 @@ __global__ void __launch_bounds__(256) k_qk_rope_store(float *__restrict__ q, si
         return;
     }
     if (k) {
-        float *vd = slot_base[sd.slot] + v_off + (size_t)pos * kv_heads * vdim;
+        float *vd = slot_base[sd.slot] + v_off + (size_t)pos * v_heads * vdim;
         const float *vs = v + (size_t)t * ldv;
-        for (int c = tid; c < kv_heads * vdim; c += blockDim.x) vd[c] = vs[c];
+        for (int c = tid; c < v_heads * vdim; c += blockDim.x) vd[c] = vs[c];
     }
 }
 
@@ -575,21 +577,30 @@ int ifa_attention_kv_f32(const void *q_f32, size_t ldq, int heads, int kv_heads,
                             max_keys, ws_f32, ws_bytes, stream);
 }
 
-int ifa_qk_rope_store_f32(void *q_f32, size_t ldq, int heads, const void *k_f32, size_t ldk, const void *v_f32, size_t ldv, int kv_heads, int dim, int vdim,
-                          const void *q_norm_w_bf16, const void *k_norm_w_bf16, float eps, int rot_dims, const double *freq_f64_dev, const void *seqs_dev,
-                          const int *row_seq_dev, size_t rows, void *const *slot_base_dev, size_t k_off, size_t v_off, ifa_stream stream)
+int ifa_qk_rope_store_pairs_f32(int pairing, void *q_f32, size_t ldq, int heads, const void *k_f32, size_t ldk, const void *v_f32, size_t ldv, int k_heads, int v_heads,
+                                int dim, int vdim, const void *q_norm_w_bf16, const void *k_norm_w_bf16, float eps, int rot_dims, const double *freq_f64_dev,
+                                const void *seqs_dev, const int *row_seq_dev, size_t rows, void *const *slot_base_dev, size_t k_off, size_t v_off, ifa_stream stream)
 {
     IFA_REQUIRE(q_f32 && seqs_dev && row_seq_dev && slot_base_dev && (!k_f32 || v_f32), "ifa_qk_rope_store_f32: null pointer");
-    IFA_REQUIRE(heads > 0 && kv_heads > 0 && dim > 0 && dim <= 1024 && vdim > 0 && rows > 0 && rot_dims >= 0 && rot_dims <= dim && rot_dims % 2 == 0
-                && (rot_dims == 0 || freq_f64_dev), "ifa_qk_rope_store_f32: bad shape (head size %d, %d rotated)", dim, rot_dims);
-    IFA_REQUIRE(ldq >= (size_t)heads * dim && (!k_f32 || (ldk >= (size_t)kv_heads * dim && ldv >= (size_t)kv_heads * vdim)), "ifa_qk_rope_store_f32: row strides too small");
+    IFA_REQUIRE(heads > 0 && k_heads > 0 && v_heads > 0 && dim > 0 && dim <= 1024 && vdim > 0 && rows > 0 && rot_dims >= 0 && rot_dims <= dim && rot_dims % 2 == 0
+                && (rot_dims == 0 || freq_f64_dev) && (pairing == 0 || pairing == 1), "ifa_qk_rope_store_f32: bad shape (head size %d, %d rotated)", dim, rot_dims);
+    IFA_REQUIRE(ldq >= (size_t)heads * dim && (!k_f32 || (ldk >= (size_t)k_heads * dim && ldv >= (size_t)v_heads * vdim)), "ifa_qk_rope_store_f32: row strides too small");
 #define IFA_RS(N) hipLaunchKernelGGL((k_qk_rope_store<N, false>), dim3((unsigned)rows), dim3(256), (size_t)std::max(rot_dims, 2) * 4, ifa_s(stream), (float *)q_f32, ldq, heads, \
-                                     (const float *)k_f32, ldk, (const float *)v_f32, ldv, kv_heads, dim, vdim, (const bf16_t *)q_norm_w_bf16, (const bf16_t *)k_norm_w_bf16, eps, \
-                                     rot_dims, freq_f64_dev, (const SeqDesc *)seqs_dev, row_seq_dev, (float *const *)slot_base_dev, k_off, v_off, 0, (const double *)nullptr)
+                                     (const float *)k_f32, ldk, (const float *)v_f32, ldv, k_heads, dim, vdim, (const bf16_t *)q_norm_w_bf16, (const bf16_t *)k_norm_w_bf16, eps, \
+                                     rot_dims, freq_f64_dev, (const SeqDesc *)seqs_dev, row_seq_dev, (float *const *)slot_base_dev, k_off, v_off, 0, (const double *)nullptr, \
+                                     pairing, v_heads)
     if (dim <= 128) IFA_RS(2); else if (dim <= 256) IFA_RS(4); else IFA_RS(16);
 #undef IFA_RS
     IFA_LAUNCH_CHECK();
     return IFA_OK;
+}
+
+int ifa_qk_rope_store_f32(void *q_f32, size_t ldq, int heads, const void *k_f32, size_t ldk, const void *v_f32, size_t ldv, int kv_heads, int dim, int vdim,
+                          const void *q_norm_w_bf16, const void *k_norm_w_bf16, float eps, int rot_dims, const double *freq_f64_dev, const void *seqs_dev,
+                          const int *row_seq_dev, size_t rows, void *const *slot_base_dev, size_t k_off, size_t v_off, ifa_stream stream)
+{
+    return ifa_qk_rope_store_pairs_f32(0, q_f32, ldq, heads, k_f32, ldk, v_f32, ldv, kv_heads, kv_heads, dim, vdim, q_norm_w_bf16, k_norm_w_bf16, eps, rot_dims, freq_f64_dev,
+                                       seqs_dev, row_seq_dev, rows, slot_base_dev, k_off, v_off, stream);
 }
 
 int ifa_qkv_rope_store_f32(void *q_f32, size_t ldq, int heads, const void *k_f32, size_t ldk, const void *v_f32, size_t ldv, int kv_heads, int dim, int vdim,
@@ -604,7 +615,7 @@ int ifa_qkv_rope_store_f32(void *q_f32, size_t ldq, int heads, const void *k_f32
     const size_t smem = ((size_t)std::max(rot_dims, 2) + (size_t)vdim + 2) * 4;
 #define IFA_RS(N) hipLaunchKernelGGL((k_qk_rope_store<N, true>), dim3((unsigned)rows, k_f32 ? 2u : 1u), dim3(256), smem, ifa_s(stream), (float *)q_f32, ldq, heads, \
                                      (const float *)k_f32, ldk, (const float *)v_f32, ldv, kv_heads, dim, vdim, (const bf16_t *)q_norm_w_bf16, (const bf16_t *)k_norm_w_bf16, eps, \
-                                     rot_dims, freq_f64_dev, (const SeqDesc *)seqs_dev, row_seq_dev, (float *const *)slot_base_dev, k_off, v_off, v_norm ? 1 : 0, v_freq_f64_dev)
+                                     rot_dims, freq_f64_dev, (const SeqDesc *)seqs_dev, row_seq_dev, (float *const *)slot_base_dev, k_off, v_off, v_norm ? 1 : 0, v_freq_f64_dev, 0, kv_heads)
     if (dim <= 128) IFA_RS(2); else if (dim <= 256) IFA_RS(4); else IFA_RS(16);
 #undef IFA_RS
     IFA_LAUNCH_CHECK();

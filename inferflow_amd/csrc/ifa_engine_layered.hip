@@ -20,10 +20,12 @@
 // inputs in the slot), put a grouped RMS norm on each sub-layer's OUTPUT (x <- x + norm(sub(x'))), mix with latent attention (cache row
 // [latent | rotated key part] per position; single tokens take the absorbed form, prompts expanded keys / values and the tiled
 // kernel), feed forward through a mixture of experts, and hand the next layer a learned average over the depth of the stack.
-// Layers wired IFA_BLOCK_SANDWICH carry an RMS norm with weight (1 + w) before and after each sub-layer (x <- x + norm1b(mixer(norm1(x))),
+// Layers wired IFA_BLOCK_SANDWICH carry an RMS norm with weight (1 + w) -- or w, norm_plain -- before and after each sub-layer (x <- x + norm1b(mixer(norm1(x))),
 // x <- x + norm2b(ffn(norm2(x)))), mix with softmax attention over rotated queries and keys (IFA_MIX_ROTARY: K rows normed and rotated,
 // V rows of their own size; a layer may read the rows an earlier layer has written instead of projecting keys and values), and feed
-// forward through the clamped gated form or a mixture of gated experts with a router on the logits and a shared, sigmoid-gated expert.
+// forward through the clamped gated form, the squared-relu form without a gate, or a mixture of gated experts with a router on the logits and a shared,
+// sigmoid-gated expert.  The same wiring takes latent attention (with a learned sink per head; a layer may read an earlier layer's cache rows) and
+// differential attention (IFA_MIX_DIFF: two softmax maps per head over the same values, chunked or windowed; K rows [kv_heads][2][dim] turned in pairs).
 // Stem 2 adds a hashed token-pair embedding whose previous token lives in the slot.
 // Layers wired IFA_BLOCK_PRENORM put a Dynamic Tanh norm (tanh(alpha x) w + b) in front of each sub-layer (x <- x + mixer(norm1(x)),
 // x <- x + ffn(norm2(x))), mix with the rotary attention (here with a learned sink per head, a sliding window, scaled frequencies, normed
@@ -71,6 +73,8 @@ struct LLayer {
     // PRENORM: frequencies of the rotated values; generalized delta rule: columns of r | k | v | g | a | bottleneck in the fused product;
     // a layer of a looped group repeats its part of the arena per pass, pass_stride floats apart
     double *freq_v = nullptr;
+    // differential attention: column of the head gates in the fused product, factor of the second map
+    size_t c_ag = 0; float diff_lambda = 0.0f;
     size_t c_cr = 0, c_ck = 0, c_cv = 0, c_cg = 0, c_ca = 0, c_cw = 0, pass_stride = 0;
     // (the state space's projection is one matrix already: z at column 0, x | B | C behind it, then dt)
     LTensor &T(int id) { return t[id - IFA_LT_NORM1]; }
@@ -142,6 +146,7 @@ bool expected_shape(const LayeredNet *n, const ifa_layer_spec &s, int li, int id
     vec = false;
     const bool par = s.mixer == IFA_MIX_WINDOW_LINEAR, del = s.mixer == IFA_MIX_GATED_DELTA, lat = s.mixer == IFA_MIX_LATENT, rot = s.mixer == IFA_MIX_ROTARY;
     const bool post = s.block == IFA_BLOCK_POSTNORM, sand = s.block == IFA_BLOCK_SANDWICH, pre = s.block == IFA_BLOCK_PRENORM, moe = has_moe(s);
+    const bool dif = s.mixer == IFA_MIX_DIFF, relu2 = s.ffn_kind == IFA_FFN_RELU2, own_lat = lat && s.m_kv_layer == 0;
     const bool chan = s.mixer == IFA_MIX_CHAN_DELTA, ssm = s.mixer == IFA_MIX_SSM, strm = s.block == IFA_BLOCK_STREAMS, hc = strm && n->cfg.streams > 0;
     const size_t SI = (size_t)s.s_heads * s.s_vdim, SC = SI + 2 * (size_t)s.s_groups * s.s_state, NS = (size_t)n->cfg.streams;
     const size_t CH = (size_t)s.c_heads * s.c_dim;
@@ -173,7 +178,9 @@ bool expected_shape(const LayeredNet *n, const ifa_layer_spec &s, int li, int id
     case IFA_LT_S_O: r = W; c = SI; return ssm;
     case IFA_LT_NORM1B: r = 1; c = W; vec = true; return sand;
     case IFA_LT_NORM2B: r = 1; c = W; vec = true; return sand && any_ffn;
-    case IFA_LT_A_V: r = (size_t)s.a_kv_heads * s.a_vdim; c = W; return own_kv;
+    case IFA_LT_A_V: r = (size_t)s.a_kv_heads * s.a_vdim; c = W; return own_kv || dif;
+    case IFA_LT_A_G: r = (size_t)s.a_heads; c = W; return dif && s.a_gate;
+    case IFA_LT_A_LQ1: case IFA_LT_A_LK1: case IFA_LT_A_LQ2: case IFA_LT_A_LK2: r = 1; c = (size_t)s.a_dim; vec = true; return dif;
     case IFA_LT_A_Q_B: r = 1; c = (size_t)s.a_heads * s.a_dim; vec = true; return rot;
     case IFA_LT_A_K_B: r = 1; c = (size_t)s.a_kv_heads * s.a_dim; vec = true; return own_kv;
     case IFA_LT_A_V_B: r = 1; c = (size_t)s.a_kv_heads * s.a_vdim; vec = true; return own_kv;
@@ -190,8 +197,9 @@ bool expected_shape(const LayeredNet *n, const ifa_layer_spec &s, int li, int id
     case IFA_LT_M_DQ: r = (size_t)s.m_q_rank; c = W; return lat && s.m_q_rank > 0;
     case IFA_LT_M_DQ_NORM: r = 1; c = (size_t)s.m_q_rank; vec = true; return lat && s.m_q_rank > 0;
     case IFA_LT_M_UQ: r = MQ; c = (size_t)s.m_q_rank; return lat && s.m_q_rank > 0;
-    case IFA_LT_M_DKV: r = MR + (size_t)s.m_rot_dim; c = W; return lat;
-    case IFA_LT_M_DKV_NORM: r = 1; c = MR; vec = true; return lat;
+    case IFA_LT_M_DKV: r = MR + (size_t)s.m_rot_dim; c = W; return own_lat;
+    case IFA_LT_M_DKV_NORM: r = 1; c = MR; vec = true; return own_lat;
+    case IFA_LT_M_SINK: r = 1; c = MH; vec = true; return lat && s.m_sink;
     case IFA_LT_M_UK: r = MH * (size_t)s.m_dim; c = MR; return lat;
     case IFA_LT_M_UV: r = MH * (size_t)s.m_vdim; c = MR; return lat;
     case IFA_LT_M_G: r = s.m_gate == 2 ? MH * (size_t)s.m_vdim : MH; c = W; return lat && s.m_gate;
@@ -201,14 +209,15 @@ bool expected_shape(const LayeredNet *n, const ifa_layer_spec &s, int li, int id
     case IFA_LT_X_UP: r = (size_t)s.x_experts * s.x_ff * (s.x_gated ? 2 : 1); c = W; return moe && s.x_experts > 0;
     case IFA_LT_X_DOWN: r = (size_t)s.x_experts * W; c = (size_t)s.x_ff; return moe && s.x_experts > 0;
     case IFA_LT_LS2: case IFA_LT_FFN_DOWN_B: r = 1; c = W; vec = true; return gated;
-    case IFA_LT_FFN_GATE: case IFA_LT_FFN_UP: r = (size_t)s.ffn; c = W; return s.ffn > 0;
+    case IFA_LT_FFN_GATE: r = (size_t)s.ffn; c = W; return s.ffn > 0 && !relu2;
+    case IFA_LT_FFN_UP: r = (size_t)s.ffn; c = W; return s.ffn > 0;
     case IFA_LT_FFN_GATE_B: case IFA_LT_FFN_UP_B: r = 1; c = (size_t)s.ffn; vec = true; return gated;
     case IFA_LT_FFN_DOWN: r = W; c = (size_t)s.ffn; return s.ffn > 0;
-    case IFA_LT_A_Q: r = (size_t)s.a_heads * s.a_dim; c = W; return par || rot;
-    case IFA_LT_A_K: r = (size_t)s.a_kv_heads * s.a_dim; c = W; return par || own_kv;
+    case IFA_LT_A_Q: r = (size_t)s.a_heads * s.a_dim * (dif ? 2 : 1); c = W; return par || rot || dif;
+    case IFA_LT_A_K: r = (size_t)s.a_kv_heads * s.a_dim * (dif ? 2 : 1); c = W; return par || own_kv || dif;
     case IFA_LT_A_REL: r = (size_t)s.a_buckets; c = (size_t)s.a_heads; return par;
     case IFA_LT_A_SINK: r = 1; c = (size_t)s.a_heads; vec = true; return par || (rot && s.a_sink == 2);
-    case IFA_LT_A_O: r = W; c = (size_t)s.a_heads * (rot ? s.a_vdim : s.a_dim); return par || rot;
+    case IFA_LT_A_O: r = W; c = (size_t)s.a_heads * (rot || dif ? s.a_vdim : s.a_dim); return par || rot || dif;
     case IFA_LT_L_Q: case IFA_LT_L_K: r = (size_t)s.l_heads * s.l_dim; c = W; return par;
     case IFA_LT_L_V: case IFA_LT_L_G: r = (size_t)s.l_heads * s.l_vdim; c = W; return par;
     case IFA_LT_L_O: r = W; c = (size_t)s.l_heads * s.l_vdim; return par;
@@ -286,10 +295,11 @@ int ensure_rows(ifa_model *m, size_t T, size_t nseq)
         const size_t W = (size_t)n->cfg.width;
         const size_t sz[] = {W * streams_of(n), W, n->n_in_max, n->mix_max, n->mix_max, std::max<size_t>(n->ffn_max, 4), std::max<size_t>(n->heads_max, 4), std::max<size_t>(n->heads_max, 4)};
         for (size_t i = 0; i < 8; i++) IFA_HIP_CHECK(hipMalloc((void **)bufs[i], T * sz[i] * 4));
-        {   // the single-row latent attention leaves at least one partial result per (row, head) in the workspace
+        {   // the single-row forms of latent and differential attention leave at least one partial result per (row, head) in the workspace
             size_t need = 0;
             for (const LLayer &L : n->layers)
                 if (L.spec.mixer == IFA_MIX_LATENT) need = std::max(need, T * (size_t)L.spec.m_heads * ((size_t)L.spec.m_kv_rank + 2) * 4);
+                else if (L.spec.mixer == IFA_MIX_DIFF) need = std::max(need, T * (size_t)L.spec.a_heads * 2 * ((size_t)L.spec.a_vdim + 2) * 4);
             if (need > n->attn_ws_bytes) {
                 lay_free(n->attn_ws); n->attn_ws = nullptr;
                 IFA_HIP_CHECK(hipMalloc((void **)&n->attn_ws, need));
@@ -332,6 +342,9 @@ int ensure_logits(ifa_model *m, size_t rows)
     return IFA_OK;
 }
 
+// what the norms of SANDWICH layers and of stem 2 add to their stored weights
+float norm_offset_of(const LayeredNet *n) { return n->cfg.norm_plain ? 0.0f : 1.0f; }
+
 int linear(ifa_model *m, const bf16_t *W, size_t N, size_t K, const float *A, size_t lda, size_t T, const bf16_t *bias, const bf16_t *mul, float alpha,
            int accumulate, float *C, size_t ldc, int silu0 = 0, int silu1 = 0)
 {
@@ -367,7 +380,8 @@ int run_latent_mixer(ifa_model *m, LLayer &L, size_t T, const float *hin, size_t
     LayeredNet *n = m->lay;
     const ifa_layered_config &c = n->cfg;
     const ifa_layer_spec &sp = L.spec;
-    const size_t W = (size_t)c.width, NI = L.n_in, o_c = L.o_c + pass_off;
+    const bool own = sp.m_kv_layer == 0;
+    const size_t W = (size_t)c.width, NI = L.n_in, o_c = (own ? L.o_c : n->layers[(size_t)sp.m_kv_layer - 1].o_c) + pass_off;
     ifa_stream s = (ifa_stream)m->stream;
     void *const *slots = (void *const *)n->slot_base_dev;
     int rc;
@@ -381,8 +395,12 @@ int run_latent_mixer(ifa_model *m, LLayer &L, size_t T, const float *hin, size_t
         if ((rc = linear(m, (const bf16_t *)L.T(IFA_LT_M_UQ).data, QD, QR, n->m3, QR, T, nullptr, nullptr, 1.0f, 0, n->m1, QD))) return rc;
         q = n->m1; ldq = QD;
     }
-    if ((rc = ifa_latent_prepare_pairs_f32(sp.m_rot_halves, n->proj + L.c_mkv, NI, R, dr, sp.m_rot_dims, L.T(IFA_LT_M_DKV_NORM).data, c.eps, q, ldq, H, dn, L.freq, L.rot_mult,
-                                     n->seqs_dev, n->row_seq_dev, T, slots, o_c, s))) return rc;
+    if (own)
+        rc = ifa_latent_prepare_pairs_f32(sp.m_rot_halves, n->proj + L.c_mkv, NI, R, dr, sp.m_rot_dims, L.T(IFA_LT_M_DKV_NORM).data, c.eps, q, ldq, H, dn, L.freq, L.rot_mult,
+                                          n->seqs_dev, n->row_seq_dev, T, slots, o_c, s);
+    else rc = ifa_latent_rotate_q_f32(sp.m_rot_halves, dr, sp.m_rot_dims, q, ldq, H, dn, L.freq, L.rot_mult, n->seqs_dev, n->row_seq_dev, T, s);      // (the cache rows of an earlier layer)
+    if (rc) return rc;
+    const void *sink = sp.m_sink ? L.T(IFA_LT_M_SINK).data : nullptr;
     const float *gate = sp.m_gate ? n->proj + L.c_mg : nullptr;
     if (n->step_expand) {
         // keys and values of every position of the step's sequences from their cached latents, then the tiled kernel
@@ -394,14 +412,14 @@ int run_latent_mixer(ifa_model *m, LLayer &L, size_t T, const float *hin, size_t
             if ((rc = linear(m, (const bf16_t *)L.T(IFA_LT_M_UK).data, ldk, (size_t)R, lat, CR, ctx, nullptr, nullptr, 1.0f, 0, n->kx + r0 * ldk, ldk))) return rc;
             if ((rc = linear(m, (const bf16_t *)L.T(IFA_LT_M_UV).data, ldv, (size_t)R, lat, CR, ctx, nullptr, nullptr, 1.0f, 0, n->vx + r0 * ldv, ldv))) return rc;
         }
-        if ((rc = ifa_attention_latent_tile_gated_f32(sp.m_gate == 2, q, ldq, H, dn, dr, dv, R, sp.m_scale, n->kx, ldk, n->vx, ldv, n->ctx0_dev, gate, NI, n->seqs_dev, n->seqs_host.data(),
+        if ((rc = ifa_attention_latent_tile_sinks_f32(sp.m_gate == 2, q, ldq, H, dn, dr, dv, R, sp.m_scale, sink, n->kx, ldk, n->vx, ldv, n->ctx0_dev, gate, NI, n->seqs_dev, n->seqs_host.data(),
                                                 (int)n->seqs_host.size(), slots, o_c, n->m5, OV, s))) return rc;
     } else {
         // absorbed form: the cache rows are keys (whole) and values (latent part) of ONE head that all query heads share
         const size_t QA = (size_t)H * CR;
         if ((rc = ifa_latent_absorb_q_f32(q, ldq, H, dn, dr, R, L.T(IFA_LT_M_UK).data, T, n->m2, QA, s))) return rc;
-        if ((rc = ifa_attention_latent_rows_f32(n->m2, QA, H, R, dr, sp.m_scale, n->seqs_dev, n->row_seq_dev, T, slots, o_c, c.max_ctx, n->attn_ws, n->attn_ws_bytes,
-                                                n->m4, (size_t)H * R, s))) return rc;
+        if ((rc = ifa_attention_latent_rows_sinks_f32(n->m2, QA, H, R, dr, sp.m_scale, sink, n->seqs_dev, n->row_seq_dev, T, slots, o_c, c.max_ctx, n->attn_ws, n->attn_ws_bytes,
+                                                      n->m4, (size_t)H * R, s))) return rc;
         if ((rc = ifa_latent_expand_out_gated_f32(sp.m_gate == 2, n->m4, (size_t)H * R, R, H, dv, R, L.T(IFA_LT_M_UV).data, gate, NI, T, n->m5, OV, s))) return rc;
     }
     if ((rc = linear(m, (const bf16_t *)L.T(IFA_LT_M_O).data, W, OV, n->m5, OV, T, nullptr, nullptr, 1.0f, 0, out, W))) return rc;
@@ -453,8 +471,28 @@ int run_postnorm_layer(ifa_model *m, LLayer &L, size_t li, size_t T, int nseq, b
     return post_step(m, T, nseq, fused, n->m1, L.T(IFA_LT_NORM2).data, depth_of, li, ncw, ntaps, noff);
 }
 
-// one SANDWICH layer over T rows: x <- x + norm1b(attention(norm1(x))); x <- x + norm2b(ffn(norm2(x))), every norm an RMS norm with
-// weight (1 + w).  The keys enter the cache normed and rotated; a layer with a_kv_layer reads the rows that layer has written in this step.
+// differential attention over T rows of h -> out (the output product)
+int run_diff_mixer(ifa_model *m, LLayer &L, size_t T, const float *h, float *out)
+{
+    LayeredNet *n = m->lay;
+    const ifa_layered_config &c = n->cfg;
+    const ifa_layer_spec &sp = L.spec;
+    const int H = sp.a_heads, G = sp.a_kv_heads, D = sp.a_dim, DV = sp.a_vdim;
+    const size_t W = (size_t)c.width, NI = L.n_in, OV = (size_t)H * DV;
+    ifa_stream s = (ifa_stream)m->stream;
+    void *const *slots = (void *const *)n->slot_base_dev;
+    int rc;
+    if ((rc = linear(m, L.w_in, NI, W, h, W, T, nullptr, nullptr, 1.0f, 0, n->proj, NI))) return rc;
+    if ((rc = ifa_qk_rope_store_pairs_f32(sp.a_rot_pairs, n->proj + L.c_aq, NI, 2 * H, n->proj + L.c_ak, NI, n->proj + L.c_av, NI, 2 * G, G, D, DV, nullptr, nullptr, c.eps, sp.a_rot_dims,
+                                          L.freq, n->seqs_dev, n->row_seq_dev, T, slots, L.o_k, L.o_v, s))) return rc;
+    if ((rc = ifa_attention_diff_f32(n->proj + L.c_aq, NI, H, G, D, DV, sp.a_scale, sp.a_window, sp.a_chunk, L.diff_lambda, 1.0f - sp.a_diff, c.eps,
+                                     sp.a_gate ? n->proj + L.c_ag : nullptr, NI, n->seqs_dev, n->row_seq_dev, T, slots, L.o_k, L.o_v, n->m1, OV, n->seqs_host.data(),
+                                     (int)n->seqs_host.size(), n->opt_attn_tile_min, c.max_ctx, n->attn_ws, n->attn_ws_bytes, s))) return rc;
+    return linear(m, (const bf16_t *)L.T(IFA_LT_A_O).data, W, OV, n->m1, OV, T, nullptr, nullptr, 1.0f, 0, out, W);
+}
+
+// one SANDWICH layer over T rows: x <- x + norm1b(mixer(norm1(x))); x <- x + norm2b(ffn(norm2(x))), every norm an RMS norm with
+// weight (1 + w), or w (norm_plain).  Rotary attention: the keys enter the cache normed and rotated; a layer with a_kv_layer reads the rows that layer has written in this step.
 // The norm behind a sub-layer and the norm in front of the next one run as ONE launch (option fuse_post): h_ready says that the layer
 // before has left norm1(x) in n->h, *next_h_ready that this layer has done so for `next`.
 int run_sandwich_layer(ifa_model *m, LLayer &L, size_t T, int nseq, bool h_ready, const LLayer *next, bool *next_h_ready)
@@ -466,22 +504,25 @@ int run_sandwich_layer(ifa_model *m, LLayer &L, size_t T, int nseq, bool h_ready
     ifa_stream s = (ifa_stream)m->stream;
     void *const *slots = (void *const *)n->slot_base_dev;
     const bool fused = n->opt_fuse_post != 0, moe = has_moe(sp), any_ffn = sp.ffn > 0 || moe;
+    const float w_off = norm_offset_of(n);
     const void *next_norm = fused && next && next->spec.block == IFA_BLOCK_SANDWICH ? next->T(IFA_LT_NORM1).data : nullptr;
     *next_h_ready = next_norm != nullptr;
     // x += norm_after(sub); h = norm_before(x) for whatever comes next
     auto close_sub = [&](const float *sub, const void *w_after, const void *w_before) -> int {
-        if (fused) return ifa_norm_add_norm_f32(n->x, W, T, W, sub, W, w_after, w_before, 1.0f, c.eps, n->h, W, s);
-        int r = ifa_rmsnorm_offset_f32(sub, W, T, W, w_after, 1.0f, c.eps, 1, n->x, W, s);
-        if (!r && w_before) r = ifa_rmsnorm_offset_f32(n->x, W, T, W, w_before, 1.0f, c.eps, 0, n->h, W, s);
+        if (fused) return ifa_norm_add_norm_f32(n->x, W, T, W, sub, W, w_after, w_before, w_off, c.eps, n->h, W, s);
+        int r = ifa_rmsnorm_offset_f32(sub, W, T, W, w_after, w_off, c.eps, 1, n->x, W, s);
+        if (!r && w_before) r = ifa_rmsnorm_offset_f32(n->x, W, T, W, w_before, w_off, c.eps, 0, n->h, W, s);
         return r;
     };
     int rc;
-    {
+    if (!h_ready && (rc = ifa_rmsnorm_offset_f32(n->x, W, T, W, L.T(IFA_LT_NORM1).data, w_off, c.eps, 0, n->h, W, s))) return rc;
+    if (sp.mixer == IFA_MIX_LATENT) { if ((rc = run_latent_mixer(m, L, T, n->h, 0, n->m2))) return rc; }
+    else if (sp.mixer == IFA_MIX_DIFF) { if ((rc = run_diff_mixer(m, L, T, n->h, n->m2))) return rc; }
+    else {
         const int H = sp.a_heads, G = sp.a_kv_heads, D = sp.a_dim, DV = sp.a_vdim;
         const size_t OV = (size_t)H * DV;
         const bool own = sp.a_kv_layer == 0;
         const LLayer &KV = own ? L : n->layers[(size_t)sp.a_kv_layer - 1];
-        if (!h_ready && (rc = ifa_rmsnorm_offset_f32(n->x, W, T, W, L.T(IFA_LT_NORM1).data, 1.0f, c.eps, 0, n->h, W, s))) return rc;
         if ((rc = linear(m, L.w_in, NI, W, n->h, W, T, L.b_in, nullptr, 1.0f, 0, n->proj, NI))) return rc;
         if ((rc = ifa_qk_rope_store_f32(n->proj + L.c_aq, NI, H, own ? n->proj + L.c_ak : nullptr, NI, own ? n->proj + L.c_av : nullptr, NI, G, D, DV,
                                         L.T(IFA_LT_A_Q_NORM).data, own ? L.T(IFA_LT_A_K_NORM).data : nullptr, c.eps, sp.a_rot_dims, L.freq, n->seqs_dev, n->row_seq_dev, T,
@@ -490,10 +531,15 @@ int run_sandwich_layer(ifa_model *m, LLayer &L, size_t T, int nseq, bool h_ready
                                        n->row_seq_dev, T, slots, KV.o_k, KV.o_v, n->m1, OV, n->seqs_host.data(), (int)n->seqs_host.size(), n->opt_attn_tile_min,
                                        c.max_ctx, n->attn_ws, n->attn_ws_bytes, s))) return rc;
         if ((rc = linear(m, (const bf16_t *)L.T(IFA_LT_A_O).data, W, OV, n->m1, OV, T, nullptr, nullptr, 1.0f, 0, n->m2, W))) return rc;
-        if ((rc = close_sub(n->m2, L.T(IFA_LT_NORM1B).data, any_ffn ? L.T(IFA_LT_NORM2).data : next_norm))) return rc;
     }
+    if ((rc = close_sub(n->m2, L.T(IFA_LT_NORM1B).data, any_ffn ? L.T(IFA_LT_NORM2).data : next_norm))) return rc;
     if (!any_ffn) return IFA_OK;
     const size_t N2 = L.n_in2;
+    if (sp.ffn_kind == IFA_FFN_RELU2) {      // the square of relu in the epilogue of the up-projection
+        if ((rc = ifa_linear_bf16w_act(L.w_in2, N2, W, n->h, W, T, nullptr, 2, c.ops32, n->proj, N2, s))) return rc;
+        if ((rc = linear(m, (const bf16_t *)L.T(IFA_LT_FFN_DOWN).data, W, (size_t)sp.ffn, n->proj, N2, T, nullptr, nullptr, 1.0f, 0, n->m2, W))) return rc;
+        return close_sub(n->m2, L.T(IFA_LT_NORM2B).data, next_norm);
+    }
     if ((rc = linear(m, L.w_in2, N2, W, n->h, W, T, L.b_in2, nullptr, 1.0f, 0, n->proj, N2))) return rc;
     if (!moe) {
         const size_t F = (size_t)sp.ffn;
@@ -695,8 +741,9 @@ int run_layers(ifa_model *m, size_t T, int nseq)
         if ((rc = ifa_group_rmsnorm_f32(n->h, W, T, W, c.norm_groups, n->embd_norm.data, c.eps, 0, n->x, W, s))) return rc;
         if (n->any_depth_avg && (rc = ifa_group_rmsnorm_f32(n->h, W, T, W, c.norm_groups, n->embd_norm.data, c.eps, 0, n->stack, W, s))) return rc;      // plane 0
     } else if (c.stem == 2) {
-        if ((rc = ifa_embed_pair_f32(n->embd.data, c.vocab, c.width, c.bigram_buckets > 0 ? n->bigram.data : nullptr, c.bigram_buckets, c.bigram_mul_prev, c.bigram_mul_cur,
-                                     n->tokens_dev, n->seqs_dev, n->row_seq_dev, T, slots, n->o_prev, n->x, s))) return rc;
+        if ((rc = ifa_embed_pair_scaled_f32(n->embd.data, c.vocab, c.width, c.embed_scale != 0.0f ? c.embed_scale : 1.0f, c.bigram_buckets > 0 ? n->bigram.data : nullptr,
+                                            c.bigram_buckets, c.bigram_mul_prev, c.bigram_mul_cur, n->tokens_dev, n->seqs_dev, n->row_seq_dev, T, slots, n->o_prev, n->x,
+                                            nullptr, s))) return rc;
     } else if (c.stem == 3) {
         if ((rc = ifa_embed_pair_scaled_f32(n->embd.data, c.vocab, c.width, c.embed_scale != 0.0f ? c.embed_scale : 1.0f, c.bigram_buckets > 0 ? n->bigram.data : nullptr,
                                             c.bigram_buckets, c.bigram_mul_prev, c.bigram_mul_cur, n->tokens_dev, n->seqs_dev, n->row_seq_dev, T, slots, n->o_prev, n->x,
@@ -804,13 +851,13 @@ int run_layers(ifa_model *m, size_t T, int nseq)
 
 float logit_scale_of(const LayeredNet *n) { return n->cfg.stem == 3 && n->cfg.logit_scale != 0.0f ? n->cfg.logit_scale : 1.0f; }
 
-// the norm in front of lm_head: (stem 3) the Dynamic Tanh norm, layer norm without bias, (stem 1) the grouped RMS norm, or (stem 2) the RMS norm with weight (1 + w)
+// the norm in front of lm_head: (stem 3) the Dynamic Tanh norm, layer norm without bias, (stem 1) the grouped RMS norm, or (stem 2) the RMS norm with weight (1 + w) or w
 int out_norm_rows(ifa_model *m, const float *src, size_t rows, float *dst)
 {
     LayeredNet *n = m->lay;
     const size_t W = (size_t)n->cfg.width;
     if (n->cfg.stem == 1) return ifa_group_rmsnorm_f32(src, W, rows, W, n->cfg.norm_groups, n->out_norm.data, n->cfg.eps, 0, dst, W, (ifa_stream)m->stream);
-    if (n->cfg.stem == 2) return ifa_rmsnorm_offset_f32(src, W, rows, W, n->out_norm.data, 1.0f, n->cfg.eps, 0, dst, W, (ifa_stream)m->stream);
+    if (n->cfg.stem == 2) return ifa_rmsnorm_offset_f32(src, W, rows, W, n->out_norm.data, norm_offset_of(n), n->cfg.eps, 0, dst, W, (ifa_stream)m->stream);
     if (n->cfg.stem == 4)      // (the sum of a row's streams)
         return ifa_streams_step_f32((void *)src, rows, (int)streams_of(n), W, nullptr, nullptr, 0, 1.0f, nullptr, 0, nullptr, nullptr, 1.0f, nullptr, n->out_norm.data, n->cfg.eps, dst,
                                     W, nullptr, 0, (ifa_stream)m->stream);
@@ -910,7 +957,7 @@ int lay_finalize(ifa_model *m)
         int rc;
         if (sp.mixer == IFA_MIX_LATENT) {
             if ((rc = cat_rows(w, b, L.T(sp.m_q_rank > 0 ? IFA_LT_M_DQ : IFA_LT_M_Q), nullptr, W, L.c_mq, m->stream))
-                || (rc = cat_rows(w, b, L.T(IFA_LT_M_DKV), nullptr, W, L.c_mkv, m->stream))
+                || (sp.m_kv_layer == 0 && (rc = cat_rows(w, b, L.T(IFA_LT_M_DKV), nullptr, W, L.c_mkv, m->stream)))
                 || (sp.m_gate && (rc = cat_rows(w, b, L.T(IFA_LT_M_G), nullptr, W, L.c_mg, m->stream)))) return rc;
             // rotation frequencies in double: base^(-2i / dims), YaRN: the scaled and the plain frequency blended by a ramp over i
             const int half = sp.m_rot_dims / 2;
@@ -931,7 +978,7 @@ int lay_finalize(ifa_model *m)
             IFA_HIP_CHECK(hipMalloc((void **)&L.freq, fr.size() * 8));
             IFA_HIP_CHECK(hipMemcpy(L.freq, fr.data(), fr.size() * 8, hipMemcpyHostToDevice));
             const size_t CR = (size_t)(sp.m_kv_rank + sp.m_rot_dim), H = (size_t)sp.m_heads;
-            L.o_c = off; off += align4((size_t)n->cfg.max_ctx * CR);
+            if (sp.m_kv_layer == 0) { L.o_c = off; off += align4((size_t)n->cfg.max_ctx * CR); }
             if (sp.canon_taps > 1) { L.o_cv1 = off; off += align4((size_t)(sp.canon_taps - 1) * W); }
             n->mix_max = std::max({n->mix_max, H * (size_t)(sp.m_dim + sp.m_rot_dim), H * CR, H * (size_t)sp.m_vdim, W, (size_t)sp.m_q_rank});
             n->ffn_max = std::max(n->ffn_max, (size_t)sp.m_q_rank);
@@ -981,40 +1028,33 @@ int lay_finalize(ifa_model *m)
                 L.o_v = off; off += align4((size_t)n->cfg.max_ctx * sp.a_kv_heads * sp.a_vdim);
             }
             n->mix_max = std::max({n->mix_max, (size_t)sp.a_heads * sp.a_dim, (size_t)sp.a_heads * sp.a_vdim, W});
-            // the second product and the sizes of the feed-forward's buffers
-            std::vector<bf16_t> w2, b2;
-            size_t dummy;
-            if (sp.block == IFA_BLOCK_PRENORM) {      // (the router stays a product of its own: its choice takes it in for steps of a few rows)
-                if (has_moe(sp)) {
-                    n->mix_max = std::max(n->mix_max, (size_t)sp.x_experts);
-                    n->top_max = std::max(n->top_max, (size_t)sp.x_top);
-                    n->any_moe = true;
-                }
-            } else
-            if (has_moe(sp)) {
-                if ((rc = cat_rows(w2, b2, L.T(IFA_LT_X_ROUTER), sp.x_route == 1 ? &L.T(IFA_LT_X_ROUTER_B) : nullptr, W, L.c2_router, m->stream))) return rc;
-                if (sp.x_shared_ff > 0) {
-                    LTensor sg = L.T(IFA_LT_X_SH_SG); sg.rows = 1; sg.cols = W;
-                    if ((rc = cat_rows(w2, b2, sg, nullptr, W, L.c2_sg, m->stream))) return rc;
-                    while (b2.size() % 4) { w2.resize(w2.size() + W, 0); b2.push_back(0); }
-                    if ((rc = cat_rows(w2, b2, L.T(IFA_LT_X_SH_GATE), nullptr, W, L.c2_shg, m->stream)) || (rc = cat_rows(w2, b2, L.T(IFA_LT_X_SH_UP), nullptr, W, dummy, m->stream))) return rc;
-                    n->ffn_max = std::max(n->ffn_max, (size_t)sp.x_shared_ff);
-                }
+            if (sp.block == IFA_BLOCK_PRENORM && has_moe(sp)) {      // (the router stays a product of its own: its choice takes it in for steps of a few rows)
+                n->mix_max = std::max(n->mix_max, (size_t)sp.x_experts);
                 n->top_max = std::max(n->top_max, (size_t)sp.x_top);
                 n->any_moe = true;
-            } else if (sp.ffn > 0) {
-                if ((rc = cat_rows(w2, b2, L.T(IFA_LT_FFN_GATE), nullptr, W, L.c2_fg, m->stream)) || (rc = cat_rows(w2, b2, L.T(IFA_LT_FFN_UP), nullptr, W, dummy, m->stream))) return rc;
-                n->ffn_max = std::max(n->ffn_max, (size_t)sp.ffn);
             }
-            if (!b2.empty()) {
-                while (b2.size() % 4) { w2.resize(w2.size() + W, 0); b2.push_back(0); }
-                L.n_in2 = b2.size();
-                IFA_HIP_CHECK(hipMalloc((void **)&L.w_in2, w2.size() * 2));
-                IFA_HIP_CHECK(hipMalloc((void **)&L.b_in2, b2.size() * 2));
-                IFA_HIP_CHECK(hipMemcpy(L.w_in2, w2.data(), w2.size() * 2, hipMemcpyHostToDevice));
-                IFA_HIP_CHECK(hipMemcpy(L.b_in2, b2.data(), b2.size() * 2, hipMemcpyHostToDevice));
-                n->n_in_max = std::max(n->n_in_max, L.n_in2);
+        } else if (sp.mixer == IFA_MIX_DIFF) {
+            for (const auto &part : {std::make_pair((int)IFA_LT_A_Q, &L.c_aq), std::make_pair((int)IFA_LT_A_K, &L.c_ak), std::make_pair((int)IFA_LT_A_V, &L.c_av)}) {
+                if ((rc = cat_rows(w, b, L.T(part.first), nullptr, W, *part.second, m->stream))) return rc;
+                while (b.size() % 4) { w.resize(w.size() + W, 0); b.push_back(0); }      // (each part starts on a 16-byte border of the product's rows)
             }
+            if (sp.a_gate && (rc = cat_rows(w, b, L.T(IFA_LT_A_G), nullptr, W, L.c_ag, m->stream))) return rc;
+            const int half = sp.a_rot_dims / 2;
+            std::vector<double> fr((size_t)std::max(half, 1), 0.0);
+            for (int i = 0; i < half; i++) fr[(size_t)i] = std::pow((double)sp.a_rot_base, -2.0 * i / (double)sp.a_rot_dims);
+            IFA_HIP_CHECK(hipMalloc((void **)&L.freq, fr.size() * 8));
+            IFA_HIP_CHECK(hipMemcpy(L.freq, fr.data(), fr.size() * 8, hipMemcpyHostToDevice));
+            double dot[2] = {0.0, 0.0};      // the factor of the second map: one number for the layer
+            for (int k = 0; k < 2; k++) {
+                std::vector<bf16_t> lq((size_t)sp.a_dim), lk((size_t)sp.a_dim);
+                IFA_HIP_CHECK(hipMemcpy(lq.data(), L.T(k ? IFA_LT_A_LQ2 : IFA_LT_A_LQ1).data, lq.size() * 2, hipMemcpyDeviceToHost));
+                IFA_HIP_CHECK(hipMemcpy(lk.data(), L.T(k ? IFA_LT_A_LK2 : IFA_LT_A_LK1).data, lk.size() * 2, hipMemcpyDeviceToHost));
+                for (size_t e = 0; e < lq.size(); e++) dot[k] += (double)ifa32::bf2f(lq[e]) * (double)ifa32::bf2f(lk[e]);
+            }
+            L.diff_lambda = (float)(std::exp(dot[0]) - std::exp(dot[1]) + (double)sp.a_diff);
+            L.o_k = off; off += align4((size_t)n->cfg.max_ctx * sp.a_kv_heads * 2 * sp.a_dim);
+            L.o_v = off; off += align4((size_t)n->cfg.max_ctx * sp.a_kv_heads * sp.a_vdim);
+            n->mix_max = std::max({n->mix_max, (size_t)sp.a_heads * sp.a_vdim, W});
         } else if (sp.mixer == IFA_MIX_CHAN_DELTA) {
             if ((rc = cat_rows(w, b, L.T(IFA_LT_C_R), nullptr, W, L.c_cr, m->stream)) || (rc = cat_rows(w, b, L.T(IFA_LT_C_K), nullptr, W, L.c_ck, m->stream))
                 || (rc = cat_rows(w, b, L.T(IFA_LT_C_V), nullptr, W, L.c_cv, m->stream)) || (rc = cat_rows(w, b, L.T(IFA_LT_C_G), nullptr, W, L.c_cg, m->stream))
@@ -1068,6 +1108,37 @@ int lay_finalize(ifa_model *m)
             n->mix_max = std::max({n->mix_max, (size_t)L.conv_ch, DV});
             n->heads_max = std::max(n->heads_max, (size_t)sp.d_heads);
         }
+        if (sp.block == IFA_BLOCK_SANDWICH) {      // the second product (what reads norm2) and the sizes of the feed-forward's buffers
+            std::vector<bf16_t> w2, b2;
+            size_t dummy;
+            n->mix_max = std::max(n->mix_max, W);
+            if (has_moe(sp)) {
+                if ((rc = cat_rows(w2, b2, L.T(IFA_LT_X_ROUTER), sp.x_route == 1 ? &L.T(IFA_LT_X_ROUTER_B) : nullptr, W, L.c2_router, m->stream))) return rc;
+                if (sp.x_shared_ff > 0) {
+                    LTensor sg = L.T(IFA_LT_X_SH_SG); sg.rows = 1; sg.cols = W;
+                    if ((rc = cat_rows(w2, b2, sg, nullptr, W, L.c2_sg, m->stream))) return rc;
+                    while (b2.size() % 4) { w2.resize(w2.size() + W, 0); b2.push_back(0); }
+                    if ((rc = cat_rows(w2, b2, L.T(IFA_LT_X_SH_GATE), nullptr, W, L.c2_shg, m->stream)) || (rc = cat_rows(w2, b2, L.T(IFA_LT_X_SH_UP), nullptr, W, dummy, m->stream))) return rc;
+                    n->ffn_max = std::max(n->ffn_max, (size_t)sp.x_shared_ff);
+                }
+                n->top_max = std::max(n->top_max, (size_t)sp.x_top);
+                n->any_moe = true;
+            } else if (sp.ffn > 0 && sp.ffn_kind == IFA_FFN_RELU2) {
+                if ((rc = cat_rows(w2, b2, L.T(IFA_LT_FFN_UP), nullptr, W, L.c2_fg, m->stream))) return rc;
+            } else if (sp.ffn > 0) {
+                if ((rc = cat_rows(w2, b2, L.T(IFA_LT_FFN_GATE), nullptr, W, L.c2_fg, m->stream)) || (rc = cat_rows(w2, b2, L.T(IFA_LT_FFN_UP), nullptr, W, dummy, m->stream))) return rc;
+                n->ffn_max = std::max(n->ffn_max, (size_t)sp.ffn);
+            }
+            if (!b2.empty()) {
+                while (b2.size() % 4) { w2.resize(w2.size() + W, 0); b2.push_back(0); }
+                L.n_in2 = b2.size();
+                IFA_HIP_CHECK(hipMalloc((void **)&L.w_in2, w2.size() * 2));
+                IFA_HIP_CHECK(hipMalloc((void **)&L.b_in2, b2.size() * 2));
+                IFA_HIP_CHECK(hipMemcpy(L.w_in2, w2.data(), w2.size() * 2, hipMemcpyHostToDevice));
+                IFA_HIP_CHECK(hipMemcpy(L.b_in2, b2.data(), b2.size() * 2, hipMemcpyHostToDevice));
+                n->n_in_max = std::max(n->n_in_max, L.n_in2);
+            }
+        }
         if (sp.block == IFA_BLOCK_STREAMS) {      // buffers of the feed-forward; dense: gate | up as one product of what norm2 leaves
             n->ffn_max = std::max(n->ffn_max, W);          // (m3 takes the mixer's output)
             n->mix_max = std::max(n->mix_max, W);
@@ -1110,7 +1181,7 @@ int lay_finalize(ifa_model *m)
         for (int id : {IFA_LT_A_Q, IFA_LT_A_K, IFA_LT_L_Q, IFA_LT_L_K, IFA_LT_L_V, IFA_LT_L_G, IFA_LT_D_Q, IFA_LT_D_K, IFA_LT_D_V, IFA_LT_D_B, IFA_LT_D_A,
                        IFA_LT_D_G, IFA_LT_FFN_GATE, IFA_LT_FFN_UP, IFA_LT_M_Q, IFA_LT_M_DQ, IFA_LT_M_DKV, IFA_LT_M_G, IFA_LT_A_V, IFA_LT_A_Q_B, IFA_LT_A_K_B,
                        IFA_LT_A_V_B, IFA_LT_X_ROUTER_B, IFA_LT_X_SH_GATE, IFA_LT_X_SH_UP, IFA_LT_X_SH_SG, IFA_LT_C_R, IFA_LT_C_K, IFA_LT_C_V, IFA_LT_C_G, IFA_LT_C_A,
-                       IFA_LT_C_A_B, IFA_LT_C_W1, IFA_LT_S_IN}) {
+                       IFA_LT_C_A_B, IFA_LT_C_W1, IFA_LT_S_IN, IFA_LT_A_G}) {
             LTensor &t = L.T(id);
             if (t.data) { lay_free(t.data); t.data = nullptr; }
         }
@@ -1121,6 +1192,7 @@ int lay_finalize(ifa_model *m)
         for (const LLayer &L : n->layers)
             if (L.spec.mixer == IFA_MIX_WINDOW_LINEAR) per_row = std::max(per_row, (size_t)L.spec.a_heads * 32 * ((size_t)L.spec.a_dim + 2) * 4);
             else if (L.spec.mixer == IFA_MIX_ROTARY) per_row = std::max(per_row, (size_t)L.spec.a_heads * 32 * ((size_t)L.spec.a_vdim + 2) * 4);
+            else if (L.spec.mixer == IFA_MIX_DIFF) per_row = std::max(per_row, (size_t)L.spec.a_heads * 16 * 2 * ((size_t)L.spec.a_vdim + 2) * 4);
             else if (L.spec.mixer == IFA_MIX_LATENT) per_row = std::max(per_row, (size_t)L.spec.m_heads * 16 * ((size_t)L.spec.m_kv_rank + 2) * 4);
         n->attn_ws_bytes = per_row * 64;
         if (n->attn_ws_bytes) IFA_HIP_CHECK(hipMalloc((void **)&n->attn_ws, n->attn_ws_bytes));
@@ -1436,6 +1508,19 @@ int ifa_model_create_layered(const ifa_layered_config *cfg, const ifa_layer_spec
                         "ifa_model_create_layered: layer %d: bad latent-attention sizes", l);
             IFA_REQUIRE(s.m_yarn_factor == 0.0f || (s.m_yarn_factor > 0.0f && s.m_yarn_original > 0.0f && s.m_yarn_fast > 0.0f && s.m_yarn_slow > 0.0f),
                         "ifa_model_create_layered: layer %d: bad frequency scaling", l);
+            if (s.m_kv_layer != 0) {
+                IFA_REQUIRE(s.m_kv_layer >= 1 && s.m_kv_layer <= l, "ifa_model_create_layered: layer %d reads the latent of layer %d, which is not an earlier layer", l, s.m_kv_layer - 1);
+                const ifa_layer_spec &o = layers[s.m_kv_layer - 1];
+                IFA_REQUIRE(o.mixer == IFA_MIX_LATENT && o.m_kv_layer == 0 && o.m_kv_rank == s.m_kv_rank && o.m_rot_dim == s.m_rot_dim && o.m_rot_dims == s.m_rot_dims
+                            && o.m_rot_base == s.m_rot_base && o.m_rot_halves == s.m_rot_halves && o.m_yarn_factor == s.m_yarn_factor && o.m_yarn_original == s.m_yarn_original
+                            && o.m_yarn_fast == s.m_yarn_fast && o.m_yarn_slow == s.m_yarn_slow && s.block == IFA_BLOCK_SANDWICH,
+                            "ifa_model_create_layered: layer %d: layer %d has no latent of its own in this layer's shape", l, s.m_kv_layer - 1);
+            }
+        } else if (s.mixer == IFA_MIX_DIFF) {
+            IFA_REQUIRE(s.a_heads > 0 && s.a_kv_heads > 0 && s.a_heads % s.a_kv_heads == 0 && s.a_dim > 0 && s.a_dim <= 1024 && s.a_vdim > 0 && s.a_vdim <= 1024
+                        && s.a_window >= 0 && s.a_chunk >= 0 && s.a_kv_layer == 0 && s.a_rot_dims >= 0 && s.a_rot_dims <= s.a_dim && s.a_rot_dims % 2 == 0
+                        && (s.a_rot_dims == 0 || s.a_rot_base > 0.0f) && (s.a_rot_pairs == 0 || s.a_rot_pairs == 1),
+                        "ifa_model_create_layered: layer %d: bad sizes of the differential attention", l);
         } else if (s.mixer == IFA_MIX_ROTARY) {
             IFA_REQUIRE(s.a_heads > 0 && s.a_kv_heads > 0 && s.a_heads % s.a_kv_heads == 0 && s.a_dim > 0 && s.a_dim <= 1024 && s.a_vdim > 0 && s.a_vdim <= 1024
                         && s.a_window >= 0 && s.a_keep_first >= 0 && s.a_rot_dims >= 0 && s.a_rot_dims <= s.a_dim && s.a_rot_dims % 2 == 0
@@ -1457,7 +1542,8 @@ int ifa_model_create_layered(const ifa_layered_config *cfg, const ifa_layer_spec
                         && s.s_norm_groups > 0 && ((size_t)s.s_heads * s.s_vdim) % (size_t)s.s_norm_groups == 0,
                         "ifa_model_create_layered: layer %d: bad state-space sizes", l);
         } else return ifa_fail(IFA_ERR_ARG, "ifa_model_create_layered: layer %d: unknown mixer %d", l, s.mixer);
-        const bool wired = s.mixer == IFA_MIX_LATENT ? (s.block == IFA_BLOCK_POSTNORM || s.block == IFA_BLOCK_STREAMS)
+        const bool wired = s.mixer == IFA_MIX_LATENT ? (s.block == IFA_BLOCK_POSTNORM || s.block == IFA_BLOCK_STREAMS || s.block == IFA_BLOCK_SANDWICH)
+                           : s.mixer == IFA_MIX_DIFF ? s.block == IFA_BLOCK_SANDWICH
                            : s.mixer == IFA_MIX_SSM ? s.block == IFA_BLOCK_STREAMS
                            : s.mixer == IFA_MIX_ROTARY ? (s.block == IFA_BLOCK_SANDWICH || s.block == IFA_BLOCK_PRENORM)
                            : s.mixer == IFA_MIX_CHAN_DELTA ? s.block == IFA_BLOCK_PRENORM : s.block == IFA_BLOCK_PARALLEL;
@@ -1481,7 +1567,8 @@ int ifa_model_create_layered(const ifa_layered_config *cfg, const ifa_layer_spec
             if (s.ffn_kind == IFA_FFN_MOE && s.x_experts + s.x_identity > 0)
                 IFA_REQUIRE(s.ffn == 0 && s.x_identity == 0 && s.x_gated == 1 && s.x_route == 1 && s.x_experts >= 1 && s.x_experts <= 4096 && s.x_top >= 1 && s.x_top <= s.x_experts
                             && s.x_ff > 0 && s.x_shared_ff >= 0, "ifa_model_create_layered: layer %d: bad mixture-of-experts sizes", l);
-            else IFA_REQUIRE(s.ffn == 0 || (s.ffn_kind == IFA_FFN_CLAMPED && s.f_limit > 0.0f), "ifa_model_create_layered: layer %d: this wiring takes the clamped feed-forward or a mixture", l);
+            else IFA_REQUIRE(s.ffn == 0 || (s.ffn_kind == IFA_FFN_CLAMPED && s.f_limit > 0.0f) || s.ffn_kind == IFA_FFN_RELU2,
+                             "ifa_model_create_layered: layer %d: this wiring takes the clamped or the squared-relu feed-forward or a mixture", l);
         } else
         if (s.block == IFA_BLOCK_POSTNORM) {
             IFA_REQUIRE(s.ffn == 0 && s.canon_taps >= 0 && s.canon_taps <= 64 && cfg->norm_groups >= 1 && cfg->width % cfg->norm_groups == 0,

@@ -85,6 +85,16 @@ __device__ __forceinline__ float gelu_tanh_f(float z)
 }
 __device__ __forceinline__ float softplus_f(float z) { return z > 20.0f ? z : log1pf(expf(z)); }
 
+// First key position that the query at position i sees: a sliding window (window <= 0: none) and / or chunks of `chunk` positions counted from
+// position 0 (chunk <= 0: none); the last one is i itself.
+__host__ __device__ __forceinline__ int first_visible(int i, int window, int chunk)
+{
+    int lo = 0;
+    if (window > 0 && i - window + 1 > lo) lo = i - window + 1;
+    if (chunk > 0 && i - i % chunk > lo) lo = i - i % chunk;
+    return lo;
+}
+
 // One sequence of a step: rows [row0, row0 + n) of the step's activation tensors are the tokens at positions
 // [pos0, pos0 + n) of the sequence whose cache / state lives in slot `slot`.
 struct SeqDesc { int row0, n, pos0, slot; };

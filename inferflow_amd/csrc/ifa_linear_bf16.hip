@@ -32,7 +32,7 @@ struct LinArgs {
     // grouped product (k_lin_mfma only): tile blockIdx.y serves rows [row0, row0 + n) of group g (tile_map {g, row0, n}; *n_tiles valid
     // tiles) with the matrix W + g * N * K; activation row of output row r: A[a_rows[r]] (a_rows null: r); row_scale per output row
     const int *tile_map, *n_tiles, *a_rows; const float *row_scale;
-    int act_kind;                              // 1: every output passes the exact (erf) GELU after the bias
+    int act_kind;                              // every output after the bias passes 1: the exact (erf) GELU, 2: the square of relu
 };
 
 __device__ __forceinline__ void lin_store(const LinArgs &P, int t, int n, float acc)
@@ -40,6 +40,7 @@ __device__ __forceinline__ void lin_store(const LinArgs &P, int t, int n, float 
     if (P.bias) acc += bf2f(P.bias[n]);
     if (n >= P.act_c0 && n < P.act_c1) acc = silu_exact(acc);
     if (P.act_kind == 1) acc = 0.5f * acc * (1.0f + erff(acc * 0.70710678118654752f));
+    if (P.act_kind == 2) { acc = fmaxf(acc, 0.0f); acc *= acc; }
     if (P.row_scale) acc *= P.row_scale[t];
     if (P.mul) acc *= bf2f(P.mul[n]);
     acc *= P.alpha;
@@ -226,7 +227,7 @@ __global__ void __launch_bounds__(256) k_lin_rows(LinArgs P)
 
 static int linear_launch(const void *w_bf16, size_t rows, size_t cols, const void *a_f32, size_t lda, size_t tokens, const void *bias_bf16,
                          const void *mul_bf16, float alpha, int accumulate, int ops32, void *c_f32, size_t ldc, int silu_col0, int silu_col1, int prologue,
-                         const void *norm_w_bf16, float norm_eps, ifa_stream stream, const char *who)
+                         const void *norm_w_bf16, float norm_eps, ifa_stream stream, const char *who, int act = 0)
 {
     IFA_REQUIRE(w_bf16 && a_f32 && c_f32, "%s: null pointer", who);
     IFA_REQUIRE(rows > 0 && cols > 0 && tokens > 0 && lda >= cols * (prologue == 2 ? 2 : 1) && ldc >= rows, "%s: bad shape (%zu x %zu, %zu tokens, lda %zu, ldc %zu)", who, rows, cols, tokens, lda, ldc);
@@ -237,7 +238,7 @@ static int linear_launch(const void *w_bf16, size_t rows, size_t cols, const voi
     P.T = (int)tokens; P.N = (int)rows; P.K = (int)cols; P.lda = (int)lda; P.ldc = (int)ldc;
     P.alpha = alpha; P.accumulate = accumulate ? 1 : 0; P.act_c0 = silu_col0; P.act_c1 = silu_col1;
     P.norm_w = (const bf16_t *)norm_w_bf16; P.norm_eps = norm_eps;
-    P.tile_map = P.n_tiles = P.a_rows = nullptr; P.row_scale = nullptr; P.act_kind = 0;
+    P.tile_map = P.n_tiles = P.a_rows = nullptr; P.row_scale = nullptr; P.act_kind = act;
     // 16-byte requests need whole 8-element pieces in every row of both operands
     P.vec = (cols % 8 == 0 && lda % 4 == 0 && ((uintptr_t)a_f32 & 15) == 0 && ((uintptr_t)w_bf16 & 15) == 0) ? 1 : 0;
     hipStream_t s = ifa_s(stream);
@@ -268,6 +269,13 @@ extern "C" int ifa_linear_bf16w(const void *w_bf16, size_t rows, size_t cols, co
 {
     return linear_launch(w_bf16, rows, cols, a_f32, lda, tokens, bias_bf16, mul_bf16, alpha, accumulate, ops32, c_f32, ldc, silu_col0, silu_col1, 0, nullptr, 0.0f,
                          stream, "ifa_linear_bf16w");
+}
+
+extern "C" int ifa_linear_bf16w_act(const void *w_bf16, size_t rows, size_t cols, const void *a_f32, size_t lda, size_t tokens, const void *bias_bf16, int act,
+                                    int ops32, void *c_f32, size_t ldc, ifa_stream stream)
+{
+    IFA_REQUIRE(act >= 0 && act <= 2, "ifa_linear_bf16w_act: activation %d", act);
+    return linear_launch(w_bf16, rows, cols, a_f32, lda, tokens, bias_bf16, nullptr, 1.0f, 0, ops32, c_f32, ldc, 0, 0, 0, nullptr, 0.0f, stream, "ifa_linear_bf16w_act", act);
 }
 
 extern "C" int ifa_linear_bf16w_rows(int prologue, const void *norm_w_bf16, float norm_eps, const void *w_bf16, size_t rows, size_t cols, const void *a_f32,

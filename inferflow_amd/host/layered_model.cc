@@ -40,6 +40,15 @@
 //   "latent_attention"  queries straight from the input, rotation in halves, one cached row per position, a sigmoid gate per output column
 //   "mamba2"            selective state space behind a short convolution with bias, SiLU gate in front of an RMS norm in norm_groups parts
 // and a feed-forward of kind "dense" (SiLU-gated) or "moe" (sigmoid scores, renormalized over the chosen and multiplied by router.scale), or none.
+//
+// Rosilix: width / vocab / norm.eps / embedding.scale; the scaled token embedding, an RMS norm (plain weight) before and after each sub-layer and in front
+// of the head; mixer types
+//   "attention"         differential attention: two softmax maps per head over the same values (queries and keys [head][map][dim]), grouped queries, rotation
+//                       of the first rot.dims dimensions of each map in pairs (2i, 2i + 1), chunks of mask.size positions, the second map times a learned
+//                       factor (lq1, lk1, lq2, lk2, diff) taken off the first, the difference normed per head, a sigmoid gate per head
+//   "latent_attention"  queries straight from the input, rotation in pairs, one cached row per position, a learned sink and a sigmoid gate per head;
+//                       "kv_from": j = the layer has no down-projection and reads the cache rows of layer j
+// and a feed-forward of kind "dense" (down(relu(up)^2), no gate), or none.
 #include <cmath>
 #include <cstdio>
 #include <cstring>
@@ -445,6 +454,92 @@ void KamelornNames(const LayeredDesc &d, std::vector<std::pair<std::string, std:
     }
 }
 
+// ---- Rosilix
+bool ParseRosilix(const JsonValue &root, LayeredDesc &d)
+{
+    memset(&d.cfg, 0, sizeof(d.cfg));
+    if (!Need(root, "width", d.cfg.width, "config") || !Need(root, "vocab", d.cfg.vocab, "config")) return false;
+    const JsonValue *norm = root.Get("norm");
+    if (!norm || !Need(*norm, "eps", d.cfg.eps, "norm")) { if (!norm) EngineSetError("config.json: norm is missing"); return false; }
+    d.cfg.stem = 2; d.cfg.norm_plain = 1;
+    d.cfg.embed_scale = 1.0f;
+    if (const JsonValue *emb = root.Get("embedding")) emb->GetNumber("scale", d.cfg.embed_scale);
+    const JsonValue *layers = root.Get("layers");
+    if (!layers || layers->type != JsonValue::Array || layers->arr.empty()) { EngineSetError("config.json: layers is missing or empty"); return false; }
+    for (size_t li = 0; li < layers->arr.size(); li++) {
+        const JsonValue &L = layers->arr[li];
+        ifa_layer_spec s; memset(&s, 0, sizeof(s));
+        std::string type;
+        const JsonValue *mx = L.Get("mixer");
+        if (!L.GetString("type", type) || !mx || mx->type != JsonValue::Object) { EngineSetError("config.json: layer %zu has no type / mixer", li); return false; }
+        s.block = IFA_BLOCK_SANDWICH;
+        const JsonValue *rot = mx->Get("rot");
+        const bool rotated = rot && rot->type == JsonValue::Object;
+        int from = -1;
+        const bool shared = mx->GetNumber("kv_from", from);
+        if (type == "attention") {
+            s.mixer = IFA_MIX_DIFF; s.a_gate = 1; s.a_rot_pairs = 1;
+            if (!Need(*mx, "heads", s.a_heads, "mixer") || !Need(*mx, "kv_heads", s.a_kv_heads, "mixer") || !Need(*mx, "dim", s.a_dim, "mixer")
+                || !Need(*mx, "vdim", s.a_vdim, "mixer") || !Need(*mx, "scale", s.a_scale, "mixer") || !Need(*mx, "diff", s.a_diff, "mixer")) return false;
+            if (rotated && (!Need(*rot, "base", s.a_rot_base, "mixer.rot") || !Need(*rot, "dims", s.a_rot_dims, "mixer.rot"))) return false;
+            const JsonValue *mask = mx->Get("mask");
+            if (mask && mask->type == JsonValue::Object) {
+                if (!Need(*mask, "size", s.a_chunk, "mixer.mask")) return false;
+                if (s.a_chunk < 1) { EngineSetError("config.json: layer %zu: mask.size %d", li, s.a_chunk); return false; }
+            }
+            if (shared) { EngineSetError("config.json: layer %zu: kv_from is for latent_attention", li); return false; }
+        } else if (type == "latent_attention") {
+            s.mixer = IFA_MIX_LATENT; s.m_gate = 1; s.m_sink = 1;
+            if (!Need(*mx, "heads", s.m_heads, "mixer") || !Need(*mx, "dim", s.m_dim, "mixer") || !Need(*mx, "rot_dim", s.m_rot_dim, "mixer") || !Need(*mx, "vdim", s.m_vdim, "mixer")
+                || !Need(*mx, "kv_rank", s.m_kv_rank, "mixer") || !Need(*mx, "scale", s.m_scale, "mixer")) return false;
+            if (!rotated || !Need(*rot, "base", s.m_rot_base, "mixer.rot") || !Need(*rot, "dims", s.m_rot_dims, "mixer.rot")) {
+                if (!rotated) EngineSetError("config.json: layer %zu: mixer.rot is missing", li);
+                return false;
+            }
+            if (shared) {
+                if (from < 0 || from >= (int)li) { EngineSetError("config.json: layer %zu: kv_from %d is not an earlier layer", li, from); return false; }
+                s.m_kv_layer = from + 1;
+            }
+        } else { EngineSetError("config.json: layer %zu: unknown type \"%s\"", li, type.c_str()); return false; }
+        const JsonValue *mlp = L.Get("mlp");
+        if (mlp && mlp->type == JsonValue::Object) {
+            std::string kind;
+            if (!mlp->GetString("kind", kind) || kind != "dense") { EngineSetError("config.json: layer %zu: mlp.kind \"%s\" is not supported (dense)", li, kind.c_str()); return false; }
+            s.ffn_kind = IFA_FFN_RELU2;
+            if (!Need(*mlp, "ff", s.ffn, "mlp")) return false;
+        }
+        d.layers.push_back(s);
+        d.decays.push_back(std::vector<float>());
+    }
+    d.cfg.n_layers = (int)d.layers.size();
+    return true;
+}
+
+void RosilixNames(const LayeredDesc &d, std::vector<std::pair<std::string, std::pair<int, int>>> &out)
+{
+    out.push_back({"embed", {-1, IFA_T_EMBD}}); out.push_back({"final.norm", {-1, IFA_T_OUT_NORM}}); out.push_back({"head", {-1, IFA_T_LM_HEAD}});
+    for (size_t li = 0; li < d.layers.size(); li++) {
+        const ifa_layer_spec &s = d.layers[li];
+        const std::string p = "l" + std::to_string(li) + ".";
+        const int l = (int)li;
+        out.push_back({p + "norm1", {l, IFA_LT_NORM1}}); out.push_back({p + "norm1b", {l, IFA_LT_NORM1B}});
+        if (s.mixer == IFA_MIX_LATENT) {
+            out.push_back({p + "mix.q", {l, IFA_LT_M_Q}});
+            if (s.m_kv_layer == 0) { out.push_back({p + "mix.dkv", {l, IFA_LT_M_DKV}}); out.push_back({p + "mix.dkv.norm", {l, IFA_LT_M_DKV_NORM}}); }
+            out.push_back({p + "mix.uk", {l, IFA_LT_M_UK}}); out.push_back({p + "mix.uv", {l, IFA_LT_M_UV}}); out.push_back({p + "mix.sink", {l, IFA_LT_M_SINK}});
+            out.push_back({p + "mix.g", {l, IFA_LT_M_G}}); out.push_back({p + "mix.o", {l, IFA_LT_M_O}});
+        } else {
+            out.push_back({p + "mix.q", {l, IFA_LT_A_Q}}); out.push_back({p + "mix.k", {l, IFA_LT_A_K}}); out.push_back({p + "mix.v", {l, IFA_LT_A_V}});
+            out.push_back({p + "mix.lq1", {l, IFA_LT_A_LQ1}}); out.push_back({p + "mix.lk1", {l, IFA_LT_A_LK1}});
+            out.push_back({p + "mix.lq2", {l, IFA_LT_A_LQ2}}); out.push_back({p + "mix.lk2", {l, IFA_LT_A_LK2}});
+            out.push_back({p + "mix.g", {l, IFA_LT_A_G}}); out.push_back({p + "mix.o", {l, IFA_LT_A_O}});
+        }
+        if (s.ffn <= 0) continue;
+        out.push_back({p + "norm2", {l, IFA_LT_NORM2}}); out.push_back({p + "norm2b", {l, IFA_LT_NORM2B}});
+        out.push_back({p + "mlp.up", {l, IFA_LT_FFN_UP}}); out.push_back({p + "mlp.down", {l, IFA_LT_FFN_DOWN}});
+    }
+}
+
 void SopulornNames(const LayeredDesc &d, std::vector<std::pair<std::string, std::pair<int, int>>> &out)
 {
     out.push_back({"embed", {-1, IFA_T_EMBD}});
@@ -566,7 +661,8 @@ const ArchEntry kArchitectures[] = {{"Gelarax", ParseGelarax, GelaraxSizesFromTe
                                     {"Muzopel", ParseMuzopel, NoSizesFromTensors, MuzopelNames},
                                     {"Sopulorn", ParseSopulorn, NoSizesFromTensors, SopulornNames},
                                     {"Bogupel", ParseBogupel, BogupelSizesFromTensors, BogupelNames},
-                                    {"Kamelorn", ParseKamelorn, NoSizesFromTensors, KamelornNames}};
+                                    {"Kamelorn", ParseKamelorn, NoSizesFromTensors, KamelornNames},
+                                    {"Rosilix", ParseRosilix, NoSizesFromTensors, RosilixNames}};
 
 const ArchEntry *FindArch(const std::string &name)
 {

@@ -37,7 +37,9 @@ def test_layered_only_library_builds_and_declines_the_standard_network():
              "ifa_qkv_rope_store_f32", "ifa_rotate_heads_f32", "ifa_attention_kv_sinks_f32", "ifa_chan_delta_gates_f32", "ifa_state_scan_chan_f32",
              "ifa_moe_dyt_route_rows_f32", "ifa_moe_experts_glu_f32", "ifa_streams_step_f32", "ifa_conv_ring_silu_f32", "ifa_ssm_gates_ring_f32", "ifa_ssm_step_f32",
              "ifa_ssm_chunked_f32", "ifa_state_scan_ssm_f32", "ifa_gate_groupnorm_f32", "ifa_latent_prepare_pairs_f32", "ifa_latent_expand_out_gated_f32",
-             "ifa_attention_latent_tile_gated_f32", "ifa_moe_route_renorm_f32", "ifa_moe_experts_routed_rows_f32")
+             "ifa_attention_latent_tile_gated_f32", "ifa_moe_route_renorm_f32", "ifa_moe_experts_routed_rows_f32",
+             "ifa_attention_diff_f32", "ifa_qk_rope_store_pairs_f32", "ifa_latent_rotate_q_f32", "ifa_attention_latent_rows_sinks_f32", "ifa_attention_latent_tile_sinks_f32",
+             "ifa_linear_bf16w_act")
     r = subprocess.run([sys.executable, "-c", code, path, ",".join(names)], capture_output=True, text=True, timeout=120)
     assert r.returncode == 0, r.stderr[-2000:]
     assert r.stdout.startswith("[] -4 ") and "standard network" in r.stdout, r.stdout
