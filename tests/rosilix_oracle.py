@@ -39,11 +39,16 @@ def turn_pairs(z, positions, dims, base):
     return out
 
 
-def visible(T, chunk=None):
-    """[i, j]: row i sees key j: never a later one, with `chunk` only keys of its own chunk of positions (counted from 0)"""
+def visible(T, chunk=None, window=None):
+    """[i, j]: row i sees key j: never a later one, with `chunk` only keys of its own chunk of positions (counted from 0), with `window` only
+    keys less than that far back"""
     i, j = np.arange(T)[:, None], np.arange(T)[None, :]
     see = j <= i
-    return see & (i // chunk == j // chunk) if chunk else see
+    if chunk:
+        see = see & (i // chunk == j // chunk)
+    if window:
+        see = see & (i - j < window)
+    return see
 
 
 def softmax(s, sink=None):
@@ -65,6 +70,20 @@ def difference(a1, a2, lam, diff, eps):
     return rms_unit(a1 - lam * a2, eps) * (1.0 - diff)
 
 
+def two_map_attention(q, k, v, see, scale, lam, diff, gate, eps):
+    """q [T, H, 2, d], k [T, G, 2, d], v [T, G, dv], see [T, T], gate [T, H]: every head's combined, normed and gated output [T, H, dv]"""
+    T, H, G = q.shape[0], q.shape[1], k.shape[1]
+    out = np.zeros((T, H, v.shape[-1]))
+    for hd in range(H):
+        g = hd // (H // G)
+        maps = []
+        for m in range(2):
+            s = (q[:, hd, m] @ k[:, g, m].T) * scale
+            maps.append(softmax(np.where(see, s, -np.inf)) @ v[:, g])
+        out[:, hd] = difference(maps[0], maps[1], lam, diff, eps) * gate[:, hd:hd + 1]
+    return out
+
+
 def attention(h, W, p, mx, eps):
     """differential attention inside chunks"""
     T, H, G, d, dv = h.shape[0], mx["heads"], mx["kv_heads"], mx["dim"], mx["vdim"]
@@ -73,18 +92,8 @@ def attention(h, W, p, mx, eps):
     q = turn_pairs((h @ W[p + "q"].T).reshape(T, H, 2, d), pos, rot["dims"], rot["base"])
     k = turn_pairs((h @ W[p + "k"].T).reshape(T, G, 2, d), pos, rot["dims"], rot["base"])
     v = (h @ W[p + "v"].T).reshape(T, G, dv)
-    hidden = ~visible(T, (mx.get("mask") or {}).get("size"))
     lam = mixing_factor(W[p + "lq1"], W[p + "lk1"], W[p + "lq2"], W[p + "lk2"], mx["diff"])
-    gate = logistic(h @ W[p + "g"].T)
-    out = np.zeros((T, H, dv))
-    for hd in range(H):
-        g = hd // (H // G)
-        maps = []
-        for m in range(2):
-            s = (q[:, hd, m] @ k[:, g, m].T) * mx["scale"]
-            s[hidden] = -np.inf
-            maps.append(softmax(s) @ v[:, g])
-        out[:, hd] = difference(maps[0], maps[1], lam, mx["diff"], eps) * gate[:, hd:hd + 1]
+    out = two_map_attention(q, k, v, visible(T, (mx.get("mask") or {}).get("size")), mx["scale"], lam, mx["diff"], logistic(h @ W[p + "g"].T), eps)
     return out.reshape(T, H * dv) @ W[p + "o"].T
 
 
