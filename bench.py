@@ -402,8 +402,16 @@ KAMELORN_SIZES = {  # --arch kamelorn: six layers in eight layer runs (latent at
 }
 
 
+ROSILIX_SIZES = {   # --arch rosilix: eight layers (latent attention, latent attention on the first one's rows, two layers of differential attention in chunks; twice), dense feed-forwards
+    "w1024": dict(width=1024, heads=8, kv_heads=2, dim=64, vdim=128, rot_dims=64, chunk=1280, lat_heads=8, lat_dim=96, lat_rot_dim=32, lat_vdim=128, kv_rank=256, ff=4096),
+    "w2048": dict(width=2048, heads=16, kv_heads=4, dim=64, vdim=128, rot_dims=64, chunk=1280, lat_heads=16, lat_dim=128, lat_rot_dim=64, lat_vdim=128, kv_rank=512, ff=8192),
+}
+
+
 def run_arch_bench(args):
-    """--arch gelarax | muzopel | sopulorn | bogupel | kamelorn: see run_gelarax_bench / run_muzopel_bench"""
+    """--arch gelarax | muzopel | sopulorn | bogupel | kamelorn | rosilix: see run_gelarax_bench / run_muzopel_bench"""
+    if args.arch.lower() == "rosilix":
+        return run_muzopel_bench(args, "rosilix")
     if args.arch.lower() == "kamelorn":
         return run_muzopel_bench(args, "kamelorn")
     if args.arch.lower() == "muzopel":
@@ -416,7 +424,7 @@ def run_arch_bench(args):
 
 
 def run_muzopel_bench(args, design="muzopel"):
-    """--arch muzopel | sopulorn | bogupel | kamelorn: prefill and decode throughput of models of that design with random bfloat16 weights (layer-list worker: latent attention
+    """--arch muzopel | sopulorn | bogupel | kamelorn | rosilix: prefill and decode throughput of models of that design with random bfloat16 weights (layer-list worker: latent attention
     or rotary attention with shared key / value rows, mixture of experts, fp32 residual) beside the closest standard model of this framework at equal
     width / heads / KV heads / layers / experts / expert width (Mixtral wiring: attention with an F16 KV cache, gated experts, F16 weights).  One JSON
     line; `value` = decode tokens/s of the largest size."""
@@ -440,10 +448,10 @@ def run_muzopel_bench(args, design="muzopel"):
 
     sop = design == "sopulorn"
     label = design.capitalize()
-    size_table = {"sopulorn": SOPULORN_SIZES, "muzopel": MUZOPEL_SIZES, "bogupel": BOGUPEL_SIZES, "kamelorn": KAMELORN_SIZES}[design]
-    make_cfg = {"sopulorn": synth.sopulorn_config, "muzopel": synth.muzopel_config, "bogupel": synth.bogupel_config, "kamelorn": synth.kamelorn_config}[design]
-    write_dir = {"sopulorn": synth.write_sopulorn_dir, "muzopel": synth.write_muzopel_dir, "bogupel": synth.write_bogupel_dir, "kamelorn": synth.write_kamelorn_dir}[design]
-    shapes_of = {"sopulorn": synth.sopulorn_tensor_shapes, "muzopel": synth.muzopel_tensor_shapes, "bogupel": synth.bogupel_tensor_shapes, "kamelorn": synth.kamelorn_tensor_shapes}[design]
+    size_table = {"sopulorn": SOPULORN_SIZES, "muzopel": MUZOPEL_SIZES, "bogupel": BOGUPEL_SIZES, "kamelorn": KAMELORN_SIZES, "rosilix": ROSILIX_SIZES}[design]
+    make_cfg = {"sopulorn": synth.sopulorn_config, "muzopel": synth.muzopel_config, "bogupel": synth.bogupel_config, "kamelorn": synth.kamelorn_config, "rosilix": synth.rosilix_config}[design]
+    write_dir = {"sopulorn": synth.write_sopulorn_dir, "muzopel": synth.write_muzopel_dir, "bogupel": synth.write_bogupel_dir, "kamelorn": synth.write_kamelorn_dir, "rosilix": synth.write_rosilix_dir}[design]
+    shapes_of = {"sopulorn": synth.sopulorn_tensor_shapes, "muzopel": synth.muzopel_tensor_shapes, "bogupel": synth.bogupel_tensor_shapes, "kamelorn": synth.kamelorn_tensor_shapes, "rosilix": synth.rosilix_tensor_shapes}[design]
     def layered_rates(cfg, write_dir, shapes):
         d = tempfile.mkdtemp(prefix="ifa_%s_" % design, dir="/dev/shm" if os.path.isdir("/dev/shm") else None)
         try:
@@ -477,9 +485,20 @@ def run_muzopel_bench(args, design="muzopel"):
             mz = synth.muzopel_config(width=sz["width"], vocab=32000, heads=sz["heads"], dim=sz["dim"], rot_dim=sz["rot_dim"], vdim=sz["vdim"], kv_rank=sz["kv_rank"],
                                       q_rank=3 * sz["kv_rank"] // 2, experts=sz["experts"], identity=0, top=sz["top"], ff=sz["ff"])
             extra["closest_layered_model"] = {"design": "Muzopel", **layered_rates(mz, synth.write_muzopel_dir, synth.muzopel_tensor_shapes(mz))}
+        if design == "rosilix":      # the closest layer-list models, a gated feed-forward of as many parameters (three matrices for two): rotary attention with the same wiring of
+            # norms and heads of the same size (2 dim), and latent attention of the same sizes in each of eight layers
+            gated = (2 * sz["ff"] // 3 + 255) // 256 * 256
+            sp = synth.sopulorn_config(width=sz["width"], vocab=32000, heads=sz["heads"], kv_heads=sz["kv_heads"], dim=2 * sz["dim"], vdim=sz["vdim"], rot_dims=sz["rot_dims"],
+                                       dense_ff=gated, experts=1, top=1, ff=8, shared_ff=8)
+            sp["layers"] = [sp["layers"][0]] * 8
+            extra["closest_layered_model"] = {"design": "Sopulorn, dense", **layered_rates(sp, synth.write_sopulorn_dir, synth.sopulorn_tensor_shapes(sp))}
+            km = synth.kamelorn_config(width=sz["width"], vocab=32000, heads=sz["lat_heads"], dim=sz["lat_dim"], rot_dim=sz["lat_rot_dim"], vdim=sz["lat_vdim"], kv_rank=sz["kv_rank"],
+                                       dense_ff=gated, streams=1)
+            km["layers"] = [km["layers"][0]] * 8; km.pop("loop")
+            extra["closest_latent_model"] = {"design": "Kamelorn, latent attention and dense", **layered_rates(km, synth.write_kamelorn_dir, synth.kamelorn_tensor_shapes(km))}
         # the closest standard model: same width, heads, layer count, experts, choices per token and expert width, F16 weights
-        synth.SHAPES["cmp_" + name] = dict(dim=sz["width"], layers=8, heads=sz["heads"], kv_heads=sz.get("kv_heads", sz["heads"]), head_dim=128, ffn=sz["ff"], vocab=32000,
-                                           experts=sz["experts"], moe_top_k=sz["top"])
+        synth.SHAPES["cmp_" + name] = dict(dim=sz["width"], layers=8, heads=sz["heads"], kv_heads=sz.get("kv_heads", sz["heads"]), head_dim=128, vocab=32000,
+                                           **(dict(ffn=sz["ff"], experts=sz["experts"], moe_top_k=sz["top"]) if "experts" in sz else dict(ffn=gated)))
         wk, _, _ = synth.build("cmp_" + name, dt.F16, dt.F16, ctx, quant_threshold=1 << 62)
         c = {"prefill_tok_s": {}}
         for n in lens:
@@ -589,13 +608,13 @@ def main():
                     "a functional check of the N > 1 step logic on a one-GPU box, not a scaling number")
     ap.add_argument("--no-cpu-baseline", action="store_true")
     ap.add_argument("--cpu-tokens", type=int, default=0, help="CPU baseline sample size (0 = auto)")
-    ap.add_argument("--arch", default="", help="'gelarax', 'muzopel', 'sopulorn', 'bogupel' or 'kamelorn': instead of the headline workload, prefill / decode rates of models of that design beside the "
+    ap.add_argument("--arch", default="", help="'gelarax', 'muzopel', 'sopulorn', 'bogupel', 'kamelorn' or 'rosilix': instead of the headline workload, prefill / decode rates of models of that design beside the "
                     "closest standard model at equal size (one GPU; --prefill-lens, --steps, --warmup apply)")
     ap.add_argument("--arch-sizes", default="w1024,w2048")
     args = ap.parse_args()
     if args.arch:
-        if args.arch.lower() not in ("gelarax", "muzopel", "sopulorn", "bogupel", "kamelorn"):
-            raise SystemExit("unknown --arch %s (gelarax, muzopel, sopulorn, bogupel, kamelorn)" % args.arch)
+        if args.arch.lower() not in ("gelarax", "muzopel", "sopulorn", "bogupel", "kamelorn", "rosilix"):
+            raise SystemExit("unknown --arch %s (gelarax, muzopel, sopulorn, bogupel, kamelorn, rosilix)" % args.arch)
         if args.gpus > 1 or int(os.environ.get("WORLD_SIZE", "1")) > 1:
             raise SystemExit("--arch runs on one GPU")
         return run_arch_bench(args)

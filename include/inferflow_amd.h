@@ -793,6 +793,12 @@ int ifa_attention_diff_f32(const void *q_f32, size_t ldq, int heads, int kv_head
                            float eps, const void *g_f32, size_t ldg, const void *seqs_dev, const int *row_seq_dev, size_t rows, void *const *slot_base_dev, size_t k_off,
                            size_t v_off, void *out_f32, size_t ldo, const void *seqs_host, int n_seqs, int tile_min_rows, int max_keys, void *ws_f32, size_t ws_bytes,
                            ifa_stream stream);
+/* rows of 32-bit values rounded to bfloat16 (to nearest even), zero from cols to ldy (a multiple of 8) */
+int ifa_rows_to_bf16(const void *x_f32, size_t ldx, size_t rows, size_t cols, void *y_bf16, size_t ldy, ifa_stream stream);
+/* ifa_linear_bf16w (ops32 0) over activations that are bfloat16 already: a_bf16 [tokens][lda], lda = cols rounded up to whole 64s, zero beyond cols (cols % 8 ==
+ * 0, cols >= 64).  act as ifa_linear_bf16w_act; c_bf16 (not null, act 2 only): the output in bfloat16 instead of c_f32.  The same sums in the same order as ifa_linear_bf16w. */
+int ifa_linear_bf16_both(const void *w_bf16, size_t rows, size_t cols, const void *a_bf16, size_t lda, size_t tokens, const void *bias_bf16, const void *mul_bf16,
+                         float alpha, int accumulate, int act, void *c_f32, void *c_bf16, size_t ldc, int silu_col0, int silu_col1, ifa_stream stream);
 /* ifa_linear_bf16w with an activation of every output after the bias: act 0 none, 1 erf-GELU, 2 relu(z)^2 */
 int ifa_linear_bf16w_act(const void *w_bf16, size_t rows, size_t cols, const void *a_f32, size_t lda, size_t tokens, const void *bias_bf16, int act, int ops32,
                          void *c_f32, size_t ldc, ifa_stream stream);

@@ -46,6 +46,13 @@ __global__ void __launch_bounds__(256) k_attn_diff_rows(DiffArgs P)
     const int split = blockIdx.z, tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
     const SeqDesc sd = P.seqs[P.row_seq[t]];
     const int i = sd.pos0 + t - sd.row0, lo = first_visible(i, P.window, P.chunk), nk = i - lo + 1;
+    if (split * 64 >= nk) {          // no keys for this share: an empty one (the combine does not read its values)
+        if (tid < 2 * nh) {
+            float *dst = P.ws + ((((size_t)t * P.heads + h0 + (tid >> 1)) * P.nsplit + split) * 2 + (tid & 1)) * (dv + 2);
+            dst[0] = -INFINITY; dst[1] = 0.0f;
+        }
+        return;
+    }
     for (int e = tid; e < HB * D2; e += blockDim.x) qs[e] = e < nh * D2 ? P.q[(size_t)t * P.ldq + (size_t)h0 * D2 + e] : 0.0f;
     __syncthreads();
     const size_t kvd = (size_t)P.kv_heads * D2, vvd = (size_t)P.kv_heads * dv;
@@ -107,10 +114,10 @@ __global__ void __launch_bounds__(256) k_attn_diff_rows(DiffArgs P)
 #pragma unroll
             for (int mp = 0; mp < 2; mp++) {
                 const float sc = quad_sum(s[hh][mp]) * P.scale, x = valid ? sc : -INFINITY;
-                const float m_new = fmaxf(m[hh][mp], wave_max(x));          // finite: the chunk holds at least one visible key
+                const float m_new = fmaxf(m[hh][mp], quads_max(x));          // finite: the chunk holds at least one visible key
                 p[hh][mp] = valid ? expf(x - m_new) : 0.0f;
                 const float corr = m[hh][mp] == -INFINITY ? 0.0f : expf(m[hh][mp] - m_new);
-                l[hh][mp] = l[hh][mp] * corr + wave_sum(sub == 0 ? p[hh][mp] : 0.0f);
+                l[hh][mp] = l[hh][mp] * corr + quads_sum(p[hh][mp]);
 #pragma unroll
                 for (int e = 0; e < CPL; e++) acc[hh][mp][e] *= corr;
                 m[hh][mp] = m_new;
@@ -147,15 +154,18 @@ __global__ void __launch_bounds__(256) k_attn_diff_rows(DiffArgs P)
             for (int e = 0; e < CPL; e++) { const int c = lane + 64 * e; if (c < dv) wacc[(size_t)w * dv + c] = acc[hh][mp][e]; }
         }
     __syncthreads();
-    for (int hm = 0; hm < 2 * nh; hm++) {
+    for (int hm = wave; hm < 2 * nh; hm += 4) {          // (a wave per head and map)
         float M = -INFINITY;
+#pragma unroll
         for (int w = 0; w < 4; w++) M = fmaxf(M, wm[w * 2 * HB + hm]);
         float L = 0.0f, f[4];
+#pragma unroll
         for (int w = 0; w < 4; w++) { const float mw = wm[w * 2 * HB + hm]; f[w] = mw == -INFINITY ? 0.0f : expf(mw - M); L += wl[w * 2 * HB + hm] * f[w]; }
         float *dst = P.ws + ((((size_t)t * P.heads + h0 + (hm >> 1)) * P.nsplit + split) * 2 + (hm & 1)) * (dv + 2);
-        if (tid == 0) { dst[0] = M; dst[1] = L; }
-        for (int c = tid; c < dv; c += blockDim.x) {
+        if (lane == 0) { dst[0] = M; dst[1] = L; }
+        for (int c = lane; c < dv; c += 64) {
             float o = 0.0f;
+#pragma unroll
             for (int w = 0; w < 4; w++) o = fmaf(wacc[(size_t)(w * 2 * HB + hm) * dv + c], f[w], o);
             dst[2 + c] = o;
         }
@@ -191,7 +201,8 @@ __global__ void __launch_bounds__(256) k_attn_diff_combine(DiffArgs P)
             for (int u = 0; u < 4; u++) {
                 const int sp = min(s0 + 4 * u, nsplit - 1);
                 const float f1 = __shfl(f[0], sp, 64), f2 = __shfl(f[1], sp, 64);
-                if (s0 + 4 * u < nsplit) { o1 = fmaf(v1[u], f1, o1); o2 = fmaf(v2[u], f2, o2); }
+                if (s0 + 4 * u < nsplit && f1 > 0.0f) o1 = fmaf(v1[u], f1, o1);          // (an empty share's values are not there)
+                if (s0 + 4 * u < nsplit && f2 > 0.0f) o2 = fmaf(v2[u], f2, o2);
             }
         }
         if (c0 + lane < dv) { part[(size_t)(wave * 2) * dv + c] = o1; part[(size_t)(wave * 2 + 1) * dv + c] = o2; }

@@ -391,7 +391,9 @@ __global__ void __launch_bounds__(256) k_qk_rope_store(float *__restrict__ q, si
     }
     __syncthreads();
     const int n_items = do_qk ? heads + (k ? kv_heads : 0) : 0;
-    for (int it = wave; it < n_items; it += nw) {
+    // (steps of a few rows: a row's heads are shared out over gridDim.z workgroups)
+    const int w0 = blockIdx.z * nw + wave, wn = nw * gridDim.z;
+    for (int it = w0; it < n_items; it += wn) {
         const bool is_q = it < heads;
         const int hd = is_q ? it : it - heads;
         const float *src = is_q ? q + (size_t)t * ldq + (size_t)hd * dim : k + (size_t)t * ldk + (size_t)hd * dim;
@@ -430,7 +432,7 @@ __global__ void __launch_bounds__(256) k_qk_rope_store(float *__restrict__ q, si
     if (VX) {
         if (!k || !do_v) return;
         // a wave per value head: weightless RMS norm, then the turn by the position (a lane reads both members of a pair from the input row)
-        for (int hd = wave; hd < kv_heads; hd += nw) {
+        for (int hd = w0; hd < kv_heads; hd += wn) {
             const float *src = v + (size_t)t * ldv + (size_t)hd * vdim;
             float *dst = slot_base[sd.slot] + v_off + ((size_t)pos * kv_heads + hd) * vdim;
             float r = 1.0f;
@@ -454,7 +456,7 @@ __global__ void __launch_bounds__(256) k_qk_rope_store(float *__restrict__ q, si
     if (k) {
         float *vd = slot_base[sd.slot] + v_off + (size_t)pos * v_heads * vdim;
         const float *vs = v + (size_t)t * ldv;
-        for (int c = tid; c < v_heads * vdim; c += blockDim.x) vd[c] = vs[c];
+        for (int c = blockIdx.z * blockDim.x + tid; c < v_heads * vdim; c += blockDim.x * gridDim.z) vd[c] = vs[c];
     }
 }
 
@@ -577,6 +579,9 @@ int ifa_attention_kv_f32(const void *q_f32, size_t ldq, int heads, int kv_heads,
                             max_keys, ws_f32, ws_bytes, stream);
 }
 
+// workgroups that share a row's heads: one head per wave for steps of a few rows
+static unsigned rope_parts(size_t rows, int heads, int k_heads) { return rows <= 8 ? (unsigned)std::min(16, (heads + k_heads + 3) / 4) : 1u; }
+
 int ifa_qk_rope_store_pairs_f32(int pairing, void *q_f32, size_t ldq, int heads, const void *k_f32, size_t ldk, const void *v_f32, size_t ldv, int k_heads, int v_heads,
                                 int dim, int vdim, const void *q_norm_w_bf16, const void *k_norm_w_bf16, float eps, int rot_dims, const double *freq_f64_dev,
                                 const void *seqs_dev, const int *row_seq_dev, size_t rows, void *const *slot_base_dev, size_t k_off, size_t v_off, ifa_stream stream)
@@ -585,7 +590,7 @@ int ifa_qk_rope_store_pairs_f32(int pairing, void *q_f32, size_t ldq, int heads,
     IFA_REQUIRE(heads > 0 && k_heads > 0 && v_heads > 0 && dim > 0 && dim <= 1024 && vdim > 0 && rows > 0 && rot_dims >= 0 && rot_dims <= dim && rot_dims % 2 == 0
                 && (rot_dims == 0 || freq_f64_dev) && (pairing == 0 || pairing == 1), "ifa_qk_rope_store_f32: bad shape (head size %d, %d rotated)", dim, rot_dims);
     IFA_REQUIRE(ldq >= (size_t)heads * dim && (!k_f32 || (ldk >= (size_t)k_heads * dim && ldv >= (size_t)v_heads * vdim)), "ifa_qk_rope_store_f32: row strides too small");
-#define IFA_RS(N) hipLaunchKernelGGL((k_qk_rope_store<N, false>), dim3((unsigned)rows), dim3(256), (size_t)std::max(rot_dims, 2) * 4, ifa_s(stream), (float *)q_f32, ldq, heads, \
+#define IFA_RS(N) hipLaunchKernelGGL((k_qk_rope_store<N, false>), dim3((unsigned)rows, 1u, rope_parts(rows, heads, k_f32 ? k_heads : 0)), dim3(256), (size_t)std::max(rot_dims, 2) * 4, ifa_s(stream), (float *)q_f32, ldq, heads, \
                                      (const float *)k_f32, ldk, (const float *)v_f32, ldv, k_heads, dim, vdim, (const bf16_t *)q_norm_w_bf16, (const bf16_t *)k_norm_w_bf16, eps, \
                                      rot_dims, freq_f64_dev, (const SeqDesc *)seqs_dev, row_seq_dev, (float *const *)slot_base_dev, k_off, v_off, 0, (const double *)nullptr, \
                                      pairing, v_heads)
@@ -613,7 +618,7 @@ int ifa_qkv_rope_store_f32(void *q_f32, size_t ldq, int heads, const void *k_f32
                 && (rot_dims == 0 || freq_f64_dev) && (!v_freq_f64_dev || vdim % 2 == 0), "ifa_qkv_rope_store_f32: bad shape (head sizes %d / %d, %d rotated)", dim, vdim, rot_dims);
     IFA_REQUIRE(ldq >= (size_t)heads * dim && (!k_f32 || (ldk >= (size_t)kv_heads * dim && ldv >= (size_t)kv_heads * vdim)), "ifa_qkv_rope_store_f32: row strides too small");
     const size_t smem = ((size_t)std::max(rot_dims, 2) + (size_t)vdim + 2) * 4;
-#define IFA_RS(N) hipLaunchKernelGGL((k_qk_rope_store<N, true>), dim3((unsigned)rows, k_f32 ? 2u : 1u), dim3(256), smem, ifa_s(stream), (float *)q_f32, ldq, heads, \
+#define IFA_RS(N) hipLaunchKernelGGL((k_qk_rope_store<N, true>), dim3((unsigned)rows, k_f32 ? 2u : 1u, rope_parts(rows, heads, k_f32 ? kv_heads : 0)), dim3(256), smem, ifa_s(stream), (float *)q_f32, ldq, heads, \
                                      (const float *)k_f32, ldk, (const float *)v_f32, ldv, kv_heads, dim, vdim, (const bf16_t *)q_norm_w_bf16, (const bf16_t *)k_norm_w_bf16, eps, \
                                      rot_dims, freq_f64_dev, (const SeqDesc *)seqs_dev, row_seq_dev, (float *const *)slot_base_dev, k_off, v_off, v_norm ? 1 : 0, v_freq_f64_dev, 0, kv_heads)
     if (dim <= 128) IFA_RS(2); else if (dim <= 256) IFA_RS(4); else IFA_RS(16);

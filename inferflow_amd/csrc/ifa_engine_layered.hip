@@ -113,6 +113,7 @@ struct LayeredNet {
                                            // SANDWICH layers, every step size: the norm behind a sub-layer and the norm in front of the next one in one launch
                                            // PRENORM layers: the start of a looped pass inside the norm's launch; steps of at most 8 rows: the norm inside the router's launch
     float *attn_ws = nullptr; size_t attn_ws_bytes = 0;      // partial results of the windowed attention when a (row, head)'s keys are shared out
+    bf16_t *a16 = nullptr; size_t a16_cap = 0; int opt_a16_min = 17;          // activations of a prompt's product rounded to bfloat16; steps of at least this many rows (0: never)
     int opt_attn_tile_min = 16;            // steps of at least this many rows run the windowed attention through the tiled kernel
     std::vector<ifa_seq_desc> seqs_host;   // the current step's sequences (the tiled attention's grid is sized from them)
     // POSTNORM layers: two more mixer buffers, the planes of the depth average ([layers + 1][scratch_rows * width]), the router's choices,
@@ -345,9 +346,32 @@ int ensure_logits(ifa_model *m, size_t rows)
 // what the norms of SANDWICH layers and of stem 2 add to their stored weights
 float norm_offset_of(const LayeredNet *n) { return n->cfg.norm_plain ? 0.0f : 1.0f; }
 
+// Products of prompts with bfloat16 operands: the activations are rounded once, into n->a16 (rows of whole 64s), and both operands go to LDS as they are.
+bool takes_a16(const LayeredNet *n, size_t K, size_t T) { return !n->cfg.ops32 && n->opt_a16_min > 0 && T >= (size_t)n->opt_a16_min && K % 8 == 0 && K >= 64; }
+size_t a16_stride(size_t K) { return (K + 63) & ~(size_t)63; }
+
+int ensure_a16(ifa_model *m, size_t T, size_t K)
+{
+    LayeredNet *n = m->lay;
+    const size_t need = T * a16_stride(K);
+    if (need <= n->a16_cap) return IFA_OK;
+    IFA_HIP_CHECK(hipStreamSynchronize(m->stream));
+    lay_free(n->a16); n->a16 = nullptr; n->a16_cap = 0;
+    IFA_HIP_CHECK(hipMalloc((void **)&n->a16, need * 2));
+    n->a16_cap = need;
+    return IFA_OK;
+}
+
 int linear(ifa_model *m, const bf16_t *W, size_t N, size_t K, const float *A, size_t lda, size_t T, const bf16_t *bias, const bf16_t *mul, float alpha,
            int accumulate, float *C, size_t ldc, int silu0 = 0, int silu1 = 0)
 {
+    LayeredNet *n = m->lay;
+    if (takes_a16(n, K, T)) {
+        int rc = ensure_a16(m, T, K);
+        if (!rc) rc = ifa_rows_to_bf16(A, lda, T, K, n->a16, a16_stride(K), (ifa_stream)m->stream);
+        if (!rc) rc = ifa_linear_bf16_both(W, N, K, n->a16, a16_stride(K), T, bias, mul, alpha, accumulate, 0, C, nullptr, ldc, silu0, silu1, (ifa_stream)m->stream);
+        return rc;
+    }
     return ifa_linear_bf16w(W, N, K, A, lda, T, bias, mul, alpha, accumulate, m->lay->cfg.ops32, C, ldc, silu0, silu1, (ifa_stream)m->stream);
 }
 
@@ -536,6 +560,15 @@ int run_sandwich_layer(ifa_model *m, LLayer &L, size_t T, int nseq, bool h_ready
     if (!any_ffn) return IFA_OK;
     const size_t N2 = L.n_in2;
     if (sp.ffn_kind == IFA_FFN_RELU2) {      // the square of relu in the epilogue of the up-projection
+        const size_t F = (size_t)sp.ffn;
+        if (takes_a16(n, W, T) && takes_a16(n, F, T) && F % 64 == 0) {      // ... which then leaves the down-projection's operand as it is read
+            if ((rc = ensure_a16(m, T, W + F))) return rc;
+            bf16_t *h16 = n->a16, *u16 = n->a16 + T * a16_stride(W);
+            if ((rc = ifa_rows_to_bf16(n->h, W, T, W, h16, a16_stride(W), s))) return rc;
+            if ((rc = ifa_linear_bf16_both(L.w_in2, N2, W, h16, a16_stride(W), T, nullptr, nullptr, 1.0f, 0, 2, nullptr, u16, F, 0, 0, s))) return rc;
+            if ((rc = ifa_linear_bf16_both(L.T(IFA_LT_FFN_DOWN).data, W, F, u16, F, T, nullptr, nullptr, 1.0f, 0, 0, n->m2, nullptr, W, 0, 0, s))) return rc;
+            return close_sub(n->m2, L.T(IFA_LT_NORM2B).data, next_norm);
+        }
         if ((rc = ifa_linear_bf16w_act(L.w_in2, N2, W, n->h, W, T, nullptr, 2, c.ops32, n->proj, N2, s))) return rc;
         if ((rc = linear(m, (const bf16_t *)L.T(IFA_LT_FFN_DOWN).data, W, (size_t)sp.ffn, n->proj, N2, T, nullptr, nullptr, 1.0f, 0, n->m2, W))) return rc;
         return close_sub(n->m2, L.T(IFA_LT_NORM2B).data, next_norm);
@@ -908,7 +941,7 @@ int lay_destroy(ifa_model *m)
     for (float *p : n->slot_ptr) lay_free(p);
     lay_free(n->slot_base_dev);
     if (n->tab_pin) (void)hipHostFree(n->tab_pin);
-    lay_free(n->attn_ws);
+    lay_free(n->attn_ws); lay_free(n->a16);
     lay_free(n->tab_dev); lay_free(n->excl_dev); lay_free(n->next_dev); lay_free(n->ring_dev);
     float *bufs[] = {n->x, n->h, n->proj, n->m1, n->m2, n->m3, n->beta, n->decay, n->logits, n->taps};
     for (float *b : bufs) lay_free(b);
@@ -1248,10 +1281,11 @@ int lay_set_option(ifa_model *m, const char *name, int value)
     if (!strcmp(name, "fuse_rows")) { n->opt_fuse_rows = value; drop_step_graph(n); return IFA_OK; }
     if (!strcmp(name, "fuse_post")) { n->opt_fuse_post = value; drop_step_graph(n); return IFA_OK; }
     if (!strcmp(name, "ssm_chunk_min")) { n->opt_ssm_chunk_min = value; return IFA_OK; }
+    if (!strcmp(name, "a16_min")) { n->opt_a16_min = value; return IFA_OK; }
     if (!strcmp(name, "attn_tile_min")) { n->opt_attn_tile_min = value; return IFA_OK; }
     if (!strcmp(name, "graph")) { n->opt_graph = value; drop_step_graph(n); return IFA_OK; }
     if (!strcmp(name, "ops32")) { IFA_HIP_CHECK(hipStreamSynchronize(m->stream)); n->cfg.ops32 = value ? 1 : 0; drop_step_graph(n); return IFA_OK; }
-    return ifa_fail(IFA_ERR_ARG, "ifa_model_set_option: unknown option '%s' (layer-list model: tap_layers, graph, ops32, attn_tile_min, fuse_rows, fuse_post, ssm_chunk_min)", name);
+    return ifa_fail(IFA_ERR_ARG, "ifa_model_set_option: unknown option '%s' (layer-list model: tap_layers, graph, ops32, attn_tile_min, a16_min, fuse_rows, fuse_post, ssm_chunk_min)", name);
 }
 
 int lay_set_excluded(ifa_model *m, const int *ids_host, int cnt)
@@ -1448,6 +1482,7 @@ int lay_decode(ifa_model *m, int first_token, int start_pos, int n_steps, int *o
     if (n->opt_graph && !n->opt_tap_layers && !n->step_exec) {      // (the slot is read from the device tables: one capture serves every slot)
         drop_step_graph(n);
         n->step_expand = false;
+        n->seqs_host.assign(1, ifa_seq_desc{0, 1, start_pos, n->cur_slot});      // (the launches are shaped by it: one sequence, one row)
         IFA_HIP_CHECK(hipStreamSynchronize(m->stream));
         IFA_HIP_CHECK(hipStreamBeginCapture(m->stream, hipStreamCaptureModeThreadLocal));
         rc = enqueue_decode_step(m);

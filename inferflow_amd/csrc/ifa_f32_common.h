@@ -63,6 +63,22 @@ __device__ __forceinline__ float hex_sum(float v)
     return v;
 }
 
+// sum / maximum over the sixteen quads of a wave, for values that are equal within each quad (two DPP steps inside a row, two exchanges between rows)
+__device__ __forceinline__ float quads_sum(float v)
+{
+    v += __int_as_float(__builtin_amdgcn_mov_dpp(__float_as_int(v), 0x141, 0xF, 0xF, true));
+    v += __int_as_float(__builtin_amdgcn_mov_dpp(__float_as_int(v), 0x128, 0xF, 0xF, true));
+    v += __shfl_xor(v, 16, 64);
+    return v + __shfl_xor(v, 32, 64);
+}
+__device__ __forceinline__ float quads_max(float v)
+{
+    v = fmaxf(v, __int_as_float(__builtin_amdgcn_mov_dpp(__float_as_int(v), 0x141, 0xF, 0xF, true)));
+    v = fmaxf(v, __int_as_float(__builtin_amdgcn_mov_dpp(__float_as_int(v), 0x128, 0xF, 0xF, true)));
+    v = fmaxf(v, __shfl_xor(v, 16, 64));
+    return fmaxf(v, __shfl_xor(v, 32, 64));
+}
+
 // sum over a workgroup of up to 1024 threads; red: 17 floats of LDS; every thread gets the result
 __device__ __forceinline__ float block_sum(float v, float *red)
 {

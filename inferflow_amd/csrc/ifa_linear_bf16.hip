@@ -9,8 +9,11 @@
 //   T  > 8    k_lin_mfma: 64 x 64 output tiles, K in steps of 32 through LDS, four waves of 32 x 32 sub-tiles;
 //             OPS32 = false: operands rounded to bfloat16, v_mfma_f32_32x32x16_bf16;
 //             OPS32 = true : operands stay 32-bit, v_mfma_f32_32x32x2_f32 (the exact mode of the worker)
+//   prompts   k_lin_tile<BM, BN> (ifa_linear_bf16_both: activations rounded to bfloat16 beforehand, by their producer or by k_rows_to_bf16): tiles of up to
+//             128 x 128, both operands straight to LDS; the same sums in the same order as k_lin_mfma<false>
 // Accumulation is fp32 in every path.  No atomics, no split K: a result does not depend on what else runs.
 #include <algorithm>
+#include <cstring>
 #include "ifa_host.h"
 #include "ifa_f32_common.h"
 
@@ -32,6 +35,7 @@ struct LinArgs {
     // grouped product (k_lin_mfma only): tile blockIdx.y serves rows [row0, row0 + n) of group g (tile_map {g, row0, n}; *n_tiles valid
     // tiles) with the matrix W + g * N * K; activation row of output row r: A[a_rows[r]] (a_rows null: r); row_scale per output row
     const int *tile_map, *n_tiles, *a_rows; const float *row_scale;
+    bf16_t *C16;                               // (k_lin_tile with act_kind 2: the output in bfloat16 instead of C)
     int act_kind;                              // every output after the bias passes 1: the exact (erf) GELU, 2: the square of relu
 };
 
@@ -146,6 +150,160 @@ __global__ void __launch_bounds__(256) k_lin_mfma(LinArgs P)
     }
 }
 
+// ---- prompts, both operands in bfloat16 already: BM x BN output tiles, K in steps of 64, double-buffered in LDS.  Both operands go from memory to LDS
+// directly (global_load_lds_dwordx4: a wave moves 8 rows x 128 bytes per instruction, a step ahead); both images are [rows][64 halfs] with the eight
+// 16-byte pieces of row r at slot c ^ ((r >> 1) & 7), so that the fragment reads of 16 consecutive lanes (16 rows, one piece) are free of bank conflicts; the
+// loads write LDS linearly, the permutation sits in their SOURCE addresses.  The step's barrier stands before its last group of products: every wave has read
+// its last fragments by then, and the first fragments of the next buffer land under that group.
+// Workgroups are dealt to the eight XCDs round-robin: the id is remapped so that an XCD works on a compact block of tiles whose operands its L2 shares.
+// A's rows are K rounded up to whole steps long, zero beyond K (what W's requests bring in there -- held inside the row -- does not count).
+constexpr int LT_BK = 64;
+typedef __attribute__((address_space(3))) void lt_lds_t;
+typedef const __attribute__((address_space(1))) void lt_glb_t;
+
+template <int BM, int BN>
+__global__ void __launch_bounds__(256, 2) k_lin_tile(LinArgs P, const bf16_t *__restrict__ A16, int lda16, int tiles_m, int tiles_n)
+{
+    constexpr int TA = BM / 64, TB = BN / 64, AI = BM / 32, WI = BN / 32, ROWB = 2 * LT_BK, STEPB = (BM + BN) * ROWB;
+    __shared__ __attribute__((aligned(16))) char smem[2 * STEPB];          // [2 steps][BM rows of A, BN rows of W]
+    const int tid = threadIdx.x, lane = tid & 63, wave = __builtin_amdgcn_readfirstlane(tid >> 6), i = lane & 31, g = lane >> 5, wm = wave & 1, wn = wave >> 1;
+    int t0, n0;
+    {
+        const int nwg = tiles_m * tiles_n, orig = blockIdx.x, xcd = orig & 7, q = nwg >> 3, r = nwg & 7;
+        const int wg = (xcd < r ? xcd * (q + 1) : r * (q + 1) + (xcd - r) * q) + (orig >> 3);
+        constexpr int GM = 1024 / BM;          // bands of 1024 rows of C, the row tiles of a band fastest
+        const int band = wg / (GM * tiles_n), within = wg % (GM * tiles_n), band_m = min(GM, tiles_m - band * GM);
+        t0 = (band * GM + within % band_m) * BM; n0 = (within / band_m) * BN;
+    }
+    auto swz = [](int r) { return (r >> 1) & 7; };
+    const bf16_t *asrc[AI], *wsrc[WI];
+    int wlim[WI];          // furthest step offset of the lane's piece inside a row of W
+#pragma unroll
+    for (int j = 0; j < AI; j++) {
+        const int row = (wave * AI + j) * 8 + (lane >> 3), c = (lane & 7) ^ swz(row);
+        asrc[j] = A16 + (size_t)min(t0 + row, P.T - 1) * lda16 + c * 8;          // (rows beyond the last: repeated, not stored)
+    }
+#pragma unroll
+    for (int j = 0; j < WI; j++) {
+        const int row = (wave * WI + j) * 8 + (lane >> 3), c = (lane & 7) ^ swz(row);
+        wsrc[j] = P.W + (size_t)min(n0 + row, P.N - 1) * P.K + c * 8;
+        wlim[j] = P.K - 8 - c * 8;
+    }
+    auto stage = [&](int step, int buf) {
+        char *As = smem + buf * STEPB, *Ws = As + BM * ROWB;
+#pragma unroll
+        for (int j = 0; j < AI; j++)
+            __builtin_amdgcn_global_load_lds((lt_glb_t *)(asrc[j] + step * LT_BK), (lt_lds_t *)(As + (wave * AI + j) * 1024), 16, 0, 0);
+#pragma unroll
+        for (int j = 0; j < WI; j++)
+            __builtin_amdgcn_global_load_lds((lt_glb_t *)(wsrc[j] + min(step * LT_BK, wlim[j])), (lt_lds_t *)(Ws + (wave * WI + j) * 1024), 16, 0, 0);
+    };
+    const int lc = g ^ swz(i), a_off = (wm * (BM / 2) + i) * ROWB, w_off = (BM + wn * (BN / 2) + i) * ROWB;          // (tile rows start at multiples of 32)
+    f32x16v acc[TA][TB];
+#pragma unroll
+    for (int a = 0; a < TA; a++)
+#pragma unroll
+        for (int b = 0; b < TB; b++)
+#pragma unroll
+            for (int r = 0; r < 16; r++) acc[a][b][r] = 0.0f;
+    bf16x8v af[2][TA], wf[2][TB];
+    auto frags = [&](int buf, int ks, bf16x8v (&fa)[TA], bf16x8v (&fw)[TB]) {
+        const char *base = smem + buf * STEPB;
+        const int so = ((2 * ks) ^ lc) << 4;
+#pragma unroll
+        for (int a = 0; a < TA; a++) fa[a] = *reinterpret_cast<const bf16x8v *>(base + a_off + a * 32 * ROWB + so);
+#pragma unroll
+        for (int b = 0; b < TB; b++) fw[b] = *reinterpret_cast<const bf16x8v *>(base + w_off + b * 32 * ROWB + so);
+    };
+    auto mma = [&](const bf16x8v (&fa)[TA], const bf16x8v (&fw)[TB]) {
+#pragma unroll
+        for (int a = 0; a < TA; a++)
+#pragma unroll
+            for (int b = 0; b < TB; b++) acc[a][b] = __builtin_amdgcn_mfma_f32_32x32x16_bf16(fa[a], fw[b], acc[a][b], 0, 0, 0);
+    };
+    const int nsteps = lda16 / LT_BK;
+    stage(0, 0);
+    __syncthreads();
+    frags(0, 0, af[0], wf[0]);
+    for (int step = 0; step + 1 < nsteps; step++) {
+        const int cur = step & 1;
+        stage(step + 1, cur ^ 1);
+#pragma unroll
+        for (int ks = 0; ks < 3; ks++) {
+            frags(cur, ks + 1, af[(ks + 1) & 1], wf[(ks + 1) & 1]);
+            mma(af[ks & 1], wf[ks & 1]);
+        }
+        __syncthreads();
+        frags(cur ^ 1, 0, af[0], wf[0]);
+        mma(af[1], wf[1]);
+    }
+    {
+        const int cur = (nsteps - 1) & 1;
+#pragma unroll
+        for (int ks = 0; ks < 3; ks++) {
+            frags(cur, ks + 1, af[(ks + 1) & 1], wf[(ks + 1) & 1]);
+            mma(af[ks & 1], wf[ks & 1]);
+        }
+        mma(af[1], wf[1]);
+    }
+    // every (row, column) of the wave's tile: f(C element's place, value behind the bias)
+    auto each = [&](auto f) {
+#pragma unroll
+        for (int b = 0; b < TB; b++) {
+            const int n = n0 + wn * (BN / 2) + 32 * b + i;
+            if (n >= P.N) continue;
+            const float bv = P.bias ? bf2f(P.bias[n]) : 0.0f, mv = P.alpha * (P.mul ? bf2f(P.mul[n]) : 1.0f);
+#pragma unroll
+            for (int a = 0; a < TA; a++)
+#pragma unroll
+                for (int r = 0; r < 16; r++) {
+                    const int t = t0 + wm * (BM / 2) + 32 * a + (r & 3) + 8 * (r >> 2) + 4 * g;
+                    if (t < P.T) f((size_t)t * P.ldc + n, n, acc[a][b][r] + bv, mv);
+                }
+        }
+    };
+    if (P.act_kind == 2) {
+        if (P.C16) each([&](size_t at, int, float v, float mv) { v = fmaxf(v, 0.0f); P.C16[at] = __builtin_bit_cast(bf16_t, (__bf16)(v * v * mv)); });
+        else each([&](size_t at, int, float v, float mv) { v = fmaxf(v, 0.0f); P.C[at] = v * v * mv; });
+    } else if (P.act_kind == 0 && P.act_c0 >= P.act_c1) {
+        if (P.accumulate) each([&](size_t at, int, float v, float mv) { P.C[at] += v * mv; });
+        else each([&](size_t at, int, float v, float mv) { P.C[at] = v * mv; });
+    } else {
+        each([&](size_t at, int n, float v, float mv) {
+            if (n >= P.act_c0 && n < P.act_c1) v = silu_exact(v);
+            if (P.act_kind == 1) v = 0.5f * v * (1.0f + erff(v * 0.70710678118654752f));
+            P.C[at] = P.accumulate ? P.C[at] + v * mv : v * mv;
+        });
+    }
+}
+
+template <int BM, int BN>
+void launch_lin_tile(const LinArgs &P, const bf16_t *a16, size_t lda16, hipStream_t s)
+{
+    const int tm = (P.T + BM - 1) / BM, tn = (P.N + BN - 1) / BN;
+    hipLaunchKernelGGL((k_lin_tile<BM, BN>), dim3((unsigned)tm * (unsigned)tn), dim3(256), 0, s, P, a16, (int)lda16, tm, tn);
+}
+
+// rows of 32-bit values to bfloat16, zero up to ldy (a multiple of 8)
+__global__ void __launch_bounds__(256) k_rows_to_bf16(const float *__restrict__ x, size_t ldx, int cols, bf16_t *__restrict__ y, int ldy, int vec)
+{
+    const float *xr = x + (size_t)blockIdx.y * ldx;
+    const int c = (blockIdx.x * 256 + threadIdx.x) * 8;
+    if (c >= ldy) return;
+    float v[8];
+    if (vec && c + 8 <= cols) {
+        const float4 a = *reinterpret_cast<const float4 *>(xr + c), b = *reinterpret_cast<const float4 *>(xr + c + 4);
+        v[0] = a.x; v[1] = a.y; v[2] = a.z; v[3] = a.w; v[4] = b.x; v[5] = b.y; v[6] = b.z; v[7] = b.w;
+    } else {
+#pragma unroll
+        for (int e = 0; e < 8; e++) v[e] = c + e < cols ? xr[c + e] : 0.0f;
+    }
+    bf16x8v h;
+#pragma unroll
+    for (int e = 0; e < 8; e++) h[e] = (__bf16)v[e];
+    *reinterpret_cast<bf16x8v *>(y + (size_t)blockIdx.y * ldy + c) = h;
+}
+
 // T <= TT rows; one wave per output row at a time.  PRO: what the activations pass as they are read (steps of a few rows are bound
 // by launches and dependent loads, not arithmetic, so the neighbouring element-wise launch is folded in here):
 //   1  layer norm without bias: a = (x - mean) / sqrt(var + eps) * w[k]   (every wave forms mean and variance of the T rows itself)
@@ -238,7 +396,7 @@ static int linear_launch(const void *w_bf16, size_t rows, size_t cols, const voi
     P.T = (int)tokens; P.N = (int)rows; P.K = (int)cols; P.lda = (int)lda; P.ldc = (int)ldc;
     P.alpha = alpha; P.accumulate = accumulate ? 1 : 0; P.act_c0 = silu_col0; P.act_c1 = silu_col1;
     P.norm_w = (const bf16_t *)norm_w_bf16; P.norm_eps = norm_eps;
-    P.tile_map = P.n_tiles = P.a_rows = nullptr; P.row_scale = nullptr; P.act_kind = act;
+    P.tile_map = P.n_tiles = P.a_rows = nullptr; P.row_scale = nullptr; P.act_kind = act; P.C16 = nullptr;
     // 16-byte requests need whole 8-element pieces in every row of both operands
     P.vec = (cols % 8 == 0 && lda % 4 == 0 && ((uintptr_t)a_f32 & 15) == 0 && ((uintptr_t)w_bf16 & 15) == 0) ? 1 : 0;
     hipStream_t s = ifa_s(stream);
@@ -271,6 +429,45 @@ extern "C" int ifa_linear_bf16w(const void *w_bf16, size_t rows, size_t cols, co
                          stream, "ifa_linear_bf16w");
 }
 
+extern "C" int ifa_rows_to_bf16(const void *x_f32, size_t ldx, size_t rows, size_t cols, void *y_bf16, size_t ldy, ifa_stream stream)
+{
+    IFA_REQUIRE(x_f32 && y_bf16, "ifa_rows_to_bf16: null pointer");
+    IFA_REQUIRE(rows > 0 && rows < 65536u * 16u && cols > 0 && ldx >= cols && ldy >= cols && ldy % 8 == 0 && ldy < (1u << 30) && ((uintptr_t)y_bf16 & 15) == 0, "ifa_rows_to_bf16: bad shape");
+    const int vec = ldx % 4 == 0 && ((uintptr_t)x_f32 & 15) == 0;
+    for (size_t r0 = 0; r0 < rows; r0 += 65535) {
+        const size_t n = std::min<size_t>(65535, rows - r0);
+        hipLaunchKernelGGL(k_rows_to_bf16, dim3(ifa_cdiv(ldy / 8, 256), (unsigned)n), dim3(256), 0, ifa_s(stream), (const float *)x_f32 + r0 * ldx, ldx, (int)cols,
+                           (bf16_t *)y_bf16 + r0 * ldy, (int)ldy, vec);
+    }
+    IFA_LAUNCH_CHECK();
+    return IFA_OK;
+}
+
+extern "C" int ifa_linear_bf16_both(const void *w_bf16, size_t rows, size_t cols, const void *a_bf16, size_t lda, size_t tokens, const void *bias_bf16, const void *mul_bf16,
+                                    float alpha, int accumulate, int act, void *c_f32, void *c_bf16, size_t ldc, int silu_col0, int silu_col1, ifa_stream stream)
+{
+    IFA_REQUIRE(w_bf16 && a_bf16 && (c_f32 || c_bf16), "ifa_linear_bf16_both: null pointer");
+    IFA_REQUIRE(rows > 0 && cols >= (size_t)LT_BK && cols % 8 == 0 && tokens > 0 && lda % 64 == 0 && lda >= cols && lda - cols < 64 && ldc >= rows && act >= 0 && act <= 2,
+                "ifa_linear_bf16_both: bad shape (%zu x %zu, %zu tokens, lda %zu)", rows, cols, tokens, lda);
+    IFA_REQUIRE(!c_bf16 || (act == 2 && !accumulate), "ifa_linear_bf16_both: a bfloat16 output goes with the squared relu and no accumulation");
+    IFA_REQUIRE(rows < (1u << 30) && cols < (1u << 30) && tokens < (1u << 30) && (((uintptr_t)a_bf16 | (uintptr_t)w_bf16) & 15) == 0, "ifa_linear_bf16_both: dimension too large or unaligned operand");
+    LinArgs P;
+    memset(&P, 0, sizeof(P));
+    P.W = (const bf16_t *)w_bf16; P.C = (float *)c_f32; P.C16 = (bf16_t *)c_bf16; P.bias = (const bf16_t *)bias_bf16; P.mul = (const bf16_t *)mul_bf16;
+    P.T = (int)tokens; P.N = (int)rows; P.K = (int)cols; P.ldc = (int)ldc; P.alpha = alpha; P.accumulate = accumulate ? 1 : 0; P.act_c0 = silu_col0; P.act_c1 = silu_col1;
+    P.act_kind = act;
+    hipStream_t s = ifa_s(stream);
+    const bf16_t *a = (const bf16_t *)a_bf16;
+    // the largest tile that still gives every compute unit its share of workgroups
+    const size_t t128 = (tokens + 127) / 128, n128 = (rows + 127) / 128, n64 = (rows + 63) / 64;
+    IFA_REQUIRE(((tokens + 63) / 64) * n64 < (1u << 31), "ifa_linear_bf16_both: too many tiles");
+    if (t128 * n128 >= 384) launch_lin_tile<128, 128>(P, a, lda, s);
+    else if (t128 * n64 >= 256) launch_lin_tile<128, 64>(P, a, lda, s);
+    else launch_lin_tile<64, 64>(P, a, lda, s);
+    IFA_LAUNCH_CHECK();
+    return IFA_OK;
+}
+
 extern "C" int ifa_linear_bf16w_act(const void *w_bf16, size_t rows, size_t cols, const void *a_f32, size_t lda, size_t tokens, const void *bias_bf16, int act,
                                     int ops32, void *c_f32, size_t ldc, ifa_stream stream)
 {
@@ -301,7 +498,7 @@ extern "C" int ifa_linear_bf16w_grouped(const void *w_bf16, size_t rows, size_t 
     P.W = (const bf16_t *)w_bf16; P.A = (const float *)a_f32; P.C = (float *)c_f32; P.bias = nullptr; P.mul = nullptr;
     P.T = 0; P.N = (int)rows; P.K = (int)cols; P.lda = (int)lda; P.ldc = (int)ldc; P.alpha = 1.0f; P.accumulate = 0; P.act_c0 = P.act_c1 = 0;
     P.norm_w = nullptr; P.norm_eps = 0.0f;
-    P.tile_map = tile_map_dev; P.n_tiles = n_tiles_dev; P.a_rows = a_rows_dev; P.row_scale = (const float *)row_scale_f32; P.act_kind = act;
+    P.tile_map = tile_map_dev; P.n_tiles = n_tiles_dev; P.a_rows = a_rows_dev; P.row_scale = (const float *)row_scale_f32; P.act_kind = act; P.C16 = nullptr;
     P.vec = (cols % 8 == 0 && lda % 4 == 0 && ((uintptr_t)a_f32 & 15) == 0 && ((uintptr_t)w_bf16 & 15) == 0 && (rows * cols) % 8 == 0) ? 1 : 0;
     const dim3 grid(ifa_cdiv(rows, LM_N), (unsigned)max_tiles);
     if (ops32) hipLaunchKernelGGL(k_lin_mfma<true>, grid, dim3(256), 0, ifa_s(stream), P);

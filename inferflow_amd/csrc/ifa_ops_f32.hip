@@ -189,6 +189,63 @@ __global__ void __launch_bounds__(256) k_norm_add_norm(float *__restrict__ x, si
     for (int c = threadIdx.x; c < cols; c += blockDim.x) hr[c] = xr[c] * rinv2 * (w_off + bf2f(w_before[c]));
 }
 
+// The same (m null: h alone) with the row in registers: every thread holds PIECES pieces of four values, and everything the row needs (x, m, both weights) is requested
+// before the first reduction.  cols % 4 == 0, cols <= 4 PIECES blockDim, 16-byte aligned rows, 8-byte aligned weights.
+template <int PIECES>
+__global__ void __launch_bounds__(1024) k_norm_add_norm_reg(float *__restrict__ x, size_t ldx, int cols, const float *__restrict__ m, size_t ldm,
+                                                            const bf16_t *__restrict__ w_after, const bf16_t *__restrict__ w_before, float w_off, float eps,
+                                                            float *__restrict__ h, size_t ldh)
+{
+    __shared__ float red[17];
+    float *xr = x + (size_t)blockIdx.x * ldx;
+    const float *mr = m ? m + (size_t)blockIdx.x * ldm : xr;
+    float xv[PIECES][4], mv[PIECES][4];
+    uint2 wa[PIECES], wb[PIECES];
+    float q = 0.0f;
+#pragma unroll
+    for (int p = 0; p < PIECES; p++) {
+        const int c = 4 * (threadIdx.x + p * blockDim.x);
+        float4 a = make_float4(0.f, 0.f, 0.f, 0.f), b = a;
+        wa[p] = wb[p] = make_uint2(0u, 0u);
+        if (c < cols) {
+            a = *reinterpret_cast<const float4 *>(mr + c); b = *reinterpret_cast<const float4 *>(xr + c);
+            if (m) wa[p] = *reinterpret_cast<const uint2 *>(w_after + c);
+            if (w_before) wb[p] = *reinterpret_cast<const uint2 *>(w_before + c);
+        }
+        mv[p][0] = a.x; mv[p][1] = a.y; mv[p][2] = a.z; mv[p][3] = a.w; xv[p][0] = b.x; xv[p][1] = b.y; xv[p][2] = b.z; xv[p][3] = b.w;
+    }
+#pragma unroll
+    for (int p = 0; p < PIECES; p++)
+#pragma unroll
+        for (int e = 0; e < 4; e++) q = fmaf(mv[p][e], mv[p][e], q);
+    auto weight = [&](const uint2 &w, int e) { const uint32_t u = e < 2 ? w.x : w.y; return w_off + __uint_as_float((e & 1) ? (u & 0xFFFF0000u) : (u << 16)); };
+    const float rinv = 1.0f / sqrtf(block_sum(q, red) / (float)cols + eps);
+    float rinv2 = rinv;
+    if (m) {
+        float q2 = 0.0f;
+#pragma unroll
+        for (int p = 0; p < PIECES; p++) {
+            const int c = 4 * (threadIdx.x + p * blockDim.x);
+            if (c >= cols) continue;
+#pragma unroll
+            for (int e = 0; e < 4; e++) { xv[p][e] += mv[p][e] * rinv * weight(wa[p], e); q2 = fmaf(xv[p][e], xv[p][e], q2); }
+            *reinterpret_cast<float4 *>(xr + c) = make_float4(xv[p][0], xv[p][1], xv[p][2], xv[p][3]);
+        }
+        if (!w_before) return;
+        rinv2 = 1.0f / sqrtf(block_sum(q2, red) / (float)cols + eps);
+    }
+    float *hr = h + (size_t)blockIdx.x * ldh;
+#pragma unroll
+    for (int p = 0; p < PIECES; p++) {
+        const int c = 4 * (threadIdx.x + p * blockDim.x);
+        if (c >= cols) continue;
+        float o[4];
+#pragma unroll
+        for (int e = 0; e < 4; e++) o[e] = xv[p][e] * rinv2 * weight(wb[p], e);
+        *reinterpret_cast<float4 *>(hr + c) = make_float4(o[0], o[1], o[2], o[3]);
+    }
+}
+
 // one workgroup per row (ifa_streams.h)
 template <int SMAX, bool VEC>
 __global__ void __launch_bounds__(1024) k_streams_step(StreamArgs P)
@@ -243,11 +300,21 @@ __global__ void __launch_bounds__(1024) k_argmax_f32(const float *__restrict__ l
     int ex[3] = {-1, -1, -1};
     if (excluded) { const int ne = min(excluded[0], 3); for (int e = 0; e < ne; e++) ex[e] = excluded[1 + e]; }
     float best = -INFINITY; int idx = 0x7FFFFFFF;
-    for (int c = threadIdx.x; c < n; c += blockDim.x) {
-        if (c == ex[0] || c == ex[1] || c == ex[2]) continue;
-        const float v = r[c];
-        if (v > best || (v == best && c < idx)) { best = v; idx = c; }
+    auto take = [&](float v, int c) { if (c != ex[0] && c != ex[1] && c != ex[2] && (v > best || (v == best && c < idx))) { best = v; idx = c; } };
+    int c0 = 0;
+    if (((uintptr_t)r & 15) == 0) {          // 16-byte pieces, four requested side by side
+        for (; c0 + 16 * (int)blockDim.x <= n; c0 += 16 * blockDim.x) {
+            float4 v[4];
+#pragma unroll
+            for (int u = 0; u < 4; u++) v[u] = *reinterpret_cast<const float4 *>(r + c0 + 4 * (threadIdx.x + u * blockDim.x));
+#pragma unroll
+            for (int u = 0; u < 4; u++) {
+                const int c = c0 + 4 * (threadIdx.x + u * blockDim.x);
+                take(v[u].x, c); take(v[u].y, c + 1); take(v[u].z, c + 2); take(v[u].w, c + 3);
+            }
+        }
     }
+    for (int c = c0 + threadIdx.x; c < n; c += blockDim.x) take(r[c], c);
     for (int o = 32; o > 0; o >>= 1) {
         const float ov = __shfl_xor(best, o, 64); const int oi = __shfl_xor(idx, o, 64);
         if (ov > best || (ov == best && oi < idx)) { best = ov; idx = oi; }
@@ -413,12 +480,33 @@ int ifa_add_rows_vec_f32(void *x_f32, size_t ldx, size_t rows, size_t cols, cons
     return IFA_OK;
 }
 
+// launches k_norm_add_norm_reg where the row fits the registers and every access is aligned; false: nothing launched
+static bool norm_add_norm_reg(void *x, size_t ldx, size_t rows, size_t cols, const void *m, size_t ldm, const void *w_after, const void *w_before, float w_offset, float eps,
+                              void *h, size_t ldh, ifa_stream stream)
+{
+    const size_t quads = cols / 4;
+    const bool vec = cols % 4 == 0 && ldx % 4 == 0 && (!m || ldm % 4 == 0) && (((uintptr_t)x | (uintptr_t)m) & 15) == 0 && ((uintptr_t)w_after & 7) == 0
+                     && (!w_before || (ldh % 4 == 0 && ((uintptr_t)h & 15) == 0 && ((uintptr_t)w_before & 7) == 0));
+    if (!vec || quads > 2048) return false;
+    const int pieces = quads <= 1024 ? 1 : 2;          // one piece of four values per thread up to 4096 columns, two beyond
+    const unsigned threads = (unsigned)((quads + 64 * pieces - 1) / (64 * pieces)) * 64;
+#define IFA_NAN(P) hipLaunchKernelGGL(k_norm_add_norm_reg<P>, dim3((unsigned)rows), dim3(threads), 0, ifa_s(stream), (float *)x, ldx, (int)cols, (const float *)m, ldm, \
+                                      (const bf16_t *)w_after, (const bf16_t *)w_before, w_offset, eps, (float *)h, ldh)
+    if (pieces == 1) IFA_NAN(1); else IFA_NAN(2);
+#undef IFA_NAN
+    return true;
+}
+
 int ifa_rmsnorm_offset_f32(const void *x_f32, size_t ldx, size_t rows, size_t cols, const void *w_bf16, float w_offset, float eps, int accumulate,
                            void *y_f32, size_t ldy, ifa_stream stream)
 {
     IFA_REQUIRE(x_f32 && y_f32, "ifa_rmsnorm_offset_f32: null pointer");
     IFA_REQUIRE(rows > 0 && cols > 0 && ldx >= cols && ldy >= cols, "ifa_rmsnorm_offset_f32: bad arguments");
     IFA_REQUIRE(!accumulate || x_f32 != y_f32, "ifa_rmsnorm_offset_f32: accumulating a row's norm into the row itself");
+    if (!accumulate && w_bf16 && norm_add_norm_reg((void *)x_f32, ldx, rows, cols, nullptr, 0, nullptr, w_bf16, w_offset, eps, y_f32, ldy, stream)) {
+        IFA_LAUNCH_CHECK();
+        return IFA_OK;
+    }
     hipLaunchKernelGGL(k_rmsnorm_offset, dim3((unsigned)rows), dim3(256), 0, ifa_s(stream), (const float *)x_f32, ldx, (int)cols, (const bf16_t *)w_bf16, w_offset, eps,
                        accumulate ? 1 : 0, (float *)y_f32, ldy);
     IFA_LAUNCH_CHECK();
@@ -469,6 +557,10 @@ int ifa_norm_add_norm_f32(void *x_f32, size_t ldx, size_t rows, size_t cols, con
 {
     IFA_REQUIRE(x_f32 && m_f32 && w_after_bf16 && (!w_before_bf16 || h_f32), "ifa_norm_add_norm_f32: null pointer");
     IFA_REQUIRE(rows > 0 && cols > 0 && ldx >= cols && ldm >= cols && (!w_before_bf16 || ldh >= cols) && x_f32 != m_f32, "ifa_norm_add_norm_f32: bad arguments");
+    if (norm_add_norm_reg(x_f32, ldx, rows, cols, m_f32, ldm, w_after_bf16, w_before_bf16, w_offset, eps, h_f32, ldh, stream)) {
+        IFA_LAUNCH_CHECK();
+        return IFA_OK;
+    }
     hipLaunchKernelGGL(k_norm_add_norm, dim3((unsigned)rows), dim3(256), 0, ifa_s(stream), (float *)x_f32, ldx, (int)cols, (const float *)m_f32, ldm,
                        (const bf16_t *)w_after_bf16, (const bf16_t *)w_before_bf16, w_offset, eps, (float *)h_f32, ldh);
     IFA_LAUNCH_CHECK();

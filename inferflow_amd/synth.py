@@ -341,6 +341,48 @@ def kamelorn_tensor_shapes(cfg):
     return s
 
 
+def rosilix_config(width=2048, vocab=32000, heads=16, kv_heads=4, dim=64, vdim=128, rot_dims=64, chunk=1280, lat_heads=16, lat_dim=128, lat_rot_dim=64, lat_vdim=128,
+                   kv_rank=512, ff=8192):
+    """eight layers: twice (latent attention, latent attention on the first one's rows, differential attention, differential attention), each with the dense
+    feed-forward"""
+    def lat(kv_from=None):
+        mx = {"heads": lat_heads, "dim": lat_dim, "rot_dim": lat_rot_dim, "vdim": lat_vdim, "kv_rank": kv_rank, "scale": float((lat_dim + lat_rot_dim) ** -0.5),
+              "rot": {"base": 1e6, "dims": lat_rot_dim}}
+        if kv_from is not None:
+            mx["kv_from"] = kv_from
+        return {"type": "latent_attention", "mixer": mx, "mlp": {"kind": "dense", "ff": ff}}
+    att = {"type": "attention", "mlp": {"kind": "dense", "ff": ff},
+           "mixer": {"heads": heads, "kv_heads": kv_heads, "dim": dim, "vdim": vdim, "scale": float(dim ** -0.5), "diff": 0.5, "mask": {"size": chunk},
+                     "rot": {"base": 10000.0, "dims": rot_dims}}}
+    return {"architecture": "Rosilix", "width": width, "vocab": vocab, "norm": {"eps": 1e-6}, "embedding": {"scale": float(width ** 0.5)},
+            "layers": [lat(), lat(0), att, att, lat(), lat(4), att, att]}
+
+
+def rosilix_tensor_shapes(cfg):
+    W_, V = cfg["width"], cfg["vocab"]
+    s = {"embed": (V, W_), "final.norm": (W_,), "head": (V, W_)}
+    for li, L in enumerate(cfg["layers"]):
+        p, m = "l%d." % li, L["mixer"]
+        s.update({p + "norm1": (W_,), p + "norm1b": (W_,)})
+        if L["type"] == "latent_attention":
+            H, dn, dr, dv, R = m["heads"], m["dim"], m["rot_dim"], m["vdim"], m["kv_rank"]
+            s.update({p + "mix.q": (H * (dn + dr), W_), p + "mix.uk": (H * dn, R), p + "mix.uv": (H * dv, R), p + "mix.sink": (H,), p + "mix.g": (H, W_), p + "mix.o": (W_, H * dv)})
+            if m.get("kv_from") is None:
+                s.update({p + "mix.dkv": (R + dr, W_), p + "mix.dkv.norm": (R,)})
+        else:
+            H, G, D, DV = m["heads"], m["kv_heads"], m["dim"], m["vdim"]
+            s.update({p + "mix.q": (2 * H * D, W_), p + "mix.k": (2 * G * D, W_), p + "mix.v": (G * DV, W_), p + "mix.lq1": (D,), p + "mix.lk1": (D,), p + "mix.lq2": (D,),
+                      p + "mix.lk2": (D,), p + "mix.g": (H, W_), p + "mix.o": (W_, H * DV)})
+        if L.get("mlp"):
+            F = L["mlp"]["ff"]
+            s.update({p + "norm2": (W_,), p + "norm2b": (W_,), p + "mlp.up": (F, W_), p + "mlp.down": (W_, F)})
+    return s
+
+
+def write_rosilix_dir(path, cfg, seed=0):
+    return write_gelarax_dir(path, cfg, seed, rosilix_tensor_shapes(cfg))
+
+
 def write_kamelorn_dir(path, cfg, seed=0):
     return write_gelarax_dir(path, cfg, seed, kamelorn_tensor_shapes(cfg))
 
@@ -384,7 +426,7 @@ def write_gelarax_dir(path, cfg, seed=0, shapes=None):
             leaf = name.split(".")[-1]
             if cfg.get("architecture") == "Sopulorn" and len(shape) == 1 and (leaf in ("norm1", "norm2", "norm1b", "norm2b") or name == "final.norm"):
                 a = 0.05 * rng.standard_normal(shape, dtype=np.float32)          # (this design's norms multiply by one plus the stored weight)
-            elif len(shape) == 1 and leaf in ("norm1", "norm2", "norm", "ls1", "ls2"):
+            elif len(shape) == 1 and leaf in ("norm1", "norm2", "norm1b", "norm2b", "norm", "ls1", "ls2"):
                 a = 1.0 + 0.05 * rng.standard_normal(shape, dtype=np.float32)
             elif leaf == "alpha":
                 a = np.full(shape, 0.5, np.float32)          # (the scalar of an element-wise tanh norm)

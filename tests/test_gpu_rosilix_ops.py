@@ -266,7 +266,57 @@ def test_squared_relu_in_the_epilogue(T, N, K):
     assert capi().ifa_linear_bf16w_act(p(devbf(Wm)), N, K, p(dev32(A)), K + 4, T, None, 3, 1, p(out), N + 2, None) != 0
 
 
-@pytest.mark.parametrize("rows,cols", [(1, 64), (5, 97), (3, 4096)])
+@pytest.mark.parametrize("T,N,K", [(1, 1, 64), (17, 64, 64), (200, 70, 80), (65, 130, 136), (1100, 1930, 200), (1025, 2049, 72), (2500, 2600, 72), (2561, 2432, 328), (300, 520, 2048)])
+def test_products_of_prompts_in_every_tile(T, N, K):
+    """row and column counts on both sides of the tiles' borders, inner sizes that are no multiple of a step; every epilogue; the same numbers as the product that
+    rounds its activations itself"""
+    rng = np.random.default_rng(T + N + K)
+    Wm, A, b = bf16_round(rng.standard_normal((N, K))), rng.standard_normal((T, K + 4)).astype(np.float32), bf16_round(rng.standard_normal(N))
+    mul, C0 = bf16_round(rng.standard_normal(N)), rng.standard_normal((T, N + 2)).astype(np.float32)
+    prod = orc.f64(bf16_round(A)[:, :K]) @ orc.f64(Wm).T
+    wd, ad, bd, md, L = devbf(Wm), dev32(A), devbf(b), devbf(mul), capi()
+    ld = (K + 63) // 64 * 64
+    a16 = torch.full((T, ld), -1, dtype=torch.int16, device="cuda")
+    ia.check(L.ifa_rows_to_bf16(p(ad), K + 4, T, K, p(a16), ld, None)); sync()
+    bits = a16.cpu().numpy().view(np.uint16)
+    assert np.array_equal((bits.astype(np.uint32) << 16).view(np.float32)[:, :K], bf16_round(A)[:, :K]) and np.all(bits[:, K:] == 0)
+    # bias, SiLU on a column range, scale per column, accumulation
+    c = dev32(C0)
+    ia.check(L.ifa_linear_bf16_both(p(wd), N, K, p(a16), ld, T, p(bd), p(md), 0.7, 1, 0, p(c), None, N + 2, 3, min(N, 41), None)); sync()
+    want = prod + orc.f64(b)
+    want[:, 3:min(N, 41)] *= orc.logistic(want[:, 3:min(N, 41)])
+    assert near(c.cpu().numpy()[:, :N], C0[:, :N] + want * orc.f64(mul) * 0.7, 1e-5) and np.array_equal(c.cpu().numpy()[:, N:], C0[:, N:])
+    # plain, against the other product too (from 9 rows on it rounds its activations)
+    out, other = (torch.full((T, N), 7.0, dtype=torch.float32, device="cuda") for _ in range(2))
+    ia.check(L.ifa_linear_bf16_both(p(wd), N, K, p(a16), ld, T, None, None, 1.0, 0, 0, p(out), None, N, 0, 0, None))
+    ia.check(L.ifa_linear_bf16w(p(wd), N, K, p(ad), K + 4, T, None, None, 1.0, 0, 0, p(other), N, 0, 0, None)); sync()
+    assert near(out.cpu().numpy(), prod, 1e-5) and (T <= 8 or torch.equal(out, other))
+    # residual update; the squared relu in both output formats; erf-GELU
+    ia.check(L.ifa_linear_bf16_both(p(wd), N, K, p(a16), ld, T, p(bd), None, 1.0, 1, 0, p(out), None, N, 0, 0, None)); sync()
+    assert near(out.cpu().numpy(), 2 * prod + orc.f64(b), 1e-5)
+    h = torch.zeros((T, N), dtype=torch.int16, device="cuda")
+    ia.check(L.ifa_linear_bf16_both(p(wd), N, K, p(a16), ld, T, None, None, 1.0, 0, 2, p(out), None, N, 0, 0, None))
+    ia.check(L.ifa_linear_bf16_both(p(wd), N, K, p(a16), ld, T, None, None, 1.0, 0, 2, None, p(h), N, 0, 0, None)); sync()
+    assert near(out.cpu().numpy(), np.maximum(prod, 0) ** 2, 1e-5)
+    assert np.array_equal((h.cpu().numpy().view(np.uint16).astype(np.uint32) << 16).view(np.float32), bf16_round(out.cpu().numpy()))
+    ia.check(L.ifa_linear_bf16_both(p(wd), N, K, p(a16), ld, T, p(bd), None, 1.0, 0, 1, p(out), None, N, 0, 0, None)); sync()
+    z = torch.from_numpy(prod + orc.f64(b))
+    assert near(out.cpu().numpy(), torch.nn.functional.gelu(z).numpy(), 1e-5)
+
+
+def test_products_of_prompts_decline_bad_arguments():
+    L = capi()
+    z = torch.zeros(1 << 16, dtype=torch.float32, device="cuda")
+
+    def rc(N=8, K=64, ld=64, T=4, acc=0, act=0, c=True, h=False, ldc=8):
+        return L.ifa_linear_bf16_both(p(z), N, K, p(z), ld, T, None, None, 1.0, acc, act, p(z) if c else None, p(z) if h else None, ldc, 0, 0, None)
+    assert rc() == 0
+    for bad in (dict(K=56), dict(K=68), dict(ld=72), dict(ld=128), dict(T=0), dict(act=3), dict(c=False), dict(h=True), dict(h=True, act=2, acc=1), dict(ldc=7)):
+        assert rc(**bad) != 0, bad
+    sync()
+
+
+@pytest.mark.parametrize("rows,cols", [(1, 64), (5, 97), (3, 4096), (2, 4100), (3, 8192), (2, 9000), (9, 12)])
 def test_norms_on_both_sides_with_plain_weights(rows, cols):
     rng = np.random.default_rng(cols)
     x, m = (rng.standard_normal((rows, cols)).astype(np.float32) for _ in range(2))
