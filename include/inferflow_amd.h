@@ -766,14 +766,14 @@ int ifa_attention_latent_tile_gated_f32(int gate_cols, const void *q_f32, size_t
                                         const void *seqs_dev, const void *seqs_host, int n_seqs, void *const *slot_base_dev, size_t cache_off,
                                         void *out_f32, size_t ldo, ifa_stream stream);
 /* the two forms above with a learned sink per head (sink_bf16 [heads], null: none): exp(sink[h]) joins the softmax's denominator, once, unscaled, with no
- * key and no value */
+ * key and no value; out_bf16 (not null): the tiled form's output in bfloat16 instead of out_f32 */
 int ifa_attention_latent_rows_sinks_f32(const void *qa_f32, size_t ldqa, int heads, int kv_rank, int rot_dim, float scale, const void *sink_bf16, const void *seqs_dev,
                                         const int *row_seq_dev, size_t rows, void *const *slot_base_dev, size_t cache_off, int max_keys, void *ws_f32,
                                         size_t ws_bytes, void *out_f32, size_t ldo, ifa_stream stream);
 int ifa_attention_latent_tile_sinks_f32(int gate_cols, const void *q_f32, size_t ldq, int heads, int dim, int rot_dim, int vdim, int kv_rank, float scale,
                                         const void *sink_bf16, const void *kx_f32, size_t ldkx, const void *vx_f32, size_t ldvx, const int *ctx0_dev, const void *g_f32,
                                         size_t ldg, const void *seqs_dev, const void *seqs_host, int n_seqs, void *const *slot_base_dev, size_t cache_off, void *out_f32,
-                                        size_t ldo, ifa_stream stream);
+                                        void *out_bf16, size_t ldo, ifa_stream stream);
 /* the queries' part of ifa_latent_prepare_pairs_f32 alone (a layer that reads another layer's cache rows): the rotated part of every query head in place */
 int ifa_latent_rotate_q_f32(int pairing, int rot_dim, int rot_dims, void *q_f32, size_t ldq, int heads, int dim, const double *freq_f64_dev, float rot_mult,
                             const void *seqs_dev, const int *row_seq_dev, size_t rows, ifa_stream stream);
@@ -788,11 +788,16 @@ int ifa_qk_rope_store_pairs_f32(int pairing, void *q_f32, size_t ldq, int heads,
  * out = o / sqrt(mean(o^2) + eps) * out_scale * sigmoid(g[t][h]) (g null: no gate).  Steps whose longest sequence brings tile_min_rows rows or more run 64
  * queries of one sequence per workgroup on the fp32 matrix cores (dim <= 128, vdim <= 128 or 193 .. 256); others a workgroup per (row, up to four heads
  * of a group, share of the keys) through ws_f32 (rows * heads * shares * 2 * (vdim + 2) floats; max_keys > 0 bounds the shares) and a second launch that merges
- * the shares, takes the difference, norms and gates.  dim, vdim <= 1024. */
+ * the shares, takes the difference, norms and gates.  out_bf16 (not null, tiled form only): the output in bfloat16 instead of out_f32.  dim, vdim <= 1024. */
 int ifa_attention_diff_f32(const void *q_f32, size_t ldq, int heads, int kv_heads, int dim, int vdim, float scale, int window, int chunk, float lambda, float out_scale,
                            float eps, const void *g_f32, size_t ldg, const void *seqs_dev, const int *row_seq_dev, size_t rows, void *const *slot_base_dev, size_t k_off,
-                           size_t v_off, void *out_f32, size_t ldo, const void *seqs_host, int n_seqs, int tile_min_rows, int max_keys, void *ws_f32, size_t ws_bytes,
-                           ifa_stream stream);
+                           size_t v_off, void *out_f32, void *out_bf16, size_t ldo, const void *seqs_host, int n_seqs, int tile_min_rows, int max_keys, void *ws_f32,
+                           size_t ws_bytes, ifa_stream stream);
+/* 1 if the tiled form serves these head sizes */
+int ifa_attention_diff_tile_fits(int dim, int vdim);
+/* ifa_norm_add_norm_f32 with h in bfloat16 (what a product over bfloat16 activations reads); m_f32 null: h alone.  cols % 4 == 0, at most 8192 */
+int ifa_norm_add_norm_to_bf16(void *x_f32, size_t ldx, size_t rows, size_t cols, const void *m_f32, size_t ldm, const void *w_after_bf16, const void *w_before_bf16,
+                              float w_offset, float eps, void *h_bf16, size_t ldh, ifa_stream stream);
 /* rows of 32-bit values rounded to bfloat16 (to nearest even), zero from cols to ldy (a multiple of 8) */
 int ifa_rows_to_bf16(const void *x_f32, size_t ldx, size_t rows, size_t cols, void *y_bf16, size_t ldy, ifa_stream stream);
 /* ifa_linear_bf16w (ops32 0) over activations that are bfloat16 already: a_bf16 [tokens][lda], lda = cols rounded up to whole 64s, zero beyond cols (cols % 8 ==

@@ -215,10 +215,12 @@ SIGNATURES = {
     "ifa_latent_expand_out_gated_f32": (_i, [_i, _vp, _sz, _i, _i, _i, _i, _vp, _vp, _sz, _sz, _vp, _sz, _vp]),
     "ifa_attention_latent_tile_gated_f32": (_i, [_i, _vp, _sz, _i, _i, _i, _i, _i, _f, _vp, _sz, _vp, _sz, _vp, _vp, _sz, _vp, _vp, _i, _vp, _sz, _vp, _sz, _vp]),
     "ifa_attention_latent_rows_sinks_f32": (_i, [_vp, _sz, _i, _i, _i, _f, _vp, _vp, _vp, _sz, _vp, _sz, _i, _vp, _sz, _vp, _sz, _vp]),
-    "ifa_attention_latent_tile_sinks_f32": (_i, [_i, _vp, _sz, _i, _i, _i, _i, _i, _f, _vp, _vp, _sz, _vp, _sz, _vp, _vp, _sz, _vp, _vp, _i, _vp, _sz, _vp, _sz, _vp]),
+    "ifa_attention_latent_tile_sinks_f32": (_i, [_i, _vp, _sz, _i, _i, _i, _i, _i, _f, _vp, _vp, _sz, _vp, _sz, _vp, _vp, _sz, _vp, _vp, _i, _vp, _sz, _vp, _vp, _sz, _vp]),
     "ifa_latent_rotate_q_f32": (_i, [_i, _i, _i, _vp, _sz, _i, _i, _vp, _f, _vp, _vp, _sz, _vp]),
     "ifa_qk_rope_store_pairs_f32": (_i, [_i, _vp, _sz, _i, _vp, _sz, _vp, _sz, _i, _i, _i, _i, _vp, _vp, _f, _i, _vp, _vp, _vp, _sz, _vp, _sz, _sz, _vp]),
-    "ifa_attention_diff_f32": (_i, [_vp, _sz, _i, _i, _i, _i, _f, _i, _i, _f, _f, _f, _vp, _sz, _vp, _vp, _sz, _vp, _sz, _sz, _vp, _sz, _vp, _i, _i, _i, _vp, _sz, _vp]),
+    "ifa_attention_diff_f32": (_i, [_vp, _sz, _i, _i, _i, _i, _f, _i, _i, _f, _f, _f, _vp, _sz, _vp, _vp, _sz, _vp, _sz, _sz, _vp, _vp, _sz, _vp, _i, _i, _i, _vp, _sz, _vp]),
+    "ifa_attention_diff_tile_fits": (_i, [_i, _i]),
+    "ifa_norm_add_norm_to_bf16": (_i, [_vp, _sz, _sz, _sz, _vp, _sz, _vp, _vp, _f, _f, _vp, _sz, _vp]),
     "ifa_rows_to_bf16": (_i, [_vp, _sz, _sz, _sz, _vp, _sz, _vp]),
     "ifa_linear_bf16_both": (_i, [_vp, _sz, _sz, _vp, _sz, _sz, _vp, _vp, _f, _i, _i, _vp, _vp, _sz, _i, _i, _vp]),
     "ifa_linear_bf16w_act": (_i, [_vp, _sz, _sz, _vp, _sz, _sz, _vp, _i, _i, _vp, _sz, _vp]),

@@ -28,6 +28,7 @@ struct DiffArgs {
     const SeqDesc *seqs; const int *row_seq; float *const *slot_base; size_t k_off, v_off;
     float *out; size_t ldo;                      // [rows][heads * vdim]
     float *ws; int nsplit;                       // [rows][heads][nsplit][2 maps][vdim + 2]: maximum, sum, weighted values relative to the maximum
+    bf16_t *out16;                               // tiled form: the output in bfloat16 instead
     int vec, n_seqs;
 };
 
@@ -381,6 +382,17 @@ __global__ void __launch_bounds__(256) k_attn_diff_tile(DiffArgs P)
     const float gate = P.g ? sigmoid_f(P.g[row * P.ldg + h]) : 1.0f;
     const float rs = P.out_scale * gate / sqrtf(ss / (float)dv + P.eps);
     float *dst = P.out + row * P.ldo + (size_t)h * dv;
+    if (P.out16) {
+        bf16_t *d16 = P.out16 + row * P.ldo + (size_t)h * dv;
+#pragma unroll
+        for (int nt = 0; nt < NTV; nt++)
+#pragma unroll
+            for (int r = 0; r < 16; r++) {
+                const int c = 32 * nt + (r & 3) + 8 * (r >> 2) + 4 * g;
+                if (c < dv) d16[c] = f2bf(o[nt][r] * rs);
+            }
+        return;
+    }
 #pragma unroll
     for (int nt = 0; nt < NTV; nt++)
 #pragma unroll
@@ -435,19 +447,21 @@ void dispatch_diff_rows_c(const DiffArgs &P, unsigned rows, hipStream_t s)
 
 extern "C" {
 
+int ifa_attention_diff_tile_fits(int dim, int vdim) { return dim >= 1 && dim <= 128 && vdim >= 1 && (vdim <= 128 || (vdim > 192 && vdim <= 256)) ? 1 : 0; }
+
 int ifa_attention_diff_f32(const void *q_f32, size_t ldq, int heads, int kv_heads, int dim, int vdim, float scale, int window, int chunk, float lambda, float out_scale,
                            float eps, const void *g_f32, size_t ldg, const void *seqs_dev, const int *row_seq_dev, size_t rows, void *const *slot_base_dev, size_t k_off,
-                           size_t v_off, void *out_f32, size_t ldo, const void *seqs_host, int n_seqs, int tile_min_rows, int max_keys, void *ws_f32, size_t ws_bytes,
-                           ifa_stream stream)
+                           size_t v_off, void *out_f32, void *out_bf16, size_t ldo, const void *seqs_host, int n_seqs, int tile_min_rows, int max_keys, void *ws_f32,
+                           size_t ws_bytes, ifa_stream stream)
 {
-    IFA_REQUIRE(q_f32 && seqs_dev && row_seq_dev && slot_base_dev && out_f32 && seqs_host, "ifa_attention_diff_f32: null pointer");
+    IFA_REQUIRE(q_f32 && seqs_dev && row_seq_dev && slot_base_dev && (out_f32 || out_bf16) && seqs_host, "ifa_attention_diff_f32: null pointer");
     IFA_REQUIRE(heads > 0 && heads < 65536 && kv_heads > 0 && heads % kv_heads == 0 && dim > 0 && dim <= 1024 && vdim > 0 && vdim <= 1024 && rows > 0 && window >= 0 && chunk >= 0
                 && n_seqs > 0, "ifa_attention_diff_f32: bad shape (%d / %d heads of %d / %d)", heads, kv_heads, dim, vdim);
     IFA_REQUIRE(ldq >= (size_t)heads * 2 * dim && ldo >= (size_t)heads * vdim && (!g_f32 || ldg >= (size_t)heads), "ifa_attention_diff_f32: row strides too small");
     DiffArgs P;
     P.q = (const float *)q_f32; P.ldq = ldq; P.heads = heads; P.kv_heads = kv_heads; P.dim = dim; P.vdim = vdim; P.scale = scale; P.window = window; P.chunk = chunk;
     P.lambda = lambda; P.out_scale = out_scale; P.eps = eps; P.g = (const float *)g_f32; P.ldg = ldg; P.seqs = (const SeqDesc *)seqs_dev; P.row_seq = row_seq_dev;
-    P.slot_base = (float *const *)slot_base_dev; P.k_off = k_off; P.v_off = v_off; P.out = (float *)out_f32; P.ldo = ldo; P.ws = (float *)ws_f32; P.nsplit = 1; P.n_seqs = n_seqs;
+    P.slot_base = (float *const *)slot_base_dev; P.k_off = k_off; P.v_off = v_off; P.out = (float *)out_f32; P.out16 = (bf16_t *)out_bf16; P.ldo = ldo; P.ws = (float *)ws_f32; P.nsplit = 1; P.n_seqs = n_seqs;
     const ifa_seq_desc *sh = (const ifa_seq_desc *)seqs_host;
     hipStream_t s = ifa_s(stream);
     int longest = 0;
@@ -455,13 +469,14 @@ int ifa_attention_diff_f32(const void *q_f32, size_t ldq, int heads, int kv_head
     for (int q = 0; q < n_seqs; q++) { longest = std::max(longest, sh[q].n); tiles += ((size_t)sh[q].n + DT_Q - 1) / DT_Q; }
     // 16-byte requests: every key and value head of a cache row on a 16-byte boundary (arena bases are 256-byte aligned)
     P.vec = (dim % 4 == 0 && vdim % 4 == 0 && k_off % 4 == 0 && v_off % 4 == 0 && ldo % 4 == 0 && ((uintptr_t)out_f32 & 15) == 0) ? 1 : 0;
-    if (longest >= std::max(tile_min_rows, 1) && dim <= 128 && (vdim <= 128 || (vdim > 192 && vdim <= 256))) {
+    if (longest >= std::max(tile_min_rows, 1) && ifa_attention_diff_tile_fits(dim, vdim)) {
         IFA_REQUIRE(tiles < 65536, "ifa_attention_diff_f32: %zu query tiles in one step", tiles);
         if (dim <= 32) return dispatch_diff_tile_v<1>(P, (unsigned)tiles, s);
         if (dim <= 64) return dispatch_diff_tile_v<2>(P, (unsigned)tiles, s);
         if (dim <= 96) return dispatch_diff_tile_v<3>(P, (unsigned)tiles, s);
         return dispatch_diff_tile_v<4>(P, (unsigned)tiles, s);
     }
+    IFA_REQUIRE(!out_bf16, "ifa_attention_diff_f32: a bfloat16 output comes from the tiled form only");
     // key shares: 64 keys a share over the most keys a row can see (the same for every step, so that a captured step replays), fewer where many rows
     // already fill the chip or the workspace is small
     const int group = heads / kv_heads;

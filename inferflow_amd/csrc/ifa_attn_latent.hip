@@ -320,6 +320,7 @@ struct LatTileArgs {
     float *out; size_t ldo;
     int vec;
     const bf16_t *sink;          // [heads] or null
+    bf16_t *out16;               // the output in bfloat16 instead
 };
 
 template <int NTK, int NTV>
@@ -468,7 +469,8 @@ __global__ void __launch_bounds__(256) k_attn_latent_tile(LatTileArgs P)
             if (e < dv) {
                 const size_t c = (size_t)h * dv + e;
                 const float v = o[nt][r] * sc;
-                P.out[row * P.ldo + c] = P.gate_cols ? v * sigmoid_f(P.g[row * P.ldg + c]) : v;
+                const float vg = P.gate_cols ? v * sigmoid_f(P.g[row * P.ldg + c]) : v;
+                if (P.out16) P.out16[row * P.ldo + c] = f2bf(vg); else P.out[row * P.ldo + c] = vg;
             }
         }
 }
@@ -633,15 +635,15 @@ int ifa_attention_latent_tile_gated_f32(int gate_cols, const void *q_f32, size_t
                                         void *out_f32, size_t ldo, ifa_stream stream)
 {
     return ifa_attention_latent_tile_sinks_f32(gate_cols, q_f32, ldq, heads, dim, rot_dim, vdim, kv_rank, scale, nullptr, kx_f32, ldkx, vx_f32, ldvx, ctx0_dev, g_f32, ldg,
-                                               seqs_dev, seqs_host, n_seqs, slot_base_dev, cache_off, out_f32, ldo, stream);
+                                               seqs_dev, seqs_host, n_seqs, slot_base_dev, cache_off, out_f32, nullptr, ldo, stream);
 }
 
 int ifa_attention_latent_tile_sinks_f32(int gate_cols, const void *q_f32, size_t ldq, int heads, int dim, int rot_dim, int vdim, int kv_rank, float scale,
                                         const void *sink_bf16, const void *kx_f32, size_t ldkx, const void *vx_f32, size_t ldvx, const int *ctx0_dev, const void *g_f32,
                                         size_t ldg, const void *seqs_dev, const void *seqs_host, int n_seqs, void *const *slot_base_dev, size_t cache_off, void *out_f32,
-                                        size_t ldo, ifa_stream stream)
+                                        void *out_bf16, size_t ldo, ifa_stream stream)
 {
-    IFA_REQUIRE(q_f32 && kx_f32 && vx_f32 && ctx0_dev && seqs_dev && seqs_host && slot_base_dev && out_f32, "ifa_attention_latent_tile_f32: null pointer");
+    IFA_REQUIRE(q_f32 && kx_f32 && vx_f32 && ctx0_dev && seqs_dev && seqs_host && slot_base_dev && (out_f32 || out_bf16), "ifa_attention_latent_tile_f32: null pointer");
     IFA_REQUIRE(heads > 0 && heads < 65536 && dim > 0 && rot_dim >= 0 && vdim > 0 && kv_rank > 0 && n_seqs > 0 && ldq >= (size_t)heads * (dim + rot_dim)
                 && ldkx >= (size_t)heads * dim && ldvx >= (size_t)heads * vdim && ldo >= (size_t)heads * vdim && (!g_f32 || ldg >= (size_t)heads * (gate_cols ? vdim : 1)) && (!gate_cols || g_f32),
                 "ifa_attention_latent_tile_f32: bad shape");
@@ -650,7 +652,7 @@ int ifa_attention_latent_tile_sinks_f32(int gate_cols, const void *q_f32, size_t
     LatTileArgs P;
     P.q = (const float *)q_f32; P.ldq = ldq; P.heads = heads; P.dim = dim; P.dr = rot_dim; P.vdim = vdim; P.R = kv_rank; P.scale = scale;
     P.kx = (const float *)kx_f32; P.ldkx = ldkx; P.vx = (const float *)vx_f32; P.ldvx = ldvx; P.ctx0 = ctx0_dev; P.g = (const float *)g_f32; P.ldg = ldg; P.gate_cols = gate_cols ? 1 : 0;
-    P.sink = (const bf16_t *)sink_bf16;
+    P.sink = (const bf16_t *)sink_bf16; P.out16 = (bf16_t *)out_bf16;
     P.seqs = (const SeqDesc *)seqs_dev; P.n_seqs = n_seqs; P.slot_base = (float *const *)slot_base_dev; P.cache_off = cache_off; P.out = (float *)out_f32; P.ldo = ldo;
     // 16-byte requests: every source row and every part of a row starts on a 16-byte boundary
     P.vec = (dim % 4 == 0 && rot_dim % 4 == 0 && vdim % 4 == 0 && kv_rank % 4 == 0 && ldq % 4 == 0 && ldkx % 4 == 0 && ldvx % 4 == 0 && cache_off % 4 == 0

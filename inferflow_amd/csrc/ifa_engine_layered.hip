@@ -113,7 +113,7 @@ struct LayeredNet {
                                            // SANDWICH layers, every step size: the norm behind a sub-layer and the norm in front of the next one in one launch
                                            // PRENORM layers: the start of a looped pass inside the norm's launch; steps of at most 8 rows: the norm inside the router's launch
     float *attn_ws = nullptr; size_t attn_ws_bytes = 0;      // partial results of the windowed attention when a (row, head)'s keys are shared out
-    bf16_t *a16 = nullptr; size_t a16_cap = 0; int opt_a16_min = 17;          // activations of a prompt's product rounded to bfloat16; steps of at least this many rows (0: never)
+    bf16_t *a16 = nullptr, *h16 = nullptr; size_t a16_cap = 0, h16_cap = 0; int opt_a16_min = 17;          // activations of a prompt's product rounded to bfloat16; steps of at least this many rows (0: never)
     int opt_attn_tile_min = 16;            // steps of at least this many rows run the windowed attention through the tiled kernel
     std::vector<ifa_seq_desc> seqs_host;   // the current step's sequences (the tiled attention's grid is sized from them)
     // POSTNORM layers: two more mixer buffers, the planes of the depth average ([layers + 1][scratch_rows * width]), the router's choices,
@@ -350,17 +350,18 @@ float norm_offset_of(const LayeredNet *n) { return n->cfg.norm_plain ? 0.0f : 1.
 bool takes_a16(const LayeredNet *n, size_t K, size_t T) { return !n->cfg.ops32 && n->opt_a16_min > 0 && T >= (size_t)n->opt_a16_min && K % 8 == 0 && K >= 64; }
 size_t a16_stride(size_t K) { return (K + 63) & ~(size_t)63; }
 
-int ensure_a16(ifa_model *m, size_t T, size_t K)
+int ensure_halfs(ifa_model *m, bf16_t *&buf, size_t &cap, size_t need)
 {
-    LayeredNet *n = m->lay;
-    const size_t need = T * a16_stride(K);
-    if (need <= n->a16_cap) return IFA_OK;
+    if (need <= cap) return IFA_OK;
     IFA_HIP_CHECK(hipStreamSynchronize(m->stream));
-    lay_free(n->a16); n->a16 = nullptr; n->a16_cap = 0;
-    IFA_HIP_CHECK(hipMalloc((void **)&n->a16, need * 2));
-    n->a16_cap = need;
+    lay_free(buf); buf = nullptr; cap = 0;
+    IFA_HIP_CHECK(hipMalloc((void **)&buf, need * 2));
+    cap = need;
     return IFA_OK;
 }
+int ensure_a16(ifa_model *m, size_t T, size_t K) { return ensure_halfs(m, m->lay->a16, m->lay->a16_cap, T * a16_stride(K)); }
+// norms that leave what only products read in bfloat16 (n->h16) at once
+bool norms_leave_h16(const LayeredNet *n, size_t T) { return takes_a16(n, (size_t)n->cfg.width, T) && n->cfg.width % 64 == 0 && n->cfg.width <= 8192; }
 
 int linear(ifa_model *m, const bf16_t *W, size_t N, size_t K, const float *A, size_t lda, size_t T, const bf16_t *bias, const bf16_t *mul, float alpha,
            int accumulate, float *C, size_t ldc, int silu0 = 0, int silu1 = 0)
@@ -373,6 +374,13 @@ int linear(ifa_model *m, const bf16_t *W, size_t N, size_t K, const float *A, si
         return rc;
     }
     return ifa_linear_bf16w(W, N, K, A, lda, T, bias, mul, alpha, accumulate, m->lay->cfg.ops32, C, ldc, silu0, silu1, (ifa_stream)m->stream);
+}
+
+// product of what a norm has left: bfloat16 rows (h16) or 32-bit rows
+int linear_in(ifa_model *m, const bf16_t *W, size_t N, size_t K, const float *h, const bf16_t *h16, size_t T, const bf16_t *bias, float *C, size_t ldc)
+{
+    if (h16) return ifa_linear_bf16_both(W, N, K, h16, K, T, bias, nullptr, 1.0f, 0, 0, C, nullptr, ldc, 0, 0, (ifa_stream)m->stream);
+    return linear(m, W, N, K, h, K, T, bias, nullptr, 1.0f, 0, C, ldc);
 }
 
 // What lies between two sub-layers of a POSTNORM block: x += gnorm(sub) * norm_w; [depth average]; [h = x + conv(x), tail advanced].
@@ -399,7 +407,7 @@ int post_step(ifa_model *m, size_t T, int nseq, bool fused, const float *sub, co
 }
 
 // latent attention over T rows of hin -> out (the output product): pass_off = offset of this pass's copy of the layer's part of the arena
-int run_latent_mixer(ifa_model *m, LLayer &L, size_t T, const float *hin, size_t pass_off, float *out)
+int run_latent_mixer(ifa_model *m, LLayer &L, size_t T, const float *hin, const bf16_t *hin16, size_t pass_off, float *out)
 {
     LayeredNet *n = m->lay;
     const ifa_layered_config &c = n->cfg;
@@ -411,7 +419,7 @@ int run_latent_mixer(ifa_model *m, LLayer &L, size_t T, const float *hin, size_t
     int rc;
     const int H = sp.m_heads, dn = sp.m_dim, dr = sp.m_rot_dim, dv = sp.m_vdim, R = sp.m_kv_rank;
     const size_t QD = (size_t)H * (dn + dr), CR = (size_t)(R + dr), OV = (size_t)H * dv;
-    if ((rc = linear(m, L.w_in, NI, W, hin, W, T, nullptr, nullptr, 1.0f, 0, n->proj, NI))) return rc;
+    if ((rc = linear_in(m, L.w_in, NI, W, hin, hin16, T, nullptr, n->proj, NI))) return rc;
     float *q = n->proj + L.c_mq; size_t ldq = NI;
     if (sp.m_q_rank > 0) {      // queries through their own normed latent
         const size_t QR = (size_t)sp.m_q_rank;
@@ -433,11 +441,20 @@ int run_latent_mixer(ifa_model *m, LLayer &L, size_t T, const float *hin, size_t
             const ifa_seq_desc &sd = n->seqs_host[qi];
             const float *lat = n->slot_ptr[(size_t)sd.slot] + o_c;
             const size_t ctx = (size_t)sd.pos0 + sd.n, r0 = (size_t)n->ctx0_host[qi];
+            if (takes_a16(n, (size_t)R, ctx)) {      // (the latents rounded once for both products)
+                if ((rc = ensure_a16(m, ctx, (size_t)R)) || (rc = ifa_rows_to_bf16(lat, CR, ctx, (size_t)R, n->a16, a16_stride((size_t)R), s))) return rc;
+                if ((rc = ifa_linear_bf16_both(L.T(IFA_LT_M_UK).data, ldk, (size_t)R, n->a16, a16_stride((size_t)R), ctx, nullptr, nullptr, 1.0f, 0, 0, n->kx + r0 * ldk, nullptr, ldk, 0, 0, s))) return rc;
+                if ((rc = ifa_linear_bf16_both(L.T(IFA_LT_M_UV).data, ldv, (size_t)R, n->a16, a16_stride((size_t)R), ctx, nullptr, nullptr, 1.0f, 0, 0, n->vx + r0 * ldv, nullptr, ldv, 0, 0, s))) return rc;
+                continue;
+            }
             if ((rc = linear(m, (const bf16_t *)L.T(IFA_LT_M_UK).data, ldk, (size_t)R, lat, CR, ctx, nullptr, nullptr, 1.0f, 0, n->kx + r0 * ldk, ldk))) return rc;
             if ((rc = linear(m, (const bf16_t *)L.T(IFA_LT_M_UV).data, ldv, (size_t)R, lat, CR, ctx, nullptr, nullptr, 1.0f, 0, n->vx + r0 * ldv, ldv))) return rc;
         }
+        bf16_t *out16 = nullptr;          // the attention's output as the output product reads it
+        if (takes_a16(n, OV, T) && OV % 64 == 0) { if ((rc = ensure_a16(m, T, OV))) return rc; out16 = n->a16; }
         if ((rc = ifa_attention_latent_tile_sinks_f32(sp.m_gate == 2, q, ldq, H, dn, dr, dv, R, sp.m_scale, sink, n->kx, ldk, n->vx, ldv, n->ctx0_dev, gate, NI, n->seqs_dev, n->seqs_host.data(),
-                                                (int)n->seqs_host.size(), slots, o_c, n->m5, OV, s))) return rc;
+                                                (int)n->seqs_host.size(), slots, o_c, n->m5, out16, OV, s))) return rc;
+        if (out16) return linear_in(m, (const bf16_t *)L.T(IFA_LT_M_O).data, W, OV, nullptr, out16, T, nullptr, out, W);
     } else {
         // absorbed form: the cache rows are keys (whole) and values (latent part) of ONE head that all query heads share
         const size_t QA = (size_t)H * CR;
@@ -472,7 +489,7 @@ int run_postnorm_layer(ifa_model *m, LLayer &L, size_t li, size_t T, int nseq, b
         if (!h_ready && (rc = post_step(m, T, nseq, fused, nullptr, nullptr, nullptr, li, L.T(IFA_LT_CANON1).data, sp.canon_taps, L.o_cv1))) return rc;
         hin = n->h;
     }
-    if ((rc = run_latent_mixer(m, L, T, hin, 0, n->m1))) return rc;
+    if ((rc = run_latent_mixer(m, L, T, hin, nullptr, 0, n->m1))) return rc;
     const LLayer *depth_of = sp.depth_avg ? &L : nullptr;
     const void *ncw = next_conv ? next->T(IFA_LT_CANON1).data : nullptr;
     const int ntaps = next_conv ? next->spec.canon_taps : 0;
@@ -496,7 +513,7 @@ int run_postnorm_layer(ifa_model *m, LLayer &L, size_t li, size_t T, int nseq, b
 }
 
 // differential attention over T rows of h -> out (the output product)
-int run_diff_mixer(ifa_model *m, LLayer &L, size_t T, const float *h, float *out)
+int run_diff_mixer(ifa_model *m, LLayer &L, size_t T, const float *h, const bf16_t *h16, float *out)
 {
     LayeredNet *n = m->lay;
     const ifa_layered_config &c = n->cfg;
@@ -506,12 +523,17 @@ int run_diff_mixer(ifa_model *m, LLayer &L, size_t T, const float *h, float *out
     ifa_stream s = (ifa_stream)m->stream;
     void *const *slots = (void *const *)n->slot_base_dev;
     int rc;
-    if ((rc = linear(m, L.w_in, NI, W, h, W, T, nullptr, nullptr, 1.0f, 0, n->proj, NI))) return rc;
+    if ((rc = linear_in(m, L.w_in, NI, W, h, h16, T, nullptr, n->proj, NI))) return rc;
     if ((rc = ifa_qk_rope_store_pairs_f32(sp.a_rot_pairs, n->proj + L.c_aq, NI, 2 * H, n->proj + L.c_ak, NI, n->proj + L.c_av, NI, 2 * G, G, D, DV, nullptr, nullptr, c.eps, sp.a_rot_dims,
                                           L.freq, n->seqs_dev, n->row_seq_dev, T, slots, L.o_k, L.o_v, s))) return rc;
+    int longest = 0;
+    for (const ifa_seq_desc &sd : n->seqs_host) longest = std::max(longest, sd.n);
+    bf16_t *out16 = nullptr;          // (tiled form: the output as the output product reads it)
+    if (takes_a16(n, OV, T) && OV % 64 == 0 && longest >= n->opt_attn_tile_min && ifa_attention_diff_tile_fits(D, DV)) { if ((rc = ensure_a16(m, T, OV))) return rc; out16 = n->a16; }
     if ((rc = ifa_attention_diff_f32(n->proj + L.c_aq, NI, H, G, D, DV, sp.a_scale, sp.a_window, sp.a_chunk, L.diff_lambda, 1.0f - sp.a_diff, c.eps,
-                                     sp.a_gate ? n->proj + L.c_ag : nullptr, NI, n->seqs_dev, n->row_seq_dev, T, slots, L.o_k, L.o_v, n->m1, OV, n->seqs_host.data(),
+                                     sp.a_gate ? n->proj + L.c_ag : nullptr, NI, n->seqs_dev, n->row_seq_dev, T, slots, L.o_k, L.o_v, n->m1, out16, OV, n->seqs_host.data(),
                                      (int)n->seqs_host.size(), n->opt_attn_tile_min, c.max_ctx, n->attn_ws, n->attn_ws_bytes, s))) return rc;
+    if (out16) return linear_in(m, (const bf16_t *)L.T(IFA_LT_A_O).data, W, OV, nullptr, out16, T, nullptr, out, W);
     return linear(m, (const bf16_t *)L.T(IFA_LT_A_O).data, W, OV, n->m1, OV, T, nullptr, nullptr, 1.0f, 0, out, W);
 }
 
@@ -531,23 +553,32 @@ int run_sandwich_layer(ifa_model *m, LLayer &L, size_t T, int nseq, bool h_ready
     const float w_off = norm_offset_of(n);
     const void *next_norm = fused && next && next->spec.block == IFA_BLOCK_SANDWICH ? next->T(IFA_LT_NORM1).data : nullptr;
     *next_h_ready = next_norm != nullptr;
+    // steps whose products read bfloat16 rows: the norms leave them so (n->h16), but where a mixture of experts reads the rows itself
+    const bool in16 = fused && norms_leave_h16(n, T);
+    if (in16) { const int r = ensure_halfs(m, n->h16, n->h16_cap, T * W); if (r) return r; }
+    const bf16_t *h16 = in16 ? n->h16 : nullptr;
     // x += norm_after(sub); h = norm_before(x) for whatever comes next
-    auto close_sub = [&](const float *sub, const void *w_after, const void *w_before) -> int {
+    auto close_sub = [&](const float *sub, const void *w_after, const void *w_before, bool to16) -> int {
+        if (fused && to16 && w_before) return ifa_norm_add_norm_to_bf16(n->x, W, T, W, sub, W, w_after, w_before, w_off, c.eps, n->h16, W, s);
         if (fused) return ifa_norm_add_norm_f32(n->x, W, T, W, sub, W, w_after, w_before, w_off, c.eps, n->h, W, s);
         int r = ifa_rmsnorm_offset_f32(sub, W, T, W, w_after, w_off, c.eps, 1, n->x, W, s);
         if (!r && w_before) r = ifa_rmsnorm_offset_f32(n->x, W, T, W, w_before, w_off, c.eps, 0, n->h, W, s);
         return r;
     };
     int rc;
-    if (!h_ready && (rc = ifa_rmsnorm_offset_f32(n->x, W, T, W, L.T(IFA_LT_NORM1).data, w_off, c.eps, 0, n->h, W, s))) return rc;
-    if (sp.mixer == IFA_MIX_LATENT) { if ((rc = run_latent_mixer(m, L, T, n->h, 0, n->m2))) return rc; }
-    else if (sp.mixer == IFA_MIX_DIFF) { if ((rc = run_diff_mixer(m, L, T, n->h, n->m2))) return rc; }
+    if (!h_ready) {
+        rc = in16 ? ifa_norm_add_norm_to_bf16(n->x, W, T, W, nullptr, 0, nullptr, L.T(IFA_LT_NORM1).data, w_off, c.eps, n->h16, W, s)
+                  : ifa_rmsnorm_offset_f32(n->x, W, T, W, L.T(IFA_LT_NORM1).data, w_off, c.eps, 0, n->h, W, s);
+        if (rc) return rc;
+    }
+    if (sp.mixer == IFA_MIX_LATENT) { if ((rc = run_latent_mixer(m, L, T, n->h, h16, 0, n->m2))) return rc; }
+    else if (sp.mixer == IFA_MIX_DIFF) { if ((rc = run_diff_mixer(m, L, T, n->h, h16, n->m2))) return rc; }
     else {
         const int H = sp.a_heads, G = sp.a_kv_heads, D = sp.a_dim, DV = sp.a_vdim;
         const size_t OV = (size_t)H * DV;
         const bool own = sp.a_kv_layer == 0;
         const LLayer &KV = own ? L : n->layers[(size_t)sp.a_kv_layer - 1];
-        if ((rc = linear(m, L.w_in, NI, W, n->h, W, T, L.b_in, nullptr, 1.0f, 0, n->proj, NI))) return rc;
+        if ((rc = linear_in(m, L.w_in, NI, W, n->h, h16, T, L.b_in, n->proj, NI))) return rc;
         if ((rc = ifa_qk_rope_store_f32(n->proj + L.c_aq, NI, H, own ? n->proj + L.c_ak : nullptr, NI, own ? n->proj + L.c_av : nullptr, NI, G, D, DV,
                                         L.T(IFA_LT_A_Q_NORM).data, own ? L.T(IFA_LT_A_K_NORM).data : nullptr, c.eps, sp.a_rot_dims, L.freq, n->seqs_dev, n->row_seq_dev, T,
                                         slots, KV.o_k, KV.o_v, s))) return rc;
@@ -556,24 +587,28 @@ int run_sandwich_layer(ifa_model *m, LLayer &L, size_t T, int nseq, bool h_ready
                                        c.max_ctx, n->attn_ws, n->attn_ws_bytes, s))) return rc;
         if ((rc = linear(m, (const bf16_t *)L.T(IFA_LT_A_O).data, W, OV, n->m1, OV, T, nullptr, nullptr, 1.0f, 0, n->m2, W))) return rc;
     }
-    if ((rc = close_sub(n->m2, L.T(IFA_LT_NORM1B).data, any_ffn ? L.T(IFA_LT_NORM2).data : next_norm))) return rc;
+    if ((rc = close_sub(n->m2, L.T(IFA_LT_NORM1B).data, any_ffn ? L.T(IFA_LT_NORM2).data : next_norm, in16 && !(any_ffn && moe)))) return rc;
+    if (any_ffn && moe) h16 = nullptr;
     if (!any_ffn) return IFA_OK;
     const size_t N2 = L.n_in2;
     if (sp.ffn_kind == IFA_FFN_RELU2) {      // the square of relu in the epilogue of the up-projection
         const size_t F = (size_t)sp.ffn;
         if (takes_a16(n, W, T) && takes_a16(n, F, T) && F % 64 == 0) {      // ... which then leaves the down-projection's operand as it is read
-            if ((rc = ensure_a16(m, T, W + F))) return rc;
-            bf16_t *h16 = n->a16, *u16 = n->a16 + T * a16_stride(W);
-            if ((rc = ifa_rows_to_bf16(n->h, W, T, W, h16, a16_stride(W), s))) return rc;
-            if ((rc = ifa_linear_bf16_both(L.w_in2, N2, W, h16, a16_stride(W), T, nullptr, nullptr, 1.0f, 0, 2, nullptr, u16, F, 0, 0, s))) return rc;
+            if ((rc = ensure_a16(m, T, F + a16_stride(W)))) return rc;
+            bf16_t *u16 = n->a16, *in = n->a16 + T * F;
+            if (!h16 && (rc = ifa_rows_to_bf16(n->h, W, T, W, in, a16_stride(W), s))) return rc;
+            if ((rc = ifa_linear_bf16_both(L.w_in2, N2, W, h16 ? h16 : in, a16_stride(W), T, nullptr, nullptr, 1.0f, 0, 2, nullptr, u16, F, 0, 0, s))) return rc;
             if ((rc = ifa_linear_bf16_both(L.T(IFA_LT_FFN_DOWN).data, W, F, u16, F, T, nullptr, nullptr, 1.0f, 0, 0, n->m2, nullptr, W, 0, 0, s))) return rc;
-            return close_sub(n->m2, L.T(IFA_LT_NORM2B).data, next_norm);
+            return close_sub(n->m2, L.T(IFA_LT_NORM2B).data, next_norm, in16);
         }
+        if (h16) {      // (the down-projection reads 32-bit rows)
+            if ((rc = ifa_linear_bf16_both(L.w_in2, N2, W, h16, W, T, nullptr, nullptr, 1.0f, 0, 2, n->proj, nullptr, N2, 0, 0, s))) return rc;
+        } else
         if ((rc = ifa_linear_bf16w_act(L.w_in2, N2, W, n->h, W, T, nullptr, 2, c.ops32, n->proj, N2, s))) return rc;
-        if ((rc = linear(m, (const bf16_t *)L.T(IFA_LT_FFN_DOWN).data, W, (size_t)sp.ffn, n->proj, N2, T, nullptr, nullptr, 1.0f, 0, n->m2, W))) return rc;
-        return close_sub(n->m2, L.T(IFA_LT_NORM2B).data, next_norm);
+        if ((rc = linear(m, (const bf16_t *)L.T(IFA_LT_FFN_DOWN).data, W, F, n->proj, N2, T, nullptr, nullptr, 1.0f, 0, n->m2, W))) return rc;
+        return close_sub(n->m2, L.T(IFA_LT_NORM2B).data, next_norm, in16);
     }
-    if ((rc = linear(m, L.w_in2, N2, W, n->h, W, T, L.b_in2, nullptr, 1.0f, 0, n->proj, N2))) return rc;
+    if ((rc = linear_in(m, L.w_in2, N2, W, n->h, h16, T, L.b_in2, n->proj, N2))) return rc;
     if (!moe) {
         const size_t F = (size_t)sp.ffn;
         if ((rc = ifa_glu_ex_f32(3, sp.f_limit, n->proj + L.c2_fg, N2, T, F, nullptr, 0, n->m3, F, s))) return rc;
@@ -589,7 +624,7 @@ int run_sandwich_layer(ifa_model *m, LLayer &L, size_t T, int nseq, bool h_ready
             if ((rc = linear(m, (const bf16_t *)L.T(IFA_LT_X_SH_DOWN).data, W, SF, n->m3, SF, T, nullptr, nullptr, 1.0f, 1, n->m2, W))) return rc;
         }
     }
-    return close_sub(n->m2, L.T(IFA_LT_NORM2B).data, next_norm);
+    return close_sub(n->m2, L.T(IFA_LT_NORM2B).data, next_norm, in16);
 }
 
 // one PRENORM layer over T rows: x <- x + mixer(dyt1(x)); x <- x + experts(dyt2(x)), dyt(x) = tanh(alpha x) w + b.  pass: which copy of the
@@ -730,7 +765,7 @@ int run_streams_layer(ifa_model *m, LLayer &L, size_t T, int nseq, int pass, LLa
     const bool moe = has_moe(sp), any_ffn = sp.ffn > 0 || moe;
     const void *next_in = next ? next->T(IFA_LT_HC1_IN).data : nullptr, *next_norm = next ? next->T(IFA_LT_NORM1).data : n->out_norm.data;
     int rc;
-    if ((rc = sp.mixer == IFA_MIX_LATENT ? run_latent_mixer(m, L, T, n->h, po, n->m3) : run_ssm_mixer(m, L, T, nseq, n->h, po, n->m3))) return rc;
+    if ((rc = sp.mixer == IFA_MIX_LATENT ? run_latent_mixer(m, L, T, n->h, nullptr, po, n->m3) : run_ssm_mixer(m, L, T, nseq, n->h, po, n->m3))) return rc;
     if ((rc = streams_step(m, T, false, n->m3, &L, 1, any_ffn ? L.T(IFA_LT_HC2_IN).data : next_in, any_ffn ? L.T(IFA_LT_NORM2).data : next_norm))) return rc;
     if (!any_ffn) return IFA_OK;
     if (!moe) {
@@ -941,7 +976,7 @@ int lay_destroy(ifa_model *m)
     for (float *p : n->slot_ptr) lay_free(p);
     lay_free(n->slot_base_dev);
     if (n->tab_pin) (void)hipHostFree(n->tab_pin);
-    lay_free(n->attn_ws); lay_free(n->a16);
+    lay_free(n->attn_ws); lay_free(n->a16); lay_free(n->h16);
     lay_free(n->tab_dev); lay_free(n->excl_dev); lay_free(n->next_dev); lay_free(n->ring_dev);
     float *bufs[] = {n->x, n->h, n->proj, n->m1, n->m2, n->m3, n->beta, n->decay, n->logits, n->taps};
     for (float *b : bufs) lay_free(b);

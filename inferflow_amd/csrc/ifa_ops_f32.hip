@@ -189,12 +189,12 @@ __global__ void __launch_bounds__(256) k_norm_add_norm(float *__restrict__ x, si
     for (int c = threadIdx.x; c < cols; c += blockDim.x) hr[c] = xr[c] * rinv2 * (w_off + bf2f(w_before[c]));
 }
 
-// The same (m null: h alone) with the row in registers: every thread holds PIECES pieces of four values, and everything the row needs (x, m, both weights) is requested
+// The same (m null: h alone; h16 not null: h in bfloat16) with the row in registers: every thread holds PIECES pieces of four values, and everything the row needs (x, m, both weights) is requested
 // before the first reduction.  cols % 4 == 0, cols <= 4 PIECES blockDim, 16-byte aligned rows, 8-byte aligned weights.
 template <int PIECES>
 __global__ void __launch_bounds__(1024) k_norm_add_norm_reg(float *__restrict__ x, size_t ldx, int cols, const float *__restrict__ m, size_t ldm,
                                                             const bf16_t *__restrict__ w_after, const bf16_t *__restrict__ w_before, float w_off, float eps,
-                                                            float *__restrict__ h, size_t ldh)
+                                                            float *__restrict__ h, bf16_t *__restrict__ h16, size_t ldh)
 {
     __shared__ float red[17];
     float *xr = x + (size_t)blockIdx.x * ldx;
@@ -234,7 +234,6 @@ __global__ void __launch_bounds__(1024) k_norm_add_norm_reg(float *__restrict__ 
         if (!w_before) return;
         rinv2 = 1.0f / sqrtf(block_sum(q2, red) / (float)cols + eps);
     }
-    float *hr = h + (size_t)blockIdx.x * ldh;
 #pragma unroll
     for (int p = 0; p < PIECES; p++) {
         const int c = 4 * (threadIdx.x + p * blockDim.x);
@@ -242,7 +241,10 @@ __global__ void __launch_bounds__(1024) k_norm_add_norm_reg(float *__restrict__ 
         float o[4];
 #pragma unroll
         for (int e = 0; e < 4; e++) o[e] = xv[p][e] * rinv2 * weight(wb[p], e);
-        *reinterpret_cast<float4 *>(hr + c) = make_float4(o[0], o[1], o[2], o[3]);
+        if (h16) {
+            const uint32_t lo = (uint32_t)f2bf(o[0]) | ((uint32_t)f2bf(o[1]) << 16), hi = (uint32_t)f2bf(o[2]) | ((uint32_t)f2bf(o[3]) << 16);
+            *reinterpret_cast<uint2 *>(h16 + (size_t)blockIdx.x * ldh + c) = make_uint2(lo, hi);
+        } else *reinterpret_cast<float4 *>(h + (size_t)blockIdx.x * ldh + c) = make_float4(o[0], o[1], o[2], o[3]);
     }
 }
 
@@ -482,16 +484,16 @@ int ifa_add_rows_vec_f32(void *x_f32, size_t ldx, size_t rows, size_t cols, cons
 
 // launches k_norm_add_norm_reg where the row fits the registers and every access is aligned; false: nothing launched
 static bool norm_add_norm_reg(void *x, size_t ldx, size_t rows, size_t cols, const void *m, size_t ldm, const void *w_after, const void *w_before, float w_offset, float eps,
-                              void *h, size_t ldh, ifa_stream stream)
+                              void *h, void *h16, size_t ldh, ifa_stream stream)
 {
     const size_t quads = cols / 4;
     const bool vec = cols % 4 == 0 && ldx % 4 == 0 && (!m || ldm % 4 == 0) && (((uintptr_t)x | (uintptr_t)m) & 15) == 0 && ((uintptr_t)w_after & 7) == 0
-                     && (!w_before || (ldh % 4 == 0 && ((uintptr_t)h & 15) == 0 && ((uintptr_t)w_before & 7) == 0));
+                     && (!w_before || (ldh % 4 == 0 && (((uintptr_t)h | (uintptr_t)h16) & 15) == 0 && ((uintptr_t)w_before & 7) == 0));
     if (!vec || quads > 2048) return false;
     const int pieces = quads <= 1024 ? 1 : 2;          // one piece of four values per thread up to 4096 columns, two beyond
     const unsigned threads = (unsigned)((quads + 64 * pieces - 1) / (64 * pieces)) * 64;
 #define IFA_NAN(P) hipLaunchKernelGGL(k_norm_add_norm_reg<P>, dim3((unsigned)rows), dim3(threads), 0, ifa_s(stream), (float *)x, ldx, (int)cols, (const float *)m, ldm, \
-                                      (const bf16_t *)w_after, (const bf16_t *)w_before, w_offset, eps, (float *)h, ldh)
+                                      (const bf16_t *)w_after, (const bf16_t *)w_before, w_offset, eps, (float *)h, (bf16_t *)h16, ldh)
     if (pieces == 1) IFA_NAN(1); else IFA_NAN(2);
 #undef IFA_NAN
     return true;
@@ -503,7 +505,7 @@ int ifa_rmsnorm_offset_f32(const void *x_f32, size_t ldx, size_t rows, size_t co
     IFA_REQUIRE(x_f32 && y_f32, "ifa_rmsnorm_offset_f32: null pointer");
     IFA_REQUIRE(rows > 0 && cols > 0 && ldx >= cols && ldy >= cols, "ifa_rmsnorm_offset_f32: bad arguments");
     IFA_REQUIRE(!accumulate || x_f32 != y_f32, "ifa_rmsnorm_offset_f32: accumulating a row's norm into the row itself");
-    if (!accumulate && w_bf16 && norm_add_norm_reg((void *)x_f32, ldx, rows, cols, nullptr, 0, nullptr, w_bf16, w_offset, eps, y_f32, ldy, stream)) {
+    if (!accumulate && w_bf16 && norm_add_norm_reg((void *)x_f32, ldx, rows, cols, nullptr, 0, nullptr, w_bf16, w_offset, eps, y_f32, nullptr, ldy, stream)) {
         IFA_LAUNCH_CHECK();
         return IFA_OK;
     }
@@ -552,12 +554,23 @@ int ifa_streams_step_f32(void *x_f32, size_t rows, int streams, size_t cols, con
     return IFA_OK;
 }
 
+int ifa_norm_add_norm_to_bf16(void *x_f32, size_t ldx, size_t rows, size_t cols, const void *m_f32, size_t ldm, const void *w_after_bf16, const void *w_before_bf16,
+                              float w_offset, float eps, void *h_bf16, size_t ldh, ifa_stream stream)
+{
+    IFA_REQUIRE(x_f32 && w_before_bf16 && h_bf16 && (!m_f32 || w_after_bf16), "ifa_norm_add_norm_to_bf16: null pointer");
+    IFA_REQUIRE(rows > 0 && cols > 0 && ldx >= cols && (!m_f32 || ldm >= cols) && ldh >= cols && x_f32 != m_f32, "ifa_norm_add_norm_to_bf16: bad arguments");
+    IFA_REQUIRE(norm_add_norm_reg(x_f32, ldx, rows, cols, m_f32, ldm, w_after_bf16, w_before_bf16, w_offset, eps, nullptr, h_bf16, ldh, stream),
+                "ifa_norm_add_norm_to_bf16: rows of %zu columns (at most 8192, whole 16-byte pieces, aligned)", cols);
+    IFA_LAUNCH_CHECK();
+    return IFA_OK;
+}
+
 int ifa_norm_add_norm_f32(void *x_f32, size_t ldx, size_t rows, size_t cols, const void *m_f32, size_t ldm, const void *w_after_bf16,
                           const void *w_before_bf16, float w_offset, float eps, void *h_f32, size_t ldh, ifa_stream stream)
 {
     IFA_REQUIRE(x_f32 && m_f32 && w_after_bf16 && (!w_before_bf16 || h_f32), "ifa_norm_add_norm_f32: null pointer");
     IFA_REQUIRE(rows > 0 && cols > 0 && ldx >= cols && ldm >= cols && (!w_before_bf16 || ldh >= cols) && x_f32 != m_f32, "ifa_norm_add_norm_f32: bad arguments");
-    if (norm_add_norm_reg(x_f32, ldx, rows, cols, m_f32, ldm, w_after_bf16, w_before_bf16, w_offset, eps, h_f32, ldh, stream)) {
+    if (norm_add_norm_reg(x_f32, ldx, rows, cols, m_f32, ldm, w_after_bf16, w_before_bf16, w_offset, eps, h_f32, nullptr, ldh, stream)) {
         IFA_LAUNCH_CHECK();
         return IFA_OK;
     }

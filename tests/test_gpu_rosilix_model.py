@@ -366,6 +366,10 @@ CASES = {
     # many heads on one key / value head, a group that does not fill the row kernel's blocks, a feed-forward narrower and wider than the model, no latent layer
     "heads": lambda: fx.config([fx.attention_layer(heads=16, kv_heads=1, dim=8, vdim=16, chunk=29, rot_dims=8, mlp=fx.dense(8)),
                                 fx.attention_layer(heads=10, kv_heads=2, dim=36, vdim=36, chunk=64, rot_dims=12, diff=0.9, mlp=fx.dense(300))], width=40, vocab=29),
+    # sizes in whole 64s: prompts in bfloat16 hand every operand on as it is read (norms, attention outputs, the squared relu); one feed-forward that does not
+    "sixty_fours": lambda: fx.config([fx.latent_layer(heads=4, dim=24, rot_dim=8, vdim=16, kv_rank=64, mlp=fx.dense(128)), fx.attention_layer(heads=4, kv_heads=2, dim=16, vdim=32, chunk=40, rot_dims=16),
+                                      fx.latent_layer(heads=2, dim=24, rot_dim=8, vdim=32, kv_rank=64, kv_from=0, mlp=None), fx.attention_layer(heads=2, kv_heads=1, dim=16, vdim=64, rot_dims=16, mlp=fx.dense(192))],
+                                     width=128, vocab=67),
     # latent layers only, three readers of one source, the reader of another in between
     "readers": lambda: fx.config([fx.latent_layer(kv_rank=20), fx.latent_layer(kv_rank=24, rot_dim=4), fx.latent_layer(heads=1, dim=40, vdim=40, kv_rank=20, kv_from=0),
                                   fx.latent_layer(heads=6, dim=4, vdim=8, kv_rank=24, rot_dim=4, kv_from=1), fx.latent_layer(heads=2, dim=8, vdim=20, kv_rank=20, kv_from=0, mlp=None)],
@@ -448,6 +452,29 @@ def test_greedy_generation_through_the_engine(tmp_path):
     b = eng.add_query(prompt, strategy="sample.top_k", seed=5)
     out = dict(eng.infer())
     assert out[a] == out[b] and 0 <= out[a] < MIXED["vocab"]
+    eng.close()
+
+
+def test_generation_right_behind_a_step_of_several_prompts(tmp_path):
+    """the decode step is captured after a step of three long prompts: its launches must be shaped for one row, and replay on every slot"""
+    w = fx.random_weights(MIXED, 71)
+    eng = engine_for(tmp_path, MIXED, w, queries=4)
+    prompts = [tokens_for(MIXED, n, 72 + n) for n in (60, 41, 100)]
+    qs = [eng.add_query(p) for p in prompts]
+    eng.infer()
+    for q in qs[:2]:
+        eng.remove_query(q)
+    short = tokens_for(MIXED, 3, 79)
+    for prompt in (short, prompts[1], short):
+        q = eng.add_query(prompt)
+        gen, _ = eng.generate(q, 8)
+        eng.remove_query(q)
+        want = oracle_logits(MIXED, w, prompt + gen)
+        for i, tok in enumerate(gen):
+            row = want[len(prompt) - 1 + i]
+            top2 = np.sort(row)[-2:]
+            if top2[1] - top2[0] > 1e-3 * np.abs(row).max():
+                assert tok == int(row.argmax()), (len(prompt), i)
     eng.close()
 
 

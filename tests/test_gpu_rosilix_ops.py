@@ -125,9 +125,14 @@ def test_differential_attention_in_both_forms(H, G, d, dv, chunk, window):
             ldo = H * dv + (4 if rows % 2 else 3)
             out = torch.full((rows, ldo), 7.0, dtype=torch.float32, device="cuda")
             ia.check(L.ifa_attention_diff_f32(p(q), H * 2 * d, H, G, d, dv, c.scale, window, chunk, c.lam, 1.0 - c.diff, c.eps, p(g), H, p(d_), p(rs), rows, p(slots.table), k_off,
-                                              v_off, p(out), ldo, host_seqs(seqs), len(seqs), tile_min, ctx, p(ws), ws.numel() * 4, None)); sync()
+                                              v_off, p(out), None, ldo, host_seqs(seqs), len(seqs), tile_min, ctx, p(ws), ws.numel() * 4, None)); sync()
             got, r = out.cpu().numpy(), 0
             assert np.all(got[:, H * dv:] == 7.0)
+            if tile_min == 1 and L.ifa_attention_diff_tile_fits(d, dv):          # the same in bfloat16
+                half = torch.zeros((rows, ldo), dtype=torch.int16, device="cuda")
+                ia.check(L.ifa_attention_diff_f32(p(q), H * 2 * d, H, G, d, dv, c.scale, window, chunk, c.lam, 1.0 - c.diff, c.eps, p(g), H, p(d_), p(rs), rows, p(slots.table), k_off,
+                                                  v_off, None, p(half), ldo, host_seqs(seqs), len(seqs), tile_min, ctx, p(ws), ws.numel() * 4, None)); sync()
+                assert np.array_equal((half.cpu().numpy().view(np.uint16).astype(np.uint32) << 16).view(np.float32)[:, :H * dv], bf16_round(got[:, :H * dv]))
             for s, n, _ in step:
                 # (a head whose two maps nearly cancel is small before its norm: rounding relative to the norm's gain)
                 assert near(got[r:r + n, :H * dv], want[s][at[s]:at[s] + n], 1e-4), (tile_min, s, at[s], n)
@@ -168,7 +173,7 @@ def test_differential_attention_without_a_gate_and_decode_shares():
             q = dev32(np.stack([c.q[i % 3][ends[i]].reshape(-1) for i in batch]))
             ws = torch.full((rows * H * shares * 2 * (dv + 2),), float("nan"), dtype=torch.float32, device="cuda")
             out = torch.zeros((rows, H * dv), dtype=torch.float32, device="cuda")
-            ia.check(L.ifa_attention_diff_f32(p(q), H * 2 * d, H, G, d, dv, c.scale, 0, 0, c.lam, 1.0, c.eps, None, 0, p(d_), p(rs), rows, p(slots.table), 0, T * kw, p(out), H * dv,
+            ia.check(L.ifa_attention_diff_f32(p(q), H * 2 * d, H, G, d, dv, c.scale, 0, 0, c.lam, 1.0, c.eps, None, 0, p(d_), p(rs), rows, p(slots.table), 0, T * kw, p(out), None, H * dv,
                                               host_seqs(seqs), rows, 16, 64 * shares, p(ws), ws.numel() * 4, None)); sync()
             assert near(out.cpu().numpy(), np.stack([want[i] for i in batch]), 3e-5), (shares, len(batch))
 
@@ -180,7 +185,7 @@ def test_differential_attention_declines_bad_arguments():
     d_, rs, rows = seq_tables([(1, 0, 0)])
 
     def rc(H=2, G=1, d=8, dv=8, ws_bytes=4096, ldq=32):
-        return L.ifa_attention_diff_f32(p(z), ldq, H, G, d, dv, 1.0, 0, 0, 0.5, 0.5, 1e-5, None, 0, p(d_), p(rs), 1, p(slots.table), 0, 1024, p(z), H * dv, host_seqs([(1, 0, 0)]), 1, 16, 4,
+        return L.ifa_attention_diff_f32(p(z), ldq, H, G, d, dv, 1.0, 0, 0, 0.5, 0.5, 1e-5, None, 0, p(d_), p(rs), 1, p(slots.table), 0, 1024, p(z), None, H * dv, host_seqs([(1, 0, 0)]), 1, 16, 4,
                                         p(z), ws_bytes, None)
     assert rc() == 0
     for bad in (dict(H=3, G=2), dict(d=0), dict(d=1025, ldq=9000), dict(dv=0), dict(ws_bytes=16), dict(ldq=31)):
@@ -238,7 +243,7 @@ def test_latent_attention_with_sinks_over_own_and_shared_rows(H, dn, dr, dv, R):
                     ia.check(L.ifa_linear_bf16w(p(ukd), H * dn, R, lat, CR, tot, None, None, 1.0, 0, 1, p(kx), H * dn, 0, 0, None))
                     ia.check(L.ifa_linear_bf16w(p(uvd), OV, R, lat, CR, tot, None, None, 1.0, 0, 1, p(vx), OV, 0, 0, None))
                     ia.check(L.ifa_attention_latent_tile_sinks_f32(0, p(qd), QD, H, dn, dr, dv, R, scale, p(sd), p(kx), H * dn, p(vx), OV, p(devi([0])), p(gd), H, p(d), host_seqs(seqs), 1,
-                                                                   p(slots.table), 0, p(out), OV, None))
+                                                                   p(slots.table), 0, p(out), None, OV, None))
                 else:
                     qa, ol = torch.zeros((rows, H * CR), dtype=torch.float32, device="cuda"), torch.zeros((rows, H * R), dtype=torch.float32, device="cuda")
                     ws = torch.zeros(rows * H * 4 * (R + 2), dtype=torch.float32, device="cuda")
@@ -247,6 +252,11 @@ def test_latent_attention_with_sinks_over_own_and_shared_rows(H, dn, dr, dv, R):
                     ia.check(L.ifa_latent_expand_out_gated_f32(0, p(ol), H * R, R, H, dv, R, p(uvd), p(gd), H, rows, p(out), OV, None))
                 sync()
                 assert near(out.cpu().numpy(), want[at:at + n], 3e-5), (tiled, own, at, n)
+                if tiled:          # the same in bfloat16
+                    half = torch.zeros((rows, OV), dtype=torch.int16, device="cuda")
+                    ia.check(L.ifa_attention_latent_tile_sinks_f32(0, p(qd), QD, H, dn, dr, dv, R, scale, p(sd), p(kx), H * dn, p(vx), OV, p(devi([0])), p(gd), H, p(d), host_seqs(seqs), 1,
+                                                                   p(slots.table), 0, None, p(half), OV, None)); sync()
+                    assert np.array_equal((half.cpu().numpy().view(np.uint16).astype(np.uint32) << 16).view(np.float32), bf16_round(out.cpu().numpy()))
             at += n
         assert at == T
 
@@ -329,6 +339,17 @@ def test_norms_on_both_sides_with_plain_weights(rows, cols):
     assert near(xd.cpu().numpy(), new) and near(h.cpu().numpy(), orc.norm(new, orc.f64(wb), eps), 5e-6)
     ia.check(L.ifa_rmsnorm_offset_f32(p(xd), cols, rows, cols, p(devbf(wb)), 0.0, eps, 0, p(h), cols, None)); sync()
     assert near(h.cpu().numpy(), orc.norm(new, orc.f64(wb), eps), 5e-6)
+    # h in bfloat16, with and without the update in front
+    half = torch.zeros((rows, cols), dtype=torch.int16, device="cuda")
+    for upd in (0, 1):
+        xd = dev32(new if not upd else x)
+        rc = L.ifa_norm_add_norm_to_bf16(p(xd), cols, rows, cols, p(dev32(m)) if upd else None, cols, p(devbf(wa)) if upd else None, p(devbf(wb)), 0.0, eps, p(half), cols, None); sync()
+        if cols % 4 or cols > 8192:
+            assert rc != 0
+            continue
+        ia.check(rc)
+        got = (half.cpu().numpy().view(np.uint16).astype(np.uint32) << 16).view(np.float32)
+        assert near(xd.cpu().numpy(), new) and np.abs(got - orc.norm(new, orc.f64(wb), eps)).max() < 2 ** -7 * max(1.0, np.abs(got).max())
 
 
 def test_scaled_embedding():
